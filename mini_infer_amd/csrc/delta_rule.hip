@@ -4,6 +4,7 @@
 //   short_conv        y[t, c] = silu(sum_j w[c, j] * x[t - (taps-1) + j, c]) over the rows of each
 //                     request; rows before a portion's first come from the request's tail (its
 //                     last taps-1 inputs, kept in its state slot), zeros at a sequence's start.
+//                     `add_input`: y = x[t, c] + sum instead of silu(sum).
 //   short_conv_tail   the tail after the portion (runs after short_conv: it overwrites what
 //                     that one reads).
 //   gated_delta       per request and head, token by token (S is dim x vdim, float32):
@@ -31,11 +32,27 @@
 namespace {
 
 template <typename T>
+struct ConvSum {
+  using type = float;
+};
+template <>
+struct ConvSum<float> {
+  using type = double;
+};
+
+__device__ __forceinline__ float conv_result(float sum, float now, int add_input) {
+  return add_input ? now + sum : sum * mi_logistic(sum);
+}
+__device__ __forceinline__ float conv_result(double sum, float now, int add_input) {
+  return add_input ? (float)((double)now + sum) : (float)(sum / (1.0 + exp(-sum)));
+}
+
+template <typename T>
 __global__ __launch_bounds__(256) void short_conv_kernel(
     const T* __restrict__ x, int64_t x_stride, const float* __restrict__ w, const T* __restrict__ tail,
     int64_t tail_stride, const int* __restrict__ cu, const int* __restrict__ slots,
     const int* __restrict__ token_request, T* __restrict__ y, int64_t y_stride, int channels, int taps,
-    int num_slots, int row0, const float* __restrict__ bias) {
+    int num_slots, int row0, const float* __restrict__ bias, int add_input) {
   const int t = row0 + blockIdx.y;
   const int c = blockIdx.x * blockDim.x + threadIdx.x;
   if (c >= channels) return;
@@ -53,7 +70,7 @@ __global__ __launch_bounds__(256) void short_conv_kernel(
       const float v = at >= 0 ? x[(int64_t)(t - back + j) * x_stride + c] : mine[(int64_t)(back + at) * channels + c];
       sum = fma((double)wc[j], (double)v, sum);
     }
-    y[(int64_t)t * y_stride + c] = (float)(sum / (1.0 + exp(-sum)));
+    y[(int64_t)t * y_stride + c] = conv_result(sum, x[(int64_t)t * x_stride + c], add_input);
   } else {
     float sum = start;
     for (int j = 0; j < taps; ++j) {
@@ -62,7 +79,63 @@ __global__ __launch_bounds__(256) void short_conv_kernel(
                               : to_f32(mine[(int64_t)(back + at) * channels + c]);
       sum = fmaf(wc[j], v, sum);
     }
-    y[(int64_t)t * y_stride + c] = from_f32<T>(sum * mi_logistic(sum));
+    y[(int64_t)t * y_stride + c] = from_f32<T>(conv_result(sum, to_f32(x[(int64_t)t * x_stride + c]), add_input));
+  }
+}
+
+// Long steps whose rows are read four columns at a time: a thread takes CONV_RUN consecutive rows of
+// four channels with the last taps-1 inputs in registers, so a row is read once per run and not once per
+// tap.  The arithmetic is that of short_conv_kernel, term by term.
+#define CONV_RUN 16
+
+template <typename T, int TAPS>
+__global__ __launch_bounds__(256) void short_conv_runs_kernel(
+    const T* __restrict__ x, int64_t x_stride, const float* __restrict__ w, const T* __restrict__ tail,
+    int64_t tail_stride, const int* __restrict__ cu, const int* __restrict__ slots,
+    const int* __restrict__ token_request, T* __restrict__ y, int64_t y_stride, int channels, int num_tokens,
+    int num_slots, const float* __restrict__ bias, int add_input) {
+  using A = typename ConvSum<T>::type;
+  constexpr int BACK = TAPS - 1;
+  const int c = (blockIdx.x * blockDim.x + threadIdx.x) * 4;
+  if (c >= channels) return;
+  const int t0 = blockIdx.y * CONV_RUN, t1 = min(num_tokens, t0 + CONV_RUN);
+  A wc[TAPS][4], start[4];
+  float window[BACK > 0 ? BACK : 1][4];  // window[j]: the input `BACK - j` rows ago
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    start[e] = bias ? (A)bias[c + e] : (A)0;
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) wc[j][e] = (A)w[(int64_t)(c + e) * TAPS + j];
+  }
+  int of = -1;  // the request the window belongs to
+  for (int t = t0; t < t1; ++t) {
+    const int b = token_request[t];
+    if (b != of) {
+      of = b;
+      const int i = t - cu[b];
+      const int slot = slots[b];
+      const T* mine = tail + (int64_t)((slot < 0 || slot >= num_slots) ? num_slots : slot) * tail_stride;
+#pragma unroll
+      for (int j = 0; j < BACK; ++j) {
+        const int at = i - BACK + j;
+        if (at >= 0) mi_load_cols<T, 4>(x + (int64_t)(t - BACK + j) * x_stride + c, window[j]);
+        else mi_load_cols<T, 4>(mine + (int64_t)(BACK + at) * channels + c, window[j]);
+      }
+    }
+    float now[4], made[4];
+    mi_load_cols<T, 4>(x + (int64_t)t * x_stride + c, now);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      A sum = start[e];
+#pragma unroll
+      for (int j = 0; j < BACK; ++j) sum = fma(wc[j][e], (A)window[j][e], sum);
+      sum = fma(wc[BACK][e], (A)now[e], sum);
+      made[e] = conv_result(sum, now[e], add_input);
+#pragma unroll
+      for (int j = 0; j + 1 < BACK; ++j) window[j][e] = window[j + 1][e];
+      if constexpr (BACK > 0) window[BACK - 1][e] = now[e];
+    }
+    mi_store_cols<T, 4>(y + (int64_t)t * y_stride + c, made);
   }
 }
 
@@ -94,7 +167,7 @@ template <typename T>
 __global__ __launch_bounds__(256) void short_conv_walk_kernel(
     const T* __restrict__ x, int64_t x_stride, const float* __restrict__ w, T* __restrict__ tail, int64_t tail_stride,
     const int* __restrict__ cu, const int* __restrict__ slots, T* __restrict__ y, int64_t y_stride, int channels, int taps,
-    int num_slots, const float* __restrict__ bias) {
+    int num_slots, const float* __restrict__ bias, int add_input) {
   const int b = blockIdx.y;
   const int c = blockIdx.x * blockDim.x + threadIdx.x;
   if (c >= channels) return;
@@ -118,14 +191,14 @@ __global__ __launch_bounds__(256) void short_conv_walk_kernel(
       for (int j = 0; j < DELTA_MAX_TAPS; ++j)
         if (j < back) sum = fma((double)wc[j], (double)window[j], sum);
       sum = fma((double)w[(int64_t)c * taps + back], (double)now, sum);
-      y[(int64_t)t * y_stride + c] = (float)(sum / (1.0 + exp(-sum)));
+      y[(int64_t)t * y_stride + c] = conv_result(sum, now, add_input);
     } else {
       float sum = start;
 #pragma unroll
       for (int j = 0; j < DELTA_MAX_TAPS; ++j)
         if (j < back) sum = fmaf(wc[j], window[j], sum);
       sum = fmaf(w[(int64_t)c * taps + back], now, sum);
-      y[(int64_t)t * y_stride + c] = from_f32<T>(sum * mi_logistic(sum));
+      y[(int64_t)t * y_stride + c] = from_f32<T>(conv_result(sum, now, add_input));
     }
 #pragma unroll
     for (int j = 0; j < DELTA_MAX_TAPS - 1; ++j)
@@ -416,11 +489,11 @@ static void delta_layout(int dim, int vdim, int* lanes, int* rows) {
 
 // x: the projections [tokens, >= channels] (row stride); w float32 [channels, taps]; tail
 // [slots + 1, (taps-1) * channels] in the element type (row stride); y [tokens, channels]; bias float32
-// [channels] or null.
+// [channels] or null; add_input: y = x + sum instead of silu(sum).
 extern "C" int mi_short_conv(int dtype, const void* x, int64_t x_stride, const float* w, void* tail,
                              int64_t tail_stride, const int* cu, const int* slots, const int* token_request,
                              void* y, int64_t y_stride, int num_tokens, int num_requests, int channels, int taps,
-                             int num_slots, const float* bias, hipStream_t stream) {
+                             int num_slots, const float* bias, int add_input, hipStream_t stream) {
   MI_REQUIRE(num_tokens >= 0 && num_requests >= 0 && channels > 0, "short_conv: bad sizes tokens=%d requests=%d channels=%d",
              num_tokens, num_requests, channels);
   MI_REQUIRE(taps >= 1 && taps <= DELTA_MAX_TAPS, "short_conv: taps=%d must be 1..%d", taps, DELTA_MAX_TAPS);
@@ -435,23 +508,43 @@ extern "C" int mi_short_conv(int dtype, const void* x, int64_t x_stride, const f
     dim3 grid(blocks, num_requests);
     if (dtype == MI_F32)
       short_conv_walk_kernel<float><<<grid, 256, 0, stream>>>((const float*)x, x_stride, w, (float*)tail, tail_stride, cu, slots,
-                                                              (float*)y, y_stride, channels, taps, num_slots, bias);
+                                                              (float*)y, y_stride, channels, taps, num_slots, bias, add_input);
     else
       short_conv_walk_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)x, x_stride, w, (bf16_t*)tail, tail_stride, cu,
-                                                               slots, (bf16_t*)y, y_stride, channels, taps, num_slots, bias);
+                                                               slots, (bf16_t*)y, y_stride, channels, taps, num_slots, bias, add_input);
     MI_CHECK_LAUNCH("short_conv_walk");
     return MI_OK;
   }
-  for (int first = 0; first < num_tokens; first += 65535) {
+  const size_t elem = dtype == MI_F32 ? 4 : 2;
+  const bool runs = taps >= 2 && taps <= 4 && channels % 4 == 0 && x_stride % 4 == 0 && y_stride % 4 == 0 && tail_stride % 4 == 0 &&
+                    ((uintptr_t)x | (uintptr_t)y | (uintptr_t)tail) % (4 * elem) == 0 && ceil_div(num_tokens, CONV_RUN) <= 65535;
+  if (runs) {
+    dim3 grid(ceil_div(channels, 1024), ceil_div(num_tokens, CONV_RUN));
+#define MI_CONV_RUNS(T, TAPS)                                                                                            \
+  short_conv_runs_kernel<T, TAPS><<<grid, 256, 0, stream>>>((const T*)x, x_stride, w, (const T*)tail, tail_stride, cu,   \
+                                                            slots, token_request, (T*)y, y_stride, channels, num_tokens, \
+                                                            num_slots, bias, add_input)
+    if (dtype == MI_F32) {
+      if (taps == 2) MI_CONV_RUNS(float, 2);
+      else if (taps == 3) MI_CONV_RUNS(float, 3);
+      else MI_CONV_RUNS(float, 4);
+    } else {
+      if (taps == 2) MI_CONV_RUNS(bf16_t, 2);
+      else if (taps == 3) MI_CONV_RUNS(bf16_t, 3);
+      else MI_CONV_RUNS(bf16_t, 4);
+    }
+#undef MI_CONV_RUNS
+  }
+  for (int first = runs ? num_tokens : 0; first < num_tokens; first += 65535) {
     dim3 grid(blocks, min(65535, num_tokens - first));
     if (dtype == MI_F32)
       short_conv_kernel<float><<<grid, 256, 0, stream>>>((const float*)x, x_stride, w, (const float*)tail, tail_stride, cu,
                                                          slots, token_request, (float*)y, y_stride, channels, taps,
-                                                         num_slots, first, bias);
+                                                         num_slots, first, bias, add_input);
     else
       short_conv_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)x, x_stride, w, (const bf16_t*)tail, tail_stride,
                                                           cu, slots, token_request, (bf16_t*)y, y_stride, channels, taps,
-                                                          num_slots, first, bias);
+                                                          num_slots, first, bias, add_input);
   }
   MI_CHECK_LAUNCH("short_conv");
   if (taps > 1) {

@@ -10,6 +10,9 @@
 //   gated_mul
 //       out[t, i] = act(a[t, i]) * b[t, i] for act = silu, the tanh form of gelu, or the logistic
 //       function; a and b are column ranges of rows that may be strided.
+//   gate_heads
+//       out[t, h * width + d] = x[t, h * x_head_width + d] * logistic(gate[t, h * width + d]): heads that
+//       lie apart in their rows, packed and gated.
 #include "common.h"
 
 #include <math.h>
@@ -139,7 +142,41 @@ __global__ __launch_bounds__(256) void gated_mul_vec4_kernel(const T* __restrict
   *reinterpret_cast<Four*>(out + (int64_t)t * out_stride + i) = ov;
 }
 
+template <typename T>
+__global__ __launch_bounds__(256) void gate_heads_kernel(const T* __restrict__ x, int64_t x_stride, int x_head_width,
+                                                         const T* __restrict__ gate, int64_t gate_stride, T* __restrict__ out,
+                                                         int64_t out_stride, int heads, int width) {
+  const int t = blockIdx.x;
+  for (int e = blockIdx.y * blockDim.x + threadIdx.x; e < heads * width; e += gridDim.y * blockDim.x) {
+    const int h = e / width, d = e % width;
+    out[(int64_t)t * out_stride + e] = from_f32<T>(act_times<T>(ACT_LOGISTIC, to_f32(gate[(int64_t)t * gate_stride + e]),
+                                                                to_f32(x[(int64_t)t * x_stride + (int64_t)h * x_head_width + d])));
+  }
+}
+
 }  // namespace
+
+// x: rows of heads x_head_width columns apart of which the first `width` are read; gate, out: [tokens, heads * width].
+extern "C" int mi_gate_heads(int dtype, const void* x, int64_t x_stride, int x_head_width, const void* gate,
+                             int64_t gate_stride, void* out, int64_t out_stride, int num_tokens, int heads, int width,
+                             hipStream_t stream) {
+  MI_REQUIRE(num_tokens >= 0 && heads > 0 && width > 0 && x_head_width >= width, "gate_heads: bad sizes tokens=%d heads=%d width=%d", num_tokens,
+             heads, width);
+  MI_REQUIRE(x_stride >= (int64_t)(heads - 1) * x_head_width + width && gate_stride >= (int64_t)heads * width &&
+                 out_stride >= (int64_t)heads * width && (int64_t)heads * width <= 0x3fffffff,
+             "gate_heads: row strides shorter than a row");
+  MI_REQUIRE(dtype == MI_F32 || dtype == MI_BF16, "gate_heads: unknown dtype %d", dtype);
+  if (num_tokens == 0) return MI_OK;
+  dim3 grid(num_tokens, min(8, ceil_div(heads * width, 1024)));
+  if (dtype == MI_F32)
+    gate_heads_kernel<float><<<grid, 256, 0, stream>>>((const float*)x, x_stride, x_head_width, (const float*)gate, gate_stride,
+                                                       (float*)out, out_stride, heads, width);
+  else
+    gate_heads_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)x, x_stride, x_head_width, (const bf16_t*)gate, gate_stride,
+                                                        (bf16_t*)out, out_stride, heads, width);
+  MI_CHECK_LAUNCH("gate_heads");
+  return MI_OK;
+}
 
 // qkv rows: [q heads | k heads | v heads], q and k heads head_dim wide, v heads v_head_dim wide.
 // q_weight, k_weight: float32 [head_dim] or null (that side is not normed).

@@ -2,12 +2,14 @@
 // router, and the results are added with the router's weights.
 //
 //   route_top_k         per token: logits z = R x (R float32, sums float32; 64-bit in the 32-bit
-//                       engine), scores s = softmax(z) over all router outputs, choice = s +
-//                       correction, the `top` largest choices (the lower index wins a tie); leaves
-//                       the chosen indices and their weights s * route_scale (not renormalized),
-//                       and, where a gate row is given, logistic(gate . x) for a shared expert.
-//   expert_gate_up      few rows: for every (token, chosen expert) pair the expert's stacked
-//                       gate|up product and silu(gate) * up, the weights read by expert index.
+//                       engine), scores s = softmax(z) over all router outputs or logistic(z) one by
+//                       one, choice = s + correction, the `top` largest choices (the lower index wins
+//                       a tie; logistic scores without a correction are ranked by z itself, of which
+//                       they are a rising function); leaves the chosen indices and their weights
+//                       s * route_scale (not renormalized), and, where a gate row is given,
+//                       logistic(gate . x) for a shared expert.
+//   expert_gate_up      few rows: for every (token, chosen expert) pair the expert's first product and
+//                       its activation, the weights read by expert index.
 //   expert_down_combine few rows: y[t] = sum_k w[t, k] * (W_down[e_k] act[t, k])  (+ shared_gate[t] *
 //                       shared[t]); a chosen index past the real experts is an identity expert,
 //                       whose output is the token's input row itself.
@@ -15,7 +17,13 @@
 //                       by expert (sorted by expert; `where` maps a pair to its sorted row).
 //
 // Expert weights are stacked: gate|up [experts, 2 * ff, width] (an expert's gate rows, then its up
-// rows), down [experts, width, ff].
+// rows), or up [experts, ff, width] where experts have no gate; down [experts, width, ff].
+//
+// What the first product of an expert ends with (MODE):
+//   EXPERT_SILU_GATED    silu(gate . x) * (up . x)
+//   EXPERT_SQUARED_RELU  relu(w * (up . x))^2, w the pair's router weight: the weight multiplies what the
+//                        expert reads, and W (w x) = w (W x), so no weighted copy of the rows is made
+// and EXPERT_PLAIN, the second product alone.
 #include "common.h"
 
 #include <math.h>
@@ -43,13 +51,30 @@ __device__ __forceinline__ double exp_of(double z) { return exp(z); }
 
 #define MI_ROUTER_MAX_OUTPUTS 1024
 
+enum ExpertMode { EXPERT_PLAIN = 0, EXPERT_SILU_GATED = 1, EXPERT_SQUARED_RELU = 2 };
+
+// what is written for a feature whose sums are `a` (and, gated, `b`), float32 or 64-bit; `weight` is the pair's
+template <typename T, int MODE, typename A>
+__device__ __forceinline__ T expert_feature(A a, A b, A weight) {
+  if constexpr (MODE == EXPERT_SILU_GATED) {
+    // the two products as the element type holds them, then silu(gate) * up
+    const A g = (A)to_f32(from_f32<T>((float)a)), u = (A)to_f32(from_f32<T>((float)b));
+    return from_f32<T>((float)(g / ((A)1 + exp_of(-g)) * u));
+  } else if constexpr (MODE == EXPERT_SQUARED_RELU) {
+    const A z = weight * a;
+    return from_f32<T>((float)(z > (A)0 ? z * z : (A)0));
+  } else {
+    return from_f32<T>((float)a);
+  }
+}
+
 // R tokens a block: their rows wait in LDS while every wave walks router rows (16 bytes a lane, each
 // router row read once for all R tokens), then thread r ranks token r's outputs.
 template <typename T, int R>
 __global__ __launch_bounds__(1024) void route_top_k_kernel(
     const T* __restrict__ x, int64_t x_stride, const float* __restrict__ router, const float* __restrict__ correction,
     const float* __restrict__ gate_row, int* __restrict__ chosen, float* __restrict__ weights,
-    float* __restrict__ shared_gate, int num_tokens, int width, int outputs, int top, float route_scale) {
+    float* __restrict__ shared_gate, int num_tokens, int width, int outputs, int top, float route_scale, int logistic) {
   using A = typename SumOf<T>::type;
   extern __shared__ __align__(16) unsigned char lds_bytes[];
   A* z = reinterpret_cast<A*>(lds_bytes);                         // [R][outputs + 1]
@@ -107,6 +132,23 @@ __global__ __launch_bounds__(1024) void route_top_k_kernel(
   if (r >= R || t >= num_tokens) return;
   A* mine = z + r * (outputs + 1);
   if (gate_row != nullptr) shared_gate[t] = (float)((A)1 / ((A)1 + exp_of(-mine[outputs])));
+  if (logistic) {
+    const A taken = -(A)INFINITY;
+    for (int k = 0; k < top; ++k) {
+      int best = -1;
+      A best_choice = 0;
+      for (int e = 0; e < outputs; ++e) {
+        if (mine[e] == taken) continue;
+        const A choice = correction != nullptr ? (A)1 / ((A)1 + exp_of(-mine[e])) + (A)correction[e] : mine[e];
+        if (best < 0 || choice > best_choice) best = e, best_choice = choice;
+      }
+      if (best < 0) best = 0;  // (logits that are no numbers, or more infinite ones than there are choices)
+      chosen[(int64_t)t * top + k] = best;
+      weights[(int64_t)t * top + k] = (float)((A)route_scale / ((A)1 + exp_of(-mine[best])));
+      mine[best] = taken;
+    }
+    return;
+  }
   A most = mine[0];
   for (int e = 1; e < outputs; ++e) most = mine[e] > most ? mine[e] : most;
   A sum = 0;
@@ -150,10 +192,10 @@ __device__ __forceinline__ A dot_lds(const T* __restrict__ w, const T* __restric
 
 #define MI_EXPERT_FEATURES 16  // features (or columns) a block of four waves makes
 
-template <typename T>
+template <typename T, int MODE>
 __global__ __launch_bounds__(256) void expert_gate_up_kernel(
     const T* __restrict__ x, int64_t x_stride, const T* __restrict__ gate_up, const int* __restrict__ chosen,
-    T* __restrict__ act, int width, int ff, int experts, int top) {
+    const float* __restrict__ pair_weight, T* __restrict__ act, int width, int ff, int experts, int top) {
   using A = typename SumOf<T>::type;
   extern __shared__ __align__(16) unsigned char lds_bytes[];
   T* row = reinterpret_cast<T*>(lds_bytes);
@@ -164,16 +206,14 @@ __global__ __launch_bounds__(256) void expert_gate_up_kernel(
   for (int c = threadIdx.x; c < width; c += blockDim.x) row[c] = src[c];
   __syncthreads();
   const int wave = threadIdx.x / MI_WAVE, lane = threadIdx.x % MI_WAVE, waves = blockDim.x / MI_WAVE;
-  const T* w = gate_up + (int64_t)e * 2 * ff * width;
+  constexpr bool GATED = MODE == EXPERT_SILU_GATED;
+  const T* w = gate_up + (int64_t)e * (GATED ? 2 : 1) * ff * width;
+  const A weight = MODE == EXPERT_SQUARED_RELU && pair_weight != nullptr ? (A)pair_weight[pair] : (A)1;
   const int first = blockIdx.y * MI_EXPERT_FEATURES;
   for (int f = first + wave; f < min(first + MI_EXPERT_FEATURES, ff); f += waves) {
     const A g = dot_lds<T, A>(w + (int64_t)f * width, row, width, lane);
-    const A u = dot_lds<T, A>(w + (int64_t)(ff + f) * width, row, width, lane);
-    if (lane == 0) {
-      // the two products as the element type holds them, then silu(g) * u
-      const A gr = (A)to_f32(from_f32<T>((float)g)), ur = (A)to_f32(from_f32<T>((float)u));
-      act[(int64_t)pair * ff + f] = from_f32<T>((float)(gr / ((A)1 + exp_of(-gr)) * ur));
-    }
+    const A u = GATED ? dot_lds<T, A>(w + (int64_t)(ff + f) * width, row, width, lane) : (A)0;
+    if (lane == 0) act[(int64_t)pair * ff + f] = expert_feature<T, MODE, A>(g, u, weight);
   }
 }
 
@@ -197,7 +237,7 @@ __global__ __launch_bounds__(256) void expert_down_combine_kernel(
     A sum = 0;
     for (int k = 0; k < top; ++k) {
       const int e = chosen[(int64_t)t * top + k];
-      const A weight = (A)weights[(int64_t)t * top + k];
+      const A weight = weights != nullptr ? (A)weights[(int64_t)t * top + k] : (A)1;
       if (e >= experts) {
         sum += weight * (A)to_f32(x[(int64_t)t * x_stride + c]);
       } else if (e >= 0) {
@@ -228,7 +268,7 @@ __global__ __launch_bounds__(256) void expert_combine_kernel(
       const T* src = e >= experts ? x + (int64_t)t * x_stride : made + (int64_t)(where != nullptr ? where[pair] : pair) * width;
       float v[VEC];
       mi_load_cols<T, VEC>(src + c, v);
-      const A weight = (A)weights[pair];
+      const A weight = weights != nullptr ? (A)weights[pair] : (A)1;
 #pragma unroll
       for (int j = 0; j < VEC; ++j) sum[j] += weight * (A)v[j];
     }
@@ -289,12 +329,13 @@ __global__ __launch_bounds__(256) void expert_sort_kernel(const int* __restrict_
   }
 }
 
-template <typename T, int R, bool GATED>
+template <typename T, int R, int MODE>
 __global__ __launch_bounds__(256) void expert_rows_kernel(
     const T* __restrict__ src, int64_t src_stride, int src_div, const T* __restrict__ weight, int64_t expert_stride,
-    const int* __restrict__ listed, const int* __restrict__ first, T* __restrict__ out, int64_t out_stride, int k_dim,
-    int features) {
+    const int* __restrict__ listed, const int* __restrict__ first, const float* __restrict__ pair_weight,
+    T* __restrict__ out, int64_t out_stride, int k_dim, int features) {
   using A = typename SumOf<T>::type;
+  constexpr bool GATED = MODE == EXPERT_SILU_GATED;
   constexpr int FW = 4;             // features a wave
   constexpr int WR = GATED ? 2 : 1;  // weight rows a feature
   constexpr int V = 16 / sizeof(T);
@@ -356,14 +397,9 @@ __global__ __launch_bounds__(256) void expert_rows_kernel(
         A a = lanes_total(sum[f][0][r]);
         A b = GATED ? lanes_total(sum[f][WR - 1][r]) : (A)0;
         if (lane == 0 && r < n && f0 + f < features) {
-          T* o = out + (int64_t)listed[chunk + r] * out_stride + f0 + f;
-          if constexpr (GATED) {
-            // the two products as the element type holds them, then silu(gate) * up
-            const A gr = (A)to_f32(from_f32<T>((float)a)), ur = (A)to_f32(from_f32<T>((float)b));
-            *o = from_f32<T>((float)(gr / ((A)1 + exp_of(-gr)) * ur));
-          } else {
-            *o = from_f32<T>((float)a);
-          }
+          const int pair = listed[chunk + r];
+          const A pw = MODE == EXPERT_SQUARED_RELU && pair_weight != nullptr ? (A)pair_weight[pair] : (A)1;
+          out[(int64_t)pair * out_stride + f0 + f] = expert_feature<T, MODE, A>(a, b, pw);
         }
       }
   }
@@ -378,11 +414,12 @@ __global__ __launch_bounds__(256) void expert_rows_kernel(
 // pair col.  Needs K a multiple of 32.
 typedef float f32x4_e __attribute__((ext_vector_type(4)));
 
-template <bool GATED>
+template <int MODE>
 __global__ __launch_bounds__(256) void expert_rows_mfma_kernel(
     const bf16_t* __restrict__ src, int64_t src_stride, int src_div, const bf16_t* __restrict__ weight,
-    int64_t expert_stride, const int* __restrict__ listed, const int* __restrict__ first, bf16_t* __restrict__ out,
-    int64_t out_stride, int k_dim, int features) {
+    int64_t expert_stride, const int* __restrict__ listed, const int* __restrict__ first,
+    const float* __restrict__ pair_weight, bf16_t* __restrict__ out, int64_t out_stride, int k_dim, int features) {
+  constexpr bool GATED = MODE == EXPERT_SILU_GATED;
   __shared__ f32x4_e meet[GATED ? 2 : 1][3][MI_WAVE];
   const int e = blockIdx.y;  // (feature tiles run fastest: a chosen expert's blocks follow one another and spread over all XCDs)
   const int begin = first[e], end = first[e + 1];
@@ -443,17 +480,11 @@ __global__ __launch_bounds__(256) void expert_rows_mfma_kernel(
         if constexpr (GATED) acc_u += meet[1][w][lane];
       }
       bf16_t* o = out + (int64_t)pair * out_stride;
+      const float pw = MODE == EXPERT_SQUARED_RELU && pair_weight != nullptr ? pair_weight[pair] : 1.f;
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int f = f0 + 4 * quad + r;
-        if (f >= features) continue;
-        if constexpr (GATED) {
-          // the two products as bfloat16 holds them, then silu(gate) * up
-          const float g = to_f32(from_f32<bf16_t>(acc_g[r])), u = to_f32(from_f32<bf16_t>(acc_u[r]));
-          o[f] = from_f32<bf16_t>(g / (1.f + expf(-g)) * u);
-        } else {
-          o[f] = from_f32<bf16_t>(acc_g[r]);
-        }
+        if (f < features) o[f] = expert_feature<bf16_t, MODE, float>(acc_g[r], acc_u[r], pw);
       }
     }
   }
@@ -464,11 +495,12 @@ __global__ __launch_bounds__(256) void expert_rows_mfma_kernel(
 // reads its 16 weight rows once (16 bytes a lane) and the four row tiles' input rows (the same for the
 // block's four waves, so three of four reads hit the cache), and makes 4 (gated: 8) MFMA 16x16x32.  An
 // expert's weights are read once per 64 of its rows and its rows once per 64 of its features.
-template <bool GATED>
+template <int MODE>
 __global__ __launch_bounds__(256) void expert_tiles_mfma_kernel(
     const bf16_t* __restrict__ src, int64_t src_stride, int src_div, const bf16_t* __restrict__ weight,
-    int64_t expert_stride, const int* __restrict__ listed, const int* __restrict__ first, bf16_t* __restrict__ out,
-    int64_t out_stride, int k_dim, int features) {
+    int64_t expert_stride, const int* __restrict__ listed, const int* __restrict__ first,
+    const float* __restrict__ pair_weight, bf16_t* __restrict__ out, int64_t out_stride, int k_dim, int features) {
+  constexpr bool GATED = MODE == EXPERT_SILU_GATED;
   constexpr int RT = 4;  // row tiles of 16
   const int e = blockIdx.y;
   const int begin = first[e], end = first[e + 1];
@@ -519,26 +551,32 @@ __global__ __launch_bounds__(256) void expert_tiles_mfma_kernel(
     for (int t = 0; t < RT; ++t) {
       if (pair[t] < 0) continue;
       bf16_t* o = out + (int64_t)pair[t] * out_stride;
+      const float pw = MODE == EXPERT_SQUARED_RELU && pair_weight != nullptr ? pair_weight[pair[t]] : 1.f;
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int f = f0 + 4 * quad + r;
-        if (f >= features) continue;
-        if constexpr (GATED) {
-          const float g = to_f32(from_f32<bf16_t>(acc_g[t][r])), u = to_f32(from_f32<bf16_t>(acc_u[t][r]));
-          o[f] = from_f32<bf16_t>(g / (1.f + expf(-g)) * u);
-        } else {
-          o[f] = from_f32<bf16_t>(acc_g[t][r]);
-        }
+        if (f < features) o[f] = expert_feature<bf16_t, MODE, float>(acc_g[t][r], acc_u[t][r], pw);
       }
     }
   }
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void weighted_squared_relu_kernel(const T* __restrict__ z, int64_t z_stride,
+                                                                    const float* __restrict__ weight, T* __restrict__ out,
+                                                                    int64_t out_stride, int width) {
+  using A = typename SumOf<T>::type;
+  const int row = blockIdx.x, i = blockIdx.y * blockDim.x + threadIdx.x;
+  if (i >= width) return;
+  out[(int64_t)row * out_stride + i] =
+      expert_feature<T, EXPERT_SQUARED_RELU, A>((A)to_f32(z[(int64_t)row * z_stride + i]), (A)0, (A)weight[row]);
 }
 
 }  // namespace
 
 extern "C" int mi_route_top_k(int dtype, const void* x, int64_t x_stride, const float* router, const float* correction,
                               const float* gate_row, int* chosen, float* weights, float* shared_gate, int num_tokens,
-                              int width, int outputs, int top, float route_scale, hipStream_t stream) {
+                              int width, int outputs, int top, float route_scale, int logistic, hipStream_t stream) {
   MI_REQUIRE(num_tokens >= 0 && width > 0 && x_stride >= width, "route_top_k: bad sizes tokens=%d width=%d", num_tokens, width);
   MI_REQUIRE(outputs > 0 && outputs <= MI_ROUTER_MAX_OUTPUTS && top > 0 && top <= outputs,
              "route_top_k: %d router outputs (at most %d) of which %d are chosen", outputs, MI_ROUTER_MAX_OUTPUTS, top);
@@ -555,7 +593,7 @@ extern "C" int mi_route_top_k(int dtype, const void* x, int64_t x_stride, const 
 #define MI_ROUTE(T, R)                                                                                               \
   route_top_k_kernel<T, R><<<blocks, threads, lds_for(R), stream>>>((const T*)x, x_stride, router, correction, gate_row, \
                                                                     chosen, weights, shared_gate, num_tokens, width,    \
-                                                                    outputs, top, route_scale)
+                                                                    outputs, top, route_scale, logistic)
   if (dtype == MI_F32) {
     if (per_block == 4) MI_ROUTE(float, 4);
     else if (per_block == 2) MI_ROUTE(float, 2);
@@ -570,23 +608,31 @@ extern "C" int mi_route_top_k(int dtype, const void* x, int64_t x_stride, const 
   return MI_OK;
 }
 
-// act: [num_tokens * top, ff]; rows of pairs whose expert is an identity expert are not written.
-extern "C" int mi_expert_gate_up(int dtype, const void* x, int64_t x_stride, const void* gate_up, const int* chosen,
-                                 void* act, int num_tokens, int width, int ff, int experts, int top, hipStream_t stream) {
+// act: [num_tokens * top, ff]; rows of pairs whose expert is an identity expert are not written.  mode: 1 silu
+// gated, 2 squared relu of the weighted product (pair_weight float32 [num_tokens * top] or null: 1).
+extern "C" int mi_expert_gate_up(int dtype, int mode, const void* x, int64_t x_stride, const void* gate_up, const int* chosen,
+                                 const float* pair_weight, void* act, int num_tokens, int width, int ff, int experts,
+                                 int top, hipStream_t stream) {
   MI_REQUIRE(num_tokens >= 0 && width > 0 && ff > 0 && experts > 0 && top > 0 && x_stride >= width,
              "expert_gate_up: bad sizes tokens=%d width=%d ff=%d experts=%d top=%d", num_tokens, width, ff, experts, top);
   MI_REQUIRE(dtype == MI_F32 || dtype == MI_BF16, "expert_gate_up: unknown dtype %d", dtype);
+  MI_REQUIRE(mode == EXPERT_SILU_GATED || (mode == EXPERT_SQUARED_RELU), "expert_gate_up: mode %d", mode);
   const size_t lds = (size_t)width * (dtype == MI_F32 ? 4 : 2);
   MI_REQUIRE(lds <= 64 * 1024, "expert_gate_up: rows of %d do not fit the block's staging", width);
   MI_REQUIRE((int64_t)num_tokens * top <= 0x7fffffff / 2 && ceil_div(ff, MI_EXPERT_FEATURES) <= 65535, "expert_gate_up: too many pairs or features");
   if (num_tokens == 0) return MI_OK;
   dim3 grid(num_tokens * top, ceil_div(ff, MI_EXPERT_FEATURES));
-  if (dtype == MI_F32)
-    expert_gate_up_kernel<float><<<grid, 256, lds, stream>>>((const float*)x, x_stride, (const float*)gate_up, chosen,
-                                                             (float*)act, width, ff, experts, top);
-  else
-    expert_gate_up_kernel<bf16_t><<<grid, 256, lds, stream>>>((const bf16_t*)x, x_stride, (const bf16_t*)gate_up, chosen,
-                                                              (bf16_t*)act, width, ff, experts, top);
+#define MI_GATE_UP(T, MODE)                                                                                              \
+  expert_gate_up_kernel<T, MODE><<<grid, 256, lds, stream>>>((const T*)x, x_stride, (const T*)gate_up, chosen, pair_weight, \
+                                                             (T*)act, width, ff, experts, top)
+  if (dtype == MI_F32) {
+    if (mode == EXPERT_SILU_GATED) MI_GATE_UP(float, EXPERT_SILU_GATED);
+    else MI_GATE_UP(float, EXPERT_SQUARED_RELU);
+  } else {
+    if (mode == EXPERT_SILU_GATED) MI_GATE_UP(bf16_t, EXPERT_SILU_GATED);
+    else MI_GATE_UP(bf16_t, EXPERT_SQUARED_RELU);
+  }
+#undef MI_GATE_UP
   MI_CHECK_LAUNCH("expert_gate_up");
   return MI_OK;
 }
@@ -662,64 +708,90 @@ extern "C" int mi_expert_rows_at_once(int dtype, int k_dim) {
   return 0;
 }
 
-// gated = 1: weight [experts, 2 * features, k_dim], out[pair, f] = silu(gate_f . row) * (up_f . row) with the row of
-// pair p at src[p / src_div]; gated = 0: weight [experts, features, k_dim], out[pair, f] = w_f . src[p / src_div].
+// mode 1 (silu gated): weight [experts, 2 * features, k_dim], out[pair, f] = silu(gate_f . row) * (up_f . row) with
+// the row of pair p at src[p / src_div]; mode 2: weight [experts, features, k_dim], out[pair, f] =
+// relu(pair_weight[pair] * (w_f . row))^2 (pair_weight null: 1); mode 0: out[pair, f] = w_f . row.
 // many_rows = 1 (bfloat16 with k_dim a multiple of 32 only): blocks of 64 features that take 64 rows a pass.
-extern "C" int mi_expert_rows(int dtype, int gated, const void* src, int64_t src_stride, int src_div, const void* weight,
-                              const int* listed, const int* first, void* out, int64_t out_stride, int experts, int k_dim,
-                              int features, int many_rows, hipStream_t stream) {
+extern "C" int mi_expert_rows(int dtype, int mode, const void* src, int64_t src_stride, int src_div, const void* weight,
+                              const int* listed, const int* first, const float* pair_weight, void* out, int64_t out_stride,
+                              int experts, int k_dim, int features, int many_rows, hipStream_t stream) {
   MI_REQUIRE(experts > 0 && experts <= 65535 && k_dim > 0 && features > 0 && src_div > 0 && src_stride >= k_dim && out_stride >= features,
              "expert_rows: bad sizes experts=%d k=%d features=%d", experts, k_dim, features);
   MI_REQUIRE(dtype == MI_F32 || dtype == MI_BF16, "expert_rows: unknown dtype %d", dtype);
+  MI_REQUIRE(mode == EXPERT_PLAIN || mode == EXPERT_SILU_GATED || (mode == EXPERT_SQUARED_RELU),
+             "expert_rows: mode %d", mode);
   const int elem = dtype == MI_F32 ? 4 : 2, step = 16 / elem;
   MI_REQUIRE(k_dim % step == 0 && src_stride % step == 0 && is_aligned16(src) && is_aligned16(weight),
              "expert_rows: rows of %d elements are not read 16 bytes at a time", k_dim);
-  const int64_t expert_stride = (int64_t)(gated ? 2 : 1) * features * k_dim;
+  const int64_t expert_stride = (int64_t)(mode == EXPERT_SILU_GATED ? 2 : 1) * features * k_dim;
   dim3 grid(ceil_div(features, 16), experts);
-  if (dtype == MI_BF16 && k_dim % 32 == 0 && many_rows) {
-    dim3 tiles(ceil_div(features, 64), experts);
-    if (gated)
-      expert_tiles_mfma_kernel<true><<<tiles, 256, 0, stream>>>((const bf16_t*)src, src_stride, src_div, (const bf16_t*)weight,
-                                                                expert_stride, listed, first, (bf16_t*)out, out_stride, k_dim, features);
-    else
-      expert_tiles_mfma_kernel<false><<<tiles, 256, 0, stream>>>((const bf16_t*)src, src_stride, src_div, (const bf16_t*)weight,
-                                                                 expert_stride, listed, first, (bf16_t*)out, out_stride, k_dim, features);
-    MI_CHECK_LAUNCH("expert_tiles_mfma");
-    return MI_OK;
-  }
+#define MI_BY_MODE(LAUNCH)                                   \
+  do {                                                       \
+    if (mode == EXPERT_SILU_GATED) LAUNCH(EXPERT_SILU_GATED); \
+    else if (mode == EXPERT_SQUARED_RELU) LAUNCH(EXPERT_SQUARED_RELU); \
+    else LAUNCH(EXPERT_PLAIN);                               \
+  } while (0)
   if (dtype == MI_BF16 && k_dim % 32 == 0) {  // the matrix cores
-    if (gated)
-      expert_rows_mfma_kernel<true><<<grid, 256, 0, stream>>>((const bf16_t*)src, src_stride, src_div, (const bf16_t*)weight,
-                                                              expert_stride, listed, first, (bf16_t*)out, out_stride, k_dim, features);
-    else
-      expert_rows_mfma_kernel<false><<<grid, 256, 0, stream>>>((const bf16_t*)src, src_stride, src_div, (const bf16_t*)weight,
-                                                               expert_stride, listed, first, (bf16_t*)out, out_stride, k_dim, features);
+    dim3 tiles(ceil_div(features, 64), experts);
+#define MI_TILES(MODE)                                                                                              \
+  expert_tiles_mfma_kernel<MODE><<<tiles, 256, 0, stream>>>((const bf16_t*)src, src_stride, src_div, (const bf16_t*)weight, \
+                                                            expert_stride, listed, first, pair_weight, (bf16_t*)out,  \
+                                                            out_stride, k_dim, features)
+#define MI_MFMA(MODE)                                                                                               \
+  expert_rows_mfma_kernel<MODE><<<grid, 256, 0, stream>>>((const bf16_t*)src, src_stride, src_div, (const bf16_t*)weight, \
+                                                          expert_stride, listed, first, pair_weight, (bf16_t*)out,    \
+                                                          out_stride, k_dim, features)
+    if (many_rows) MI_BY_MODE(MI_TILES);
+    else MI_BY_MODE(MI_MFMA);
+#undef MI_TILES
+#undef MI_MFMA
     MI_CHECK_LAUNCH("expert_rows_mfma");
     return MI_OK;
   }
   const int at_once = mi_expert_rows_at_once(dtype, k_dim);
   MI_REQUIRE(at_once > 0, "expert_rows: rows of %d do not fit the block's staging", k_dim);
   const size_t lds = (size_t)at_once * k_dim * elem;
-#define MI_ROWS(T, R)                                                                                                     \
-  do {                                                                                                                    \
-    if (gated)                                                                                                            \
-      expert_rows_kernel<T, R, true><<<grid, 256, lds, stream>>>((const T*)src, src_stride, src_div, (const T*)weight,    \
-                                                                 expert_stride, listed, first, (T*)out, out_stride, k_dim, \
-                                                                 features);                                                \
-    else                                                                                                                  \
-      expert_rows_kernel<T, R, false><<<grid, 256, lds, stream>>>((const T*)src, src_stride, src_div, (const T*)weight,   \
-                                                                  expert_stride, listed, first, (T*)out, out_stride, k_dim, \
-                                                                  features);                                               \
-  } while (0)
+#define MI_ROWS_OF(T, R, MODE)                                                                                    \
+  expert_rows_kernel<T, R, MODE><<<grid, 256, lds, stream>>>((const T*)src, src_stride, src_div, (const T*)weight, \
+                                                             expert_stride, listed, first, pair_weight, (T*)out,   \
+                                                             out_stride, k_dim, features)
+#define MI_ROWS_F4(MODE) MI_ROWS_OF(float, 4, MODE)
+#define MI_ROWS_F2(MODE) MI_ROWS_OF(float, 2, MODE)
+#define MI_ROWS_B8(MODE) MI_ROWS_OF(bf16_t, 8, MODE)
+#define MI_ROWS_B4(MODE) MI_ROWS_OF(bf16_t, 4, MODE)
+#define MI_ROWS_B2(MODE) MI_ROWS_OF(bf16_t, 2, MODE)
   if (dtype == MI_F32) {
-    if (at_once == 4) MI_ROWS(float, 4);
-    else MI_ROWS(float, 2);
+    if (at_once == 4) MI_BY_MODE(MI_ROWS_F4);
+    else MI_BY_MODE(MI_ROWS_F2);
   } else {
-    if (at_once == 8) MI_ROWS(bf16_t, 8);
-    else if (at_once == 4) MI_ROWS(bf16_t, 4);
-    else MI_ROWS(bf16_t, 2);
+    if (at_once == 8) MI_BY_MODE(MI_ROWS_B8);
+    else if (at_once == 4) MI_BY_MODE(MI_ROWS_B4);
+    else MI_BY_MODE(MI_ROWS_B2);
   }
-#undef MI_ROWS
+#undef MI_ROWS_OF
+#undef MI_ROWS_F4
+#undef MI_ROWS_F2
+#undef MI_ROWS_B8
+#undef MI_ROWS_B4
+#undef MI_ROWS_B2
+#undef MI_BY_MODE
   MI_CHECK_LAUNCH("expert_rows");
+  return MI_OK;
+}
+
+// out[row, f] = relu(z * weight[row])^2 for rows of a product made by others (row stride z_stride).
+extern "C" int mi_weighted_squared_relu(int dtype, const void* z, int64_t z_stride, const float* weight, void* out,
+                                        int64_t out_stride, int num_rows, int width, hipStream_t stream) {
+  MI_REQUIRE(num_rows >= 0 && width > 0 && z_stride >= width && out_stride >= width, "weighted_squared_relu: bad sizes rows=%d width=%d",
+             num_rows, width);
+  MI_REQUIRE(ceil_div(width, 256) <= 65535, "weighted_squared_relu: width %d is too large", width);
+  MI_REQUIRE(dtype == MI_F32 || dtype == MI_BF16, "weighted_squared_relu: unknown dtype %d", dtype);
+  if (num_rows == 0) return MI_OK;
+  dim3 grid(num_rows, ceil_div(width, 256));
+  if (dtype == MI_F32)
+    weighted_squared_relu_kernel<float><<<grid, 256, 0, stream>>>((const float*)z, z_stride, weight, (float*)out, out_stride, width);
+  else
+    weighted_squared_relu_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)z, z_stride, weight, (bf16_t*)out, out_stride, width);
+  MI_CHECK_LAUNCH("weighted_squared_relu");
   return MI_OK;
 }

@@ -115,7 +115,7 @@ class DecoderModel:
         """Per call in `order`: what its own cache must hold, or None if it reads another's; then,
         if the embedding keeps state, its needs."""
         needs = [
-            None if call.reads_cache_of is not None else self.blocks[call.layer].mixer.cache_needs(page_size)
+            None if call.reads_cache_of is not None else self.blocks[call.layer].cache_needs(page_size)
             for call in self.spec.order
         ]
         # an embedding that keeps state of its own gets one more cache, behind the calls'

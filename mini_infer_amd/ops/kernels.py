@@ -1645,11 +1645,11 @@ def linear_geglu(x: torch.Tensor, gate_up_weight: torch.Tensor) -> torch.Tensor:
 
 def short_conv(
     x: torch.Tensor, channels: int, taps_weight: torch.Tensor, tail: torch.Tensor, cu_seqlens: torch.Tensor,
-    slots: torch.Tensor, token_request: torch.Tensor, bias: torch.Tensor | None = None,
+    slots: torch.Tensor, token_request: torch.Tensor, bias: torch.Tensor | None = None, add_input: bool = False,
 ) -> torch.Tensor:
     """A causal convolution over time per channel, then silu, on the first `channels` columns of
     `x` [T, >= channels]: `y[t, c] = silu(bias[c] + sum_j w[c, j] * x[t - (taps-1) + j, c])` within each
-    request.  `tail` [slots + 1, taps - 1, channels] (compute dtype, rows may be strided) holds
+    request (`add_input`: `y = x + bias + sum` instead of the silu).  `tail` [slots + 1, taps - 1, channels] (compute dtype, rows may be strided) holds
     each request's last taps-1 inputs and is advanced in place; `taps_weight` is float32
     [channels, taps], last column the current token's."""
     _need_cuda(x, taps_weight, tail, cu_seqlens, slots, token_request, bias)
@@ -1678,7 +1678,8 @@ def short_conv(
     library.check(
         library.load().mi_short_conv(
             _dtype_code(x), _ptr(x), x.stride(0), _ptr(taps_weight), _ptr(tail), tail.stride(0), _ptr(cu_seqlens), _ptr(slots),
-            _ptr(token_request), _ptr(y), y.stride(0), tokens, requests, channels, taps, tail.shape[0] - 1, _ptr(bias), _stream(),
+            _ptr(token_request), _ptr(y), y.stride(0), tokens, requests, channels, taps, tail.shape[0] - 1, _ptr(bias), int(add_input),
+            _stream(),
         )
     )
     return y
@@ -1820,19 +1821,31 @@ def latent_expand(
     return qkv
 
 
-def linear_per_head(x: torch.Tensor, weight: torch.Tensor, out: torch.Tensor) -> None:
+PER_HEAD_MAX_ROWS = 256  # rows up to which the engine's own product head by head is taken
+
+
+def linear_per_head(x: torch.Tensor, weight: torch.Tensor, out: torch.Tensor, weight_kn: torch.Tensor | None = None,
+                    gate: torch.Tensor | None = None) -> None:
     """`out[:, h, :] = x[:, h, :] @ weight[h].T` for every head h: x [T, heads, K], weight
     [heads, N, K], out [T, heads, N]; x and out may be views into wider rows (unit inner
-    stride).  float32: the true-float32 product, head by head; bfloat16: one batched product of
-    the vendor library (the weight-streaming product has no batched form; head by head it costs a
-    launch a head, which at few rows is all a step's time)."""
-    _need_cuda(x, weight, out)
+    stride).  With `gate` [T, heads, N] the result (rounded to the element type) is multiplied by
+    `logistic(gate)`.
+
+    float32: the true-float32 product, head by head.  bfloat16: up to `PER_HEAD_MAX_ROWS` rows that are
+    read 16 bytes at a time run as one kernel, gate included; otherwise one batched product of the
+    vendor library, whose right operand is `weight_kn` (`weight` with its last two axes exchanged,
+    [heads, K, N], contiguous; made here if it is not given)."""
+    _need_cuda(x, weight, out, weight_kn, gate)
     if x.dim() != 3 or weight.dim() != 3 or out.dim() != 3 or x.stride(2) != 1 or out.stride(2) != 1 or weight.stride(2) != 1:
         raise KernelShapeError("linear_per_head: x [T, heads, K], weight [heads, N, K], out [T, heads, N], unit inner strides")
     tokens, heads, k = x.shape
     n = weight.shape[1]
     if tuple(weight.shape) != (heads, n, k) or tuple(out.shape) != (tokens, heads, n) or not (x.dtype == weight.dtype == out.dtype):
         raise KernelShapeError(f"linear_per_head: shapes {tuple(x.shape)}, {tuple(weight.shape)}, {tuple(out.shape)} do not fit")
+    if weight_kn is not None and (tuple(weight_kn.shape) != (heads, k, n) or not weight_kn.is_contiguous() or weight_kn.dtype != x.dtype):
+        raise KernelShapeError(f"linear_per_head: weight_kn is {x.dtype} [{heads}, {k}, {n}], contiguous, got {tuple(weight_kn.shape)}")
+    if gate is not None and (gate.dim() != 3 or tuple(gate.shape) != (tokens, heads, n) or gate.stride(2) != 1 or gate.dtype != x.dtype):
+        raise KernelShapeError(f"linear_per_head: the gate is {x.dtype} [{tokens}, {heads}, {n}] with unit inner stride")
     if tokens == 0:
         return
     lib = library.load()
@@ -1840,8 +1853,38 @@ def linear_per_head(x: torch.Tensor, weight: torch.Tensor, out: torch.Tensor) ->
         for h in range(heads):
             library.check(lib.mi_gemm_f32(_ptr(x[:, h]), x.stride(0), _ptr(weight[h]), weight.stride(1), _ptr(out[:, h]),
                                           out.stride(0), tokens, n, k, _stream()))
+    elif (tokens <= PER_HEAD_MAX_ROWS and k % 8 == 0 and x.stride(0) % 8 == 0 and x.stride(1) % 8 == 0 and x.data_ptr() % 16 == 0
+          and weight.is_contiguous() and weight.data_ptr() % 16 == 0):
+        library.check(lib.mi_per_head_bf16(
+            _ptr(x), x.stride(0), x.stride(1), _ptr(weight), _ptr(gate), 0 if gate is None else gate.stride(0),
+            0 if gate is None else gate.stride(1), _ptr(out), out.stride(0), out.stride(1), tokens, heads, k, n, _stream()))
         return
-    torch.bmm(x.transpose(0, 1), weight.transpose(1, 2), out=out.transpose(0, 1))
+    else:
+        if weight_kn is None:
+            weight_kn = weight.transpose(1, 2).contiguous()
+        torch.bmm(x.transpose(0, 1), weight_kn, out=out.transpose(0, 1))
+    if gate is not None:
+        gate_heads(out, gate, out)
+
+
+def gate_heads(x: torch.Tensor, gate: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
+    """`out[t, h, d] = x[t, h, d] * logistic(gate[t, h, d])` for the first `width` entries of every head:
+    x [T, heads, >= width] (heads may lie apart in wider rows), gate and out [T, heads, width] with heads
+    side by side.  `out` may be `x`."""
+    _need_cuda(x, gate, out)
+    if x.dim() != 3 or gate.dim() != 3 or tuple(out.shape) != tuple(gate.shape) or tuple(x.shape[:2]) != tuple(gate.shape[:2]):
+        raise KernelShapeError(f"gate_heads: x {tuple(x.shape)}, gate {tuple(gate.shape)}, out {tuple(out.shape)} do not fit")
+    tokens, heads, width = gate.shape
+    if x.shape[2] < width or not (x.dtype == gate.dtype == out.dtype) or x.stride(2) != 1:
+        raise KernelShapeError("gate_heads: heads at least as wide as the gate's, of one dtype, with unit inner stride")
+    for name, t in (("gate", gate), ("out", out)):
+        if t.stride(2) != 1 or (heads > 1 and t.stride(1) != width):
+            raise KernelShapeError(f"gate_heads: the heads of {name} lie side by side, got strides {t.stride()}")
+    library.check(
+        library.load().mi_gate_heads(_dtype_code(x), _ptr(x), x.stride(0), x.stride(1) if heads > 1 else x.shape[2], _ptr(gate),
+                                     gate.stride(0), _ptr(out), out.stride(0), tokens, heads, width, _stream())
+    )
+    return out
 
 
 def sample(
@@ -2336,17 +2379,23 @@ def qkv_norm_write(
 # ----------------------------------------------------------------------------
 
 ROUTER_MAX_OUTPUTS = 1024
+ROUTER_SCORES = ("softmax", "logistic")
+# an expert's activation -> (mode of its first product's kernel, weight rows a feature of that product has)
+EXPERT_ACTIVATIONS = {"silu_gated": (1, 2), "squared_relu": (2, 1)}
 
 
 def route_top_k(
     x: torch.Tensor, router: torch.Tensor, correction: torch.Tensor | None, gate_row: torch.Tensor | None, *, top: int,
-    route_scale: float,
+    route_scale: float, scores: str = "softmax",
 ) -> tuple[torch.Tensor, torch.Tensor, torch.Tensor | None]:
     """Per row of `x` [T, W]: scores `softmax(router @ x)` over all router outputs (`router` float32
     [outputs, W]), the `top` outputs with the largest `score + correction` (`correction` float32
     [outputs] or None; the lower index wins a tie) -> their indices int32 [T, top] and weights
     `score * route_scale` float32 [T, top] (not renormalized); with `gate_row` (float32 [W]) also
-    `logistic(gate_row . x)` float32 [T]."""
+    `logistic(gate_row . x)` float32 [T].  `scores="logistic"`: every output's score is `logistic(z)` of its
+    own logit."""
+    if scores not in ROUTER_SCORES:
+        raise KernelShapeError(f"route_top_k: scores {scores!r}; built: {ROUTER_SCORES}")
     _need_cuda(x, router, correction, gate_row)
     for name, t in (("router", router), ("correction", correction), ("gate_row", gate_row)):
         _need_contiguous(name, t)
@@ -2369,13 +2418,18 @@ def route_top_k(
     library.check(
         library.load().mi_route_top_k(
             _dtype_code(x), _ptr(x), x.stride(0), _ptr(router), _ptr(correction), _ptr(gate_row), _ptr(chosen), _ptr(weights),
-            _ptr(gates), tokens, width, outputs, int(top), float(route_scale), _stream(),
+            _ptr(gates), tokens, width, outputs, int(top), float(route_scale), int(scores == "logistic"), _stream(),
         )
     )
     return chosen, weights, gates
 
 
-def _check_experts(x, gate_up, down, chosen, weights, shared, shared_gate):
+def _check_experts(x, gate_up, down, chosen, weights, shared, shared_gate, activation, weight_on):
+    if activation not in EXPERT_ACTIVATIONS or weight_on not in ("input", "output"):
+        raise KernelShapeError(f"routed experts: activation {activation!r} (built: {sorted(EXPERT_ACTIVATIONS)}), weights on {weight_on!r}")
+    if weight_on == "input" and activation != "squared_relu":
+        raise KernelShapeError(f"routed experts: weights on an expert's input are not built for {activation}")
+    rows = EXPERT_ACTIVATIONS[activation][1]
     _need_cuda(x, gate_up, down, chosen, weights, shared, shared_gate)
     for name, t in (("gate_up", gate_up), ("down", down), ("chosen", chosen), ("weights", weights), ("shared_gate", shared_gate)):
         _need_contiguous(name, t)
@@ -2385,9 +2439,9 @@ def _check_experts(x, gate_up, down, chosen, weights, shared, shared_gate):
     if x.dim() != 2 or x.stride(1) != 1:
         raise KernelShapeError("routed experts: rows with unit inner stride")
     tokens, width = x.shape
-    if gate_up.dim() != 3 or down.dim() != 3 or gate_up.shape[2] != width or gate_up.shape[1] % 2 or gate_up.dtype != x.dtype or down.dtype != x.dtype:
-        raise KernelShapeError(f"routed experts: gate|up is {x.dtype} [experts, 2*ff, {width}], got {gate_up.dtype} {tuple(gate_up.shape)}")
-    experts, ff = gate_up.shape[0], gate_up.shape[1] // 2
+    if gate_up.dim() != 3 or down.dim() != 3 or gate_up.shape[2] != width or gate_up.shape[1] % rows or gate_up.dtype != x.dtype or down.dtype != x.dtype:
+        raise KernelShapeError(f"routed experts: the first matrices are {x.dtype} [experts, {rows}*ff, {width}], got {gate_up.dtype} {tuple(gate_up.shape)}")
+    experts, ff = gate_up.shape[0], gate_up.shape[1] // rows
     if tuple(down.shape) != (experts, width, ff):
         raise KernelShapeError(f"routed experts: down is [{experts}, {width}, {ff}], got {tuple(down.shape)}")
     if chosen.dim() != 2 or chosen.shape[0] != tokens or tuple(weights.shape) != tuple(chosen.shape):
@@ -2398,33 +2452,63 @@ def _check_experts(x, gate_up, down, chosen, weights, shared, shared_gate):
     return tokens, width, experts, ff, chosen.shape[1]
 
 
+def _expert_weights(activation: str, weights: torch.Tensor, weight_on: str):
+    """(mode of the first product, weights it applies to what an expert reads, weights of the final sum)."""
+    mode = EXPERT_ACTIVATIONS[activation][0]
+    return (mode, weights, None) if weight_on == "input" else (mode, None, weights)
+
+
+@dataclasses.dataclass
+class SummedRows:
+    """A sum that has not been made yet: row t of the result is the sum of rows `t * pieces` ..
+    `(t + 1) * pieces - 1` of `rows` [T * pieces, W], in that order.  A norm that knows it adds them up on its way
+    (`gated_update_norm`); anything else calls `finish()`."""
+
+    rows: torch.Tensor
+    pieces: int
+
+    def finish(self) -> torch.Tensor:
+        if self.pieces == 1:
+            return self.rows
+        wide = self.rows.view(-1, self.pieces, self.rows.shape[1])
+        total = wide[:, 0].float()
+        for p in range(1, self.pieces):
+            total = total + wide[:, p].float()
+        return total.to(self.rows.dtype)
+
+
 def experts_few_rows(
     x: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, chosen: torch.Tensor, weights: torch.Tensor,
-    shared: torch.Tensor | None = None, shared_gate: torch.Tensor | None = None,
+    shared: torch.Tensor | None = None, shared_gate: torch.Tensor | None = None, *, activation: str = "silu_gated",
+    weight_on: str = "output",
 ) -> torch.Tensor:
     """`y[t] = sum_k weights[t, k] * expert_{chosen[t, k]}(x[t]) (+ shared_gate[t] * shared[t])` with
     every (row, chosen expert) pair worked on its own, the expert's weights read by index: two
     launches whatever the rows hold, and nothing the host has to know.  An index past the real
     experts is an identity expert (its output is `x[t]`).  `gate_up` [experts, 2*ff, W] (gate rows,
-    then up rows), `down` [experts, W, ff]; an expert is `down(silu(gate(x)) * up(x))`."""
-    tokens, width, experts, ff, top = _check_experts(x, gate_up, down, chosen, weights, shared, shared_gate)
+    then up rows), `down` [experts, W, ff]; an expert is `down(silu(gate(x)) * up(x))`.
+
+    `activation="squared_relu"`: experts without a gate, `gate_up` [experts, ff, W], `down(relu(up(x))^2)`.
+    `weight_on="input"`: the weight multiplies what the expert reads, `y[t] = sum_k expert(weights * x[t])`."""
+    tokens, width, experts, ff, top = _check_experts(x, gate_up, down, chosen, weights, shared, shared_gate, activation, weight_on)
+    mode, on_input, on_output = _expert_weights(activation, weights, weight_on)
     act = torch.empty((tokens * top, ff), dtype=x.dtype, device=x.device)
     out = torch.empty((tokens, width), dtype=x.dtype, device=x.device)
     lib = library.load()
-    library.check(lib.mi_expert_gate_up(_dtype_code(x), _ptr(x), x.stride(0), _ptr(gate_up), _ptr(chosen), _ptr(act), tokens,
-                                        width, ff, experts, top, _stream()))
+    library.check(lib.mi_expert_gate_up(_dtype_code(x), mode, _ptr(x), x.stride(0), _ptr(gate_up), _ptr(chosen), _ptr(on_input),
+                                        _ptr(act), tokens, width, ff, experts, top, _stream()))
     library.check(lib.mi_expert_down_combine(
-        _dtype_code(x), _ptr(act), _ptr(down), _ptr(chosen), _ptr(weights), _ptr(x), x.stride(0), _ptr(shared),
+        _dtype_code(x), _ptr(act), _ptr(down), _ptr(chosen), _ptr(on_output), _ptr(x), x.stride(0), _ptr(shared),
         0 if shared is None else shared.stride(0), _ptr(shared_gate), _ptr(out), tokens, width, ff, experts, top, _stream()))
     return out
 
 
-def experts_by_expert_take(x: torch.Tensor, gate_up: torch.Tensor) -> bool:
+def experts_by_expert_take(x: torch.Tensor, gate_up: torch.Tensor, activation: str = "silu_gated") -> bool:
     """Whether `experts_by_expert` takes these sizes: rows and expert rows read 16 bytes at a time, and
     a few of them fit a block's staging."""
     if x.dim() != 2 or gate_up.dim() != 3 or x.dtype not in (torch.float32, torch.bfloat16):
         return False
-    width, ff = x.shape[1], gate_up.shape[1] // 2
+    width, ff = x.shape[1], gate_up.shape[1] // EXPERT_ACTIVATIONS[activation][1]
     step = 16 // x.element_size()
     lib = library.load()
     code = _dtype_code(x)
@@ -2438,54 +2522,68 @@ GROUPED_ROWS_STEP = 64  # the sorted form's products run over row counts rounded
 
 def experts_by_expert(
     x: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, chosen: torch.Tensor, weights: torch.Tensor,
-    shared: torch.Tensor | None = None, shared_gate: torch.Tensor | None = None, many_rows: bool | None = None,
-) -> torch.Tensor:
+    shared: torch.Tensor | None = None, shared_gate: torch.Tensor | None = None, many_rows: bool | None = None, *,
+    activation: str = "silu_gated", weight_on: str = "output", combine: bool = True,
+) -> "torch.Tensor | SummedRows":
     """The same sum as `experts_few_rows`, expert by expert without the host knowing anything: one small
     kernel lists the (row, expert) pairs by expert, then every chosen expert's block streams its
     weights once for up to eight of the expert's rows at a time (the rows wait in LDS), and one kernel adds
     a row's results in the order of its choices.  Four launches; an expert that many rows chose is read once
     per sixteen of them, not once per row.  `many_rows` (default: by the average number of rows an expert
-    gets): blocks of 64 features that take 64 of an expert's rows a pass, for prompts (bfloat16)."""
-    tokens, width, experts, ff, top = _check_experts(x, gate_up, down, chosen, weights, shared, shared_gate)
-    if not experts_by_expert_take(x, gate_up):
+    gets): blocks of 64 features that take 64 of an expert's rows a pass, for prompts (bfloat16).  `combine=False`
+    (weights on the input, no shared or identity experts): the rows are left for a norm to add up (`SummedRows`)."""
+    tokens, width, experts, ff, top = _check_experts(x, gate_up, down, chosen, weights, shared, shared_gate, activation, weight_on)
+    mode, on_input, on_output = _expert_weights(activation, weights, weight_on)
+    if not combine and (weight_on != "input" or shared is not None):
+        raise KernelShapeError("experts_by_expert: rows are left apart only where the final sum is a plain one")
+    if not experts_by_expert_take(x, gate_up, activation):
         raise KernelShapeError(f"experts_by_expert: rows of {width} and {ff} are not read 16 bytes at a time, or do not fit")
     pairs = tokens * top
     listed = torch.empty((pairs,), dtype=torch.int32, device=x.device)
     first = torch.empty((experts + 1,), dtype=torch.int32, device=x.device)
     act = torch.empty((pairs, ff), dtype=x.dtype, device=x.device)
     made = torch.empty((pairs, width), dtype=x.dtype, device=x.device)
-    out = torch.empty((tokens, width), dtype=x.dtype, device=x.device)
     lib, code = library.load(), _dtype_code(x)
     if many_rows is None:
         many_rows = pairs >= EXPERT_TILES_MIN_ROWS * experts
     many = int(bool(many_rows))
     library.check(lib.mi_expert_sort(_ptr(chosen), _ptr(listed), _ptr(first), pairs, experts, _stream()))
-    library.check(lib.mi_expert_rows(code, 1, _ptr(x), x.stride(0), top, _ptr(gate_up), _ptr(listed), _ptr(first), _ptr(act), ff,
-                                     experts, width, ff, many, _stream()))
-    library.check(lib.mi_expert_rows(code, 0, _ptr(act), ff, 1, _ptr(down), _ptr(listed), _ptr(first), _ptr(made), width,
+    library.check(lib.mi_expert_rows(code, mode, _ptr(x), x.stride(0), top, _ptr(gate_up), _ptr(listed), _ptr(first),
+                                     _ptr(on_input), _ptr(act), ff, experts, width, ff, many, _stream()))
+    library.check(lib.mi_expert_rows(code, 0, _ptr(act), ff, 1, _ptr(down), _ptr(listed), _ptr(first), None, _ptr(made), width,
                                      experts, ff, width, many, _stream()))
+    if not combine:
+        return SummedRows(made, top)
+    out = torch.empty((tokens, width), dtype=x.dtype, device=x.device)
     library.check(lib.mi_expert_combine(
-        code, _ptr(made), None, _ptr(chosen), _ptr(weights), _ptr(x), x.stride(0), _ptr(shared),
+        code, _ptr(made), None, _ptr(chosen), _ptr(on_output), _ptr(x), x.stride(0), _ptr(shared),
         0 if shared is None else shared.stride(0), _ptr(shared_gate), _ptr(out), tokens, width, experts, top, _stream()))
     return out
 
 
 def experts_grouped(
     x: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, chosen: torch.Tensor, weights: torch.Tensor,
-    shared: torch.Tensor | None = None, shared_gate: torch.Tensor | None = None,
+    shared: torch.Tensor | None = None, shared_gate: torch.Tensor | None = None, *, activation: str = "silu_gated",
+    weight_on: str = "output",
 ) -> torch.Tensor:
     """The same sum for many rows: the (row, expert) pairs are sorted by expert, every expert that
     was chosen runs its two products once over all its rows (the engine's own products, so each
     expert's weights are read once), and one kernel adds a row's results in the order of its
     choices.  The host reads how many rows each expert got, so this form is not for a step that
     is being recorded."""
-    tokens, width, experts, ff, top = _check_experts(x, gate_up, down, chosen, weights, shared, shared_gate)
+    tokens, width, experts, ff, top = _check_experts(x, gate_up, down, chosen, weights, shared, shared_gate, activation, weight_on)
+    _, on_input, on_output = _expert_weights(activation, weights, weight_on)
+    first_rows = gate_up.shape[1]
+    sorted_weights = None  # of the sorted pairs, for the first product's activation
     flat = chosen.reshape(-1).long()
     order = torch.argsort(flat, stable=True)
     counts = torch.bincount(flat, minlength=experts)[:experts].tolist()
     where = torch.empty_like(order, dtype=torch.int32)
     where[order] = torch.arange(order.numel(), dtype=torch.int32, device=x.device)
     real = sum(counts)
+    if activation == "squared_relu":
+        given = on_input.reshape(-1) if on_input is not None else torch.ones_like(weights).reshape(-1)
+        sorted_weights = torch.cat([given[order][:real], given.new_zeros(GROUPED_ROWS_STEP)])
     if x.dtype == torch.bfloat16:
         # The vendor library's product expert by expert, straight into one buffer for all experts' rows, one
         # activation launch.  Every product runs over its expert's rows rounded UP to a multiple of 64: the
@@ -2498,7 +2596,7 @@ def experts_grouped(
         sorted_rows = torch.empty((pairs + step, width), dtype=x.dtype, device=x.device)
         sorted_rows[pairs:].zero_()
         torch.index_select(x, 0, torch.div(order, top, rounding_mode="floor"), out=sorted_rows[:pairs])
-        stacked = torch.empty((real + step, 2 * ff), dtype=x.dtype, device=x.device)
+        stacked = torch.empty((real + step, first_rows), dtype=x.dtype, device=x.device)
         rows = torch.empty((real + step, width), dtype=x.dtype, device=x.device)
         at = 0
         for e, count in enumerate(counts):
@@ -2507,7 +2605,7 @@ def experts_grouped(
                 torch.matmul(sorted_rows[at:upto], gate_up[e].t(), out=stacked[at:upto])
                 at += count
         stacked[real:].zero_()
-        act = silu_mul(stacked)
+        act = silu_mul(stacked) if activation == "silu_gated" else weighted_squared_relu(stacked, sorted_weights)
         at = 0
         for e, count in enumerate(counts):
             if count:
@@ -2519,11 +2617,150 @@ def experts_grouped(
         made, at = [], 0
         for e, count in enumerate(counts):
             if count:
-                made.append(linear(linear_swiglu(sorted_rows[at:at + count], gate_up[e]), down[e]))
+                mine = sorted_rows[at:at + count]
+                if activation == "silu_gated":
+                    inner = linear_swiglu(mine, gate_up[e])
+                else:
+                    inner = weighted_squared_relu(linear(mine, gate_up[e]), sorted_weights[at:at + count].contiguous())
+                made.append(linear(inner, down[e]))
                 at += count
         rows = torch.cat(made, dim=0) if made else torch.empty((1, width), dtype=x.dtype, device=x.device)
     out = torch.empty((tokens, width), dtype=x.dtype, device=x.device)
     library.check(library.load().mi_expert_combine(
-        _dtype_code(x), _ptr(rows), _ptr(where), _ptr(chosen), _ptr(weights), _ptr(x), x.stride(0), _ptr(shared),
+        _dtype_code(x), _ptr(rows), _ptr(where), _ptr(chosen), _ptr(on_output), _ptr(x), x.stride(0), _ptr(shared),
         0 if shared is None else shared.stride(0), _ptr(shared_gate), _ptr(out), tokens, width, experts, top, _stream()))
     return out
+
+
+def weighted_squared_relu(z: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
+    """`relu(z * weight[row])^2` for rows [n, width] (`weight` float32 [n])."""
+    _need_cuda(z, weight)
+    _need_contiguous("weight", weight)
+    _need_f32("weight", weight)
+    if z.dim() != 2 or z.stride(1) != 1 or weight.numel() != z.shape[0]:
+        raise KernelShapeError(f"weighted_squared_relu: rows and one weight each, got {tuple(z.shape)} and {weight.numel()}")
+    out = torch.empty(z.shape, dtype=z.dtype, device=z.device)
+    library.check(
+        library.load().mi_weighted_squared_relu(_dtype_code(z), _ptr(z), z.stride(0), _ptr(weight), _ptr(out), out.stride(0),
+                                                z.shape[0], z.shape[1], _stream())
+    )
+    return out
+
+
+# ----------------------------------------------------------------------------
+# sublayers between two norms
+# ----------------------------------------------------------------------------
+
+
+@dataclasses.dataclass
+class GatedNormedUpdate:
+    """An update of the float32 stream that has not been made yet:
+
+        x += rms_norm(y * logistic(gate + bias)) * weight
+
+    `y`: a sublayer's result [T, H] in the compute dtype, or `SummedRows`; `gate` [T, H] (compute dtype)
+    with `bias` (float32 [H]), or neither; `weight` [H] in the compute dtype.  A norm that knows it makes
+    the update and its own statistics in one launch (`gated_update_norm`); anything else calls `finish()`,
+    which returns the right-hand side as one float32 tensor to add."""
+
+    y: "torch.Tensor | SummedRows"
+    weight: torch.Tensor
+    eps: float
+    gate: torch.Tensor | None = None
+    bias: torch.Tensor | None = None
+
+    def finish(self) -> torch.Tensor:
+        rows = self.y.rows if isinstance(self.y, SummedRows) else self.y
+        pieces = self.y.pieces if isinstance(self.y, SummedRows) else 1
+        total = torch.zeros((rows.shape[0] // pieces, rows.shape[1]), dtype=torch.float32, device=rows.device)
+        gated_update_norm(self, total, None, 1.0)
+        return total
+
+
+@dataclasses.dataclass
+class InputConvolution:
+    """What a sublayer reads instead of its norm's output h: `u = h + conv(h)`, a causal convolution per
+    channel over each request's tokens.  `weight` float32 [H, taps] (last column the current token's);
+    `tail` [slots + 1, taps - 1, H] (compute dtype) holds each request's last taps-1 rows of h, or None
+    for a single tap."""
+
+    weight: torch.Tensor
+    tail: torch.Tensor | None
+    cu_seqlens: torch.Tensor
+    slots: torch.Tensor
+    token_request: torch.Tensor
+    single_tokens: bool  # every request of the step brings exactly one token
+
+    def apply(self, h: torch.Tensor) -> torch.Tensor:
+        tail = self.tail
+        if tail is None:
+            tail = torch.empty((2, 0, h.shape[1]), dtype=h.dtype, device=h.device)
+        return short_conv(h, h.shape[1], self.weight, tail, self.cu_seqlens, self.slots, self.token_request, add_input=True)
+
+
+def gated_update_norm(
+    update: GatedNormedUpdate | None, residual: torch.Tensor, weight: torch.Tensor | None, eps: float,
+    rows: torch.Tensor | None = None, conv: InputConvolution | None = None,
+):
+    """Make `update` on the float32 stream in place (kept unless `rows`), then the RMS norm of the new
+    rows times `weight` (compute dtype) -> h [T, H] or [len(rows), H]; `weight=None`: the update alone.
+    With `conv` (all rows): `(h, u)`, `u` what the next sublayer reads; in a step of single tokens in the
+    same launch."""
+    y = gate = bias = out_weight = None
+    pieces, eps_out = 1, 1.0
+    if update is not None:
+        y, gate, bias, out_weight, eps_out = update.y, update.gate, update.bias, update.weight, update.eps
+        if isinstance(y, SummedRows):
+            y, pieces = y.rows, y.pieces
+    _need_cuda(y, gate, bias, out_weight, residual, weight, rows)
+    for name, t in (("residual", residual), ("weight", weight), ("rows", rows), ("bias", bias), ("output weight", out_weight)):
+        _need_contiguous(name, t)
+    _need_int32("rows", rows)
+    _need_f32("residual", residual)
+    _need_f32("bias", bias)
+    tokens, hidden = residual.shape
+    dtype = weight.dtype if weight is not None else (y.dtype if y is not None else torch.float32)
+    if y is not None and (y.dim() != 2 or y.stride(1) != 1 or tuple(y.shape) != (tokens * pieces, hidden) or y.dtype != dtype
+                          or out_weight.dtype != dtype):
+        raise KernelShapeError(f"gated_update_norm: {tuple(y.shape)} {y.dtype} in {pieces} pieces do not fit the stream {(tokens, hidden)} in {dtype}")
+    if gate is not None and (gate.dim() != 2 or gate.stride(1) != 1 or tuple(gate.shape) != (tokens, hidden) or gate.dtype != dtype or bias is None):
+        raise KernelShapeError(f"gated_update_norm: the gate is {dtype} {(tokens, hidden)} and comes with its bias, got {gate.dtype} {tuple(gate.shape)}")
+    for name, t in (("bias", bias), ("weight", weight), ("output weight", out_weight)):
+        if t is not None and t.numel() != hidden:
+            raise KernelShapeError(f"gated_update_norm: {name} has {t.numel()} entries for {hidden} columns")
+    if rows is not None and (weight is None or conv is not None):
+        raise KernelShapeError("gated_update_norm: a row list goes with a norm and without a convolution")
+    if conv is not None and weight is None:
+        raise KernelShapeError("gated_update_norm: a convolution goes with a norm")
+    n_out = tokens if rows is None else rows.numel()
+    h = torch.empty((n_out, hidden), dtype=dtype, device=residual.device) if weight is not None else None
+    here = conv is not None and conv.single_tokens
+    u = tail = None
+    taps = tail_stride = num_slots = 0
+    if here:
+        taps, tail = conv.weight.shape[1], conv.tail
+        _need_cuda(conv.weight, tail, conv.slots, conv.token_request)
+        _need_f32("convolution weight", conv.weight)
+        for name, t in (("convolution weight", conv.weight), ("slots", conv.slots), ("token_request", conv.token_request)):
+            _need_contiguous(name, t)
+        _need_int32("slots", conv.slots)
+        _need_int32("token_request", conv.token_request)
+        if conv.weight.shape[0] != hidden or conv.token_request.numel() != tokens or conv.slots.numel() != tokens:
+            raise KernelShapeError("gated_update_norm: single tokens have one request and one slot each, the convolution one row of taps a column")
+        if taps > 1:
+            if tail is None or tail.dtype != dtype or tail.dim() != 3 or tuple(tail.shape[1:]) != (taps - 1, hidden) or tail.shape[0] < 2 \
+                    or tail.stride(2) != 1 or tail.stride(1) != hidden:
+                raise KernelShapeError(f"gated_update_norm: the tail is {dtype} [slots + 1, {taps - 1}, {hidden}] with packed slots")
+            tail_stride, num_slots = tail.stride(0), tail.shape[0] - 1
+        u = torch.empty((tokens, hidden), dtype=dtype, device=residual.device)
+    library.check(
+        library.load().mi_gated_update_norm(
+            F32 if dtype == torch.float32 else BF16, _ptr(residual), _ptr(y), 0 if y is None else y.stride(0), pieces, _ptr(gate),
+            0 if gate is None else gate.stride(0), _ptr(bias), _ptr(out_weight), _ptr(weight), _ptr(rows), _ptr(h), n_out, hidden,
+            float(eps_out), float(eps), _ptr(conv.weight) if here else None, taps, _ptr(tail) if taps > 1 else None, tail_stride,
+            _ptr(conv.token_request) if here else None, _ptr(conv.slots) if here else None, num_slots, _ptr(u), _stream(),
+        )
+    )
+    if conv is None:
+        return h
+    return h, (u if here else conv.apply(h))

@@ -14,7 +14,7 @@ from pathlib import Path
 from mini_infer_amd.exceptions import ExtensionMissingError, KernelShapeError
 from mini_infer_amd.ops import build as _build
 
-ABI_VERSION = 35
+ABI_VERSION = 36
 
 _lib: ctypes.CDLL | None = None
 _lib_path: Path | None = None
@@ -85,7 +85,9 @@ _SIGNATURES: dict[str, list] = {
     ],
     "mi_stream_update_norm": [c_int, _P, c_int64, _P, c_int64, _P, _P, c_float, _P, _P, _P, _P, c_int, c_int, c_float, _P],
     "mi_clamped_glu": [c_int, _P, c_int64, _P, _P, c_int64, c_int, c_int, c_float, c_float, _P],
-    "mi_short_conv": [c_int, _P, c_int64, _P, _P, c_int64, _P, _P, _P, _P, c_int64, c_int, c_int, c_int, c_int, c_int, _P, _P],
+    "mi_short_conv": [
+        c_int, _P, c_int64, _P, _P, c_int64, _P, _P, _P, _P, c_int64, c_int, c_int, c_int, c_int, c_int, _P, c_int, _P,
+    ],
     "mi_gated_delta": [
         c_int, _P, c_int64, _P, c_int64, c_int, c_int, c_int, _P, _P, _P, _P, c_int64, _P, _P, _P, _P, c_int64,
         c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, _P,
@@ -121,13 +123,22 @@ _SIGNATURES: dict[str, list] = {
         c_int, _P, c_int64, _P, _P, _P, c_int64, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
         c_float, _P,
     ],
-    "mi_route_top_k": [c_int, _P, c_int64, _P, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_float, _P],
-    "mi_expert_gate_up": [c_int, _P, c_int64, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, _P],
+    "mi_route_top_k": [c_int, _P, c_int64, _P, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_float, c_int, _P],
+    "mi_expert_gate_up": [c_int, c_int, _P, c_int64, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, _P],
+    "mi_weighted_squared_relu": [c_int, _P, c_int64, _P, _P, c_int64, c_int, c_int, _P],
     "mi_expert_down_combine": [c_int, _P, _P, _P, _P, _P, c_int64, _P, c_int64, _P, _P, c_int, c_int, c_int, c_int, c_int, _P],
     "mi_expert_combine": [c_int, _P, _P, _P, _P, _P, c_int64, _P, c_int64, _P, _P, c_int, c_int, c_int, c_int, _P],
     "mi_expert_sort": [_P, _P, _P, c_int, c_int, _P],
     "mi_expert_rows_at_once": [c_int, c_int],
-    "mi_expert_rows": [c_int, c_int, _P, c_int64, c_int, _P, _P, _P, _P, c_int64, c_int, c_int, c_int, c_int, _P],
+    "mi_expert_rows": [c_int, c_int, _P, c_int64, c_int, _P, _P, _P, _P, _P, c_int64, c_int, c_int, c_int, c_int, _P],
+    "mi_gated_update_norm": [
+        c_int, _P, _P, c_int64, c_int, _P, c_int64, _P, _P, _P, _P, _P, c_int, c_int, c_float, c_float, _P, c_int, _P,
+        c_int64, _P, _P, c_int, _P, _P,
+    ],
+    "mi_gate_heads": [c_int, _P, c_int64, c_int, _P, c_int64, _P, c_int64, c_int, c_int, c_int, _P],
+    "mi_per_head_bf16": [
+        _P, c_int64, c_int64, _P, _P, c_int64, c_int64, _P, c_int64, c_int64, c_int, c_int, c_int, c_int, _P,
+    ],
 }
 
 

@@ -206,6 +206,14 @@ class Norm(Part):
     ) -> torch.Tensor:
         raise NotImplementedError
 
+    def forward_conv(self, delta, residual: torch.Tensor, conv) -> "tuple[torch.Tensor, torch.Tensor]":
+        """`forward` for a sublayer whose input passes a short convolution over time (`ops.InputConvolution`):
+        `(h, u)`, the norm's output in the compute dtype and what the sublayer reads, `h + conv(h)`.  A norm
+        with a kernel that does both says so by its own `forward_conv`."""
+        h = self.forward(delta, residual)
+        h = h.finish() if hasattr(h, "finish") else h
+        return h, conv.apply(h)
+
     def norm_sum(
         self,
         y: torch.Tensor,
@@ -383,6 +391,11 @@ class Block(Part):
 
     def enable_pending_output(self) -> None:
         pass
+
+    def cache_needs(self, page_size: int) -> CacheNeeds:
+        """What the cache manager must keep for one call of this block: its mixer's needs, and what the
+        block itself remembers of a request from step to step."""
+        return self.mixer.cache_needs(page_size)
 
     def optional_names(self, prefix: str) -> set[str]:
         """Names a checkpoint may hold for this block without the block reading them."""

@@ -8,15 +8,19 @@ feed-forward; the block's own last add is left to the next norm
 
 from __future__ import annotations
 
+import dataclasses
+
 import torch
 
 from mini_infer_amd.parts.base import (
     Block,
+    CacheNeeds,
     FeedForward,
     LayerCache,
     Mixer,
     Norm,
     ParamSpec,
+    StateNeeds,
     StepContext,
     TensorGetter,
 )
@@ -481,4 +485,158 @@ def build_post_norm_block(desc: dict, dtype: torch.dtype, device, shared: dict |
         FEED_FORWARDS.lookup(ffn["kind"])(ffn, dtype, device, shared) if ffn is not None else None,
         int(desc["hidden_size"]), float(desc.get("alpha", 1.0)), bool(desc.get("layer_scale", False)), dict(desc["names"]),
         dtype, device,
+    )
+
+
+class SandwichBlock(Block):
+    """Sublayers that stand between two norms of their own; sublayer q is the mixer, then the feed-forward
+    if the layer has one:
+
+        h = norm_q(x)      u = h + conv_q(h)      x <- x + output_norm_q( sublayer_q(u) * logistic(W_q h + b_q) )
+
+    `conv_taps`: a short causal convolution over time per channel on what a sublayer reads; a request's last
+    taps - 1 rows of h are state of the block, one tail per sublayer, beside whatever the mixer keeps (None:
+    `u = h`).  `gated`: the element-by-element gate on a sublayer's result, read from h (else none).
+
+    A sublayer's gate, output norm and add are left to whatever norm comes next (`ops.GatedNormedUpdate`): one
+    launch ends a sublayer and begins the next, convolution included where every request of the step
+    brings one token."""
+
+    takes_pending_products = False
+
+    def __init__(self, norms: dict[str, Norm | None], mixer: Mixer, feed_forward: FeedForward | None, hidden_size: int,
+                 gated: bool, conv_taps: int | None, names: dict[str, str], dtype: torch.dtype, device) -> None:
+        from mini_infer_amd.parts.linear import Linear
+
+        super().__init__(dtype, device)
+        if conv_taps is not None and not 1 <= conv_taps <= self.MAX_TAPS:
+            raise ValueError(f"input convolution: 1 to {self.MAX_TAPS} taps, got {conv_taps}")
+        self.norms, self.mixer, self.feed_forward = norms, mixer, feed_forward
+        self.hidden_size, self.gated, self.conv_taps, self.names = hidden_size, bool(gated), conv_taps, names
+        self.sublayers = ["mixer"] + (["ffn"] if feed_forward is not None else [])
+        self.gates = {q: Linear(hidden_size, hidden_size, names[f"{q}_gate"], dtype, device, suffix="") for q in self.sublayers} if gated else {}
+        self.gate_biases: dict[str, torch.Tensor] = {}
+        self.conv_weights: dict[str, torch.Tensor] = {}  # float32 [hidden, taps]
+        for q in self.sublayers:
+            if not hasattr(norms[f"{q}_output_norm"], "weight"):
+                raise ValueError("a sublayer's output norm is an RMS norm with a weight per column (the next norm makes it)")
+        if feed_forward is not None and hasattr(feed_forward, "leave_rows_apart"):
+            feed_forward.leave_rows_apart = True
+
+    MAX_TAPS = 16
+
+    def _children(self):
+        parts = [(self.names["mixer"], self.mixer)]
+        if self.feed_forward is not None:
+            parts.append((self.names["feed_forward"], self.feed_forward))
+        for q in self.sublayers:
+            parts += [(self.names[f"{q}_norm"], self.norms[f"{q}_norm"]), (self.names[f"{q}_output_norm"], self.norms[f"{q}_output_norm"])]
+        return parts
+
+    @property
+    def graph_safe(self) -> bool:  # type: ignore[override]
+        return all(part.graph_safe for _, part in self._children())
+
+    def param_specs(self, prefix: str) -> dict[str, ParamSpec]:
+        specs: dict[str, ParamSpec] = {}
+        for sub, part in self._children():
+            specs.update(part.param_specs(prefix + sub))
+        for q in self.sublayers:
+            if self.gated:
+                specs.update(self.gates[q].param_specs(prefix))
+                specs[prefix + self.names[f"{q}_gate"] + ".b"] = ParamSpec((self.hidden_size,), dtype="float32")
+            if self.conv_taps is not None:
+                specs[prefix + self.names[f"{q}_conv"]] = ParamSpec((self.hidden_size, self.conv_taps), dtype="float32")
+        return specs
+
+    def optional_names(self, prefix: str) -> set[str]:
+        """A layer without a feed-forward has no use for the second sublayer's norms, gate and convolution; a
+        checkpoint that stores them all the same is read without them."""
+        names = set(self.mixer.optional_names(prefix + self.names["mixer"]))
+        if self.feed_forward is None:
+            names |= {prefix + self.names[f"ffn_{what}"] for what in ("norm", "output_norm", "gate", "conv")}
+            names.add(prefix + self.names["ffn_gate"] + ".b")
+        return names
+
+    def load_params(self, prefix: str, get: TensorGetter) -> None:
+        for sub, part in self._children():
+            part.load_params(prefix + sub, get)
+        for q in self.sublayers:
+            if self.gated:
+                self.gates[q].load_params(prefix, get)
+                self.gate_biases[q] = get(prefix + self.names[f"{q}_gate"] + ".b").float().contiguous()
+            if self.conv_taps is not None:
+                self.conv_weights[q] = get(prefix + self.names[f"{q}_conv"]).float().contiguous()
+
+    # -- state ---------------------------------------------------------------------
+
+    def cache_needs(self, page_size: int) -> CacheNeeds:
+        """The mixer's needs, its state under names that begin with `mixer.`, beside the convolutions' tails."""
+        needs = self.mixer.cache_needs(page_size)
+        if self.conv_taps is None:
+            return needs
+        state: dict[str, StateNeeds] = {}
+        if isinstance(needs.state, StateNeeds):
+            state["mixer."] = needs.state
+        elif needs.state is not None:
+            state.update({"mixer." + name: need for name, need in needs.state.items()})
+        if self.conv_taps > 1:
+            state.update({f"{q}_conv": StateNeeds((self.conv_taps - 1, self.hidden_size), self.dtype) for q in self.sublayers})
+        return CacheNeeds(pages=needs.pages, state=state or None)
+
+    def _mixer_cache(self, cache: LayerCache) -> LayerCache:
+        """The cache as the mixer asked for it."""
+        if self.conv_taps is None or not isinstance(cache.state, dict):
+            return cache
+        own = {name[len("mixer."):]: rows for name, rows in cache.state.items() if name.startswith("mixer.")}
+        return dataclasses.replace(cache, state=own.get("", own or None))
+
+    def _begin(self, q: str, delta, residual: torch.Tensor, ctx: StepContext, cache: LayerCache):
+        """`(h, u)` of sublayer q, what was left to be added made first."""
+        from mini_infer_amd import ops
+
+        norm = self.norms[f"{q}_norm"]
+        if self.conv_taps is None:
+            h = norm.forward(delta, residual)
+            h = h.finish() if hasattr(h, "finish") else h
+            return h, h
+        single = ctx.host_cu_seqlens_q is not None and ctx.max_q_len == 1 and residual.shape[0] == ctx.state_slots.numel()
+        conv = ops.InputConvolution(self.conv_weights[q], cache.state[f"{q}_conv"] if self.conv_taps > 1 else None, ctx.cu_seqlens_q,
+                                    ctx.state_slots, ctx.token_request, single)
+        return norm.forward_conv(delta, residual, conv)
+
+    def _end(self, q: str, y, gate: torch.Tensor | None):
+        from mini_infer_amd import ops
+
+        if hasattr(y, "finish") and not isinstance(y, ops.SummedRows):
+            y = y.finish()
+        norm = self.norms[f"{q}_output_norm"]
+        return ops.GatedNormedUpdate(y, norm.weight, norm.eps, gate, self.gate_biases.get(q))
+
+    def forward(self, delta, residual: torch.Tensor, ctx: StepContext, cache: LayerCache, writes_cache: bool = True):
+        if not writes_cache and self.conv_taps is not None:
+            raise NotImplementedError("a block with input convolutions owns their tails; it cannot read another call's")
+        h, u = self._begin("mixer", delta, residual, ctx, cache)
+        gate = self.gates["mixer"].forward(h) if self.gated else None
+        pending = self._end("mixer", self.mixer.forward(u, ctx, self._mixer_cache(cache), writes_cache), gate)
+        if self.feed_forward is None:
+            return pending
+        h, u = self._begin("ffn", pending, residual, ctx, cache)
+        gate = self.gates["ffn"].forward(h) if self.gated else None
+        return self._end("ffn", self.feed_forward.forward(u, ctx), gate)
+
+
+@register_block("sandwich")
+def build_sandwich_block(desc: dict, dtype: torch.dtype, device, shared: dict | None = None) -> SandwichBlock:
+    """`desc`: `norm` (for both sublayers, in front and behind), `mixer`, optional `feed_forward`, `hidden_size`,
+    `gated` (whether sublayers' results are gated), `conv_taps` (taps of the convolutions on what sublayers
+    read, or None) and `names` (each part's name inside the layer)."""
+    shared = {} if shared is None else shared
+    ffn, norm = desc.get("feed_forward"), desc["norm"]
+    wanted = ["mixer_norm", "mixer_output_norm"] + (["ffn_norm", "ffn_output_norm"] if ffn is not None else [])
+    return SandwichBlock(
+        {which: NORMS.lookup(norm["kind"])(norm, dtype, device, shared) for which in wanted},
+        MIXERS.lookup(desc["mixer"]["kind"])(desc["mixer"], dtype, device, shared),
+        FEED_FORWARDS.lookup(ffn["kind"])(ffn, dtype, device, shared) if ffn is not None else None,
+        int(desc["hidden_size"]), bool(desc.get("gated", False)), desc.get("conv_taps"), dict(desc["names"]), dtype, device,
     )

@@ -266,7 +266,10 @@ class RoutedExperts(FeedForward):
         z = R x (float32)        s = softmax(z) over ALL router outputs        choice = s + correction
         y = sum over the `top` outputs e with the largest choice of  (s_e * route_scale) * expert_e(x)
 
-    The weights are the scores themselves (without the correction, not renormalized).  The last
+    The weights are the scores themselves (without the correction, not renormalized).  `scores="logistic"`:
+    every output's score is the logistic function of its own logit.  `activation="squared_relu"`: experts
+    have no gate, `W_down relu(W_up x)^2`.  `weight_on="input"`: the weight multiplies what an expert
+    READS, `y = sum expert_e(s_e * x)`; it is applied to the first product's sums, `W (s x) = s (W x)`.  The last
     `identity` router outputs stand for experts without tensors whose output is their input.  A
     shared expert of the same form may run for every token beside them, gated by one number a
     token, `logistic(w_sg . x)`.
@@ -286,8 +289,18 @@ class RoutedExperts(FeedForward):
 
     def __init__(self, hidden_size: int, intermediate_size: int, experts: int, top: int, dtype: torch.dtype, device, *,
                  identity: int = 0, route_scale: float = 1.0, correction: bool = True, shared_size: int | None = None,
-                 names: dict[str, str] | None = None) -> None:
+                 names: dict[str, str] | None = None, scores: str = "softmax", activation: str = "silu_gated",
+                 weight_on: str = "output") -> None:
         super().__init__(dtype, device)
+        if scores not in ops.kernels.ROUTER_SCORES or activation not in ops.kernels.EXPERT_ACTIVATIONS:
+            raise NotImplementedError(f"routed experts: scores {scores!r} (built: {ops.kernels.ROUTER_SCORES}), activation {activation!r} "
+                                      f"(built: {sorted(ops.kernels.EXPERT_ACTIVATIONS)})")
+        if weight_on not in ("input", "output") or (weight_on == "input" and activation != "squared_relu"):
+            raise NotImplementedError(f"routed experts: weights on {weight_on!r} of {activation} experts")
+        if weight_on == "input" and identity:
+            raise NotImplementedError("routed experts: identity experts take their weight on the output")
+        self.scores, self.activation, self.weight_on = scores, activation, weight_on
+        self.gated = activation == "silu_gated"
         if experts <= 0 or identity < 0 or not 0 < top <= experts + identity:
             raise ValueError(f"routed experts: {top} of {experts} experts + {identity} identity experts")
         if experts + identity > ops.kernels.ROUTER_MAX_OUTPUTS:
@@ -305,8 +318,10 @@ class RoutedExperts(FeedForward):
         self.router: torch.Tensor | None = None  # float32 [experts + identity, hidden]
         self.correction: torch.Tensor | None = None  # float32 [experts + identity]
         self.shared_gate_row: torch.Tensor | None = None  # float32 [hidden]
-        self.gate_up: torch.Tensor | None = None  # [experts, 2 * ff, hidden]
+        self.gate_up: torch.Tensor | None = None  # [experts, 2 * ff, hidden] (no gate: [experts, ff, hidden])
         self.down: torch.Tensor | None = None  # [experts, hidden, ff]
+        # set by a block whose norms add up `ops.SummedRows` on their way
+        self.leave_rows_apart = False
         self.force_form: str | None = None  # "few", "by_expert" or "grouped": for tests and measurements
 
     def _expert_name(self, prefix: str, e: int, which: str) -> str:
@@ -318,7 +333,8 @@ class RoutedExperts(FeedForward):
         if self.has_correction:
             specs[prefix + self.names["correction"]] = ParamSpec((outputs,), dtype="float32")
         for e in range(self.experts):
-            specs[self._expert_name(prefix, e, "gate")] = ParamSpec((ff, hidden))
+            if self.gated:
+                specs[self._expert_name(prefix, e, "gate")] = ParamSpec((ff, hidden))
             specs[self._expert_name(prefix, e, "up")] = ParamSpec((ff, hidden))
             specs[self._expert_name(prefix, e, "down")] = ParamSpec((hidden, ff))
         if self.shared is not None:
@@ -331,12 +347,14 @@ class RoutedExperts(FeedForward):
         if self.has_correction:
             self.correction = get(prefix + self.names["correction"]).float().contiguous()
         ff, hidden = self.intermediate_size, self.hidden_size
-        first = get(self._expert_name(prefix, 0, "gate"))
-        self.gate_up = torch.empty((self.experts, 2 * ff, hidden), dtype=first.dtype, device=first.device)
+        rows = 2 * ff if self.gated else ff
+        first = get(self._expert_name(prefix, 0, "up"))
+        self.gate_up = torch.empty((self.experts, rows, hidden), dtype=first.dtype, device=first.device)
         self.down = torch.empty((self.experts, hidden, ff), dtype=first.dtype, device=first.device)
         for e in range(self.experts):
-            self.gate_up[e, :ff] = get(self._expert_name(prefix, e, "gate"))
-            self.gate_up[e, ff:] = get(self._expert_name(prefix, e, "up"))
+            if self.gated:
+                self.gate_up[e, :ff] = get(self._expert_name(prefix, e, "gate"))
+            self.gate_up[e, rows - ff:] = get(self._expert_name(prefix, e, "up"))
             self.down[e] = get(self._expert_name(prefix, e, "down"))
         if self.shared is not None:
             self.shared.load_params(prefix, get)
@@ -348,7 +366,7 @@ class RoutedExperts(FeedForward):
         if ctx.host_cu_seqlens_q is None or torch.cuda.is_current_stream_capturing():
             return False  # (the sorted form reads the experts' row counts on the host)
         element = 2 if self.dtype == torch.bfloat16 else 4
-        expert_bytes = 3 * self.intermediate_size * self.hidden_size * element
+        expert_bytes = (3 if self.gated else 2) * self.intermediate_size * self.hidden_size * element
         return rows * self.top * expert_bytes > self.experts * self.GROUPED_BYTES_PER_EXPERT
 
     def forward(self, x, ctx: StepContext) -> torch.Tensor:
@@ -357,22 +375,26 @@ class RoutedExperts(FeedForward):
         if hasattr(x, "finish"):
             x = x.finish()
         chosen, weights, gates = ops.route_top_k(x, self.router, self.correction, self.shared_gate_row, top=self.top,
-                                                 route_scale=self.route_scale)
+                                                 route_scale=self.route_scale, scores=self.scores)
         shared = None
         if self.shared is not None:
             shared = self.shared.forward(x, ctx)
             shared = shared.finish() if hasattr(shared, "finish") else shared
+        how = {"activation": self.activation, "weight_on": self.weight_on}
         if self._grouped(x.shape[0], ctx):
             run = ops.experts_grouped
-        elif self.force_form == "by_expert" or (self.force_form is None and ops.experts_by_expert_take(x, self.gate_up)):
+        elif self.force_form == "by_expert" or (
+                self.force_form is None and ops.experts_by_expert_take(x, self.gate_up, self.activation)):
             run = ops.experts_by_expert
+            how["combine"] = not (self.leave_rows_apart and self.weight_on == "input" and shared is None)
         else:
             run = ops.experts_few_rows
-        return run(x, self.gate_up, self.down, chosen, weights, shared, gates)
+        return run(x, self.gate_up, self.down, chosen, weights, shared, gates, **how)
 
 
 @register_feed_forward("routed_experts")
 def build_routed_experts(desc: dict, dtype: torch.dtype, device, shared: dict | None = None) -> RoutedExperts:
-    extra = {k: desc[k] for k in ("identity", "route_scale", "correction", "shared_size", "names") if k in desc}
+    extra = {k: desc[k] for k in ("identity", "route_scale", "correction", "shared_size", "names", "scores", "activation", "weight_on")
+             if k in desc}
     return RoutedExperts(int(desc["hidden_size"]), int(desc["intermediate_size"]), int(desc["experts"]), int(desc["top"]),
                          dtype, device, **extra)

@@ -20,6 +20,10 @@ kv_rank + rot_dim numbers a key instead of head_dim + rot_dim.  Such a step writ
 values out per head into pages of its own and runs the matrix-core attention kernel over them
 like any other layer (bfloat16, head sizes it takes); the cache gets the same `[c | r]` rows
 either way.  The two forms differ by rounding only.
+
+With an output gate the concatenated heads are multiplied element by element by `logistic(W_g h)`
+before the last product; its columns are made with the queries' product, and the gate itself is
+part of the value map's kernel.
 """
 
 from __future__ import annotations
@@ -41,7 +45,7 @@ from mini_infer_amd.parts.linear import Linear
 from mini_infer_amd.registry import POSITION_ENCODINGS, register_mixer
 
 DEFAULT_NAMES = {"q": "q", "down": "dkv", "down_norm": "dkv.norm", "up_k": "uk", "up_v": "uv", "out": "o",
-                 "q_down": "dq", "q_down_norm": "dq.norm", "q_up": "uq", "sink": "sink"}
+                 "q_down": "dq", "q_down_norm": "dq.norm", "q_up": "uq", "sink": "sink", "gate": "g"}
 
 
 class LatentAttention(Mixer):
@@ -50,17 +54,18 @@ class LatentAttention(Mixer):
     def __init__(self, hidden_size: int, num_heads: int, head_dim: int, rot_dim: int, v_head_dim: int, kv_rank: int,
                  position: PositionEncoding, scale: float, norm_eps: float, dtype: torch.dtype, device, *,
                  names: dict[str, str] | None = None, suffix: str = "", q_rank: int | None = None, window: int | None = None,
-                 learned_sink: bool = False) -> None:
+                 learned_sink: bool = False, output_gate: bool = False) -> None:
         """`q_rank`: the queries go through a latent of their own, `q = W_uq rms_norm(W_dq h)` (tensors
         `q_down`, `q_down_norm`, `q_up` of `names`) instead of one product `W_q h`.  `window`: position i
         sees only the last `window` positions, itself included.  `learned_sink`: the softmax's
-        denominator holds `exp(sink_h)` too, `sink_h` a learned number per head (tensor `sink`)."""
+        denominator holds `exp(sink_h)` too, `sink_h` a learned number per head (tensor `sink`).
+        `output_gate`: the heads' outputs are multiplied by `logistic(W_g h)` (tensor `gate`)."""
         super().__init__(dtype, device)
         if q_rank is not None and q_rank <= 0:
             raise ValueError(f"latent attention: q_rank must be positive, got {q_rank}")
         if window is not None and window <= 0:
             raise ValueError(f"latent attention: the window must be positive, got {window}")
-        self.q_rank, self.window, self.learned_sink = q_rank, window, bool(learned_sink)
+        self.q_rank, self.window, self.learned_sink, self.output_gate = q_rank, window, bool(learned_sink), bool(output_gate)
         for what, value in (("hidden_size", hidden_size), ("num_heads", num_heads), ("head_dim", head_dim),
                             ("v_head_dim", v_head_dim), ("kv_rank", kv_rank)):
             if value <= 0:
@@ -81,14 +86,16 @@ class LatentAttention(Mixer):
         self.names = {**DEFAULT_NAMES, **(names or {})}
         n = self.names
         self.q_head_width = head_dim + rot_dim
+        gate_rows, gate_names = ([num_heads * v_head_dim], [n["gate"]]) if self.output_gate else ([], [])
         if q_rank is None:
-            # one product yields [q of every head | x_c | x_r]
-            self.q_down = Linear(hidden_size, [num_heads * self.q_head_width, kv_rank + rot_dim], [n["q"], n["down"]], dtype,
-                                 device, suffix=suffix)
+            # one product yields [q of every head | x_c | x_r | output gate]
+            self.q_down = Linear(hidden_size, [num_heads * self.q_head_width, kv_rank + rot_dim] + gate_rows,
+                                 [n["q"], n["down"]] + gate_names, dtype, device, suffix=suffix)
             self.q_up = None
         else:
-            # one product yields [the queries' latent | x_c | x_r]; the queries are a second product
-            self.q_down = Linear(hidden_size, [q_rank, kv_rank + rot_dim], [n["q_down"], n["down"]], dtype, device, suffix=suffix)
+            # one product yields [the queries' latent | x_c | x_r | output gate]; the queries are a second product
+            self.q_down = Linear(hidden_size, [q_rank, kv_rank + rot_dim] + gate_rows, [n["q_down"], n["down"]] + gate_names,
+                                 dtype, device, suffix=suffix)
             self.q_up = Linear(q_rank, num_heads * self.q_head_width, n["q_up"], dtype, device, suffix=suffix)
         self.q_latent_norm: torch.Tensor | None = None
         self.sinks: torch.Tensor | None = None
@@ -98,6 +105,9 @@ class LatentAttention(Mixer):
         self.latent_norm: torch.Tensor | None = None
         self.fold_k: torch.Tensor | None = None  # [heads, kv_rank, head_dim]: W_uk,a transposed
         self.map_v: torch.Tensor | None = None  # [heads, v_head_dim, kv_rank]
+        # the same two with their last axes exchanged, contiguous: what a batched product takes on its right
+        self.fold_k_kn: torch.Tensor | None = None
+        self.map_v_kn: torch.Tensor | None = None
         self._out_padded: torch.Tensor | None = None  # W_o with zero columns where expanded value heads are padded
 
     def param_specs(self, prefix: str) -> dict[str, ParamSpec]:
@@ -127,6 +137,9 @@ class LatentAttention(Mixer):
         assert self.up_k.weight is not None and self.up_v.weight is not None
         self.fold_k = self.up_k.weight.view(self.num_heads, self.head_dim, self.kv_rank).transpose(1, 2).contiguous()
         self.map_v = self.up_v.weight.view(self.num_heads, self.v_head_dim, self.kv_rank)
+        if self.dtype != torch.float32:
+            self.fold_k_kn = self.up_k.weight.view(self.num_heads, self.head_dim, self.kv_rank)
+            self.map_v_kn = self.map_v.transpose(1, 2).contiguous()
         self._out_padded = None
 
     def cache_needs(self, page_size: int) -> CacheNeeds:
@@ -170,8 +183,8 @@ class LatentAttention(Mixer):
             ctx.shared[key] = (both[: slots.size], both[slots.size:].view(table.shape), int(first[-1]))
         return ctx.shared[key]
 
-    def _forward_expanded(self, proj: torch.Tensor, down, c_col: int, ctx: StepContext, cache: LayerCache,
-                          writes_cache: bool) -> torch.Tensor:
+    def _forward_expanded(self, proj: torch.Tensor, down, c_col: int, gate: torch.Tensor | None, ctx: StepContext,
+                          cache: LayerCache, writes_cache: bool) -> torch.Tensor:
         heads, rank, rot, dim, vdim = self.num_heads, self.kv_rank, self.rot_dim, self.head_dim, self.v_head_dim
         width, tokens = dim + rot, proj.shape[0]
         rotary = self.position.rotary(ctx)
@@ -195,6 +208,10 @@ class LatentAttention(Mixer):
             kv_heads=heads, head_dim=width, scale=self.scale, window=self.window, max_seq_len=ctx.max_q_len, v_transposed=True,
             sinks=self.sinks,
         )
+        if gate is not None:  # (the padding of the value heads leaves with it)
+            packed = torch.empty((tokens, heads, vdim), dtype=mixed.dtype, device=mixed.device)
+            ops.gate_heads(mixed.unflatten(1, (heads, width)), gate, packed)
+            return self.out.forward(packed.view(tokens, heads * vdim))
         if self._out_padded is None:  # W_o with zero columns under the padding of every value head
             assert self.out.weight is not None
             padded = torch.zeros((self.hidden_size, heads, width), dtype=self.out.weight.dtype, device=self.out.weight.device)
@@ -211,13 +228,16 @@ class LatentAttention(Mixer):
         heads, rank, rot, width = self.num_heads, self.kv_rank, self.rot_dim, self.kv_rank + self.rot_dim
         proj = self.q_down.forward(x)
         down, c_col = None, heads * self.q_head_width
+        gate = None
+        if self.output_gate:  # (the last columns of the product)
+            gate = proj[:, proj.shape[1] - heads * self.v_head_dim:].unflatten(1, (heads, self.v_head_dim))
         if self.q_up is not None:
             # [the queries' latent | x_c | x_r]: the latent is normed, and the queries are a product of their own
             assert self.q_latent_norm is not None
             down, c_col = proj, self.q_rank
             proj = self.q_up.forward(ops.norm_rows(proj, self.q_latent_norm, self.norm_eps, width=self.q_rank))
         if self._expands(ctx):
-            return self._forward_expanded(proj, down, c_col, ctx, cache, writes_cache)
+            return self._forward_expanded(proj, down, c_col, gate, ctx, cache, writes_cache)
         tokens = proj.shape[0]
         rotary = self.position.rotary(ctx)
         queries = torch.empty((tokens, heads * width), dtype=proj.dtype, device=proj.device)
@@ -228,15 +248,16 @@ class LatentAttention(Mixer):
         )
         # the key map folded into the queries: q'_a = W_uk,a^T q_a,plain
         plain = proj[:, : heads * self.q_head_width].unflatten(1, (heads, self.q_head_width))[:, :, : self.head_dim]
-        ops.linear_per_head(plain, self.fold_k, queries.unflatten(1, (heads, width))[:, :, :rank])
+        ops.linear_per_head(plain, self.fold_k, queries.unflatten(1, (heads, width))[:, :, :rank], weight_kn=self.fold_k_kn)
         mixed = ops.paged_attention(
             queries, cache.k_pages, None, ctx.block_tables[cache.group], ctx.token_request, ctx.positions,
             ctx.cu_seqlens_q, ctx.host_cu_seqlens_q, q_heads=heads, kv_heads=1, head_dim=width, scale=self.scale,
             window=self.window, max_seq_len=ctx.max_seq_len, v_head_dim=rank, sinks=self.sinks,
         )
-        # the value map after the attention: W_uv,a (sum_j p_j c_j)
+        # the value map after the attention, W_uv,a (sum_j p_j c_j), and the output gate
         values = torch.empty((tokens, heads * self.v_head_dim), dtype=proj.dtype, device=proj.device)
-        ops.linear_per_head(mixed.unflatten(1, (heads, rank)), self.map_v, values.unflatten(1, (heads, self.v_head_dim)))
+        ops.linear_per_head(mixed.unflatten(1, (heads, rank)), self.map_v, values.unflatten(1, (heads, self.v_head_dim)),
+                            weight_kn=self.map_v_kn, gate=gate)
         return self.out.forward(values)
 
 
@@ -253,5 +274,5 @@ def build_latent_attention(desc: dict, dtype: torch.dtype, device, shared: dict 
         int(desc["hidden_size"]), int(desc["num_heads"]), int(desc["head_dim"]), int(desc["rot_dim"]),
         int(desc["v_head_dim"]), int(desc["kv_rank"]), position, float(desc["scale"]), float(desc["norm_eps"]), dtype, device,
         names=desc.get("names"), suffix=str(desc.get("suffix", "")), q_rank=desc.get("q_rank"), window=desc.get("window"),
-        learned_sink=bool(desc.get("learned_sink", False)),
+        learned_sink=bool(desc.get("learned_sink", False)), output_gate=bool(desc.get("output_gate", False)),
     )

@@ -54,6 +54,9 @@ class RMSNorm(Norm):
             # the sublayers' outputs of a layer that adds them together, scaled: the add and
             # the norm are one launch
             return ops.stream_update_norm(delta, residual, self.weight, self.eps, rows)
+        if isinstance(delta, ops.GatedNormedUpdate):
+            # a sublayer's output with a gate and a norm of its own: all of it and this norm are one launch
+            return ops.gated_update_norm(delta, residual, self.weight, self.eps, rows)
         if isinstance(delta, ops.PendingProduct):
             # few rows: the product, the add and the norm but for the rows' factors are one
             # kernel, if the part that follows has a kernel that applies the factors in this step
@@ -68,6 +71,15 @@ class RMSNorm(Norm):
                 return ops.linear_add_norm(delta, residual, self.weight, self.eps)
             delta = delta.finish()
         return ops.add_rmsnorm(delta, residual, self.weight, self.eps, rows)
+
+
+    def forward_conv(self, delta, residual, conv):
+        """The norm and the convolution on its output; a gated update and, in a step of single tokens, the
+        convolution are the norm's own launch."""
+        assert self.weight is not None, "RMSNorm used before its weight was loaded"
+        if delta is not None and not isinstance(delta, ops.GatedNormedUpdate):
+            return super().forward_conv(delta, residual, conv)
+        return ops.gated_update_norm(delta, residual, self.weight, self.eps, conv=conv)
 
 
 @register_norm("rms_norm")
