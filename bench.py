@@ -505,6 +505,25 @@ def kunudra_config(sizes: dict, layers: int) -> dict:
             "layers": [dict((latent, attention, attention, latent)[i % 4], mlp=dense if i == 0 else moe) for i in range(layers)]}
 
 
+FIGOSUN_EXPERTS = 16
+FIGOSUN_TOP = 2
+
+
+def figosun_config(sizes: dict, layers: int) -> dict:
+    """A Figosun model with the widths of a Llama configuration: every layer latent attention over all
+    keys (Llama's heads and head size, the latent four head sizes wide with half a head size of rotated
+    part) and 16 ungated experts of which a token takes 2, three eighths as wide as Llama's feed-forward (two
+    matrices that hold as much as three of a quarter of that width); gates on both sublayers, convolutions of
+    four taps on what they read."""
+    h, heads, d, ff = sizes["hidden_size"], sizes["num_attention_heads"], sizes["head_dim"], sizes["intermediate_size"]
+    layer = {"type": "latent_attention",
+             "mixer": {"heads": heads, "dim": d, "rot_dim": d // 2, "vdim": d, "kv_rank": 4 * d, "scale": (d + d // 2) ** -0.5,
+                       "rot": {"base": 10000.0, "dims": d // 2}},
+             "mlp": {"kind": "moe", "expert": {"ff": 3 * ff // 8}, "router": {"experts": FIGOSUN_EXPERTS, "top": FIGOSUN_TOP}}}
+    return {"architecture": "Figosun", "vocab": sizes["vocab_size"], "width": h, "norm": {"eps": 1e-6}, "canon": {"taps": 4},
+            "embedding": {"scale": float(h) ** 0.5}, "layers": [layer for _ in range(layers)]}
+
+
 def model_costs(model, raw: dict, tokens: int, context: float) -> dict:
     """What a step must move and compute, from the model's own list of tensors: bytes of every matrix
     a decode step streams (tables that are only gathered from are left out), multiply-adds of its
@@ -553,6 +572,23 @@ def model_costs(model, raw: dict, tokens: int, context: float) -> dict:
         expert_flops = sum(2.0 * tokens * m["router"]["top"] * share * 3 * m["expert"]["ff"] * raw["width"] for m, share in zip(routed, real_share))
         return {"matrix_values": matrix, "kv_values_per_request": kv_values, "expert_values": expert_values,
                 "experts": KUNUDRA_EXPERTS, "top": KUNUDRA_TOP,
+                "prefill_flops": 2.0 * tokens * (matrix - head) + 2.0 * head + attention_flops + expert_flops}
+    if raw.get("architecture") == "Figosun":
+        # one row [latent | rotated part] per token and layer; experts as for Kunudra (two matrices each); the
+        # convolutions' tails are read and written once a step; the embedding table is the head
+        mixers, routed = [l["mixer"] for l in raw["layers"]], [l["mlp"] for l in raw["layers"] if l["mlp"] is not None]
+        expert_values = sum(2 * m["expert"]["ff"] * raw["width"] for m in routed)
+        taps = raw["canon"]["taps"]
+        # (what is two-dimensional and no matrix of a product: the convolutions' taps)
+        matrix += head - FIGOSUN_EXPERTS * expert_values - (len(mixers) + len(routed)) * raw["width"] * taps
+        kv_values = sum((m["kv_rank"] + m["rot_dim"]) * context for m in mixers)
+        state_bytes = (len(mixers) + len(routed)) * 2 * 2 * (taps - 1) * raw["width"]
+        pairs_all = tokens * (tokens + 1) / 2
+        # a prompt that comes whole is scored per head against keys of dim + rot_dim and summed over values of vdim
+        attention_flops = sum(2.0 * pairs_all * m["heads"] * (m["dim"] + m["rot_dim"] + m["vdim"]) for m in mixers)
+        expert_flops = 2.0 * tokens * FIGOSUN_TOP * expert_values
+        return {"matrix_values": matrix, "kv_values_per_request": kv_values, "state_bytes_per_request": state_bytes,
+                "expert_values": expert_values, "experts": FIGOSUN_EXPERTS, "top": FIGOSUN_TOP,
                 "prefill_flops": 2.0 * tokens * (matrix - head) + 2.0 * head + attention_flops + expert_flops}
     if raw.get("architecture") == "Kemurax":
         # attention inside chunks: a token sees the keys of its own chunk only; the recurrences keep a
@@ -659,6 +695,8 @@ def measure_design(design: str, sizes_name: str, dtype: str, layers: int | None,
         sides = [(design, kemurax_config(sizes, layers)), ("zekonex", zekonex_config(sizes, layers)), ("llama", theirs)]
     elif design == "kunudra":  # beside the design that also has latent attention and attention with a sink, and beside Llama
         sides = [(design, kunudra_config(sizes, layers)), ("zekonex", zekonex_config(sizes, layers)), ("llama", theirs)]
+    elif design == "figosun":  # beside the other design with latent attention and routed experts, and beside Llama
+        sides = [(design, figosun_config(sizes, layers)), ("kunudra", kunudra_config(sizes, layers)), ("llama", theirs)]
     else:
         raise ValueError(f"no design {design!r} to compare")
     line = {"design": design, "sizes": f"{model_name} layer sizes", "layers": layers, "dtype": dtype, "window": DESIGN_WINDOW,
@@ -706,10 +744,10 @@ def main() -> int:
                         help="with --serving / --reference-workload: launch steps that have portions of prompts in them kernel "
                         "by kernel, however few their tokens (recorded steps of single tokens stay)")
     parser.add_argument(
-        "--design", default=None, choices=("nadosun", "zekonex", "kemurax", "kunudra"),
+        "--design", default=None, choices=("nadosun", "zekonex", "kemurax", "kunudra", "figosun"),
         help="instead of the default run: prefill (one 2,048-token prompt) and decode (batch 1, --batch and 64; --steps "
         "steps, default 64 here) of that design beside Llama at the layer sizes of --sizes and equal depth "
-        "(--layers, default 12; zekonex also beside nadosun, kemurax and kunudra beside zekonex); prints one JSON line and exits",
+        "(--layers, default 12; zekonex also beside nadosun, kemurax and kunudra beside zekonex, figosun beside kunudra); prints one JSON line and exits",
     )
     parser.add_argument("--design-alone", action="store_true", help="with --design: leave the Llama side out (for profiles)")
     parser.add_argument("--attention-batch", type=int, default=0)

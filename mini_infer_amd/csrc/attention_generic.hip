@@ -253,18 +253,20 @@ __global__ __launch_bounds__(64) void attn_generic_kernel(
   }
 }
 
-// Combine the splits of one (token, head): one wave; lanes first share the work of
-// reading the splits' (max, sum) pairs, then own output dims.  The order of the sums
-// is fixed, so the result does not depend on timing.
+// Combine the splits of one (token, head): one wave, or for heads of more than 128 dims one wave per
+// 64 dims; lanes first share the work of reading the splits' (max, sum) pairs, then own output
+// dims.  The order of the sums is fixed, so the result does not depend on timing.
+static inline int reduce_threads(int head_dim) { return head_dim <= 2 * MI_WAVE ? MI_WAVE : min(512, ceil_div(head_dim, MI_WAVE) * MI_WAVE); }
+
 template <typename T>
-__global__ __launch_bounds__(64) void attn_reduce_kernel(const float* __restrict__ part_acc,
+__global__ __launch_bounds__(512) void attn_reduce_kernel(const float* __restrict__ part_acc,
                                                          const float* __restrict__ part_ml,
                                                          T* __restrict__ out, int64_t out_row_stride,
                                                          int q_heads, int head_dim, int num_splits,
                                                          int has_sink, float sink_logit, const float* __restrict__ sinks) {
   using S = typename SumType<T>::type;
   const int t = blockIdx.x, h = blockIdx.y;
-  const int lane = threadIdx.x;
+  const int lane = threadIdx.x % MI_WAVE;
   const int64_t base = ((int64_t)t * q_heads + h) * num_splits;
   constexpr int BATCH = 8;
   // Few splits of a head of at most 128 dims (the usual decode step): every partial value
@@ -309,7 +311,7 @@ __global__ __launch_bounds__(64) void attn_reduce_kernel(const float* __restrict
     }
     return;
   }
-  for (int d0 = 0; d0 < head_dim; d0 += MI_WAVE) {  // all lanes stay in the loop for the shuffles
+  for (int d0 = threadIdx.x - lane; d0 < head_dim; d0 += blockDim.x) {  // all lanes of a wave stay in the loop for the shuffles
     const int d = d0 + lane;
     const bool active = d < head_dim;
     const float* src = part_acc + base * head_dim + (active ? d : 0);
@@ -362,7 +364,7 @@ static int attn_generic_launch(const void* q, int64_t q_row_stride, const void* 
   MI_CHECK_LAUNCH("attn_generic");
   if (num_splits > 1) {
     dim3 rgrid(num_tokens, q_heads);
-    attn_reduce_kernel<T><<<rgrid, MI_WAVE, 0, stream>>>(part_acc, part_ml, (T*)out, out_row_stride,
+    attn_reduce_kernel<T><<<rgrid, reduce_threads(v_dim), 0, stream>>>(part_acc, part_ml, (T*)out, out_row_stride,
                                                          q_heads, v_dim, num_splits, has_sink, sink_logit, sinks);
     MI_CHECK_LAUNCH("attn_reduce");
   }
@@ -466,7 +468,7 @@ extern "C" int mi_attn_reduce_bf16(const float* part_acc, const float* part_ml, 
   if (num_tokens == 0) return MI_OK;
   MI_REQUIRE(q_heads <= 65535, "attn_reduce: too many heads");
   dim3 rgrid(num_tokens, q_heads);
-  attn_reduce_kernel<bf16_t><<<rgrid, MI_WAVE, 0, stream>>>(part_acc, part_ml, (bf16_t*)out,
+  attn_reduce_kernel<bf16_t><<<rgrid, reduce_threads(head_dim), 0, stream>>>(part_acc, part_ml, (bf16_t*)out,
                                                             out_row_stride, q_heads, head_dim,
                                                             num_splits, has_sink, sink_logit, sinks);
   MI_CHECK_LAUNCH("attn_reduce");

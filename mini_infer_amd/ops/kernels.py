@@ -1190,6 +1190,83 @@ def _paged_attention_general(
     return out
 
 
+# blocks of the latent attention kernel wanted in a launch (blocks of one or two waves, two to a CU; of four, one),
+# and the keys a range has at least
+LATENT_ATTENTION_BLOCKS, LATENT_ATTENTION_BLOCKS_WIDE, LATENT_ATTENTION_MIN_KEYS = 512, 256, 64
+
+
+def latent_attention_takes(dtype: torch.dtype, rank: int, rot: int) -> bool:
+    """Whether attention over cached rows [latent (rank) | rotated part (rot)] runs on the matrix cores."""
+    return dtype == torch.bfloat16 and bool(library.load().mi_attn_latent_takes(rank, rot))
+
+
+def latent_attention(
+    q: torch.Tensor, k_pages: torch.Tensor, block_table: torch.Tensor, token_request: torch.Tensor, positions: torch.Tensor,
+    cu_seqlens_q: torch.Tensor, host_cu_seqlens_q: list[int] | None, *, heads: int, rank: int, rot: int, scale: float,
+    window: int | None, max_seq_len: int, sinks: torch.Tensor | None = None, splits: int | None = None,
+) -> torch.Tensor:
+    """Causal attention of every token over its request's latent rows: `k_pages` [num_pages, 1, page_size,
+    rank + rot], a value being the first `rank` entries of its key row; `q` [T, heads * (rank + rot)] ->
+    [T, heads * rank].  Window, sinks, request boundaries (device-only with `host_cu_seqlens_q=None`) as
+    `paged_attention`, which also is what sizes and dtypes run that the matrix-core kernel does not take."""
+    width = rank + rot
+    aligned = q.dim() == 2 and q.stride(1) == 1 and q.stride(0) % 8 == 0 and q.data_ptr() % 16 == 0
+    if not (aligned and latent_attention_takes(q.dtype, rank, rot)):
+        return paged_attention(
+            q, k_pages, None, block_table, token_request, positions, cu_seqlens_q, host_cu_seqlens_q, q_heads=heads, kv_heads=1,
+            head_dim=width, scale=scale, window=window, max_seq_len=max_seq_len, v_head_dim=rank, sinks=sinks,
+        )
+    _need_cuda(q, k_pages, block_table, positions, cu_seqlens_q, sinks)
+    for name, t in (("k_pages", k_pages), ("block_table", block_table), ("positions", positions), ("cu_seqlens_q", cu_seqlens_q), ("sinks", sinks)):
+        _need_contiguous(name, t)
+    for name, t in (("block_table", block_table), ("positions", positions), ("cu_seqlens_q", cu_seqlens_q)):
+        _need_int32(name, t)
+    _need_f32("sinks", sinks)
+    tokens = q.shape[0]
+    if q.shape[1] < heads * width or k_pages.dtype != q.dtype or k_pages.dim() != 4 or k_pages.shape[1] != 1 or k_pages.shape[3] != width:
+        raise KernelShapeError(f"latent_attention: q [T, >= {heads * width}], key pages {q.dtype} [num_pages, 1, page_size, {width}], "
+                               f"got {tuple(q.shape)}, {k_pages.dtype} {tuple(k_pages.shape)}")
+    if block_table.dim() != 2 or positions.numel() != tokens or cu_seqlens_q.numel() != block_table.shape[0] + 1:
+        raise KernelShapeError("latent_attention: one position a token, one boundary more than requests, block_table [requests, max_blocks]")
+    if k_pages.shape[0] * k_pages.shape[2] >= 1 << 31 or (sinks is not None and sinks.numel() != heads):
+        raise KernelShapeError("latent_attention: too many key rows, or not one sink per head")
+    requests = block_table.shape[0]
+    lens = None
+    if host_cu_seqlens_q is not None:
+        if len(host_cu_seqlens_q) != requests + 1 or host_cu_seqlens_q[-1] != tokens:
+            raise KernelShapeError(f"latent_attention: the boundaries end at {host_cu_seqlens_q[-1]} of {tokens} tokens")
+        lens = [host_cu_seqlens_q[b + 1] - host_cu_seqlens_q[b] for b in range(requests)]
+    lib = library.load()
+    single = lens is not None and tokens == requests and max(lens, default=0) == 1
+    longest = 1 if single else (max(lens) if lens is not None else tokens)
+    waves = lib.mi_attn_latent_waves(min(longest, tokens) * heads)
+    rows = 16 * waves
+    if single:
+        tiles = requests * -(-heads // rows)
+    elif lens is not None:
+        tiles = sum(-(-n * heads // rows) for n in lens)
+    else:
+        tiles = tokens * heads // rows + requests
+    # (no row sees more keys than a window holds; a block's rows together see a few more)
+    span = min(max_seq_len, window + longest) if window else max_seq_len
+    if splits is None:
+        wanted = LATENT_ATTENTION_BLOCKS_WIDE if waves == 4 else LATENT_ATTENTION_BLOCKS
+        splits = max(1, min(64, wanted // max(1, tiles), span // LATENT_ATTENTION_MIN_KEYS))
+    out = torch.empty((tokens, heads * rank), dtype=q.dtype, device=q.device)
+    part_acc = part_ml = None
+    if splits > 1:
+        part_acc = torch.empty((tokens * heads * splits, rank), dtype=torch.float32, device=q.device)
+        part_ml = torch.empty((tokens * heads * splits, 2), dtype=torch.float32, device=q.device)
+    library.check(
+        lib.mi_attn_latent(
+            _ptr(q), q.stride(0), _ptr(k_pages), _ptr(block_table), block_table.shape[1], _ptr(cu_seqlens_q), _ptr(positions), requests,
+            tokens, tiles, waves, _ptr(out), out.stride(0), _ptr(part_acc), _ptr(part_ml), heads, rank, rot, k_pages.shape[2],
+            float(scale), int(window or 0), splits, int(single), _ptr(sinks), _stream(),
+        )
+    )
+    return out
+
+
 # ----------------------------------------------------------------------------
 # sublayers that add their own normed output to the stream, and what goes with them
 # ----------------------------------------------------------------------------
@@ -2517,20 +2594,37 @@ def experts_by_expert_take(x: torch.Tensor, gate_up: torch.Tensor, activation: s
 
 
 EXPERT_TILES_MIN_ROWS = 48  # rows an expert gets on average from which on the 64 x 64 tiles are taken
+EXPERT_LDS_TILES_MIN_ROWS = 12  # and those staged through LDS (16 experts of 4096 x 5376, 8 / 16 rows each: 303 / 437 against 296 / 296 us)
+EXPERT_TILES = ("rows", "direct", "lds")
+
+
+def expert_tiles_take(x: torch.Tensor, ff: int) -> bool:
+    """Whether the tiles staged through LDS take rows like those of `x` and rows of `ff`."""
+    lib = library.load()
+    return x.dtype == torch.bfloat16 and bool(lib.mi_expert_tiles_take(x.shape[1])) and bool(lib.mi_expert_tiles_take(ff))
+
+
+def expert_tiles_for(x: torch.Tensor, pairs: int, experts: int, ff: int) -> str:
+    """The form in which `experts_by_expert` makes its products for `pairs` (row, choice) pairs."""
+    if pairs >= EXPERT_LDS_TILES_MIN_ROWS * experts and expert_tiles_take(x, ff):
+        return "lds"
+    return "direct" if pairs >= EXPERT_TILES_MIN_ROWS * experts else "rows"
 GROUPED_ROWS_STEP = 64  # the sorted form's products run over row counts rounded up to a multiple of this
 
 
 def experts_by_expert(
     x: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, chosen: torch.Tensor, weights: torch.Tensor,
-    shared: torch.Tensor | None = None, shared_gate: torch.Tensor | None = None, many_rows: bool | None = None, *,
+    shared: torch.Tensor | None = None, shared_gate: torch.Tensor | None = None, tiles: str | None = None, *,
     activation: str = "silu_gated", weight_on: str = "output", combine: bool = True,
 ) -> "torch.Tensor | SummedRows":
     """The same sum as `experts_few_rows`, expert by expert without the host knowing anything: one small
     kernel lists the (row, expert) pairs by expert, then every chosen expert's block streams its
     weights once for up to eight of the expert's rows at a time (the rows wait in LDS), and one kernel adds
     a row's results in the order of its choices.  Four launches; an expert that many rows chose is read once
-    per sixteen of them, not once per row.  `many_rows` (default: by the average number of rows an expert
-    gets): blocks of 64 features that take 64 of an expert's rows a pass, for prompts (bfloat16).  `combine=False`
+    per sixteen of them, not once per row.  `tiles` (default: by the average number of rows an expert
+    gets): "rows" is that form; for prompts (bfloat16) "direct", blocks of 64 features that take 64 of an
+    expert's rows a pass, and "lds", tiles of 128 rows x 128 features with both operands staged through LDS
+    (rows in steps of 64 elements).  `combine=False`
     (weights on the input, no shared or identity experts): the rows are left for a norm to add up (`SummedRows`)."""
     tokens, width, experts, ff, top = _check_experts(x, gate_up, down, chosen, weights, shared, shared_gate, activation, weight_on)
     mode, on_input, on_output = _expert_weights(activation, weights, weight_on)
@@ -2544,14 +2638,22 @@ def experts_by_expert(
     act = torch.empty((pairs, ff), dtype=x.dtype, device=x.device)
     made = torch.empty((pairs, width), dtype=x.dtype, device=x.device)
     lib, code = library.load(), _dtype_code(x)
-    if many_rows is None:
-        many_rows = pairs >= EXPERT_TILES_MIN_ROWS * experts
-    many = int(bool(many_rows))
+    if tiles is None:
+        tiles = expert_tiles_for(x, pairs, experts, ff)
+    elif tiles not in EXPERT_TILES or (tiles == "lds" and not expert_tiles_take(x, ff)):
+        raise KernelShapeError(f"experts_by_expert: tiles {tiles!r} for rows of {width} and {ff} {x.dtype}")
+    many = int(tiles == "direct")
     library.check(lib.mi_expert_sort(_ptr(chosen), _ptr(listed), _ptr(first), pairs, experts, _stream()))
-    library.check(lib.mi_expert_rows(code, mode, _ptr(x), x.stride(0), top, _ptr(gate_up), _ptr(listed), _ptr(first),
-                                     _ptr(on_input), _ptr(act), ff, experts, width, ff, many, _stream()))
-    library.check(lib.mi_expert_rows(code, 0, _ptr(act), ff, 1, _ptr(down), _ptr(listed), _ptr(first), None, _ptr(made), width,
-                                     experts, ff, width, many, _stream()))
+    if tiles == "lds":
+        library.check(lib.mi_expert_tiles(mode, _ptr(x), x.stride(0), top, _ptr(gate_up), _ptr(listed), _ptr(first),
+                                          _ptr(on_input), _ptr(act), ff, pairs, experts, width, ff, _stream()))
+        library.check(lib.mi_expert_tiles(0, _ptr(act), ff, 1, _ptr(down), _ptr(listed), _ptr(first), None, _ptr(made),
+                                          width, pairs, experts, ff, width, _stream()))
+    else:
+        library.check(lib.mi_expert_rows(code, mode, _ptr(x), x.stride(0), top, _ptr(gate_up), _ptr(listed), _ptr(first),
+                                         _ptr(on_input), _ptr(act), ff, experts, width, ff, many, _stream()))
+        library.check(lib.mi_expert_rows(code, 0, _ptr(act), ff, 1, _ptr(down), _ptr(listed), _ptr(first), None, _ptr(made),
+                                         width, experts, ff, width, many, _stream()))
     if not combine:
         return SummedRows(made, top)
     out = torch.empty((tokens, width), dtype=x.dtype, device=x.device)

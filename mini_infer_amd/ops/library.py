@@ -131,6 +131,14 @@ _SIGNATURES: dict[str, list] = {
     "mi_expert_sort": [_P, _P, _P, c_int, c_int, _P],
     "mi_expert_rows_at_once": [c_int, c_int],
     "mi_expert_rows": [c_int, c_int, _P, c_int64, c_int, _P, _P, _P, _P, _P, c_int64, c_int, c_int, c_int, c_int, _P],
+    "mi_attn_latent_takes": [c_int, c_int],
+    "mi_attn_latent_waves": [c_int],
+    "mi_attn_latent": [
+        _P, c_int64, _P, _P, c_int, _P, _P, c_int, c_int, c_int, c_int, _P, c_int64, _P, _P, c_int, c_int, c_int, c_int, c_float,
+        c_int, c_int, c_int, _P, _P,
+    ],
+    "mi_expert_tiles_take": [c_int],
+    "mi_expert_tiles": [c_int, _P, c_int64, c_int, _P, _P, _P, _P, _P, c_int64, c_int, c_int, c_int, c_int, _P],
     "mi_gated_update_norm": [
         c_int, _P, _P, c_int64, c_int, _P, c_int64, _P, _P, _P, _P, _P, c_int, c_int, c_float, c_float, _P, c_int, _P,
         c_int64, _P, _P, c_int, _P, _P,

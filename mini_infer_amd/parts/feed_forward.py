@@ -278,8 +278,9 @@ class RoutedExperts(FeedForward):
     knowing anything: the (token, expert) pairs are listed by expert on the device, and every chosen
     expert's weights are streamed once for up to eight of its rows at a time (sizes that are not read
     16 bytes at a time work each pair on its own instead, the expert's weights read by index).  Many
-    rows are sorted by expert and every chosen expert runs the engine's own products once over all
-    its rows.  Router, correction and the shared expert's gate row stay float32."""
+    rows (bfloat16, rows in steps of 64 elements) run over tiles of 128 of an expert's rows staged through
+    LDS, from the same list; sizes those do not take are sorted by expert and every chosen expert runs the
+    engine's own products once over all its rows.  Router, correction and the shared expert's gate row stay float32."""
 
     graph_safe = True
 
@@ -360,14 +361,16 @@ class RoutedExperts(FeedForward):
             self.shared.load_params(prefix, get)
             self.shared_gate_row = get(prefix + self.names["shared_gate"]).float().reshape(-1).contiguous()
 
-    def _grouped(self, rows: int, ctx: StepContext) -> bool:
+    def _grouped(self, x: torch.Tensor, ctx: StepContext) -> bool:
         if self.force_form is not None:
             return self.force_form == "grouped"
         if ctx.host_cu_seqlens_q is None or torch.cuda.is_current_stream_capturing():
             return False  # (the sorted form reads the experts' row counts on the host)
+        if ops.expert_tiles_take(x, self.intermediate_size):
+            return False  # (tiles over the device's own list of rows are faster at every size)
         element = 2 if self.dtype == torch.bfloat16 else 4
         expert_bytes = (3 if self.gated else 2) * self.intermediate_size * self.hidden_size * element
-        return rows * self.top * expert_bytes > self.experts * self.GROUPED_BYTES_PER_EXPERT
+        return x.shape[0] * self.top * expert_bytes > self.experts * self.GROUPED_BYTES_PER_EXPERT
 
     def forward(self, x, ctx: StepContext) -> torch.Tensor:
         assert self.router is not None and self.gate_up is not None and self.down is not None, \
@@ -381,7 +384,7 @@ class RoutedExperts(FeedForward):
             shared = self.shared.forward(x, ctx)
             shared = shared.finish() if hasattr(shared, "finish") else shared
         how = {"activation": self.activation, "weight_on": self.weight_on}
-        if self._grouped(x.shape[0], ctx):
+        if self._grouped(x, ctx):
             run = ops.experts_grouped
         elif self.force_form == "by_expert" or (
                 self.force_form is None and ops.experts_by_expert_take(x, self.gate_up, self.activation)):

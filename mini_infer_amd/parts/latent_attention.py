@@ -249,10 +249,10 @@ class LatentAttention(Mixer):
         # the key map folded into the queries: q'_a = W_uk,a^T q_a,plain
         plain = proj[:, : heads * self.q_head_width].unflatten(1, (heads, self.q_head_width))[:, :, : self.head_dim]
         ops.linear_per_head(plain, self.fold_k, queries.unflatten(1, (heads, width))[:, :, :rank], weight_kn=self.fold_k_kn)
-        mixed = ops.paged_attention(
-            queries, cache.k_pages, None, ctx.block_tables[cache.group], ctx.token_request, ctx.positions,
-            ctx.cu_seqlens_q, ctx.host_cu_seqlens_q, q_heads=heads, kv_heads=1, head_dim=width, scale=self.scale,
-            window=self.window, max_seq_len=ctx.max_seq_len, v_head_dim=rank, sinks=self.sinks,
+        mixed = ops.latent_attention(
+            queries, cache.k_pages, ctx.block_tables[cache.group], ctx.token_request, ctx.positions, ctx.cu_seqlens_q,
+            ctx.host_cu_seqlens_q, heads=heads, rank=rank, rot=rot, scale=self.scale, window=self.window,
+            max_seq_len=ctx.max_seq_len, sinks=self.sinks,
         )
         # the value map after the attention, W_uv,a (sum_j p_j c_j), and the output gate
         values = torch.empty((tokens, heads * self.v_head_dim), dtype=proj.dtype, device=proj.device)

@@ -384,7 +384,7 @@ def test_the_router_and_both_forms_of_the_experts(dtype, rows, width, ff, expert
     forms = [ops.experts_few_rows, ops.experts_grouped]
     if ops.experts_by_expert_take(xd, dev(gate_up, TORCH[dtype])):
         # (16 rows of an expert a pass, and the tiles of 64 rows x 64 features that prompts take)
-        forms += [lambda *a: ops.experts_by_expert(*a, many_rows=False), lambda *a: ops.experts_by_expert(*a, many_rows=True)]
+        forms += [lambda *a: ops.experts_by_expert(*a, tiles="rows"), lambda *a: ops.experts_by_expert(*a, tiles="direct")]
     assert len(forms) == 4 or width % 8 or ff % 8
     for form in forms:
         got = form(xd, dev(gate_up, TORCH[dtype]), dev(down, TORCH[dtype]), chosen, w, sd, g).float().cpu().numpy()
