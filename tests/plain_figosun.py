@@ -8,7 +8,7 @@ Notation: `x` is the stream [T, W]; `h` what a sublayer's norm made of it; `i`, 
 counted from 0.
 
 `store` (default: nothing) is applied to every tensor an engine would keep in its compute dtype
-(norm outputs, projections, activations, sublayer outputs, cached rows; never the stream or
+(norm outputs, projections, activations, sublayer outputs, cached rows, logits; never the stream or
 anything inside a softmax, a norm or a router).  With `bf16_round` the model shows how far bfloat16
 storage alone, with exact arithmetic between, moves the logits: the yardstick of the bfloat16 tests.
 """
@@ -166,7 +166,7 @@ def forward(config: dict, weights: dict, tokens, store=keep, layers_out: list | 
 def logits(config: dict, weights: dict, tokens, store=keep, layers_out: list | None = None) -> np.ndarray:
     x = forward(config, weights, tokens, store, layers_out)
     h = store(rms_norm(x, np.asarray(weights["final.norm"], dtype=np.float64), config["norm"]["eps"]))
-    return h @ np.asarray(weights["embed"], dtype=np.float64).T
+    return store(h @ np.asarray(weights["embed"], dtype=np.float64).T)
 
 
 def greedy(row: np.ndarray) -> int:
