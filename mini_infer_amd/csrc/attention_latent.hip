@@ -22,14 +22,12 @@
 // neighbouring chunks, lie in different banks.
 //
 // Keys are cut into `splits` ranges (blockIdx.y); a range leaves its accumulators, maximum (natural log
-// units) and sum as the other attention kernels do, for their combining kernel.
+// units) and sum, and `latent_combine` puts the ranges of a (token, head) together: four groups of lanes take
+// every fourth range each, four columns a lane, all their loads asked for at once, and meet in LDS in
+// group order.
 #include "common.h"
 
 #include <math.h>
-
-extern "C" int mi_attn_reduce_bf16(const float* part_acc, const float* part_ml, void* out, int64_t out_row_stride,
-                                   int num_tokens, int q_heads, int head_dim, int num_splits, int has_sink,
-                                   float sink_logit, const float* sinks, hipStream_t stream);
 
 namespace {
 
@@ -329,6 +327,50 @@ __global__ __launch_bounds__(WAVES * MI_WAVE, 1) void attn_latent_kernel(
   }
 }
 
+// lane s's value, s the same in all lanes: a register move
+__device__ __forceinline__ float of_lane(float v, int s) {
+  return __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, v), s));
+}
+
+// EACH: ranges a group takes, at most (4 * EACH >= splits)
+template <int EACH>
+__global__ __launch_bounds__(512) void latent_combine_kernel(const float* __restrict__ part_acc,
+                                                             const float* __restrict__ part_ml, bf16_t* __restrict__ out,
+                                                             int64_t out_stride, int heads, int rank, int splits,
+                                                             const float* __restrict__ sinks) {
+  __shared__ f32x4_l meet[3][128];
+  const int t = blockIdx.x, h = blockIdx.y;
+  const int lanes = blockDim.x / 4;  // of a group: whole waves
+  const int group = __builtin_amdgcn_readfirstlane(threadIdx.x / lanes), place = threadIdx.x % lanes, lane = threadIdx.x % MI_WAVE;
+  const int64_t base = ((int64_t)t * heads + h) * splits;
+  const bool active = place * 4 < rank;
+  const float* src = part_acc + base * rank + (active ? place * 4 : 0);
+  f32x4_l v[EACH];
+#pragma unroll
+  for (int i = 0; i < EACH; ++i)  // (past the last range: that one again, not counted)
+    v[i] = *reinterpret_cast<const f32x4_l*>(src + (int64_t)min(group + 4 * i, splits - 1) * rank);
+  const float m_s = lane < splits ? part_ml[(base + lane) * 2] : -INFINITY;
+  const float l_s = lane < splits ? part_ml[(base + lane) * 2 + 1] : 0.f;
+  const float top = wave_max(m_s);
+  const float w_s = lane < splits ? expf(m_s - top) : 0.f;
+  float all = wave_sum(l_s * w_s);
+  if (sinks != nullptr) all += expf(sinks[h] - top);
+  f32x4_l sum = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int i = 0; i < EACH; ++i)
+    if (group + 4 * i < splits) sum += v[i] * of_lane(w_s, group + 4 * i);
+  if (group > 0) meet[group - 1][place] = sum;
+  __syncthreads();
+  if (group > 0 || !active) return;
+#pragma unroll
+  for (int g = 0; g < 3; ++g) sum += meet[g][place];
+  const float inv = 1.0f / all;
+  float r[4];
+#pragma unroll
+  for (int j = 0; j < 4; ++j) r[j] = sum[j] * inv;
+  mi_store_cols<bf16_t, 4>(out + (int64_t)t * out_stride + (int64_t)h * rank + place * 4, r);
+}
+
 }  // namespace
 
 // Whether cached rows of rank + rot columns (bfloat16) are taken.
@@ -381,7 +423,19 @@ extern "C" int mi_attn_latent(const void* q, int64_t q_stride, const void* k_pag
 #undef MI_LATENT
 #undef MI_LATENT_W
   MI_CHECK_LAUNCH("attn_latent");
-  if (splits > 1)
-    return mi_attn_reduce_bf16(part_acc, part_ml, out, out_stride, num_tokens, heads, rank, splits, sinks != nullptr, 0.f, sinks, stream);
+  if (splits > 1) {
+    MI_REQUIRE(heads <= 65535, "attn_latent: too many heads (%d)", heads);
+    dim3 cgrid(num_tokens, heads);
+    const int threads = 4 * (rank <= 256 ? 64 : 128);
+#define MI_COMBINE(EACH) \
+  latent_combine_kernel<EACH><<<cgrid, threads, 0, stream>>>(part_acc, part_ml, (bf16_t*)out, out_stride, heads, rank, splits, sinks)
+    if (splits <= 4) MI_COMBINE(1);
+    else if (splits <= 8) MI_COMBINE(2);
+    else if (splits <= 16) MI_COMBINE(4);
+    else if (splits <= 32) MI_COMBINE(8);
+    else MI_COMBINE(16);
+#undef MI_COMBINE
+    MI_CHECK_LAUNCH("latent_combine");
+  }
   return MI_OK;
 }

@@ -104,8 +104,15 @@ __global__ __launch_bounds__(256) void short_conv_runs_kernel(
 #pragma unroll
   for (int e = 0; e < 4; ++e) {
     start[e] = bias ? (A)bias[c + e] : (A)0;
+    if constexpr (TAPS == 4) {  // (a channel's taps at once: one by one every load would touch a line a lane)
+      float taps_of[4];
+      mi_load_cols<float, 4>(w + (int64_t)(c + e) * 4, taps_of);
 #pragma unroll
-    for (int j = 0; j < TAPS; ++j) wc[j][e] = (A)w[(int64_t)(c + e) * TAPS + j];
+      for (int j = 0; j < 4; ++j) wc[j][e] = (A)taps_of[j];
+    } else {
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) wc[j][e] = (A)w[(int64_t)(c + e) * TAPS + j];
+    }
   }
   int of = -1;  // the request the window belongs to
   for (int t = t0; t < t1; ++t) {
@@ -517,7 +524,8 @@ extern "C" int mi_short_conv(int dtype, const void* x, int64_t x_stride, const f
   }
   const size_t elem = dtype == MI_F32 ? 4 : 2;
   const bool runs = taps >= 2 && taps <= 4 && channels % 4 == 0 && x_stride % 4 == 0 && y_stride % 4 == 0 && tail_stride % 4 == 0 &&
-                    ((uintptr_t)x | (uintptr_t)y | (uintptr_t)tail) % (4 * elem) == 0 && ceil_div(num_tokens, CONV_RUN) <= 65535;
+                    ((uintptr_t)x | (uintptr_t)y | (uintptr_t)tail) % (4 * elem) == 0 && (uintptr_t)w % 16 == 0 &&
+                    ceil_div(num_tokens, CONV_RUN) <= 65535;
   if (runs) {
     dim3 grid(ceil_div(channels, 1024), ceil_div(num_tokens, CONV_RUN));
 #define MI_CONV_RUNS(T, TAPS)                                                                                            \

@@ -5,7 +5,7 @@
 // MFMA 16x16x32 with weight rows as the first operand and tokens as the second: per step of 32 elements
 // a lane reads 16 bytes of weight row `lane % 16` and 16 bytes of token `lane % 16` (both at elements
 // 32 * step + 8 * (lane / 16)), which are the operands as they are.  A block owns one head.
-//   SHARE  few tokens: the block owns 16 features and its four waves share K (their sums meet in LDS in
+//   SHARE  up to 64 tokens: the block owns 16 features and its four waves share K (their sums meet in LDS in
 //          wave order), so that even a short K keeps every wave busy with one stretch of weights.
 //   else   a wave owns 16 features over all of K and RT row tiles of 16 tokens share each weight operand.
 // K is a multiple of 8; what a last, shorter step lacks counts as zero on both sides.
@@ -39,7 +39,7 @@ template <int RT, bool SHARE>
 __global__ __launch_bounds__(256) void per_head_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w,
                                                        const bf16_t* __restrict__ gate, bf16_t* __restrict__ out,
                                                        PerHeadShape s) {
-  __shared__ f32x4_h meet[SHARE ? 3 : 1][MI_WAVE];
+  __shared__ f32x4_h meet[SHARE ? 3 : 1][RT][MI_WAVE];
   const int h = blockIdx.y, t0 = blockIdx.z * 16 * RT;
   const int wave = threadIdx.x / MI_WAVE, lane = threadIdx.x % MI_WAVE;
   const int col = lane % 16, quad = lane / 16;
@@ -82,12 +82,16 @@ __global__ __launch_bounds__(256) void per_head_kernel(const bf16_t* __restrict_
     }
   }
   if constexpr (SHARE) {
-    static_assert(!SHARE || RT == 1, "the waves that share K take one tile of tokens");
-    if (wave > 0) meet[wave - 1][lane] = acc[0];
+    if (wave > 0) {
+#pragma unroll
+      for (int i = 0; i < RT; ++i) meet[wave - 1][i][lane] = acc[i];
+    }
     __syncthreads();
     if (wave > 0) return;
 #pragma unroll
-    for (int i = 0; i < 3; ++i) acc[0] += meet[i][lane];
+    for (int other = 0; other < 3; ++other)
+#pragma unroll
+      for (int i = 0; i < RT; ++i) acc[i] += meet[other][i][lane];
   }
 #pragma unroll
   for (int i = 0; i < RT; ++i) {
@@ -112,6 +116,10 @@ extern "C" int mi_per_head_bf16(const void* x, int64_t x_stride, int64_t x_head,
   if (tokens <= 16) {
     dim3 grid(ceil_div(features, 16), heads, 1);
     per_head_kernel<1, true><<<grid, 256, 0, stream>>>((const bf16_t*)x, (const bf16_t*)w, (const bf16_t*)gate, (bf16_t*)out, s);
+  } else if (tokens <= 64) {
+    dim3 grid(ceil_div(features, 16), heads, 1);
+    if (tokens <= 32) per_head_kernel<2, true><<<grid, 256, 0, stream>>>((const bf16_t*)x, (const bf16_t*)w, (const bf16_t*)gate, (bf16_t*)out, s);
+    else per_head_kernel<4, true><<<grid, 256, 0, stream>>>((const bf16_t*)x, (const bf16_t*)w, (const bf16_t*)gate, (bf16_t*)out, s);
   } else {
     MI_REQUIRE(ceil_div(tokens, 64) <= 65535, "per_head: too many tokens (%d)", tokens);
     dim3 grid(ceil_div(features, 64), heads, ceil_div(tokens, 64));

@@ -8,6 +8,7 @@
 //                       they are a rising function); leaves the chosen indices and their weights
 //                       s * route_scale (not renormalized), and, where a gate row is given,
 //                       logistic(gate . x) for a shared expert.
+//   route_logits, route_list   the same and the list of pairs by expert, for few bfloat16 tokens.
 //   expert_gate_up      few rows: for every (token, chosen expert) pair the expert's first product and
 //                       its activation, the weights read by expert index.
 //   expert_down_combine few rows: y[t] = sum_k w[t, k] * (W_down[e_k] act[t, k])  (+ shared_gate[t] *
@@ -68,8 +69,57 @@ __device__ __forceinline__ T expert_feature(A a, A b, A weight) {
   }
 }
 
+// A wave ranks a token's outputs, lane l those with e % 64 == l: the `top` largest choices and their weights.
+// `mine`: the token's logits in LDS, this wave's own (spent here: chosen ones are marked).
+template <typename A>
+__device__ __forceinline__ void rank_outputs(A* mine, const float* __restrict__ correction, int* __restrict__ chosen,
+                                             float* __restrict__ weights, int outputs, int top, float route_scale,
+                                             int logistic, int lane) {
+  const A taken = -(A)INFINITY;
+  A most = taken, total_exp = 0;
+  if (!logistic) {
+    for (int e = lane; e < outputs; e += MI_WAVE) most = mine[e] > most ? mine[e] : most;
+#pragma unroll
+    for (int off = MI_WAVE / 2; off > 0; off >>= 1) {
+      const A other = __shfl_xor(most, off, MI_WAVE);
+      most = other > most ? other : most;
+    }
+    for (int e = lane; e < outputs; e += MI_WAVE) total_exp += exp_of(mine[e] - most);
+    total_exp = lanes_total(total_exp);
+  }
+  const A inv = (A)1 / total_exp;  // (softmax)
+  auto score_of = [&](A logit) { return logistic ? (A)1 / ((A)1 + exp_of(-logit)) : exp_of(logit - most) * inv; };
+  // the choice is made on score + correction (without one on the logit, of which every score is a rising
+  // function), the weight is the score alone
+  for (int k = 0; k < top; ++k) {
+    int best = outputs;
+    A best_choice = taken;
+    for (int e = lane; e < outputs; e += MI_WAVE) {
+      const A logit = mine[e];
+      if (logit == taken) continue;
+      const A choice = correction != nullptr ? score_of(logit) + (A)correction[e] : logit;
+      if (best == outputs || choice > best_choice) best = e, best_choice = choice;
+    }
+#pragma unroll
+    for (int off = MI_WAVE / 2; off > 0; off >>= 1) {
+      const A other = __shfl_xor(best_choice, off, MI_WAVE);
+      const int index = __shfl_xor(best, off, MI_WAVE);
+      if (index < outputs && (best == outputs || other > best_choice || (other == best_choice && index < best))) best = index, best_choice = other;
+    }
+    if (best == outputs) best = 0;  // (more infinite logits than there are choices)
+    if (lane == 0) {
+      chosen[k] = best;
+      weights[k] = (float)(score_of(mine[best]) * (A)route_scale);
+    }
+    // (the same lane that ranks this output marks it; within a wave LDS is read and written in program order)
+    __builtin_amdgcn_wave_barrier();
+    if (lane == best % MI_WAVE) mine[best] = taken;
+    __builtin_amdgcn_wave_barrier();
+  }
+}
+
 // R tokens a block: their rows wait in LDS while every wave walks router rows (16 bytes a lane, each
-// router row read once for all R tokens), then thread r ranks token r's outputs.
+// router row read once for all R tokens), then wave r ranks token r's outputs.
 template <typename T, int R>
 __global__ __launch_bounds__(1024) void route_top_k_kernel(
     const T* __restrict__ x, int64_t x_stride, const float* __restrict__ router, const float* __restrict__ correction,
@@ -105,13 +155,25 @@ __global__ __launch_bounds__(1024) void route_top_k_kernel(
 #pragma unroll
     for (int r = 0; r < R; ++r) sum[r] = 0;
     if (vec) {
-#pragma unroll 4
-      for (int c = lane * 4; c < width; c += MI_WAVE * 4) {
-        const float4 w4 = *reinterpret_cast<const float4*>(w + c);
+      // (BATCH pieces of the router row are asked for before the first is used)
+      constexpr int BATCH = 8;
+      for (int c0 = lane * 4; c0 < width; c0 += MI_WAVE * 4 * BATCH) {
+        float4 w4[BATCH];
 #pragma unroll
-        for (int r = 0; r < R; ++r) {
-          const T* xr = rows + (size_t)r * width + c;
-          sum[r] += (A)w4.x * (A)to_f32(xr[0]) + (A)w4.y * (A)to_f32(xr[1]) + (A)w4.z * (A)to_f32(xr[2]) + (A)w4.w * (A)to_f32(xr[3]);
+        for (int i = 0; i < BATCH; ++i) {
+          const int c = c0 + i * MI_WAVE * 4;
+          w4[i] = c < width ? *reinterpret_cast<const float4*>(w + c) : make_float4(0.f, 0.f, 0.f, 0.f);
+        }
+#pragma unroll
+        for (int i = 0; i < BATCH; ++i) {
+          const int c = c0 + i * MI_WAVE * 4;
+          if (c >= width) continue;
+#pragma unroll
+          for (int r = 0; r < R; ++r) {
+            float xv[4];
+            mi_load_cols<T, 4>(rows + (size_t)r * width + c, xv);
+            sum[r] += (A)w4[i].x * (A)xv[0] + (A)w4[i].y * (A)xv[1] + (A)w4[i].z * (A)xv[2] + (A)w4[i].w * (A)xv[3];
+          }
         }
       }
     } else {
@@ -128,47 +190,12 @@ __global__ __launch_bounds__(1024) void route_top_k_kernel(
     }
   }
   __syncthreads();
-  const int r = threadIdx.x, t = t0 + r;
-  if (r >= R || t >= num_tokens) return;
-  A* mine = z + r * (outputs + 1);
-  if (gate_row != nullptr) shared_gate[t] = (float)((A)1 / ((A)1 + exp_of(-mine[outputs])));
-  if (logistic) {
-    const A taken = -(A)INFINITY;
-    for (int k = 0; k < top; ++k) {
-      int best = -1;
-      A best_choice = 0;
-      for (int e = 0; e < outputs; ++e) {
-        if (mine[e] == taken) continue;
-        const A choice = correction != nullptr ? (A)1 / ((A)1 + exp_of(-mine[e])) + (A)correction[e] : mine[e];
-        if (best < 0 || choice > best_choice) best = e, best_choice = choice;
-      }
-      if (best < 0) best = 0;  // (logits that are no numbers, or more infinite ones than there are choices)
-      chosen[(int64_t)t * top + k] = best;
-      weights[(int64_t)t * top + k] = (float)((A)route_scale / ((A)1 + exp_of(-mine[best])));
-      mine[best] = taken;
-    }
-    return;
-  }
-  A most = mine[0];
-  for (int e = 1; e < outputs; ++e) most = mine[e] > most ? mine[e] : most;
-  A sum = 0;
-  for (int e = 0; e < outputs; ++e) {
-    mine[e] = exp_of(mine[e] - most);
-    sum += mine[e];
-  }
-  const A inv = (A)1 / sum;
-  // the choice is made on score + correction, the weight is the score alone
-  for (int k = 0; k < top; ++k) {
-    int best = -1;
-    A best_choice = 0;
-    for (int e = 0; e < outputs; ++e) {
-      if (mine[e] < (A)0) continue;  // taken already
-      const A choice = mine[e] * inv + (correction != nullptr ? (A)correction[e] : (A)0);
-      if (best < 0 || choice > best_choice) best = e, best_choice = choice;
-    }
-    chosen[(int64_t)t * top + k] = best;
-    weights[(int64_t)t * top + k] = (float)(mine[best] * inv * (A)route_scale);
-    mine[best] = (A)-1;
+  for (int r = wave; r < R; r += waves) {
+    const int t = t0 + r;
+    if (t >= num_tokens) break;
+    A* mine = z + r * (outputs + 1);
+    if (gate_row != nullptr && lane == 0) shared_gate[t] = (float)((A)1 / ((A)1 + exp_of(-mine[outputs])));
+    rank_outputs<A>(mine, correction, chosen + (int64_t)t * top, weights + (int64_t)t * top, outputs, top, route_scale, logistic, lane);
   }
 }
 
@@ -301,8 +328,31 @@ inline bool is_aligned16(const void* p) { return ((uintptr_t)p % 16) == 0; }
 
 #define MI_SORT_MAX_EXPERTS 1024
 
-__global__ __launch_bounds__(256) void expert_sort_kernel(const int* __restrict__ chosen, int* __restrict__ listed,
-                                                          int* __restrict__ first, int pairs, int experts) {
+// The pairs counted (`count` [experts + 1] in LDS, one an expert) become the experts' places: `first` and, in
+// `count`, where an expert's next pair goes.  The block's first wave, 64 experts a turn.
+__device__ __forceinline__ void place_experts(int* count, int* __restrict__ first, int experts) {
+  if (threadIdx.x >= MI_WAVE) return;
+  const int lane = threadIdx.x;
+  int at = 0;
+  for (int base = 0; base < experts; base += MI_WAVE) {
+    const int n = base + lane < experts ? count[base + lane] : 0;
+    int upto = n;
+#pragma unroll
+    for (int off = 1; off < MI_WAVE; off <<= 1) {
+      const int other = __shfl_up(upto, off, MI_WAVE);
+      if (lane >= off) upto += other;
+    }
+    if (base + lane < experts) {
+      first[base + lane] = at + upto - n;
+      count[base + lane] = at + upto - n;
+    }
+    at += __shfl(upto, MI_WAVE - 1, MI_WAVE);
+  }
+  if (lane == 0) first[experts] = at;
+}
+
+__global__ __launch_bounds__(1024) void expert_sort_kernel(const int* __restrict__ chosen, int* __restrict__ listed,
+                                                           int* __restrict__ first, int pairs, int experts) {
   __shared__ int count[MI_SORT_MAX_EXPERTS + 1];
   for (int e = threadIdx.x; e <= experts; e += blockDim.x) count[e] = 0;
   __syncthreads();
@@ -311,18 +361,90 @@ __global__ __launch_bounds__(256) void expert_sort_kernel(const int* __restrict_
     if (e >= 0 && e < experts) atomicAdd(&count[e], 1);
   }
   __syncthreads();
-  if (threadIdx.x == 0) {
-    int at = 0;
-    for (int e = 0; e < experts; ++e) {
-      const int n = count[e];
-      first[e] = at;
-      count[e] = at;  // where the expert's next pair goes
-      at += n;
-    }
-    first[experts] = at;
-  }
+  place_experts(count, first, experts);
   __syncthreads();
   // (pairs of one expert in any order: each pair's result is its own)
+  for (int p = threadIdx.x; p < pairs; p += blockDim.x) {
+    const int e = chosen[p];
+    if (e >= 0 && e < experts) listed[atomicAdd(&count[e], 1)] = p;
+  }
+}
+
+// The router for few tokens (bfloat16), where one block a handful of tokens would leave the router's matrix to
+// the bandwidth of a CU or two: `route_logits` makes one output for eight tokens a block, its four waves sharing
+// the row, and `route_list` ranks all tokens, a wave a token, and lists the pairs by expert in the same launch.
+#define MI_ROUTE_FEW_TOKENS 32
+#define MI_ROUTE_FEW_PAIRS 2048
+
+__global__ __launch_bounds__(256) void route_logits_kernel(const bf16_t* __restrict__ x, int64_t x_stride,
+                                                           const float* __restrict__ router,
+                                                           const float* __restrict__ gate_row, float* __restrict__ logits,
+                                                           int num_tokens, int width, int outputs, int total) {
+  constexpr int TOKENS = 8;
+  __shared__ float meet[3][TOKENS];
+  const int e = blockIdx.x, t0 = blockIdx.y * TOKENS;
+  const int wave = threadIdx.x / MI_WAVE, lane = threadIdx.x % MI_WAVE;
+  const float* w = e < outputs ? router + (int64_t)e * width : gate_row;
+  float sum[TOKENS];
+#pragma unroll
+  for (int t = 0; t < TOKENS; ++t) sum[t] = 0.f;
+  constexpr int BATCH = 2;
+  for (int c0 = threadIdx.x * 4; c0 < width; c0 += 1024 * BATCH) {
+    float wv[BATCH][4], xv[BATCH][TOKENS][4];
+#pragma unroll
+    for (int i = 0; i < BATCH; ++i) {
+      const int c = min(c0 + i * 1024, width - 4);  // (past the row: its last columns again, weighed with zero)
+      mi_load_cols<float, 4>(w + c, wv[i]);
+      if (c0 + i * 1024 >= width) wv[i][0] = wv[i][1] = wv[i][2] = wv[i][3] = 0.f;
+#pragma unroll
+      for (int t = 0; t < TOKENS; ++t) mi_load_cols<bf16_t, 4>(x + (int64_t)min(t0 + t, num_tokens - 1) * x_stride + c, xv[i][t]);
+    }
+#pragma unroll
+    for (int i = 0; i < BATCH; ++i)
+#pragma unroll
+      for (int t = 0; t < TOKENS; ++t)
+        sum[t] += wv[i][0] * xv[i][t][0] + wv[i][1] * xv[i][t][1] + wv[i][2] * xv[i][t][2] + wv[i][3] * xv[i][t][3];
+  }
+#pragma unroll
+  for (int t = 0; t < TOKENS; ++t) sum[t] = wave_sum(sum[t]);
+  if (wave > 0 && lane == 0) {
+#pragma unroll
+    for (int t = 0; t < TOKENS; ++t) meet[wave - 1][t] = sum[t];
+  }
+  __syncthreads();
+  if (wave == 0 && lane == 0) {
+#pragma unroll
+    for (int t = 0; t < TOKENS; ++t)
+      if (t0 + t < num_tokens) logits[(int64_t)(t0 + t) * total + e] = sum[t] + meet[0][t] + meet[1][t] + meet[2][t];
+  }
+}
+
+__global__ __launch_bounds__(1024) void route_list_kernel(const float* __restrict__ logits, const float* __restrict__ correction,
+                                                          int* __restrict__ chosen, float* __restrict__ weights,
+                                                          float* __restrict__ shared_gate, int* __restrict__ listed,
+                                                          int* __restrict__ first, int num_tokens, int outputs, int total,
+                                                          int experts, int top, float route_scale, int logistic) {
+  extern __shared__ __align__(16) unsigned char lds_bytes[];
+  float* z = reinterpret_cast<float*>(lds_bytes);                        // [waves][outputs]
+  __shared__ int count[MI_SORT_MAX_EXPERTS + 1];
+  const int wave = threadIdx.x / MI_WAVE, lane = threadIdx.x % MI_WAVE, waves = blockDim.x / MI_WAVE;
+  for (int e = threadIdx.x; e <= experts; e += blockDim.x) count[e] = 0;
+  for (int t = wave; t < num_tokens; t += waves) {
+    float* mine = z + wave * outputs;
+    for (int e = lane; e < outputs; e += MI_WAVE) mine[e] = logits[(int64_t)t * total + e];
+    __builtin_amdgcn_wave_barrier();
+    if (total > outputs && lane == 0) shared_gate[t] = 1.f / (1.f + expf(-logits[(int64_t)t * total + outputs]));
+    rank_outputs<float>(mine, correction, chosen + t * top, weights + t * top, outputs, top, route_scale, logistic, lane);
+  }
+  __syncthreads();  // (what this block's waves have written to `chosen` is there for all of them)
+  const int pairs = num_tokens * top;
+  for (int p = threadIdx.x; p < pairs; p += blockDim.x) {
+    const int e = chosen[p];
+    if (e >= 0 && e < experts) atomicAdd(&count[e], 1);
+  }
+  __syncthreads();
+  place_experts(count, first, experts);
+  __syncthreads();
   for (int p = threadIdx.x; p < pairs; p += blockDim.x) {
     const int e = chosen[p];
     if (e >= 0 && e < experts) listed[atomicAdd(&count[e], 1)] = p;
@@ -694,8 +816,36 @@ extern "C" int mi_expert_combine(int dtype, const void* made, const int* where, 
 extern "C" int mi_expert_sort(const int* chosen, int* listed, int* first, int pairs, int experts, hipStream_t stream) {
   MI_REQUIRE(pairs >= 0 && experts > 0 && experts <= MI_SORT_MAX_EXPERTS, "expert_sort: %d pairs over %d experts (at most %d)", pairs,
              experts, MI_SORT_MAX_EXPERTS);
-  expert_sort_kernel<<<1, 256, 0, stream>>>(chosen, listed, first, pairs, experts);
+  expert_sort_kernel<<<1, pairs > 256 ? 1024 : 256, 0, stream>>>(chosen, listed, first, pairs, experts);
   MI_CHECK_LAUNCH("expert_sort");
+  return MI_OK;
+}
+
+// Whether mi_route_few takes a step of these sizes (bfloat16 only).
+extern "C" int mi_route_few_takes(int num_tokens, int width, int outputs, int top) {
+  return num_tokens > 0 && num_tokens <= MI_ROUTE_FEW_TOKENS && num_tokens * top <= MI_ROUTE_FEW_PAIRS && width >= 4 && width % 4 == 0 &&
+         outputs > 0 && outputs <= MI_ROUTER_MAX_OUTPUTS;
+}
+
+// mi_route_top_k and mi_expert_sort for few bfloat16 tokens in two launches; `logits`: scratch
+// [num_tokens, outputs + (gate row ? 1 : 0)] floats.
+extern "C" int mi_route_few(const void* x, int64_t x_stride, const float* router, const float* correction, const float* gate_row,
+                            float* logits, int* chosen, float* weights, float* shared_gate, int* listed, int* first,
+                            int num_tokens, int width, int outputs, int experts, int top, float route_scale, int logistic,
+                            hipStream_t stream) {
+  MI_REQUIRE(mi_route_few_takes(num_tokens, width, outputs, top) && x_stride >= width && x_stride % 4 == 0 && (uintptr_t)x % 8 == 0 &&
+                 is_aligned16(router) && is_aligned16(gate_row),
+             "route_few: %d tokens of %d columns, %d outputs", num_tokens, width, outputs);
+  MI_REQUIRE(top > 0 && top <= outputs && experts > 0 && experts <= outputs, "route_few: %d of %d outputs, %d experts", top, outputs, experts);
+  MI_REQUIRE(gate_row == nullptr || shared_gate != nullptr, "route_few: a gate row needs a place for the gates");
+  const int total = outputs + (gate_row != nullptr ? 1 : 0);
+  route_logits_kernel<<<dim3(total, ceil_div(num_tokens, 8)), 256, 0, stream>>>((const bf16_t*)x, x_stride, router, gate_row, logits,
+                                                                               num_tokens, width, outputs, total);
+  MI_CHECK_LAUNCH("route_logits");
+  const int threads = min(1024, num_tokens * MI_WAVE);
+  route_list_kernel<<<1, threads, (size_t)(threads / MI_WAVE) * outputs * 4, stream>>>(
+      logits, correction, chosen, weights, shared_gate, listed, first, num_tokens, outputs, total, experts, top, route_scale, logistic);
+  MI_CHECK_LAUNCH("route_list");
   return MI_OK;
 }
 

@@ -63,7 +63,7 @@ __global__ __launch_bounds__(1024) void gated_update_norm_kernel(
     int64_t gate_stride, const float* __restrict__ bias, const T* __restrict__ out_weight,
     const T* __restrict__ norm_weight, const int* __restrict__ rows, T* __restrict__ h, int hidden, float eps_out,
     float eps, const float* __restrict__ conv_weight, int taps, T* __restrict__ tail, int64_t tail_stride,
-    const int* __restrict__ token_request, const int* __restrict__ slots, int num_slots, T* __restrict__ u) {
+    const int* __restrict__ slots, int num_slots, T* __restrict__ u) {
   using A = typename WideOf<T>::type;
   __shared__ A scratch[16];
   const int t = rows != nullptr ? rows[blockIdx.x] : blockIdx.x;
@@ -139,7 +139,7 @@ __global__ __launch_bounds__(1024) void gated_update_norm_kernel(
 
   T* mine = nullptr;
   if (u != nullptr && taps > 1) {
-    const int slot = slots[token_request[t]];
+    const int slot = slots[t];  // (row t is request t's only token)
     mine = tail + (int64_t)((slot < 0 || slot >= num_slots) ? num_slots : slot) * tail_stride;
   }
   T* out = h + (int64_t)blockIdx.x * hidden;
@@ -174,17 +174,113 @@ __global__ __launch_bounds__(1024) void gated_update_norm_kernel(
         for (int j = 0; j < VEC; ++j) next[j] = r[j];
       }
 #pragma unroll
-      for (int j = 0; j < VEC; ++j) sum[j] = fma((A)conv_weight[(int64_t)(c + j) * taps + k], (A)before[j], sum[j]);
+      for (int j = 0; j < VEC; ++j) sum[j] = fma((A)conv_weight[(int64_t)k * hidden + c + j], (A)before[j], sum[j]);
       mi_store_cols<T, VEC>(mine + (int64_t)k * hidden + c, next);
     }
     float made[VEC];
 #pragma unroll
     for (int j = 0; j < VEC; ++j) {
-      sum[j] = fma((A)conv_weight[(int64_t)(c + j) * taps + back], (A)r[j], sum[j]);
+      sum[j] = fma((A)conv_weight[(int64_t)back * hidden + c + j], (A)r[j], sum[j]);
       made[j] = (float)((A)r[j] + sum[j]);
     }
     mi_store_cols<T, VEC>(u + (int64_t)t * hidden + c, made);
   }
+}
+
+// The same where a thread has one turn of four columns, at most four pieces and at most four taps (few rows, the
+// usual widths): everything the row needs is asked for at once, so the launch waits for memory once and
+// not before each of its three passes (8 rows of 4,096: 15 us one after the other).
+template <typename T>
+__global__ __launch_bounds__(1024) void gated_update_norm_early_kernel(
+    float* __restrict__ stream, const T* __restrict__ y, int64_t y_stride, int pieces, const T* __restrict__ gate,
+    int64_t gate_stride, const float* __restrict__ bias, const T* __restrict__ out_weight,
+    const T* __restrict__ norm_weight, const int* __restrict__ rows, T* __restrict__ h, int hidden, float eps_out,
+    float eps, const float* __restrict__ conv_weight, int taps, T* __restrict__ tail, int64_t tail_stride,
+    const int* __restrict__ slots, int num_slots, T* __restrict__ u) {
+  using A = typename WideOf<T>::type;
+  constexpr int MOST = 4;
+  __shared__ A scratch_out[16], scratch[16];
+  const int t = rows != nullptr ? rows[blockIdx.x] : blockIdx.x;
+  const int c = threadIdx.x * 4;
+  const bool mine_too = c < hidden;
+  const int at = mine_too ? c : 0;  // (threads past the row read its first columns, and count and write nothing)
+  float* x = stream + (int64_t)t * hidden;
+  const int back = taps - 1;
+  float part[MOST][4], z[4], b[4], wo[4], now[4], w[4], before[MOST - 1][4], wc[MOST][4];
+  mi_load_cols<float, 4>(x + at, now);
+  mi_load_cols<T, 4>(norm_weight + at, w);
+  if (y != nullptr) {
+#pragma unroll
+    for (int p = 0; p < MOST; ++p)
+      if (p < pieces) mi_load_cols<T, 4>(y + ((int64_t)t * pieces + p) * y_stride + at, part[p]);
+    if (gate != nullptr) {
+      mi_load_cols<T, 4>(gate + (int64_t)t * gate_stride + at, z);
+      mi_load_cols<float, 4>(bias + at, b);
+    }
+    mi_load_cols<T, 4>(out_weight + at, wo);
+  }
+  T* kept = nullptr;
+  if (u != nullptr) {
+    if (taps > 1) {
+      const int slot = slots[t];  // (row t is request t's only token)
+      kept = tail + (int64_t)((slot < 0 || slot >= num_slots) ? num_slots : slot) * tail_stride;
+    }
+#pragma unroll
+    for (int k = 0; k < MOST - 1; ++k)
+      if (k < back) mi_load_cols<T, 4>(kept + (int64_t)k * hidden + at, before[k]);
+#pragma unroll
+    for (int k = 0; k < MOST; ++k)
+      if (k < taps) mi_load_cols<float, 4>(conv_weight + (int64_t)k * hidden + at, wc[k]);
+  }
+
+  if (y != nullptr) {
+    A v[4], squares = 0;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      v[j] = 0;
+#pragma unroll
+      for (int p = 0; p < MOST; ++p)
+        if (p < pieces) v[j] += (A)part[p][j];
+      if (gate != nullptr) v[j] *= gate_of((A)z[j] + (A)b[j]);
+      squares += v[j] * v[j];
+    }
+    const A inv_out = inv_root_of(block_add<A>(mine_too ? squares : (A)0, scratch_out) / (A)hidden, (A)eps_out);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) now[j] = (float)((A)now[j] + (v[j] * inv_out) * (A)wo[j]);
+    if (rows == nullptr && mine_too) mi_store_cols<float, 4>(x + c, now);
+  }
+  A squares = 0;
+#pragma unroll
+  for (int j = 0; j < 4; ++j) squares += (A)now[j] * (A)now[j];
+  const A inv = inv_root_of(block_add<A>(mine_too ? squares : (A)0, scratch) / (A)hidden, (A)eps);
+  if (!mine_too) return;
+  float r[4];
+#pragma unroll
+  for (int j = 0; j < 4; ++j) r[j] = to_f32(from_f32<T>((float)(((A)now[j] * inv) * (A)w[j])));
+  mi_store_cols<T, 4>(h + (int64_t)blockIdx.x * hidden + c, r);
+  if (u == nullptr) return;
+  A sum[4];
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    sum[j] = 0;
+#pragma unroll
+    for (int k = 0; k < MOST - 1; ++k)
+      if (k < back) sum[j] = fma((A)wc[k][j], (A)before[k][j], sum[j]);
+    A last = 0;
+#pragma unroll
+    for (int k = 0; k < MOST; ++k)
+      if (k == back) last = (A)wc[k][j];
+    sum[j] = fma(last, (A)r[j], sum[j]);
+  }
+#pragma unroll
+  for (int k = 0; k < MOST - 1; ++k) {
+    if (k + 1 < back) mi_store_cols<T, 4>(kept + (int64_t)k * hidden + c, before[k + 1 < MOST - 1 ? k + 1 : k]);
+    else if (k + 1 == back) mi_store_cols<T, 4>(kept + (int64_t)k * hidden + c, r);
+  }
+  float made[4];
+#pragma unroll
+  for (int j = 0; j < 4; ++j) made[j] = (float)((A)r[j] + sum[j]);
+  mi_store_cols<T, 4>(u + (int64_t)t * hidden + c, made);
 }
 
 }  // namespace
@@ -192,13 +288,13 @@ __global__ __launch_bounds__(1024) void gated_update_norm_kernel(
 // y: [tokens * pieces, hidden] (row stride) or null (the norm alone); gate [tokens, hidden] (row stride) with
 // bias float32 [hidden], or null; out_weight [hidden]; norm_weight [hidden] or null (the update alone); rows
 // (may be null) lists the rows to norm: the stream is then left as it is and h gets the rows in list order.
-// With u [tokens, hidden]: conv_weight float32 [hidden, taps], tail [slots + 1, (taps - 1) * hidden] (row
-// stride), every token the only one of its request (token_request, slots).
+// With u [tokens, hidden]: conv_weight float32 [taps, hidden] (a tap's weights side by side), tail [slots + 1, (taps - 1) * hidden] (row
+// stride), every token the only one of its request: row t is request t's (slots).
 extern "C" int mi_gated_update_norm(int dtype, float* stream_rows, const void* y, int64_t y_stride, int pieces,
                                     const void* gate, int64_t gate_stride, const float* bias, const void* out_weight,
                                     const void* norm_weight, const int* rows, void* h, int num_rows, int hidden,
                                     float eps_out, float eps, const float* conv_weight, int taps, void* tail,
-                                    int64_t tail_stride, const int* token_request, const int* slots, int num_slots,
+                                    int64_t tail_stride, const int* slots, int num_slots,
                                     void* u, hipStream_t stream) {
   MI_REQUIRE(num_rows >= 0 && hidden > 0 && pieces >= 1 && (y == nullptr || y_stride >= hidden) &&
                  (gate == nullptr || gate_stride >= hidden),
@@ -210,22 +306,34 @@ extern "C" int mi_gated_update_norm(int dtype, float* stream_rows, const void* y
   MI_REQUIRE(u == nullptr || (rows == nullptr && norm_weight != nullptr && conv_weight != nullptr && taps >= 1 && taps <= SANDWICH_MAX_TAPS),
              "gated_update_norm: the convolution goes with the norm of all rows and 1..%d taps, got %d", SANDWICH_MAX_TAPS, taps);
   MI_REQUIRE(u == nullptr || taps == 1 ||
-                 (tail != nullptr && tail_stride >= (int64_t)(taps - 1) * hidden && token_request != nullptr && slots != nullptr && num_slots >= 1),
+                 (tail != nullptr && tail_stride >= (int64_t)(taps - 1) * hidden && slots != nullptr && num_slots >= 1),
              "gated_update_norm: the convolution needs its requests' tails");
   MI_REQUIRE(eps > 0.f && eps_out > 0.f, "gated_update_norm: eps must be positive");
   MI_REQUIRE(dtype == MI_F32 || dtype == MI_BF16, "gated_update_norm: unknown dtype %d", dtype);
   if (num_rows == 0) return MI_OK;
   const bool vec = hidden % 4 == 0 && y_stride % 4 == 0 && gate_stride % 4 == 0 && tail_stride % 4 == 0 &&
                    is_aligned16(stream_rows) && is_aligned16(y) && is_aligned16(gate) && is_aligned16(bias) && is_aligned16(out_weight) &&
-                   is_aligned16(norm_weight) && is_aligned16(h) && is_aligned16(tail) && is_aligned16(u);
+                   is_aligned16(norm_weight) && is_aligned16(h) && is_aligned16(tail) && is_aligned16(u) && is_aligned16(conv_weight);
   const int items = vec ? ceil_div(hidden, 4) : hidden;
   // few rows: a turn of the whole row at once; many rows: four waves a row, several rows to a CU
   const int threads = num_rows < 256 ? min(1024, ceil_div(items, MI_WAVE) * MI_WAVE) : 256;
+  if (vec && items <= threads && pieces <= 4 && norm_weight != nullptr && (u == nullptr || taps <= 4)) {
+#define MI_SANDWICH_EARLY(T)                                                                                              \
+  gated_update_norm_early_kernel<T><<<num_rows, threads, 0, stream>>>(                                                    \
+      stream_rows, (const T*)y, y_stride, pieces, (const T*)gate, gate_stride, bias, (const T*)out_weight,                \
+      (const T*)norm_weight, rows, (T*)h, hidden, eps_out, eps, conv_weight, taps, (T*)tail, tail_stride, slots, \
+      num_slots, (T*)u)
+    if (dtype == MI_F32) MI_SANDWICH_EARLY(float);
+    else MI_SANDWICH_EARLY(bf16_t);
+#undef MI_SANDWICH_EARLY
+    MI_CHECK_LAUNCH("gated_update_norm_early");
+    return MI_OK;
+  }
 #define MI_SANDWICH(T, VEC)                                                                                             \
   gated_update_norm_kernel<T, VEC><<<num_rows, threads, 0, stream>>>(                                                   \
       stream_rows, (const T*)y, y_stride, pieces, (const T*)gate, gate_stride, bias, (const T*)out_weight,              \
-      (const T*)norm_weight, rows, (T*)h, hidden, eps_out, eps, conv_weight, taps, (T*)tail, tail_stride, token_request, \
-      slots, num_slots, (T*)u)
+      (const T*)norm_weight, rows, (T*)h, hidden, eps_out, eps, conv_weight, taps, (T*)tail, tail_stride, slots, \
+      num_slots, (T*)u)
   if (dtype == MI_F32) {
     if (vec) MI_SANDWICH(float, 4);
     else MI_SANDWICH(float, 1);

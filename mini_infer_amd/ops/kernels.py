@@ -2461,16 +2461,29 @@ ROUTER_SCORES = ("softmax", "logistic")
 EXPERT_ACTIVATIONS = {"silu_gated": (1, 2), "squared_relu": (2, 1)}
 
 
+@dataclasses.dataclass
+class ExpertLists:
+    """The (row, choice) pairs of a step listed expert by expert, on the device: expert e's are `listed[first[e] :
+    first[e + 1]]` (int32 [pairs] and [experts + 1])."""
+
+    listed: torch.Tensor
+    first: torch.Tensor
+
+
 def route_top_k(
     x: torch.Tensor, router: torch.Tensor, correction: torch.Tensor | None, gate_row: torch.Tensor | None, *, top: int,
-    route_scale: float, scores: str = "softmax",
-) -> tuple[torch.Tensor, torch.Tensor, torch.Tensor | None]:
+    route_scale: float, scores: str = "softmax", experts: int | None = None,
+) -> "tuple[torch.Tensor, torch.Tensor, torch.Tensor | None] | tuple[torch.Tensor, torch.Tensor, torch.Tensor | None, ExpertLists]":
     """Per row of `x` [T, W]: scores `softmax(router @ x)` over all router outputs (`router` float32
     [outputs, W]), the `top` outputs with the largest `score + correction` (`correction` float32
     [outputs] or None; the lower index wins a tie) -> their indices int32 [T, top] and weights
     `score * route_scale` float32 [T, top] (not renormalized); with `gate_row` (float32 [W]) also
     `logistic(gate_row . x)` float32 [T].  `scores="logistic"`: every output's score is `logistic(z)` of its
-    own logit."""
+    own logit.
+
+    With `experts` (how many of the outputs are real experts) a fourth result is the list of (row, choice) pairs
+    by expert that `experts_by_expert` works from: for few bfloat16 rows it is made in the same launch
+    that ranks the outputs."""
     if scores not in ROUTER_SCORES:
         raise KernelShapeError(f"route_top_k: scores {scores!r}; built: {ROUTER_SCORES}")
     _need_cuda(x, router, correction, gate_row)
@@ -2492,12 +2505,30 @@ def route_top_k(
     chosen = torch.empty((tokens, top), dtype=torch.int32, device=x.device)
     weights = torch.empty((tokens, top), dtype=torch.float32, device=x.device)
     gates = torch.empty((tokens,), dtype=torch.float32, device=x.device) if gate_row is not None else None
+    lists = None
+    if experts is not None:
+        if not 0 < experts <= outputs:
+            raise KernelShapeError(f"route_top_k: {experts} experts among {outputs} outputs")
+        lists = ExpertLists(torch.empty((tokens * top,), dtype=torch.int32, device=x.device),
+                            torch.empty((experts + 1,), dtype=torch.int32, device=x.device))
+        lib = library.load()
+        if (x.dtype == torch.bfloat16 and lib.mi_route_few_takes(tokens, width, outputs, int(top)) and x.stride(0) % 4 == 0
+                and x.data_ptr() % 8 == 0 and router.data_ptr() % 16 == 0 and (gate_row is None or gate_row.data_ptr() % 16 == 0)):
+            logits = torch.empty((tokens, outputs + (gate_row is not None)), dtype=torch.float32, device=x.device)
+            library.check(lib.mi_route_few(
+                _ptr(x), x.stride(0), _ptr(router), _ptr(correction), _ptr(gate_row), _ptr(logits), _ptr(chosen), _ptr(weights),
+                _ptr(gates), _ptr(lists.listed), _ptr(lists.first), tokens, width, outputs, experts, int(top), float(route_scale),
+                int(scores == "logistic"), _stream()))
+            return chosen, weights, gates, lists
     library.check(
         library.load().mi_route_top_k(
             _dtype_code(x), _ptr(x), x.stride(0), _ptr(router), _ptr(correction), _ptr(gate_row), _ptr(chosen), _ptr(weights),
             _ptr(gates), tokens, width, outputs, int(top), float(route_scale), int(scores == "logistic"), _stream(),
         )
     )
+    if lists is not None:
+        library.check(library.load().mi_expert_sort(_ptr(chosen), _ptr(lists.listed), _ptr(lists.first), tokens * top, experts, _stream()))
+        return chosen, weights, gates, lists
     return chosen, weights, gates
 
 
@@ -2615,7 +2646,7 @@ GROUPED_ROWS_STEP = 64  # the sorted form's products run over row counts rounded
 def experts_by_expert(
     x: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, chosen: torch.Tensor, weights: torch.Tensor,
     shared: torch.Tensor | None = None, shared_gate: torch.Tensor | None = None, tiles: str | None = None, *,
-    activation: str = "silu_gated", weight_on: str = "output", combine: bool = True,
+    activation: str = "silu_gated", weight_on: str = "output", combine: bool = True, lists: ExpertLists | None = None,
 ) -> "torch.Tensor | SummedRows":
     """The same sum as `experts_few_rows`, expert by expert without the host knowing anything: one small
     kernel lists the (row, expert) pairs by expert, then every chosen expert's block streams its
@@ -2625,7 +2656,8 @@ def experts_by_expert(
     gets): "rows" is that form; for prompts (bfloat16) "direct", blocks of 64 features that take 64 of an
     expert's rows a pass, and "lds", tiles of 128 rows x 128 features with both operands staged through LDS
     (rows in steps of 64 elements).  `combine=False`
-    (weights on the input, no shared or identity experts): the rows are left for a norm to add up (`SummedRows`)."""
+    (weights on the input, no shared or identity experts): the rows are left for a norm to add up (`SummedRows`).
+    `lists`: the pairs by expert where `route_top_k` has made them already."""
     tokens, width, experts, ff, top = _check_experts(x, gate_up, down, chosen, weights, shared, shared_gate, activation, weight_on)
     mode, on_input, on_output = _expert_weights(activation, weights, weight_on)
     if not combine and (weight_on != "input" or shared is not None):
@@ -2633,8 +2665,13 @@ def experts_by_expert(
     if not experts_by_expert_take(x, gate_up, activation):
         raise KernelShapeError(f"experts_by_expert: rows of {width} and {ff} are not read 16 bytes at a time, or do not fit")
     pairs = tokens * top
-    listed = torch.empty((pairs,), dtype=torch.int32, device=x.device)
-    first = torch.empty((experts + 1,), dtype=torch.int32, device=x.device)
+    if lists is None:
+        lists = ExpertLists(torch.empty((pairs,), dtype=torch.int32, device=x.device),
+                            torch.empty((experts + 1,), dtype=torch.int32, device=x.device))
+        library.check(library.load().mi_expert_sort(_ptr(chosen), _ptr(lists.listed), _ptr(lists.first), pairs, experts, _stream()))
+    listed, first = lists.listed, lists.first
+    if listed.numel() != pairs or first.numel() != experts + 1 or listed.dtype != torch.int32 or first.dtype != torch.int32:
+        raise KernelShapeError("experts_by_expert: the lists are those of other pairs")
     act = torch.empty((pairs, ff), dtype=x.dtype, device=x.device)
     made = torch.empty((pairs, width), dtype=x.dtype, device=x.device)
     lib, code = library.load(), _dtype_code(x)
@@ -2643,7 +2680,6 @@ def experts_by_expert(
     elif tiles not in EXPERT_TILES or (tiles == "lds" and not expert_tiles_take(x, ff)):
         raise KernelShapeError(f"experts_by_expert: tiles {tiles!r} for rows of {width} and {ff} {x.dtype}")
     many = int(tiles == "direct")
-    library.check(lib.mi_expert_sort(_ptr(chosen), _ptr(listed), _ptr(first), pairs, experts, _stream()))
     if tiles == "lds":
         library.check(lib.mi_expert_tiles(mode, _ptr(x), x.stride(0), top, _ptr(gate_up), _ptr(listed), _ptr(first),
                                           _ptr(on_input), _ptr(act), ff, pairs, experts, width, ff, _stream()))
@@ -2782,16 +2818,18 @@ class GatedNormedUpdate:
 @dataclasses.dataclass
 class InputConvolution:
     """What a sublayer reads instead of its norm's output h: `u = h + conv(h)`, a causal convolution per
-    channel over each request's tokens.  `weight` float32 [H, taps] (last column the current token's);
+    channel over each request's tokens.  `weight` float32 [H, taps] (last column the current token's), `by_tap` the same
+    [taps, H];
     `tail` [slots + 1, taps - 1, H] (compute dtype) holds each request's last taps-1 rows of h, or None
     for a single tap."""
 
     weight: torch.Tensor
+    by_tap: torch.Tensor
     tail: torch.Tensor | None
     cu_seqlens: torch.Tensor
     slots: torch.Tensor
     token_request: torch.Tensor
-    single_tokens: bool  # every request of the step brings exactly one token
+    single_tokens: bool  # every request of the step brings exactly one token (row t is request t's)
 
     def apply(self, h: torch.Tensor) -> torch.Tensor:
         tail = self.tail
@@ -2840,15 +2878,14 @@ def gated_update_norm(
     u = tail = None
     taps = tail_stride = num_slots = 0
     if here:
-        taps, tail = conv.weight.shape[1], conv.tail
-        _need_cuda(conv.weight, tail, conv.slots, conv.token_request)
-        _need_f32("convolution weight", conv.weight)
-        for name, t in (("convolution weight", conv.weight), ("slots", conv.slots), ("token_request", conv.token_request)):
+        taps, tail = conv.by_tap.shape[0], conv.tail
+        _need_cuda(conv.by_tap, tail, conv.slots)
+        _need_f32("convolution weight", conv.by_tap)
+        for name, t in (("convolution weight", conv.by_tap), ("slots", conv.slots)):
             _need_contiguous(name, t)
         _need_int32("slots", conv.slots)
-        _need_int32("token_request", conv.token_request)
-        if conv.weight.shape[0] != hidden or conv.token_request.numel() != tokens or conv.slots.numel() != tokens:
-            raise KernelShapeError("gated_update_norm: single tokens have one request and one slot each, the convolution one row of taps a column")
+        if conv.by_tap.shape[1] != hidden or conv.slots.numel() != tokens:
+            raise KernelShapeError("gated_update_norm: single tokens have one slot each, the convolution one row of taps a column")
         if taps > 1:
             if tail is None or tail.dtype != dtype or tail.dim() != 3 or tuple(tail.shape[1:]) != (taps - 1, hidden) or tail.shape[0] < 2 \
                     or tail.stride(2) != 1 or tail.stride(1) != hidden:
@@ -2859,8 +2896,8 @@ def gated_update_norm(
         library.load().mi_gated_update_norm(
             F32 if dtype == torch.float32 else BF16, _ptr(residual), _ptr(y), 0 if y is None else y.stride(0), pieces, _ptr(gate),
             0 if gate is None else gate.stride(0), _ptr(bias), _ptr(out_weight), _ptr(weight), _ptr(rows), _ptr(h), n_out, hidden,
-            float(eps_out), float(eps), _ptr(conv.weight) if here else None, taps, _ptr(tail) if taps > 1 else None, tail_stride,
-            _ptr(conv.token_request) if here else None, _ptr(conv.slots) if here else None, num_slots, _ptr(u), _stream(),
+            float(eps_out), float(eps), _ptr(conv.by_tap) if here else None, taps, _ptr(tail) if taps > 1 else None, tail_stride,
+            _ptr(conv.slots) if here else None, num_slots, _ptr(u), _stream(),
         )
     )
     if conv is None:

@@ -124,6 +124,10 @@ _SIGNATURES: dict[str, list] = {
         c_float, _P,
     ],
     "mi_route_top_k": [c_int, _P, c_int64, _P, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_float, c_int, _P],
+    "mi_route_few_takes": [c_int, c_int, c_int, c_int],
+    "mi_route_few": [
+        _P, c_int64, _P, _P, _P, _P, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_float, c_int, _P,
+    ],
     "mi_expert_gate_up": [c_int, c_int, _P, c_int64, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, _P],
     "mi_weighted_squared_relu": [c_int, _P, c_int64, _P, _P, c_int64, c_int, c_int, _P],
     "mi_expert_down_combine": [c_int, _P, _P, _P, _P, _P, c_int64, _P, c_int64, _P, _P, c_int, c_int, c_int, c_int, c_int, _P],
@@ -141,7 +145,7 @@ _SIGNATURES: dict[str, list] = {
     "mi_expert_tiles": [c_int, _P, c_int64, c_int, _P, _P, _P, _P, _P, c_int64, c_int, c_int, c_int, c_int, _P],
     "mi_gated_update_norm": [
         c_int, _P, _P, c_int64, c_int, _P, c_int64, _P, _P, _P, _P, _P, c_int, c_int, c_float, c_float, _P, c_int, _P,
-        c_int64, _P, _P, c_int, _P, _P,
+        c_int64, _P, c_int, _P, _P,
     ],
     "mi_gate_heads": [c_int, _P, c_int64, c_int, _P, c_int64, _P, c_int64, c_int, c_int, c_int, _P],
     "mi_per_head_bf16": [

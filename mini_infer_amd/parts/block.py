@@ -517,6 +517,7 @@ class SandwichBlock(Block):
         self.gates = {q: Linear(hidden_size, hidden_size, names[f"{q}_gate"], dtype, device, suffix="") for q in self.sublayers} if gated else {}
         self.gate_biases: dict[str, torch.Tensor] = {}
         self.conv_weights: dict[str, torch.Tensor] = {}  # float32 [hidden, taps]
+        self.conv_by_tap: dict[str, torch.Tensor] = {}  # the same [taps, hidden]
         for q in self.sublayers:
             if not hasattr(norms[f"{q}_output_norm"], "weight"):
                 raise ValueError("a sublayer's output norm is an RMS norm with a weight per column (the next norm makes it)")
@@ -567,6 +568,7 @@ class SandwichBlock(Block):
                 self.gate_biases[q] = get(prefix + self.names[f"{q}_gate"] + ".b").float().contiguous()
             if self.conv_taps is not None:
                 self.conv_weights[q] = get(prefix + self.names[f"{q}_conv"]).float().contiguous()
+                self.conv_by_tap[q] = self.conv_weights[q].t().contiguous()
 
     # -- state ---------------------------------------------------------------------
 
@@ -601,7 +603,7 @@ class SandwichBlock(Block):
             h = h.finish() if hasattr(h, "finish") else h
             return h, h
         single = ctx.host_cu_seqlens_q is not None and ctx.max_q_len == 1 and residual.shape[0] == ctx.state_slots.numel()
-        conv = ops.InputConvolution(self.conv_weights[q], cache.state[f"{q}_conv"] if self.conv_taps > 1 else None, ctx.cu_seqlens_q,
+        conv = ops.InputConvolution(self.conv_weights[q], self.conv_by_tap[q], cache.state[f"{q}_conv"] if self.conv_taps > 1 else None, ctx.cu_seqlens_q,
                                     ctx.state_slots, ctx.token_request, single)
         return norm.forward_conv(delta, residual, conv)
 

@@ -377,18 +377,22 @@ class RoutedExperts(FeedForward):
             "feed-forward used before its weights were loaded"
         if hasattr(x, "finish"):
             x = x.finish()
-        chosen, weights, gates = ops.route_top_k(x, self.router, self.correction, self.shared_gate_row, top=self.top,
-                                                 route_scale=self.route_scale, scores=self.scores)
+        grouped = self._grouped(x, ctx)
+        by_expert = not grouped and (self.force_form == "by_expert" or (
+            self.force_form is None and ops.experts_by_expert_take(x, self.gate_up, self.activation)))
+        chosen, weights, gates, *lists = ops.route_top_k(
+            x, self.router, self.correction, self.shared_gate_row, top=self.top, route_scale=self.route_scale, scores=self.scores,
+            experts=self.experts if by_expert else None)
         shared = None
         if self.shared is not None:
             shared = self.shared.forward(x, ctx)
             shared = shared.finish() if hasattr(shared, "finish") else shared
         how = {"activation": self.activation, "weight_on": self.weight_on}
-        if self._grouped(x, ctx):
+        if grouped:
             run = ops.experts_grouped
-        elif self.force_form == "by_expert" or (
-                self.force_form is None and ops.experts_by_expert_take(x, self.gate_up, self.activation)):
+        elif by_expert:
             run = ops.experts_by_expert
+            how["lists"] = lists[0]
             how["combine"] = not (self.leave_rows_apart and self.weight_on == "input" and shared is None)
         else:
             run = ops.experts_few_rows

@@ -145,10 +145,10 @@ def test_single_tokens_pass_norm_and_convolution_in_one_launch(dtype, width, tap
     seen = []
     for _ in range(steps):
         x = rng.standard_normal((4, width)).astype(np.float32)
-        args = (dev(taps_weight), one, ints(range(5)), ints(slots), ints(range(4)), True)
+        args = (dev(taps_weight), dev(taps_weight.T), one, ints(range(5)), ints(slots), ints(range(4)), True)
         h, u = ops.gated_update_norm(None, dev(x), dev(w, TORCH[dtype]), 1e-5, conv=ops.InputConvolution(*args))
         h2, u2 = ops.gated_update_norm(None, dev(x), dev(w, TORCH[dtype]), 1e-5,
-                                       conv=ops.InputConvolution(args[0], two, *args[2:5], False))
+                                       conv=ops.InputConvolution(*args[:2], two, *args[3:6], False))
         assert torch.equal(h, h2)
         np.testing.assert_allclose(u.float().cpu().numpy(), u2.float().cpu().numpy(), rtol=0, atol=tolerance(dtype, 2))
         seen.append((h.double().cpu().numpy(), u.double().cpu().numpy()))
@@ -386,6 +386,39 @@ def test_silu_gated_experts_in_tiles_staged_through_lds(rows, width, ff, experts
     want = ops.experts_few_rows(x, gate_up, down, chosen, w).double()
     got = ops.experts_by_expert(x, gate_up, down, chosen, w, tiles="lds").double()
     assert (got - want).abs().max() < 2e-2 * max(1.0, want.abs().max())
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("scores", ["logistic", "softmax"])
+@pytest.mark.parametrize("tokens, width, outputs, experts, top, corrected, gated", [
+    (1, 64, 5, 5, 2, False, True), (8, 4096, 16, 16, 2, False, False), (13, 1028, 70, 66, 3, True, True), (32, 256, 200, 200, 7, True, False),
+    (33, 256, 12, 10, 12, False, True), (9, 90, 6, 4, 2, True, True)])
+def test_router_and_list_of_pairs_in_one_call(dtype, scores, tokens, width, outputs, experts, top, corrected, gated):
+    """The same choices and weights as without the list, and every pair of a real expert listed once, under its expert."""
+    from mini_infer_amd import ops
+
+    rng = np.random.default_rng(tokens + width)
+    x = dev(rng.standard_normal((tokens, width)), TORCH[dtype])
+    router = dev(rng.standard_normal((outputs, width)) * 2.0 / np.sqrt(width))
+    correction = dev(rng.standard_normal(outputs) * 0.2) if corrected else None
+    gate_row = dev(rng.standard_normal(width) / np.sqrt(width)) if gated else None
+    args, how = (x, router, correction, gate_row), {"top": top, "route_scale": 1.7, "scores": scores}
+    chosen, weights, gates = ops.route_top_k(*args, **how)
+    again = ops.route_top_k(*args, **how, experts=experts)
+    assert torch.equal(chosen, again[0])
+    np.testing.assert_allclose(again[1].cpu().numpy(), weights.cpu().numpy(), rtol=0, atol=4e-6)
+    z = x.double().cpu().numpy() @ router.double().cpu().numpy().T
+    s = 1 / (1 + np.exp(-z)) if scores == "logistic" else np.exp(z - z.max(axis=1, keepdims=True)) / np.exp(z - z.max(axis=1, keepdims=True)).sum(axis=1, keepdims=True)
+    picks = np.argsort(-(s + (0 if correction is None else correction.double().cpu().numpy())), axis=1, kind="stable")[:, :top]
+    np.testing.assert_array_equal(chosen.cpu().numpy(), picks)
+    np.testing.assert_allclose(weights.cpu().numpy(), 1.7 * np.take_along_axis(s, picks, axis=1), rtol=0, atol=4e-6)
+    if gated:
+        np.testing.assert_allclose(again[2].cpu().numpy(), gates.cpu().numpy(), rtol=0, atol=2e-6)
+    listed, first = again[3].listed.cpu().numpy(), again[3].first.cpu().numpy()
+    flat = picks.reshape(-1)
+    assert first[0] == 0 and first[-1] == (flat < experts).sum()
+    for e in range(experts):
+        assert sorted(listed[first[e]: first[e + 1]].tolist()) == np.flatnonzero(flat == e).tolist()
 
 
 def test_logistic_scores_that_float32_cannot_tell_apart_are_ranked_by_their_logits():
