@@ -35,7 +35,7 @@ from mini_infer_amd.cache.state_slots import StateSlots
 from mini_infer_amd.exceptions import OutOfMemoryError
 from mini_infer_amd.parts.base import CacheNeeds, LayerCache, StateNeeds
 
-RELEASED = -1  # block-table entry of a page a window has passed
+RELEASED = -1  # block-table entry of a page a window or a chunk has passed
 
 
 @dataclasses.dataclass
@@ -46,6 +46,7 @@ class PageGroup:
     head_dim: int
     window: int | None
     pool: PagePool
+    chunk: int | None = None
     value_dim: int = 0  # width of a value row; 0: the group keeps no values
     v_transposed: bool = False  # values stored [dim][slot] inside a page, as its mixers asked
     k_storage: torch.Tensor | None = None
@@ -54,9 +55,15 @@ class PageGroup:
 
     def first_live_page(self, length: int, page_size: int) -> int:
         """Index of the first page a query at position `length` (or later) can see."""
-        if self.window is None:
-            return 0
-        return max(0, length - self.window + 1) // page_size
+        first = 0 if self.window is None else max(0, length - self.window + 1)
+        if self.chunk is not None:
+            first = max(first, length // self.chunk * self.chunk)
+        return first // page_size
+
+    @property
+    def releases(self) -> bool:
+        """Whether pages of a request are given back while it lives."""
+        return self.window is not None or self.chunk is not None
 
 
 @dataclasses.dataclass
@@ -104,7 +111,7 @@ class CacheManager:
                 pages = need.pages
                 if pages.num_kv_heads <= 0 or pages.head_dim <= 0 or pages.value_dim < 0:
                     raise ValueError(f"call {call}: impossible page needs {pages}")
-                key = (pages.num_kv_heads, pages.head_dim, pages.value_dim, pages.window, pages.v_transposed)
+                key = (pages.num_kv_heads, pages.head_dim, pages.value_dim, pages.window, pages.chunk, pages.v_transposed)
                 group = by_shape.get(key)
                 if group is None:
                     group = PageGroup(
@@ -113,6 +120,7 @@ class CacheManager:
                         num_kv_heads=pages.num_kv_heads,
                         head_dim=pages.head_dim,
                         window=pages.window,
+                        chunk=pages.chunk,
                         pool=PagePool(num_pages),
                         value_dim=pages.value_dim,
                         v_transposed=pages.v_transposed,
@@ -245,13 +253,13 @@ class CacheManager:
                 self.states.push_position(self._slots[request_id])
 
     def commit(self, extents: dict[Hashable, int]) -> None:
-        """Advance lengths after a step and give back what windows have passed."""
+        """Advance lengths after a step and give back what windows and chunks have passed."""
         for request_id, new_tokens in extents.items():
             length = self._lengths[request_id] + new_tokens
             self._lengths[request_id] = length
             self.states.set_position(self._slots[request_id], length)
             for group in self.groups:
-                if group.window is None:
+                if not group.releases:
                     continue
                 table = group.tables[request_id]
                 for i in range(min(group.first_live_page(length, self.page_size), len(table))):
@@ -270,7 +278,7 @@ class CacheManager:
         keep = self.pages_for_tokens(length)
         for group in self.groups:
             table = group.tables[request_id]
-            if group.window is not None and any(
+            if group.releases and any(
                 p == RELEASED for p in table[group.first_live_page(length, self.page_size) : keep]
             ):
                 raise ValueError("a windowed group has already released pages this truncation needs")

@@ -53,6 +53,14 @@ __device__ __forceinline__ double wave_sum(double v) {
   return v;
 }
 
+// what a head's result is multiplied by: logistic(gate[at]), one number per (token, query head), or 1 without a gate
+template <typename S, typename T>
+__device__ __forceinline__ S head_gate(const T* gate, int64_t at) {
+  if (gate == nullptr) return (S)1;
+  if constexpr (sizeof(S) == 8) return 1.0 / (1.0 + exp(-(double)to_f32(gate[at])));
+  else return mi_logistic(to_f32(gate[at]));
+}
+
 // VEC: head_dim is a multiple of 16 (16-byte loads, no guards inside a row)
 template <typename T, int VPL, bool VEC>
 __global__ __launch_bounds__(64) void attn_generic_kernel(
@@ -62,7 +70,7 @@ __global__ __launch_bounds__(64) void attn_generic_kernel(
     int64_t out_row_stride, float* __restrict__ part_acc, float* __restrict__ part_ml, int q_heads,
     int kv_heads, int head_dim, int page_size, float scale, int window, int num_splits,
     const float* __restrict__ slopes, int v_dim, int64_t v_row_stride, int has_sink, float sink_logit, int mask_chunk,
-    float softcap, const float* __restrict__ sinks) {
+    float softcap, const float* __restrict__ sinks, const T* __restrict__ gate, int64_t gate_row_stride) {
   using S = typename SumType<T>::type;
   extern __shared__ __align__(8) unsigned char q_lds_bytes[];
   S* q_lds = reinterpret_cast<S*>(q_lds_bytes);  // [GT][head_dim], pre-multiplied by the scale
@@ -227,7 +235,7 @@ __global__ __launch_bounds__(64) void attn_generic_kernel(
           // a sink: one more term in the denominator, exp(sink_logit) on the scores' own scale
           // (one logit for all heads, or one per query head where `sinks` is given)
           const S sunk = has_sink ? (S)exp((double)(sinks != nullptr ? sinks[head0 + g] : sink_logit) - (double)m[g]) : (S)0;
-          const S inv = (S)1 / (l[g] + sunk);
+          const S inv = (S)1 / (l[g] + sunk) * head_gate<S>(gate, (int64_t)t * gate_row_stride + head0 + g);
 #pragma unroll
           for (int v = 0; v < VPL; ++v)
             if (VEC || lane * VPL + v < v_dim) o[v] = from_f32<T>((float)(acc[g][v] * inv));
@@ -263,7 +271,8 @@ __global__ __launch_bounds__(512) void attn_reduce_kernel(const float* __restric
                                                          const float* __restrict__ part_ml,
                                                          T* __restrict__ out, int64_t out_row_stride,
                                                          int q_heads, int head_dim, int num_splits,
-                                                         int has_sink, float sink_logit, const float* __restrict__ sinks) {
+                                                         int has_sink, float sink_logit, const float* __restrict__ sinks,
+                                                         const T* __restrict__ gate, int64_t gate_row_stride) {
   using S = typename SumType<T>::type;
   const int t = blockIdx.x, h = blockIdx.y;
   const int lane = threadIdx.x % MI_WAVE;
@@ -293,7 +302,7 @@ __global__ __launch_bounds__(512) void attn_reduce_kernel(const float* __restric
   S l_all = 0;
   for (int s = 0; s < num_splits; ++s) l_all += (S)__shfl(l_s, s, MI_WAVE) * (S)__shfl(w_s, s, MI_WAVE);
   if (has_sink) l_all += (S)exp((double)(sinks != nullptr ? sinks[h] : sink_logit) - (double)m_all);
-  const S inv = (S)1 / l_all;
+  const S inv = (S)1 / l_all * head_gate<S>(gate, (int64_t)t * gate_row_stride + h);
   // The partial accumulators are read in batches of independent loads (a load per split
   // issued one after the other's use would cost a memory latency per split) and added in
   // split order.
@@ -342,7 +351,7 @@ static int attn_generic_launch(const void* q, int64_t q_row_stride, const void* 
                                int page_size, float scale, int window, int num_splits,
                                const float* slopes, hipStream_t stream, int v_dim = 0, int64_t v_row_stride = 0,
                                int has_sink = 0, float sink_logit = 0.f, int mask_chunk = 0, float softcap = 0.f,
-                               const float* sinks = nullptr) {
+                               const float* sinks = nullptr, const void* gate = nullptr, int64_t gate_row_stride = 0) {
   // (values as wide as the keys and packed, no sink: what the callers that say nothing mean)
   if (v_dim <= 0) v_dim = head_dim;
   if (v_row_stride <= 0) v_row_stride = v_dim;
@@ -355,7 +364,7 @@ static int attn_generic_launch(const void* q, int64_t q_row_stride, const void* 
       (const T*)q, q_row_stride, (const T*)k_pages, (const T*)v_pages, block_table, max_blocks,   \
       token_request, positions, (T*)out, out_row_stride, part_acc, part_ml, q_heads, kv_heads,    \
       head_dim, page_size, scale, window, num_splits, slopes, v_dim, v_row_stride, has_sink, sink_logit, mask_chunk, \
-      softcap, sinks)
+      softcap, sinks, (const T*)gate, gate_row_stride)
   if (v_dim <= 64) { if (vec) MI_ATTN_LAUNCH(1, true); else MI_ATTN_LAUNCH(1, false); }
   else if (v_dim <= 128) { if (vec) MI_ATTN_LAUNCH(2, true); else MI_ATTN_LAUNCH(2, false); }
   else if (v_dim <= 256) { if (vec) MI_ATTN_LAUNCH(4, true); else MI_ATTN_LAUNCH(4, false); }
@@ -365,7 +374,8 @@ static int attn_generic_launch(const void* q, int64_t q_row_stride, const void* 
   if (num_splits > 1) {
     dim3 rgrid(num_tokens, q_heads);
     attn_reduce_kernel<T><<<rgrid, reduce_threads(v_dim), 0, stream>>>(part_acc, part_ml, (T*)out, out_row_stride,
-                                                         q_heads, v_dim, num_splits, has_sink, sink_logit, sinks);
+                                                         q_heads, v_dim, num_splits, has_sink, sink_logit, sinks,
+                                                         (const T*)gate, gate_row_stride);
     MI_CHECK_LAUNCH("attn_reduce");
   }
   return MI_OK;
@@ -427,7 +437,8 @@ extern "C" int mi_attn_generic(int dtype, const void* q, int64_t q_row_stride, c
 // and optionally a sink: one more term exp(sink_logit) in the softmax's denominator that
 // carries no value (`sinks`, if given, holds a logit per query head instead), a cap on the scaled
 // scores (`softcap` * tanh(score / `softcap`), taken before the distance bias; 0: none), and optionally a chunked mask: a query sees only the keys of its own
-// stretch of `mask_chunk` positions (0: none).  Queries are [token][head][head_dim], outputs [token][head][v_dim];
+// stretch of `mask_chunk` positions (0: none), and optionally a `gate` (element type, row t at
+// t * gate_row_stride, one number per query head): head h's result is multiplied by logistic(gate[t][h]).  Queries are [token][head][head_dim], outputs [token][head][v_dim];
 // part_acc holds num_tokens*q_heads*num_splits*v_dim floats.
 extern "C" int mi_attn_general(int dtype, const void* q, int64_t q_row_stride, const void* k_pages,
                                const void* v_pages, const int* block_table, int max_blocks,
@@ -436,7 +447,9 @@ extern "C" int mi_attn_general(int dtype, const void* q, int64_t q_row_stride, c
                                int num_tokens, int q_heads, int kv_heads, int head_dim, int v_dim,
                                int64_t v_row_stride, int page_size, int num_pages, float scale, int window,
                                int num_splits, const float* slopes, int has_sink, float sink_logit,
-                               int mask_chunk, float softcap, const float* sinks, hipStream_t stream) {
+                               int mask_chunk, float softcap, const float* sinks, const void* gate,
+                               int64_t gate_row_stride, hipStream_t stream) {
+  MI_REQUIRE(gate == nullptr || gate_row_stride >= q_heads, "attn_general: a gate has one number per query head");
   MI_REQUIRE(softcap >= 0.f, "attn_general: softcap=%g must be 0 (none) or positive", (double)softcap);
   MI_REQUIRE(sinks == nullptr || has_sink, "attn_general: per-head sink logits come with has_sink");
   MI_REQUIRE(mask_chunk >= 0, "attn_general: mask_chunk=%d must be 0 (none) or positive", mask_chunk);
@@ -452,25 +465,26 @@ extern "C" int mi_attn_general(int dtype, const void* q, int64_t q_row_stride, c
                                       token_request, positions, out, out_row_stride, part_acc, part_ml,
                                       num_tokens, q_heads, kv_heads, head_dim, page_size, scale, window,
                                       num_splits, slopes, stream, v_dim, v_row_stride, has_sink, sink_logit, mask_chunk,
-                                      softcap, sinks);
+                                      softcap, sinks, gate, gate_row_stride);
   return attn_generic_launch<bf16_t>(q, q_row_stride, k_pages, v_pages, block_table, max_blocks,
                                      token_request, positions, out, out_row_stride, part_acc, part_ml,
                                      num_tokens, q_heads, kv_heads, head_dim, page_size, scale, window,
                                      num_splits, slopes, stream, v_dim, v_row_stride, has_sink, sink_logit, mask_chunk,
-                                      softcap, sinks);
+                                      softcap, sinks, gate, gate_row_stride);
 }
 
 // The combining step alone, for partials written by the matrix-core kernel.
 extern "C" int mi_attn_reduce_bf16(const float* part_acc, const float* part_ml, void* out,
                                    int64_t out_row_stride, int num_tokens, int q_heads,
                                    int head_dim, int num_splits, int has_sink, float sink_logit,
-                                   const float* sinks, hipStream_t stream) {
+                                   const float* sinks, const void* gate, int64_t gate_row_stride, hipStream_t stream) {
   if (num_tokens == 0) return MI_OK;
   MI_REQUIRE(q_heads <= 65535, "attn_reduce: too many heads");
   dim3 rgrid(num_tokens, q_heads);
   attn_reduce_kernel<bf16_t><<<rgrid, reduce_threads(head_dim), 0, stream>>>(part_acc, part_ml, (bf16_t*)out,
                                                             out_row_stride, q_heads, head_dim,
-                                                            num_splits, has_sink, sink_logit, sinks);
+                                                            num_splits, has_sink, sink_logit, sinks,
+                                                            (const bf16_t*)gate, gate_row_stride);
   MI_CHECK_LAUNCH("attn_reduce");
   return MI_OK;
 }

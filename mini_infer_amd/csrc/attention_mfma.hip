@@ -29,6 +29,8 @@
 //
 // Semantics as in the reference's oracle (cache/packed_attention.py:296-338):
 // row at absolute position p sees keys 0..p, or p-window+1..p with a window.
+// Value heads may be of a width of their own (VD, ANYV below).  A head's result may be multiplied by
+// logistic(gate) of its token, one number per query head, where it is written.
 // Requires head_dim % 32 == 0 and page_size % 16 == 0; other sizes use the plain kernel.
 #include "common.h"
 
@@ -62,7 +64,9 @@ __device__ __forceinline__ float quad_sum(float v) {
 // OCC: waves per SIMD the registers are budgeted for.  SHARED: the block's waves load key
 // and value tiles together through LDS (prefill); else every wave loads its own operands
 // through two register sets (decode), the values at the start of the block that uses them.
-template <int D, int WAVES, int KW, int RG, int OCC, bool SHARED, int PS>
+// VD: the value heads' width; ANYV: they are `v_dim_arg` wide, a multiple of 16 and at most VD (the
+// value blocks past their end read its last dims again and are not written).
+template <int D, int WAVES, int KW, int RG, int OCC, bool SHARED, int PS, int VD = D, bool ANYV = false>
 __global__ __launch_bounds__(64 * WAVES * KW, OCC) void attn_mfma_kernel(
     const bf16_t* __restrict__ q, int64_t q_row_stride, const bf16_t* __restrict__ k_pages,
     const bf16_t* __restrict__ vt_pages, const int* __restrict__ block_table, int max_blocks,
@@ -71,7 +75,9 @@ __global__ __launch_bounds__(64 * WAVES * KW, OCC) void attn_mfma_kernel(
     float* __restrict__ part_ml, int q_heads, int kv_heads, int page_size_arg, unsigned page_magic, float scale_log2,
     int window, int num_splits, int heads_per_block, int tokens_per_tile, int one_tile_per_request,
     int pair_group, int first_token, int has_sink, float sink_log2, int mask_chunk,
-    const float* __restrict__ sinks, const float* __restrict__ slopes, float softcap) {
+    const float* __restrict__ sinks, const float* __restrict__ slopes, float softcap, int v_dim_arg,
+    const bf16_t* __restrict__ gate, int64_t gate_row_stride) {
+  const int v_dim = ANYV ? v_dim_arg : VD;
   constexpr int KSTEPS = D / 32;  // MFMA k-steps over the head dim for S^T
   // PS != 0: the page size is this constant (divisions become shifts, value offsets
   // immediates); PS == 0: any multiple of 16, divided by multiplying with
@@ -80,7 +86,7 @@ __global__ __launch_bounds__(64 * WAVES * KW, OCC) void attn_mfma_kernel(
   auto page_index = [&](int key) -> int {  // (keys are never negative: unsigned division is a shift)
     return PS ? (int)((unsigned)key / (unsigned)(PS ? PS : 1)) : (int)__umulhi((unsigned)key, page_magic);
   };
-  constexpr int DBLOCKS = D / 16;  // 16-dim blocks of the output
+  constexpr int DBLOCKS = VD / 16;  // 16-dim blocks of the output
 
   // ---- which tile of which request ----------------------------------------
   // Every wave finds it on its own.  With at most one tile per request (decode, short
@@ -297,6 +303,8 @@ __global__ __launch_bounds__(64 * WAVES * KW, OCC) void attn_mfma_kernel(
   };
   const int page_stride = kv_heads * page_size * D;  // elements from one page to the next
   const int head_off = kvh * page_size * D;
+  const int v_page_stride = ANYV ? kv_heads * page_size * v_dim : kv_heads * page_size * VD;
+  const int v_head_off = ANYV ? kvh * page_size * v_dim : kvh * page_size * VD;
   const unsigned k_lane_off = (unsigned)(col * D + quad * 8);
   const unsigned v_lane_off = (unsigned)(col * page_size + 4 * quad);
   // Decode shape with 16-slot pages and key rows of whole cache lines: keys and values are read
@@ -308,7 +316,8 @@ __global__ __launch_bounds__(64 * WAVES * KW, OCC) void attn_mfma_kernel(
   auto load_values = [&](const bf16_t* const v_base[2], bf16x8_t* v) {
 #pragma unroll
     for (int db = 0; db < DBLOCKS; ++db) {
-      const unsigned off = v_lane_off + (unsigned)(db * 16) * (unsigned)page_size;
+      const unsigned dim0 = ANYV ? (unsigned)min(db * 16, v_dim - 16) : (unsigned)(db * 16);
+      const unsigned off = v_lane_off + dim0 * (unsigned)page_size;
       const bf16x4_t* from0 = reinterpret_cast<const bf16x4_t*>(v_base[0] + off);
       const bf16x4_t* from1 = reinterpret_cast<const bf16x4_t*>(v_base[1] + off);
       const bf16x4_t v0 = STREAM_KV ? __builtin_nontemporal_load(from0) : *from0;
@@ -326,10 +335,9 @@ __global__ __launch_bounds__(64 * WAVES * KW, OCC) void attn_mfma_kernel(
     for (int hlf = 0; hlf < 2; ++hlf) {
       const int key0 = kb + 16 * hlf;
       const int page = max(ids.page[hlf], 0);
-      const int64_t chunk_off = (int64_t)page * page_stride + head_off;
       const int slot0 = key0 - page_index(key0) * page_size;
-      k_base[hlf] = k_pages + chunk_off + (int64_t)slot0 * D;
-      blk.v_base[hlf] = vt_pages + chunk_off + slot0;
+      k_base[hlf] = k_pages + (int64_t)page * page_stride + head_off + (int64_t)slot0 * D;
+      blk.v_base[hlf] = vt_pages + (int64_t)page * v_page_stride + v_head_off + slot0;
     }
 #pragma unroll
     for (int hlf = 0; hlf < 2; ++hlf) {
@@ -517,10 +525,10 @@ __global__ __launch_bounds__(64 * WAVES * KW, OCC) void attn_mfma_kernel(
     constexpr int CPR = D / 8;  // 16-byte chunks per key row
     constexpr int KROW = D + 8;  // elements
     constexpr int VROW = 32 + 4;
-    constexpr int K_CHUNKS = 32 * CPR, V_CHUNKS = 4 * D;
+    constexpr int K_CHUNKS = 32 * CPR, V_CHUNKS = 4 * VD;
     constexpr int K_PER = (K_CHUNKS + THREADS - 1) / THREADS, V_PER = (V_CHUNKS + THREADS - 1) / THREADS;
     __shared__ __attribute__((aligned(16))) bf16_t k_lds[2][32 * KROW];
-    __shared__ __attribute__((aligned(16))) bf16_t v_lds[2][D * VROW];
+    __shared__ __attribute__((aligned(16))) bf16_t v_lds[2][VD * VROW];
     const int tid = threadIdx.x;
     bf16x8_t k_stage[K_PER], v_stage[V_PER];
     // Which half of the tile (16 keys of one page) and which 16 bytes of it a thread fetches
@@ -532,9 +540,9 @@ __global__ __launch_bounds__(64 * WAVES * KW, OCC) void attn_mfma_kernel(
     // (Bases are made from the kernel's own pointer arguments, not picked from an array of
     // pointers: those lose their address space, become flat loads, and flat loads are
     // counted with the LDS reads, so that every wait for an operand read would wait for them.)
-    static_assert((16 * CPR) % 64 == 0 && (2 * D) % 64 == 0, "a half's chunks fill whole waves");
+    static_assert((16 * CPR) % 64 == 0 && (2 * VD) % 64 == 0, "a half's chunks fill whole waves");
     constexpr bool K_HALF_KNOWN = (16 * CPR) % THREADS == 0;  // then (tid + j * THREADS) / (16 * CPR) is j's alone
-    constexpr bool V_HALF_KNOWN = (2 * D) % THREADS == 0;
+    constexpr bool V_HALF_KNOWN = (2 * VD) % THREADS == 0;
     int k_half[K_PER], v_half[V_PER];
     unsigned k_lane_byte[K_PER], v_lane_byte[V_PER];
 #pragma unroll
@@ -546,13 +554,13 @@ __global__ __launch_bounds__(64 * WAVES * KW, OCC) void attn_mfma_kernel(
 #pragma unroll
     for (int j = 0; j < V_PER; ++j) {
       const int id = tid + j * THREADS;
-      v_half[j] = V_HALF_KNOWN ? (j * THREADS) / (2 * D) : __builtin_amdgcn_readfirstlane(id / (2 * D));
-      const int dim = (id % (2 * D)) / 2, part = id % 2;
+      v_half[j] = V_HALF_KNOWN ? (j * THREADS) / (2 * VD) : __builtin_amdgcn_readfirstlane(id / (2 * VD));
+      const int dim = ANYV ? min((id % (2 * VD)) / 2, v_dim - 1) : (id % (2 * VD)) / 2, part = id % 2;
       v_lane_byte[j] = (unsigned)(dim * page_size + part * 8) * 2u;
     }
-    const unsigned page_bytes = (unsigned)page_stride * 2u;
+    const unsigned page_bytes = (unsigned)page_stride * 2u, v_page_bytes = (unsigned)v_page_stride * 2u;
     const char* const k_head = reinterpret_cast<const char*>(k_pages + head_off);
-    const char* const v_head = reinterpret_cast<const char*>(vt_pages + head_off);
+    const char* const v_head = reinterpret_cast<const char*>(vt_pages + v_head_off);
     auto request_tile = [&](int kb, const PageIds& ids) {
       uint64_t k_base[2], v_base[2];
 #pragma unroll
@@ -562,8 +570,9 @@ __global__ __launch_bounds__(64 * WAVES * KW, OCC) void attn_mfma_kernel(
         // (tiles start at multiples of 32 keys: with pages of 16 a half is a whole page)
         const unsigned slot0 = PS == 16 ? 0u : (unsigned)(key0 - page_index(key0) * page_size);
         const uint64_t chunk = (uint64_t)page * page_bytes;
+        const uint64_t v_chunk = (!ANYV && VD == D) ? chunk : (uint64_t)page * v_page_bytes;
         k_base[hlf] = reinterpret_cast<uint64_t>(k_head) + chunk + slot0 * (unsigned)(D * 2);
-        v_base[hlf] = reinterpret_cast<uint64_t>(v_head) + chunk + slot0 * 2u;
+        v_base[hlf] = reinterpret_cast<uint64_t>(v_head) + v_chunk + slot0 * 2u;
         // (kept in scalar registers as they are: otherwise the lane offset is added to the
         // heads once and the page product is redone per load on the vector pipe, in 64 bits)
         asm("" : "+s"(k_base[hlf]));
@@ -599,7 +608,7 @@ __global__ __launch_bounds__(64 * WAVES * KW, OCC) void attn_mfma_kernel(
       for (int j = 0; j < V_PER; ++j) {
         const int id = tid + j * THREADS;
         if (V_CHUNKS % THREADS == 0 || id < V_CHUNKS) {
-          const int hlf = id / (2 * D), dim = (id % (2 * D)) / 2, part = id % 2;
+          const int hlf = id / (2 * VD), dim = (id % (2 * VD)) / 2, part = id % 2;
           bf16x4_t lo, hi;  // rows are 8-byte aligned only: two 8-byte stores
 #pragma unroll
           for (int i = 0; i < 4; ++i) {
@@ -756,10 +765,12 @@ __global__ __launch_bounds__(64 * WAVES * KW, OCC) void attn_mfma_kernel(
       // a sink: one more term in the denominator (its score, like all others here, in log2 units)
       // (one logit for all heads, or one per query head where `sinks` is given)
       const float sunk_log2 = sinks != nullptr ? sinks[head[rg]] * LOG2E : sink_log2;
-      const float inv = 1.f / (l_run[rg] + (has_sink ? exp2f(sunk_log2 - m_run[rg]) : 0.f));
-      bf16_t* o = out + (int64_t)token[rg] * out_row_stride + (int64_t)head[rg] * D + quad * 4;
+      float inv = 1.f / (l_run[rg] + (has_sink ? exp2f(sunk_log2 - m_run[rg]) : 0.f));
+      if (gate != nullptr) inv *= mi_logistic((float)gate[(int64_t)token[rg] * gate_row_stride + head[rg]]);
+      bf16_t* o = out + (int64_t)token[rg] * out_row_stride + (int64_t)head[rg] * v_dim + quad * 4;
 #pragma unroll
       for (int db = 0; db < DBLOCKS; ++db) {
+        if (ANYV && db * 16 >= v_dim) break;
         bf16x4_t packed;
 #pragma unroll
         for (int r = 0; r < 4; ++r) packed[r] = (bf16_t)(o_acc[rg][db][r] * inv);
@@ -767,9 +778,10 @@ __global__ __launch_bounds__(64 * WAVES * KW, OCC) void attn_mfma_kernel(
       }
     } else {
       const int64_t slot = ((int64_t)token[rg] * q_heads + head[rg]) * num_splits + split;
-      float* pa = part_acc + slot * D + quad * 4;
+      float* pa = part_acc + slot * v_dim + quad * 4;
 #pragma unroll
       for (int db = 0; db < DBLOCKS; ++db) {
+        if (ANYV && db * 16 >= v_dim) break;
         *reinterpret_cast<f32x4_t*>(pa + db * 16) = o_acc[rg][db];
       }
       if (quad == 0) {
@@ -783,7 +795,7 @@ __global__ __launch_bounds__(64 * WAVES * KW, OCC) void attn_mfma_kernel(
 extern "C" int mi_attn_reduce_bf16(const float* part_acc, const float* part_ml, void* out,
                                    int64_t out_row_stride, int num_tokens, int q_heads,
                                    int head_dim, int num_splits, int has_sink, float sink_logit,
-                                   const float* sinks, hipStream_t stream);
+                                   const float* sinks, const void* gate, int64_t gate_row_stride, hipStream_t stream);
 
 static int heads_per_block_for(int group, int rows) { return group < rows ? group : rows; }
 
@@ -821,6 +833,14 @@ extern "C" int mi_attn_mfma_supported(int head_dim, int page_size) {
   return (d_ok && page_size > 0 && page_size % 16 == 0) ? 1 : 0;
 }
 
+// Value heads of a width of their own: which pairs of widths have a kernel (pages of 16 slots only).
+extern "C" int mi_attn_mfma_values_supported(int head_dim, int v_dim, int page_size) {
+  if (!mi_attn_mfma_supported(head_dim, page_size)) return 0;
+  if (v_dim == head_dim) return 1;
+  return (head_dim == 64 || head_dim == 96 || head_dim == 128 || head_dim == 192) && page_size == 16 && v_dim > 0 &&
+                 v_dim % 16 == 0 && v_dim <= 128 ? 1 : 0;
+}
+
 // `num_tiles` = sum over requests of ceil(q_len / tokens_per_tile), computed by the
 // caller from the host copy of cu_seqlens_q (a larger number is harmless).
 // `one_tile_per_request` = 1 promises that no request has more than tokens_per_tile
@@ -831,8 +851,11 @@ extern "C" int mi_attn_mfma_supported(int head_dim, int page_size) {
 // those of the whole step (cu_seqlens_q holds token numbers of the whole step);
 // `first_token` is the run's first token and `num_tokens` the run's token count.
 // With num_splits > 1, part_acc holds (first_token+num_tokens)*q_heads*num_splits*head_dim
-// floats and part_ml (first_token+num_tokens)*q_heads*num_splits*2; `combine` = 0 leaves the
+// floats (v_dim floats where value heads have a width of their own) and part_ml
+// (first_token+num_tokens)*q_heads*num_splits*2; `combine` = 0 leaves the
 // key ranges' results there for the caller's next kernel to combine (`out` is not written).
+// `gate` (bfloat16, row t at t * gate_row_stride, one number per query head; may be null): head h's
+// result for token t is multiplied by logistic(gate[t][h]).
 extern "C" int mi_attn_mfma(const void* q, int64_t q_row_stride, const void* k_pages,
                             const void* vt_pages, const int* block_table, int max_blocks,
                             const int* cu_seqlens_q, const int* positions, int num_requests,
@@ -841,7 +864,12 @@ extern "C" int mi_attn_mfma(const void* q, int64_t q_row_stride, const void* k_p
                             int head_dim, int page_size, int num_pages, float scale, int window,
                             int num_splits, int shape, int one_tile_per_request,
                             int first_token, int combine, int has_sink, float sink_logit, int mask_chunk,
-                            const float* sinks, const float* slopes, float softcap, hipStream_t stream) {
+                            const float* sinks, const float* slopes, float softcap, int v_dim, const void* gate,
+                            int64_t gate_row_stride, hipStream_t stream) {
+  MI_REQUIRE(mi_attn_mfma_values_supported(head_dim, v_dim, page_size),
+             "attn_mfma: value heads of %d beside key heads of %d in pages of %d are not taken", v_dim, head_dim, page_size);
+  MI_REQUIRE(gate == nullptr || (gate_row_stride >= q_heads && (num_splits == 1 || combine)),
+             "attn_mfma: a gate has one number per query head and goes with combined results");
   MI_REQUIRE(sinks == nullptr || has_sink, "attn_mfma: per-head sink logits come with has_sink");
   MI_REQUIRE(softcap >= 0.f, "attn_mfma: softcap=%g must be 0 (none) or positive", (double)softcap);
   MI_REQUIRE(mask_chunk >= 0, "attn_mfma: mask_chunk=%d must be 0 (none) or positive", mask_chunk);
@@ -861,7 +889,7 @@ extern "C" int mi_attn_mfma(const void* q, int64_t q_row_stride, const void* k_p
   MI_REQUIRE(scale > 0.f, "attn_mfma: the score scale must be positive, got %g", (double)scale);
   MI_REQUIRE(num_splits >= 1 && num_splits <= 64, "attn_mfma: num_splits=%d must be 1..64", num_splits);
   MI_REQUIRE(num_splits == 1 || (part_acc && part_ml), "attn_mfma: split keys need partial buffers");
-  MI_REQUIRE(q_row_stride >= (int64_t)q_heads * head_dim && out_row_stride >= (int64_t)q_heads * head_dim,
+  MI_REQUIRE(q_row_stride >= (int64_t)q_heads * head_dim && out_row_stride >= (int64_t)q_heads * v_dim,
              "attn_mfma: row strides shorter than q_heads*head_dim");
   MI_REQUIRE(q_row_stride % 8 == 0 && out_row_stride % 4 == 0,
              "attn_mfma: row strides must keep 16-byte (q) and 8-byte (out) alignment");
@@ -897,14 +925,15 @@ extern "C" int mi_attn_mfma(const void* q, int64_t q_row_stride, const void* k_p
              "attn_mfma: block table of %d pages of %d is too long for this kernel", max_blocks, page_size);
   const unsigned page_magic = (unsigned)((1ull << 32) / (unsigned)page_size) + 1u;
 
-#define MI_LAUNCH(DD, WW, KK, RR, OO, SS, PP)                                                 \
-  attn_mfma_kernel<DD, WW, KK, RR, OO, SS, PP><<<grid, 64 * WW * KK, 0, stream>>>(                    \
+#define MI_LAUNCH_V(DD, WW, KK, RR, OO, SS, PP, VV, AA)                                                \
+  attn_mfma_kernel<DD, WW, KK, RR, OO, SS, PP, VV, AA><<<grid, 64 * WW * KK, 0, stream>>>(            \
       (const bf16_t*)q, q_row_stride, (const bf16_t*)k_pages, (const bf16_t*)vt_pages,            \
       block_table, max_blocks, cu_seqlens_q, positions, num_requests, (bf16_t*)out,               \
       out_row_stride, part_acc, part_ml, q_heads, kv_heads, page_size, page_magic, scale_log2,    \
       window,                                                                                     \
       num_splits, hb, tq, one_tile_per_request, pair_group, first_token, has_sink, sink_logit * LOG2E, mask_chunk, \
-      sinks, slopes, softcap)
+      sinks, slopes, softcap, v_dim, (const bf16_t*)gate, gate_row_stride)
+#define MI_LAUNCH(DD, WW, KK, RR, OO, SS, PP) MI_LAUNCH_V(DD, WW, KK, RR, OO, SS, PP, DD, false)
 // (head sizes above 128 have no wide shape and were refused above: their cases name the 128 kernel,
 // so that nothing is compiled for them)
 #define MI_LAUNCH_P(DD, PP)                                                                       \
@@ -917,23 +946,47 @@ extern "C" int mi_attn_mfma(const void* q, int64_t q_row_stride, const void* k_p
   } else {                              \
     MI_LAUNCH_P(DD, 0);                 \
   }
-  switch (head_dim) {
-    case 32: MI_LAUNCH_D(32); break;
-    case 64: MI_LAUNCH_D(64); break;
-    case 96: MI_LAUNCH_D(96); break;
-    case 128: MI_LAUNCH_D(128); break;
-    case 192: MI_LAUNCH_D(192); break;
-    default: MI_LAUNCH_D(256); break;
+// value heads of a width of their own: rounded up to 64, 96 or 128
+#define MI_LAUNCH_DV(DD, VV)                                                                               \
+  if (decode_only) MI_LAUNCH_V(DD, 1, MI_DECODE_KW, 1, 2, false, 16, VV, true);                            \
+  else if (shape == MI_SHAPE_PREFILL_WIDE)                                                                 \
+    MI_LAUNCH_V((DD <= 128 ? DD : 128), MI_WIDE_WAVES, 1, MI_PREFILL_RG, 2, true, 16, VV, true);           \
+  else MI_LAUNCH_V(DD, MI_PREFILL_WAVES, 1, MI_PREFILL_RG, MI_PREFILL_OCC(DD), true, 16, VV, true)
+#define MI_LAUNCH_ANYV(DD)                          \
+  if (v_dim <= 64) { MI_LAUNCH_DV(DD, 64); }        \
+  else if (v_dim <= 96) { MI_LAUNCH_DV(DD, 96); }   \
+  else { MI_LAUNCH_DV(DD, 128); }
+  if (v_dim != head_dim) {
+    switch (head_dim) {
+      case 64: MI_LAUNCH_ANYV(64); break;
+      case 96: MI_LAUNCH_ANYV(96); break;
+      case 128: MI_LAUNCH_ANYV(128); break;
+      default: MI_LAUNCH_ANYV(192); break;
+    }
+  } else {
+    switch (head_dim) {
+      case 32: MI_LAUNCH_D(32); break;
+      case 64: MI_LAUNCH_D(64); break;
+      case 96: MI_LAUNCH_D(96); break;
+      case 128: MI_LAUNCH_D(128); break;
+      case 192: MI_LAUNCH_D(192); break;
+      default: MI_LAUNCH_D(256); break;
+    }
   }
+#undef MI_LAUNCH_ANYV
+#undef MI_LAUNCH_DV
 #undef MI_LAUNCH_D
 #undef MI_LAUNCH_P
 #undef MI_LAUNCH
+#undef MI_LAUNCH_V
   MI_CHECK_LAUNCH("attn_mfma");
   if (num_splits > 1 && combine) {
     const int64_t first_slot = (int64_t)first_token * q_heads * num_splits;
-    return mi_attn_reduce_bf16(part_acc + first_slot * head_dim, part_ml + first_slot * 2,
+    return mi_attn_reduce_bf16(part_acc + first_slot * v_dim, part_ml + first_slot * 2,
                                (bf16_t*)out + (int64_t)first_token * out_row_stride, out_row_stride,
-                               num_tokens, q_heads, head_dim, num_splits, has_sink, sink_logit, sinks, stream);
+                               num_tokens, q_heads, v_dim, num_splits, has_sink, sink_logit, sinks,
+                               gate ? (const bf16_t*)gate + (int64_t)first_token * gate_row_stride : nullptr,
+                               gate_row_stride, stream);
   }
   return MI_OK;
 }

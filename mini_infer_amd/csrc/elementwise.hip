@@ -33,48 +33,62 @@ __device__ __forceinline__ void store4(bf16_t* p, const float v[4]) {
 }
 
 // ---------------------------------------------------------------------------
-// embedding: residual[t, :] = float(table[ids[t], :]) * scale
+// embedding: residual[t, :] = float(table[ids[t], :]) * scale (+ float(rows[positions[t], :]), a learned
+// row per position; a position past the table's last row reads the last row, callers refuse such steps)
 // ---------------------------------------------------------------------------
 
 template <typename T, int VEC>
 __global__ void embed_gather_kernel(const T* __restrict__ table, const int* __restrict__ ids,
-                                    float* __restrict__ residual, int hidden, float scale) {
+                                    float* __restrict__ residual, int hidden, float scale,
+                                    const T* __restrict__ position_rows, const int* __restrict__ positions,
+                                    int num_positions) {
   const int t = blockIdx.x;
   const T* row = table + (int64_t)ids[t] * hidden;
+  const T* more = position_rows ? position_rows + (int64_t)min(max(positions[t], 0), num_positions - 1) * hidden : nullptr;
   float* out = residual + (int64_t)t * hidden;
   if (VEC == 4) {
     for (int i = threadIdx.x * 4; i < hidden; i += blockDim.x * 4) {
-      float v[4];
+      float v[4], p[4] = {0.f, 0.f, 0.f, 0.f};
       load4(row + i, v);
+      if (more) load4(more + i, p);
 #pragma unroll
-      for (int e = 0; e < 4; ++e) v[e] *= scale;  // (times 1 changes nothing)
+      for (int e = 0; e < 4; ++e) v[e] = __builtin_fmaf(v[e], scale, p[e]);  // (times 1 plus 0 changes nothing)
       store4(out + i, v);
     }
   } else {
-    for (int i = threadIdx.x; i < hidden; i += blockDim.x) out[i] = to_f32(row[i]) * scale;
+    for (int i = threadIdx.x; i < hidden; i += blockDim.x)
+      out[i] = __builtin_fmaf(to_f32(row[i]), scale, more ? to_f32(more[i]) : 0.f);
   }
 }
 
 template <typename T>
 static int embed_gather_launch(const void* table, const int* ids, float* residual, int num_tokens,
-                               int hidden, float scale, hipStream_t stream) {
+                               int hidden, float scale, const void* position_rows, const int* positions,
+                               int num_positions, hipStream_t stream) {
   if (num_tokens == 0) return MI_OK;
   if (hidden % 4 == 0) {
-    embed_gather_kernel<T, 4><<<num_tokens, 256, 0, stream>>>((const T*)table, ids, residual, hidden, scale);
+    embed_gather_kernel<T, 4><<<num_tokens, 256, 0, stream>>>((const T*)table, ids, residual, hidden, scale,
+                                                              (const T*)position_rows, positions, num_positions);
   } else {
-    embed_gather_kernel<T, 1><<<num_tokens, 256, 0, stream>>>((const T*)table, ids, residual, hidden, scale);
+    embed_gather_kernel<T, 1><<<num_tokens, 256, 0, stream>>>((const T*)table, ids, residual, hidden, scale,
+                                                              (const T*)position_rows, positions, num_positions);
   }
   MI_CHECK_LAUNCH("embed_gather");
   return MI_OK;
 }
 
+// position_rows [num_positions, hidden] with positions [num_tokens], or both null
 extern "C" int mi_embed_gather(int dtype, const void* table, const int* ids, float* residual,
-                               int num_tokens, int hidden, int vocab, float scale, hipStream_t stream) {
+                               int num_tokens, int hidden, int vocab, float scale, const void* position_rows,
+                               const int* positions, int num_positions, hipStream_t stream) {
   MI_REQUIRE(num_tokens >= 0 && hidden > 0 && vocab > 0,
              "embed_gather: bad sizes tokens=%d hidden=%d vocab=%d", num_tokens, hidden, vocab);
+  MI_REQUIRE((position_rows == nullptr) == (positions == nullptr) && (position_rows == nullptr || num_positions > 0),
+             "embed_gather: rows by position come with the positions and at least one row");
   MI_REQUIRE(dtype == MI_F32 || dtype == MI_BF16, "embed_gather: unknown dtype %d", dtype);
-  if (dtype == MI_F32) return embed_gather_launch<float>(table, ids, residual, num_tokens, hidden, scale, stream);
-  return embed_gather_launch<bf16_t>(table, ids, residual, num_tokens, hidden, scale, stream);
+  if (dtype == MI_F32)
+    return embed_gather_launch<float>(table, ids, residual, num_tokens, hidden, scale, position_rows, positions, num_positions, stream);
+  return embed_gather_launch<bf16_t>(table, ids, residual, num_tokens, hidden, scale, position_rows, positions, num_positions, stream);
 }
 
 // ---------------------------------------------------------------------------
@@ -385,23 +399,23 @@ extern "C" int mi_add_rmsnorm(int dtype, const void* delta, float* residual, con
 
 __global__ void rope_table_kernel(const int* __restrict__ positions,
                                   const float* __restrict__ inv_freq, float* __restrict__ cos_t,
-                                  float* __restrict__ sin_t, int half) {
+                                  float* __restrict__ sin_t, int half, float amplitude) {
   const int t = blockIdx.x;
   const float pos = (float)positions[t];
   for (int j = threadIdx.x; j < half; j += blockDim.x) {
     const float angle = pos * inv_freq[j];
     float s, c;
     sincosf(angle, &s, &c);
-    cos_t[(int64_t)t * half + j] = c;
-    sin_t[(int64_t)t * half + j] = s;
+    cos_t[(int64_t)t * half + j] = c * amplitude;  // (times 1 changes nothing)
+    sin_t[(int64_t)t * half + j] = s * amplitude;
   }
 }
 
 extern "C" int mi_rope_table(const int* positions, const float* inv_freq, float* cos_t,
-                             float* sin_t, int num_tokens, int half, hipStream_t stream) {
+                             float* sin_t, int num_tokens, int half, float amplitude, hipStream_t stream) {
   MI_REQUIRE(num_tokens >= 0 && half > 0, "rope_table: bad sizes tokens=%d half=%d", num_tokens, half);
   if (num_tokens == 0) return MI_OK;
-  rope_table_kernel<<<num_tokens, 64, 0, stream>>>(positions, inv_freq, cos_t, sin_t, half);
+  rope_table_kernel<<<num_tokens, 64, 0, stream>>>(positions, inv_freq, cos_t, sin_t, half, amplitude);
   MI_CHECK_LAUNCH("rope_table");
   return MI_OK;
 }
@@ -421,7 +435,7 @@ __global__ __launch_bounds__(256) void rope_kv_write_kernel(
     T* __restrict__ qkv, int64_t row_stride, const float* __restrict__ cos_t,
     const float* __restrict__ sin_t, const int* __restrict__ slot_mapping, T* __restrict__ k_pages,
     T* __restrict__ v_pages, int q_heads, int kv_heads, int head_dim, int rotary_dim,
-    int interleaved, int page_size, int v_transposed, int v_dim) {
+    int interleaved, int page_size, int v_transposed, int v_dim, const float* __restrict__ bias) {
   const int t = blockIdx.x;
   // the blocks along y share a token's work items
   const int first = blockIdx.y * blockDim.x + threadIdx.x;
@@ -431,22 +445,35 @@ __global__ __launch_bounds__(256) void rope_kv_write_kernel(
   const float* c = cos_t + (int64_t)t * half;
   const float* s = sin_t + (int64_t)t * half;
 
+  // the projection's value at column i of the row, its bias added
+  auto biased = [&](const T* x, int column, int i) -> float {
+    return bias ? to_f32(x[i]) + bias[column + i] : to_f32(x[i]);
+  };
   for (int e = first; e < q_heads * half; e += stride) {
     const int h = e / half, j = e % half;
     const int i0 = interleaved ? 2 * j : j;
     const int i1 = interleaved ? 2 * j + 1 : j + half;
     T* x = row + h * head_dim;
-    const float x0 = to_f32(x[i0]), x1 = to_f32(x[i1]);
+    const float x0 = biased(x, h * head_dim, i0), x1 = biased(x, h * head_dim, i1);
     x[i0] = from_f32<T>(x0 * c[j] - x1 * s[j]);
     x[i1] = from_f32<T>(x1 * c[j] + x0 * s[j]);
+  }
+  const int pass = head_dim - rotary_dim;
+  if (bias) {  // (without one the dims that are not rotated stay as they are)
+    for (int e = first; e < q_heads * pass; e += stride) {
+      const int h = e / pass, d = rotary_dim + e % pass;
+      T* x = row + h * head_dim;
+      x[d] = from_f32<T>(biased(x, h * head_dim, d));
+    }
   }
 
   if (kv_heads == 0 || slot_mapping == nullptr) return;
   const int slot = slot_mapping[t];
   if (slot < 0) return;
   const int page = slot / page_size, off = slot % page_size;
-  const T* k_row = row + (int64_t)q_heads * head_dim;
-  const T* v_row = k_row + (int64_t)kv_heads * head_dim;
+  const int k_col = q_heads * head_dim, v_col = k_col + kv_heads * head_dim;
+  const T* k_row = row + k_col;
+  const T* v_row = row + v_col;
 
   for (int e = first; e < kv_heads * half; e += stride) {
     const int h = e / half, j = e % half;
@@ -454,21 +481,21 @@ __global__ __launch_bounds__(256) void rope_kv_write_kernel(
     const int i1 = interleaved ? 2 * j + 1 : j + half;
     const T* x = k_row + h * head_dim;
     T* dst = k_pages + (((int64_t)page * kv_heads + h) * page_size + off) * head_dim;
-    const float x0 = to_f32(x[i0]), x1 = to_f32(x[i1]);
+    const float x0 = biased(x, k_col + h * head_dim, i0), x1 = biased(x, k_col + h * head_dim, i1);
     dst[i0] = from_f32<T>(x0 * c[j] - x1 * s[j]);
     dst[i1] = from_f32<T>(x1 * c[j] + x0 * s[j]);
   }
-  const int pass = head_dim - rotary_dim;
   for (int e = first; e < kv_heads * pass; e += stride) {
     const int h = e / pass, d = rotary_dim + e % pass;
-    k_pages[(((int64_t)page * kv_heads + h) * page_size + off) * head_dim + d] = k_row[h * head_dim + d];
+    k_pages[(((int64_t)page * kv_heads + h) * page_size + off) * head_dim + d] =
+        from_f32<T>(biased(k_row, k_col, h * head_dim + d));
   }
   // (value heads are v_dim wide, which need not be the keys' width)
   for (int e = first; e < kv_heads * v_dim; e += stride) {
     const int h = e / v_dim, d = e % v_dim;
     const int64_t chunk = ((int64_t)page * kv_heads + h) * page_size * v_dim;
     const int64_t at = v_transposed ? chunk + (int64_t)d * page_size + off : chunk + (int64_t)off * v_dim + d;
-    v_pages[at] = v_row[h * v_dim + d];
+    v_pages[at] = from_f32<T>(biased(v_row, v_col, h * v_dim + d));
   }
 }
 
@@ -482,7 +509,7 @@ __global__ __launch_bounds__(256) void rope_kv_write_vec4_kernel(
     T* __restrict__ qkv, int64_t row_stride, const float* __restrict__ cos_t,
     const float* __restrict__ sin_t, const int* __restrict__ slot_mapping, T* __restrict__ k_pages,
     T* __restrict__ v_pages, int q_heads, int kv_heads, int head_dim, int rotary_dim, int page_size,
-    int v_transposed, int num_tokens, int blocks_y) {
+    int v_transposed, int num_tokens, int blocks_y, int v_dim, const float* __restrict__ bias) {
   const int t = blockIdx.x;
   const int first = blockIdx.y * blockDim.x + threadIdx.x;
   const int stride = blockDim.x * blocks_y;
@@ -492,10 +519,20 @@ __global__ __launch_bounds__(256) void rope_kv_write_vec4_kernel(
   const float* c = cos_t + (int64_t)t * half;
   const float* s = sin_t + (int64_t)t * half;
 
-  auto rotate4 = [&](const T* x, int j, float lo[4], float hi[4]) {
+  // four of the row's columns, their biases added
+  auto load_biased = [&](int column, float v[4]) {
+    load4(row + column, v);
+    if (bias) {
+      float more[4];
+      load4(bias + column, more);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) v[i] += more[i];
+    }
+  };
+  auto rotate4 = [&](int column, int j, float lo[4], float hi[4]) {
     float x0[4], x1[4], cj[4], sj[4];
-    load4(x + j, x0);
-    load4(x + half + j, x1);
+    load_biased(column + j, x0);
+    load_biased(column + half + j, x1);
     load4(c + j, cj);
     load4(s + j, sj);
 #pragma unroll
@@ -509,31 +546,38 @@ __global__ __launch_bounds__(256) void rope_kv_write_vec4_kernel(
     const int h = e / half4, j = (e % half4) * 4;
     T* x = row + h * head_dim;
     float lo[4], hi[4];
-    rotate4(x, j, lo, hi);
+    rotate4(h * head_dim, j, lo, hi);
     store4(x + j, lo);
     store4(x + half + j, hi);
+  }
+  const int pass4 = (head_dim - rotary_dim) / 4;
+  if (bias) {  // (without one the dims that are not rotated stay as they are)
+    for (int e = first; e < q_heads * pass4; e += stride) {
+      const int column = (e / pass4) * head_dim + rotary_dim + (e % pass4) * 4;
+      float x[4];
+      load_biased(column, x);
+      store4(row + column, x);
+    }
   }
 
   if (kv_heads == 0 || slot_mapping == nullptr) return;
   const int slot = slot_mapping[t];
   if (slot < 0) return;
   const int page = slot / page_size, off = slot % page_size;
-  const T* k_row = row + (int64_t)q_heads * head_dim;
-  const T* v_row = k_row + (int64_t)kv_heads * head_dim;
+  const int k_col = q_heads * head_dim, v_col = k_col + kv_heads * head_dim;
 
   for (int e = first; e < kv_heads * half4; e += stride) {
     const int h = e / half4, j = (e % half4) * 4;
     T* dst = k_pages + (((int64_t)page * kv_heads + h) * page_size + off) * head_dim;
     float lo[4], hi[4];
-    rotate4(k_row + h * head_dim, j, lo, hi);
+    rotate4(k_col + h * head_dim, j, lo, hi);
     store4(dst + j, lo);
     store4(dst + half + j, hi);
   }
-  const int pass4 = (head_dim - rotary_dim) / 4;
   for (int e = first; e < kv_heads * pass4; e += stride) {
     const int h = e / pass4, d = rotary_dim + (e % pass4) * 4;
     float x[4];
-    load4(k_row + h * head_dim + d, x);
+    load_biased(k_col + h * head_dim + d, x);
     store4(k_pages + (((int64_t)page * kv_heads + h) * page_size + off) * head_dim + d, x);
   }
   if (v_transposed && page_size % 8 == 0) {
@@ -548,48 +592,52 @@ __global__ __launch_bounds__(256) void rope_kv_write_vec4_kernel(
       for (int i = 0; i < page_size; ++i) whole_page = whole_page && slot_mapping[lead + i] == page * page_size + i;
     }
     if (whole_page) {
-      const int64_t v_off = (int64_t)(q_heads + kv_heads) * head_dim;
-      const int rows_each = (kv_heads * head_dim + page_size - 1) / page_size;
-      const int e_end = min((off + 1) * rows_each, kv_heads * head_dim);
+      const int rows_each = (kv_heads * v_dim + page_size - 1) / page_size;
+      const int e_end = min((off + 1) * rows_each, kv_heads * v_dim);
       for (int e = off * rows_each + first; e < e_end; e += stride) {
-        const int h = e / head_dim, d = e % head_dim;
-        T* dst = v_pages + ((int64_t)page * kv_heads + h) * page_size * head_dim + (int64_t)d * page_size;
-        const T* src = qkv + (int64_t)lead * row_stride + v_off + h * head_dim + d;
+        const int h = e / v_dim, d = e % v_dim;
+        T* dst = v_pages + ((int64_t)page * kv_heads + h) * page_size * v_dim + (int64_t)d * page_size;
+        const T* src = qkv + (int64_t)lead * row_stride + v_col + h * v_dim + d;
+        const float more = bias ? bias[v_col + h * v_dim + d] : 0.f;
         for (int i0 = 0; i0 < page_size; i0 += 8) {
           if constexpr (sizeof(T) == 2) {
             bf16x8_vec x;
 #pragma unroll
-            for (int i = 0; i < 8; ++i) x[i] = src[(int64_t)(i0 + i) * row_stride];
+            for (int i = 0; i < 8; ++i) {
+              x[i] = src[(int64_t)(i0 + i) * row_stride];
+              if (bias) x[i] = (bf16_t)((float)x[i] + more);
+            }
             *reinterpret_cast<bf16x8_vec*>(dst + i0) = x;
           } else {
 #pragma unroll
-            for (int i = 0; i < 8; ++i) dst[i0 + i] = src[(int64_t)(i0 + i) * row_stride];
+            for (int i = 0; i < 8; ++i) dst[i0 + i] = from_f32<T>(to_f32(src[(int64_t)(i0 + i) * row_stride]) + more);
           }
         }
       }
       return;
     }
   }
-  const int dim4 = head_dim / 4;
+  const int dim4 = v_dim / 4;
   for (int e = first; e < kv_heads * dim4; e += stride) {
     const int h = e / dim4, d = (e % dim4) * 4;
-    const int64_t chunk = ((int64_t)page * kv_heads + h) * page_size * head_dim;
+    const int64_t chunk = ((int64_t)page * kv_heads + h) * page_size * v_dim;
+    float x[4];
+    load_biased(v_col + h * v_dim + d, x);
     if (v_transposed) {
 #pragma unroll
-      for (int i = 0; i < 4; ++i) v_pages[chunk + (int64_t)(d + i) * page_size + off] = v_row[h * head_dim + d + i];
+      for (int i = 0; i < 4; ++i) v_pages[chunk + (int64_t)(d + i) * page_size + off] = from_f32<T>(x[i]);
     } else {
-      float x[4];
-      load4(v_row + h * head_dim + d, x);
-      store4(v_pages + chunk + (int64_t)off * head_dim + d, x);
+      store4(v_pages + chunk + (int64_t)off * v_dim + d, x);
     }
   }
 }
 
+// bias: float32 [q heads | k heads | v heads], added to the projection's columns before anything else, or null
 extern "C" int mi_rope_kv_write(int dtype, void* qkv, int64_t row_stride, const float* cos_t,
                                 const float* sin_t, const int* slot_mapping, void* k_pages,
                                 void* v_pages, int num_tokens, int q_heads, int kv_heads,
                                 int head_dim, int rotary_dim, int interleaved, int page_size,
-                                int num_pages, int v_transposed, int v_head_dim, hipStream_t stream) {
+                                int num_pages, int v_transposed, int v_head_dim, const float* bias, hipStream_t stream) {
   if (v_head_dim <= 0) v_head_dim = head_dim;  // values as wide as keys
   MI_REQUIRE(num_tokens >= 0 && q_heads >= 0 && kv_heads >= 0 && head_dim > 0,
              "rope_kv_write: bad sizes tokens=%d q_heads=%d kv_heads=%d head_dim=%d", num_tokens,
@@ -605,19 +653,19 @@ extern "C" int mi_rope_kv_write(int dtype, void* qkv, int64_t row_stride, const 
   // the usual layout, everything a multiple of 4 elements and 16-byte aligned: four elements a thread
   const size_t elem = dtype == MI_F32 ? 4 : 2;
   const bool aligned = ((uintptr_t)qkv | (uintptr_t)cos_t | (uintptr_t)sin_t | (uintptr_t)k_pages |
-                        (uintptr_t)v_pages | (uintptr_t)(row_stride * elem)) % 16 == 0;
-  if (!interleaved && aligned && head_dim % 4 == 0 && rotary_dim % 8 == 0 && v_head_dim == head_dim) {
-    const int items = max(q_heads * (rotary_dim / 8), kv_heads * (head_dim / 4));
+                        (uintptr_t)v_pages | (uintptr_t)(row_stride * elem) | (uintptr_t)bias) % 16 == 0;
+  if (!interleaved && aligned && head_dim % 4 == 0 && rotary_dim % 8 == 0 && v_head_dim % 4 == 0) {
+    const int items = max(q_heads * (rotary_dim / 8), kv_heads * (max(head_dim, v_head_dim) / 4));
     const int blocks_y = min((num_tokens >= 512) ? 2 : 16, max(1, ceil_div(items, 256)));
     dim3 grid(num_tokens, blocks_y);
     if (dtype == MI_F32) {
       rope_kv_write_vec4_kernel<float><<<grid, 256, 0, stream>>>(
           (float*)qkv, row_stride, cos_t, sin_t, slot_mapping, (float*)k_pages, (float*)v_pages,
-          q_heads, kv_heads, head_dim, rotary_dim, page_size, v_transposed, num_tokens, blocks_y);
+          q_heads, kv_heads, head_dim, rotary_dim, page_size, v_transposed, num_tokens, blocks_y, v_head_dim, bias);
     } else {
       rope_kv_write_vec4_kernel<bf16_t><<<grid, 256, 0, stream>>>(
           (bf16_t*)qkv, row_stride, cos_t, sin_t, slot_mapping, (bf16_t*)k_pages, (bf16_t*)v_pages,
-          q_heads, kv_heads, head_dim, rotary_dim, page_size, v_transposed, num_tokens, blocks_y);
+          q_heads, kv_heads, head_dim, rotary_dim, page_size, v_transposed, num_tokens, blocks_y, v_head_dim, bias);
     }
     MI_CHECK_LAUNCH("rope_kv_write");
     return MI_OK;
@@ -629,11 +677,11 @@ extern "C" int mi_rope_kv_write(int dtype, void* qkv, int64_t row_stride, const 
   if (dtype == MI_F32) {
     rope_kv_write_kernel<float><<<grid, 256, 0, stream>>>(
         (float*)qkv, row_stride, cos_t, sin_t, slot_mapping, (float*)k_pages, (float*)v_pages,
-        q_heads, kv_heads, head_dim, rotary_dim, interleaved, page_size, v_transposed, v_head_dim);
+        q_heads, kv_heads, head_dim, rotary_dim, interleaved, page_size, v_transposed, v_head_dim, bias);
   } else {
     rope_kv_write_kernel<bf16_t><<<grid, 256, 0, stream>>>(
         (bf16_t*)qkv, row_stride, cos_t, sin_t, slot_mapping, (bf16_t*)k_pages, (bf16_t*)v_pages,
-        q_heads, kv_heads, head_dim, rotary_dim, interleaved, page_size, v_transposed, v_head_dim);
+        q_heads, kv_heads, head_dim, rotary_dim, interleaved, page_size, v_transposed, v_head_dim, bias);
   }
   MI_CHECK_LAUNCH("rope_kv_write");
   return MI_OK;

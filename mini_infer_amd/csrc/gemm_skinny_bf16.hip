@@ -66,10 +66,18 @@ typedef __attribute__((__vector_size__(4 * sizeof(float)))) float f32x4_t;
 //              sumsq[block][row], and the product that consumes c (PRO_SCALED) adds them up
 //              and multiplies its own sums with the factor, which commutes with the product.
 //              The norm's launch between two products is saved.
+//   EPI_LAYER_IN  W is the stacked input projection of a whole layer whose sublayers read one norm:
+//              [q | k | v | head gates | ff gate | ff up] (k and v absent where the layer reads another's, the
+//              last two where its feed-forward is made elsewhere).  A block computes PAIRS of features as in
+//              EPI_ROPE: rotated dims with their partners, dims that pass with dims that pass, value dims
+//              with value dims, gates with gates, a feed-forward's gate feature with its up feature.
+//              Biases are added to q, k and v; queries go to c[m, q_heads*head_dim], keys and values to
+//              their slots, head gates (not activated) to their own rows, the feed-forward's
+//              activation to its own rows.
 // In every case the sums are rounded to bfloat16 before the activation or rotation,
 // exactly as when the product and the second step run as two kernels.
 enum { EPI_STORE = 0, EPI_GATED = 1, EPI_ROPE = 2, EPI_ADDNORM = 3, EPI_STORE_F32 = 4, EPI_GELU_TABLE = 5, EPI_GRU = 6,
-       EPI_GATED_CLAMPED = 7, EPI_GATED_GELU = 8 };
+       EPI_GATED_CLAMPED = 7, EPI_GATED_GELU = 8, EPI_LAYER_IN = 9 };
 // Where the activations come from: a matrix in memory, or (PRO_ATTN, few rows) the
 // uncombined key ranges of attn_mfma: each wave first combines its own columns of the
 // attention output (what attn_reduce would have written) into LDS, so the combining launch
@@ -113,7 +121,19 @@ struct FoldArgs {  // what the folded neighbours of a product need
   int64_t ld_table;
   const int* table_ids;
   int table_col;
-  // EPI_GATED_CLAMPED: float32 [2n] biases of gate and up,
+  // EPI_LAYER_IN (beside the fields of EPI_ROPE, cos/sin [m, rot_half]): rotated pairs a head, value heads'
+  // width, rows of W the head gates take (q_heads of them count), features of the feed-forward; biases
+  // float32 [q | k | v] or null; where gates [m, q_heads] and activations [m, ff] go.  The feed-forward
+  // ends as EPI_GATED_CLAMPED does (glu_limit > 0, no biases) or with silu(g) * u (glu_limit 0)
+  int rot_half, v_dim, gate_rows, ff;
+  const float* qkv_bias;
+  bf16_t* gate_out;
+  int64_t ld_gate;
+  bf16_t* act_out;
+  int64_t ld_act;
+  // EPI_STORE_F32: the rounded products are multiplied by this
+  float out_scale;
+  // EPI_GATED_CLAMPED: float32 [2n] biases of gate and up (or null),
   // out = g * logistic(slope * g) * (u + 1), g = min(gate + bias, limit), u = clamp(up + bias, -limit, limit)
   const float* glu_bias;
   float glu_limit, glu_slope;
@@ -130,6 +150,7 @@ __global__ __launch_bounds__(64 * SK_WAVES) void gemm_skinny_bf16_kernel(
     bf16_t* __restrict__ c, int64_t ldc, int m, int n, int k, int features_per_block, const FoldArgs fold) {
   constexpr bool GATED = EPI == EPI_GATED || EPI == EPI_GATED_CLAMPED || EPI == EPI_GATED_GELU;
   constexpr bool ROPE = EPI == EPI_ROPE;
+  constexpr bool LAYER_IN = EPI == EPI_LAYER_IN;
   constexpr bool ADDNORM = EPI == EPI_ADDNORM;
   constexpr bool SCALED = PRO == PRO_SCALED;
   static_assert(!ROPE || NT == 1, "the rotary epilogue takes one tile of dims and its partner tile");
@@ -137,7 +158,7 @@ __global__ __launch_bounds__(64 * SK_WAVES) void gemm_skinny_bf16_kernel(
   // RT = tiles of 16 ROWS (tokens): a weight operand once in registers is used for every row tile
   static_assert(RT == 1 || (PRO == PRO_NONE && !ADDNORM), "more than 16 rows: plain activations, no folded norm");
   constexpr bool GRU = EPI == EPI_GRU;
-  constexpr int WT = GRU ? 3 * NT : (GATED || ROPE) ? 2 * NT : NT;  // weight tiles per block
+  constexpr int WT = GRU ? 3 * NT : (GATED || ROPE || LAYER_IN) ? 2 * NT : NT;  // weight tiles per block
   __shared__ float red[SK_WAVES][WT][256];
 
   // (with LINES made uniform for the compiler: the wave's range of K and with it the loop and
@@ -157,7 +178,13 @@ __global__ __launch_bounds__(64 * SK_WAVES) void gemm_skinny_bf16_kernel(
   const int pair0 = ROPE ? blockIdx.x * features_per_block : 0;
   const int pair_end = ROPE ? min(pair0 + features_per_block, total_pairs) : 0;
   const int n0 = blockIdx.x * features_per_block;
-  const int n_end = min(n0 + features_per_block, n);
+  const int n_end = min(n0 + features_per_block, n);  // (EPI_LAYER_IN: n and these count pairs)
+  // EPI_LAYER_IN: pairs of queries and keys, of values, of head gates; first rows of values, gates, feed-forward
+  const int qk_half = LAYER_IN ? fold.head_dim / 2 : 1, v_half = LAYER_IN ? fold.v_dim / 2 : 1;
+  const int qk_pairs = LAYER_IN ? (fold.q_heads + fold.kv_heads) * qk_half : 0;
+  const int v_pairs = LAYER_IN ? fold.kv_heads * v_half : 0;
+  const int gate_pairs = LAYER_IN ? fold.gate_rows / 2 : 0;
+  const int v_row0 = 2 * qk_pairs, gate_row0 = v_row0 + 2 * v_pairs, ff_row0 = gate_row0 + 2 * gate_pairs;
 
   const int ksteps = k / 32;
   const int per_wave = (ksteps + SK_WAVES - 1) / SK_WAVES;
@@ -170,6 +197,20 @@ __global__ __launch_bounds__(64 * SK_WAVES) void gemm_skinny_bf16_kernel(
     if (ROPE) {
       const int pair = min(pair0 + c, pair_end - 1);
       return (pair / half) * fold.head_dim + pair % half + t * half;
+    }
+    if (LAYER_IN) {
+      int pair = min(n0 + (t % NT) * 16 + c, n_end - 1);
+      const int partner = t / NT;
+      if (pair < qk_pairs) {
+        const int head_row = pair / qk_half * fold.head_dim, j = pair % qk_half;
+        return j < fold.rot_half ? head_row + j + partner * fold.rot_half
+                                 : head_row + fold.rot_half + j + partner * (qk_half - fold.rot_half);
+      }
+      pair -= qk_pairs;
+      if (pair < v_pairs) return v_row0 + pair / v_half * fold.v_dim + pair % v_half + partner * v_half;
+      pair -= v_pairs;
+      if (pair < gate_pairs) return gate_row0 + pair + partner * gate_pairs;
+      return ff_row0 + (pair - gate_pairs) + partner * fold.ff;
     }
     return min(n0 + (t % NT) * 16 + c, n_end - 1) + (t / NT) * n;
   };
@@ -412,7 +453,7 @@ __global__ __launch_bounds__(64 * SK_WAVES) void gemm_skinny_bf16_kernel(
 #pragma unroll
       for (int r = 0; r < 4; ++r) sum[r] += red[wv][nt][(fq * 4 + r) * 16 + token_in_tile];
     float up[4] = {0.f, 0.f, 0.f, 0.f};  // the twin tile's sums: the up half (gated), the partner dims (rotary)
-    if (GATED || ROPE || GRU) {
+    if (GATED || ROPE || GRU || LAYER_IN) {
 #pragma unroll
       for (int wv = 0; wv < SK_WAVES; ++wv)
 #pragma unroll
@@ -461,8 +502,9 @@ __global__ __launch_bounds__(64 * SK_WAVES) void gemm_skinny_bf16_kernel(
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           const int at = min(feature + r, n - 1);
-          const float g = fminf((float)(bf16_t)sum[r] + fold.glu_bias[at], fold.glu_limit);
-          const float u = fminf(fmaxf((float)(bf16_t)up[r] + fold.glu_bias[n + at], -fold.glu_limit), fold.glu_limit);
+          const float bias_g = fold.glu_bias ? fold.glu_bias[at] : 0.f, bias_u = fold.glu_bias ? fold.glu_bias[n + at] : 0.f;
+          const float g = fminf((float)(bf16_t)sum[r] + bias_g, fold.glu_limit);
+          const float u = fminf(fmaxf((float)(bf16_t)up[r] + bias_u, -fold.glu_limit), fold.glu_limit);
           sum[r] = g * mi_logistic(fold.glu_slope * g) * (u + 1.f);
         }
       } else if constexpr (EPI == EPI_GATED_GELU) {  // (the tanh form of gelu, as gated_mul spells it)
@@ -552,12 +594,119 @@ __global__ __launch_bounds__(64 * SK_WAVES) void gemm_skinny_bf16_kernel(
       }
       continue;
     }
+    if constexpr (LAYER_IN) {
+      // this thread: four consecutive pairs of one kind (and of one head: all widths are multiples of 8), one token
+      int pair = n0 + nt * 16 + fq * 4;
+      if (pair >= n_end) continue;
+      float lo[4], hi[4];
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        lo[r] = (float)(bf16_t)sum[r];
+        hi[r] = (float)(bf16_t)up[r];
+      }
+      bf16x4_t lo_b, hi_b;
+      auto round_both = [&]() {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          lo_b[r] = (bf16_t)lo[r];
+          hi_b[r] = (bf16_t)hi[r];
+        }
+      };
+      auto add_bias = [&](int lo_row, int hi_row) {
+        if (fold.qkv_bias == nullptr) return;
+        const f32x4_t bl = *reinterpret_cast<const f32x4_t*>(fold.qkv_bias + lo_row);
+        const f32x4_t bh = *reinterpret_cast<const f32x4_t*>(fold.qkv_bias + hi_row);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          lo[r] += bl[r];
+          hi[r] += bh[r];
+        }
+      };
+      const int hd = fold.head_dim, kv_heads = fold.kv_heads, rot_half = fold.rot_half;
+      if (pair < qk_pairs) {
+        const int head = pair / qk_half, j = pair % qk_half;
+        const bool turned = j < rot_half;
+        const int lo_dim = turned ? j : rot_half + j, hi_dim = lo_dim + (turned ? rot_half : qk_half - rot_half);
+        add_bias(head * hd + lo_dim, head * hd + hi_dim);
+        if (turned) {
+          const f32x4_t cs = *reinterpret_cast<const f32x4_t*>(fold.cos_t + (int64_t)token * rot_half + j);
+          const f32x4_t sn = *reinterpret_cast<const f32x4_t*>(fold.sin_t + (int64_t)token * rot_half + j);
+#pragma unroll
+          for (int r = 0; r < 4; ++r) {
+            const float x0 = lo[r], x1 = hi[r];
+            lo[r] = x0 * cs[r] - x1 * sn[r];
+            hi[r] = x1 * cs[r] + x0 * sn[r];
+          }
+        }
+        round_both();
+        bf16_t* dst = nullptr;
+        if (head < fold.q_heads) {
+          dst = c + (int64_t)token * ldc + (int64_t)head * hd;
+        } else {
+          const int slot = fold.slot_mapping[token];
+          if (slot >= 0) {  // padding rows of a replayed step write nothing
+            const int page = slot / fold.page_size, off = slot % fold.page_size;
+            dst = fold.k_pages + (((int64_t)page * kv_heads + head - fold.q_heads) * fold.page_size + off) * hd;
+          }
+        }
+        if (dst != nullptr) {
+          *reinterpret_cast<bf16x4_t*>(dst + lo_dim) = lo_b;
+          *reinterpret_cast<bf16x4_t*>(dst + hi_dim) = hi_b;
+        }
+        continue;
+      }
+      pair -= qk_pairs;
+      if (pair < v_pairs) {
+        const int head = pair / v_half, j = pair % v_half, vd = fold.v_dim;
+        add_bias(v_row0 + head * vd + j, v_row0 + head * vd + v_half + j);
+        round_both();
+        const int slot = fold.slot_mapping[token];
+        if (slot >= 0) {
+          const int page = slot / fold.page_size, off = slot % fold.page_size;
+          bf16_t* chunk = fold.v_pages + ((int64_t)page * kv_heads + head) * fold.page_size * vd;
+          if (fold.v_transposed) {
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+              chunk[(int64_t)(j + r) * fold.page_size + off] = lo_b[r];
+              chunk[(int64_t)(v_half + j + r) * fold.page_size + off] = hi_b[r];
+            }
+          } else {
+            *reinterpret_cast<bf16x4_t*>(chunk + (int64_t)off * vd + j) = lo_b;
+            *reinterpret_cast<bf16x4_t*>(chunk + (int64_t)off * vd + v_half + j) = hi_b;
+          }
+        }
+        continue;
+      }
+      pair -= v_pairs;
+      if (pair < gate_pairs) {
+        bf16_t* dst = fold.gate_out + (int64_t)token * fold.ld_gate;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          if (pair + r < fold.q_heads) dst[pair + r] = (bf16_t)lo[r];
+          if (pair + gate_pairs + r < fold.q_heads) dst[pair + gate_pairs + r] = (bf16_t)hi[r];
+        }
+        continue;
+      }
+      pair -= gate_pairs;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        if (fold.glu_limit > 0.f) {
+          const float g = fminf(lo[r], fold.glu_limit);
+          const float u = fminf(fmaxf(hi[r], -fold.glu_limit), fold.glu_limit);
+          lo_b[r] = (bf16_t)(g * mi_logistic(fold.glu_slope * g) * (u + 1.f));
+        } else {
+          lo_b[r] = (bf16_t)(lo[r] / (1.f + expf(-lo[r])) * hi[r]);
+        }
+      }
+      *reinterpret_cast<bf16x4_t*>(fold.act_out + (int64_t)token * fold.ld_act + pair) = lo_b;
+      continue;
+    }
     const int feature = n0 + nt * 16 + fq * 4;
     if constexpr (EPI == EPI_STORE_F32) {
       float* dst32 = reinterpret_cast<float*>(c) + (int64_t)token * ldc + feature;
 #pragma unroll
       for (int r = 0; r < 4; ++r)
-        if (feature + r < n_end) dst32[r] = (float)(bf16_t)sum[r];
+        if (feature + r < n_end) dst32[r] = (float)(bf16_t)sum[r] * fold.out_scale;  // (times 1 changes nothing)
       continue;
     }
     if constexpr (EPI == EPI_GELU_TABLE) {
@@ -693,10 +842,12 @@ extern "C" int mi_gemm_skinny_bf16(const void* a, int64_t lda, const void* w, in
   return skinny_plain(a, lda, w, ldw, c, ldc, m, n, k, EPI_STORE, stream);
 }
 
-// The same product, the same values, written as float32 [m, ldc].
+// The same product, the same values times `scale`, written as float32 [m, ldc].
 extern "C" int mi_gemm_skinny_f32out_bf16(const void* a, int64_t lda, const void* w, int64_t ldw, float* c,
-                                          int64_t ldc, int m, int n, int k, hipStream_t stream) {
-  return skinny_plain(a, lda, w, ldw, c, ldc, m, n, k, EPI_STORE_F32, stream);
+                                          int64_t ldc, int m, int n, int k, float scale, hipStream_t stream) {
+  FoldArgs fold = {};
+  fold.out_scale = scale;
+  return skinny_plain(a, lda, w, ldw, c, ldc, m, n, k, EPI_STORE_F32, stream, fold);
 }
 
 // c[m, n] = gelu_tanh(a . w^T) * table[ids[row], col0 : col0 + n], bfloat16 (EPI_GELU_TABLE).
@@ -895,11 +1046,11 @@ extern "C" int mi_gemm_skinny_geglu_bf16(const void* a, int64_t lda, const void*
 }
 
 // out[m, n] = g * logistic(slope * g) * (u + 1), g = min(a . gate^T + bias[:n], limit), u = clamp(a . up^T +
-// bias[n:], -limit, limit), with w = [gate; up] stacked, [2n, k], and bias float32 [2n].
+// bias[n:], -limit, limit), with w = [gate; up] stacked, [2n, k], and bias float32 [2n] or null (none).
 extern "C" int mi_gemm_skinny_clamped_glu_bf16(const void* a, int64_t lda, const void* w, int64_t ldw, const float* bias,
                                                float limit, float slope, void* out, int64_t ldo, int m, int n, int k,
                                                hipStream_t stream) {
-  MI_REQUIRE(bias != nullptr && limit > 0.f, "gemm_skinny_clamped_glu_bf16: needs the biases and a positive limit");
+  MI_REQUIRE(limit > 0.f, "gemm_skinny_clamped_glu_bf16: needs a positive limit");
   FoldArgs fold = {};
   fold.glu_bias = bias;
   fold.glu_limit = limit;
@@ -1066,4 +1217,91 @@ extern "C" int mi_gemm_skinny_rope_scaled_bf16(const void* a, int64_t lda, const
   return rope_product("gemm_skinny_rope_scaled_bf16", a, lda, sumsq, pieces, eps, w, ldw, q_out, ldq, cos_t, sin_t,
                       slot_mapping, k_pages, v_pages, m, k, q_heads, kv_heads, head_dim, page_size, num_pages,
                       v_transposed, stream);
+}
+
+// The stacked input projection of a layer whose sublayers read one norm (EPI_LAYER_IN), for at most 32
+// rows.  w: [q heads | k heads | v heads | gate_rows | ff | ff] rows of k; kv_heads = 0: no keys and values;
+// ff = 0: no feed-forward; gate_rows = 0: no head gates (else at least q_heads, a multiple of 8).  head_dim,
+// v_dim and 2 * rot_half are multiples of 8, ff of 4.  q_out [m, q_heads*head_dim] gets the rotated queries
+// (cos/sin float32 [m, rot_half]; the dims past 2 * rot_half pass), keys and values go to their
+// slots, gates to gate_out [m, q_heads], the feed-forward's activation to act_out [m, ff]:
+// limit > 0: min(g, limit) * logistic(slope * min(g, limit)) * (clamp(u, -limit, limit) + 1), else silu(g) * u.
+// qkv_bias: float32 [q | k | v] or null.  With `sumsq` the rows are a norm's output but for their factors, as
+// in mi_gemm_skinny_rope_scaled_bf16 (16 rows at most).
+extern "C" int mi_gemm_skinny_layer_in_bf16(const void* a, int64_t lda, const float* sumsq, int pieces, float eps,
+                                            const void* w, int64_t ldw, void* q_out, int64_t ldq, const float* cos_t,
+                                            const float* sin_t, const int* slot_mapping, void* k_pages, void* v_pages,
+                                            const float* qkv_bias, void* gate_out, int64_t ld_gate, void* act_out,
+                                            int64_t ld_act, int m, int k, int q_heads, int kv_heads, int head_dim,
+                                            int v_dim, int rot_half, int gate_rows, int ff, float limit, float slope,
+                                            int page_size, int num_pages, int v_transposed, hipStream_t stream) {
+  MI_REQUIRE(q_heads >= 1 && kv_heads >= 0 && head_dim >= 8 && head_dim % 8 == 0 && v_dim >= 8 && v_dim % 8 == 0 &&
+                 rot_half >= 0 && rot_half % 4 == 0 && 2 * rot_half <= head_dim && ff >= 0 && ff % 4 == 0 &&
+                 gate_rows >= 0 && gate_rows % 8 == 0 && (gate_rows == 0 || gate_rows >= q_heads),
+             "gemm_skinny_layer_in_bf16: q_heads=%d kv_heads=%d head_dim=%d v_dim=%d rot_half=%d gate_rows=%d ff=%d not taken",
+             q_heads, kv_heads, head_dim, v_dim, rot_half, gate_rows, ff);
+  const int64_t rows = (int64_t)(q_heads + kv_heads) * head_dim + (int64_t)kv_heads * v_dim + gate_rows + 2 * (int64_t)ff;
+  MI_REQUIRE(rows < (1ll << 31) && mi_gemm_skinny_wide_bf16_supported(m, (int)rows, k, lda, ldw),
+             "gemm_skinny_layer_in_bf16: takes 1 <= m <= 32, k a multiple of 32, rows aligned to 16 bytes; "
+             "got m=%d k=%d lda=%lld ldw=%lld", m, k, (long long)lda, (long long)ldw);
+  MI_REQUIRE(lda >= k && ldw >= k && ldq >= (int64_t)q_heads * head_dim && ldq % 4 == 0,
+             "gemm_skinny_layer_in_bf16: a row stride is shorter than its row or not 8-byte aligned");
+  MI_REQUIRE(rot_half == 0 || (cos_t && sin_t), "gemm_skinny_layer_in_bf16: needs the rotation tables");
+  MI_REQUIRE(kv_heads == 0 || (slot_mapping && k_pages && v_pages && page_size > 0 && num_pages > 0),
+             "gemm_skinny_layer_in_bf16: pages and slots are needed to write keys and values");
+  MI_REQUIRE(gate_rows == 0 || (gate_out && ld_gate >= q_heads), "gemm_skinny_layer_in_bf16: the head gates have no place to go");
+  MI_REQUIRE(ff == 0 || (act_out && ld_act >= ff && ld_act % 4 == 0 && (uintptr_t)act_out % 8 == 0),
+             "gemm_skinny_layer_in_bf16: the feed-forward's activation has no place to go, or one not aligned to 8 bytes");
+  MI_REQUIRE((uintptr_t)q_out % 8 == 0 && (uintptr_t)cos_t % 16 == 0 && (uintptr_t)sin_t % 16 == 0 && (uintptr_t)qkv_bias % 16 == 0,
+             "gemm_skinny_layer_in_bf16: outputs, tables and biases must be aligned to their vector accesses");
+  MI_REQUIRE(!sumsq || (m <= SK_MAX_ROWS && pieces >= 1 && pieces <= SK_SCALE_PARTS * SK_SCALE_PIECES && eps >= 0.f),
+             "gemm_skinny_layer_in_bf16: rows with their norm factor apart come 16 at most and in 1..%d pieces, got %d and %d",
+             SK_SCALE_PARTS * SK_SCALE_PIECES, m, pieces);
+  FoldArgs fold = {};
+  fold.cos_t = cos_t;
+  fold.sin_t = sin_t;
+  fold.slot_mapping = slot_mapping;
+  fold.k_pages = (bf16_t*)k_pages;
+  fold.v_pages = (bf16_t*)v_pages;
+  fold.q_heads = q_heads;
+  fold.kv_heads = kv_heads;
+  fold.head_dim = head_dim;
+  fold.page_size = page_size;
+  fold.v_transposed = v_transposed;
+  fold.rot_half = rot_half;
+  fold.v_dim = v_dim;
+  fold.gate_rows = gate_rows;
+  fold.ff = ff;
+  fold.qkv_bias = qkv_bias;
+  fold.gate_out = (bf16_t*)gate_out;
+  fold.ld_gate = ld_gate;
+  fold.act_out = (bf16_t*)act_out;
+  fold.ld_act = ld_act;
+  fold.glu_limit = limit;
+  fold.glu_slope = slope;
+  fold.sumsq_in = sumsq;
+  fold.sumsq_pieces = pieces;
+  fold.norm_eps = eps;
+  fold.norm_width = k;
+  const int cus = compute_units();
+  MI_REQUIRE(cus > 0, "gemm_skinny_layer_in_bf16: cannot read the device's compute unit count");
+  const int n = (int)(rows / 2);  // pairs
+  const int fpb = features_per_block_for(n, cus, 2);
+  const int blocks = ceil_div(n, fpb);
+  const bool lines = whole_lines(w, ldw, rows, k);
+#define SK_LAYER_IN(NT_, U_, PRO_, LINES_, RT_)                                                               \
+  gemm_skinny_bf16_kernel<NT_, U_, EPI_LAYER_IN, PRO_, LINES_, RT_><<<blocks, 64 * SK_WAVES, 0, stream>>>( \
+      (const bf16_t*)a, lda, (const bf16_t*)w, ldw, (bf16_t*)q_out, ldq, m, n, k, fpb, fold)
+  if (fpb <= 16) {
+    if (sumsq) { if (lines) SK_LAYER_IN(1, 8, PRO_SCALED, true, 1); else SK_LAYER_IN(1, 8, PRO_SCALED, false, 1); }
+    else if (m <= 16) { if (lines) SK_LAYER_IN(1, 8, PRO_NONE, true, 1); else SK_LAYER_IN(1, 8, PRO_NONE, false, 1); }
+    else { if (lines) SK_LAYER_IN(1, 4, PRO_NONE, true, 2); else SK_LAYER_IN(1, 4, PRO_NONE, false, 2); }
+  } else {
+    if (sumsq) { if (lines) SK_LAYER_IN(2, 4, PRO_SCALED, true, 1); else SK_LAYER_IN(2, 2, PRO_SCALED, false, 1); }
+    else if (m <= 16) { if (lines) SK_LAYER_IN(2, 4, PRO_NONE, true, 1); else SK_LAYER_IN(2, 2, PRO_NONE, false, 1); }
+    else { if (lines) SK_LAYER_IN(2, 2, PRO_NONE, true, 2); else SK_LAYER_IN(2, 2, PRO_NONE, false, 2); }
+  }
+#undef SK_LAYER_IN
+  MI_CHECK_LAUNCH("gemm_skinny_layer_in_bf16");
+  return MI_OK;
 }

@@ -5,7 +5,8 @@
 //                        then RMS norm of the new rows times a weight -> compute dtype.
 //                        Any of a, b, bias, shift may be absent; so may the norm.  One launch
 //                        stands between two layers: the add that ends one and the norm that
-//                        begins the next.
+//                        begins the next.  `b` may come as several rows a token with a weight each, which
+//                        are added up here (the chosen experts' outputs of a routed feed-forward).
 //   clamped_glu          [gate | up] + biases -> min(gate, limit) * logistic(slope * gate') *
 //                        (clamp(up, -limit, limit) + 1), gate' the clamped gate.
 //
@@ -72,21 +73,43 @@ __device__ __forceinline__ void store_some(bf16_t* p, const float v[VEC]) {
   }
 }
 
-// The new values of VEC columns of a row: x + scale * (a + b + bias) + shift.
+// The new values of VEC columns of a row: x + scale * (a + b + bias) + shift, with b = sum_p
+// b_weights[p] * row p of `pieces` rows that lie b_stride apart (b_weights null: one row, as it is).
 template <typename T, int VEC>
-__device__ __forceinline__ void updated(const T* ar, const T* br, const float* bias, const float* shift, float scale,
-                                        const float* x, int c, float value[VEC]) {
+__device__ __forceinline__ void updated(const T* ar, const T* br, int64_t b_stride, const float* b_weights, int pieces,
+                                        const float* bias, const float* shift, float scale, const float* x, int c,
+                                        float value[VEC]) {
   float xv[VEC], av[VEC], bv[VEC], cv[VEC], sv[VEC];
   load_some<VEC>(x + c, xv);
 #pragma unroll
   for (int e = 0; e < VEC; ++e) av[e] = bv[e] = cv[e] = sv[e] = 0.f;
   if (ar) load_some<VEC>(ar + c, av);
-  if (br) load_some<VEC>(br + c, bv);
+  double bw[VEC];  // (float32 elements: the weighted sum in 64-bit)
+  if (b_weights) {
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) bw[e] = 0.0;
+    for (int p = 0; p < pieces; ++p) {
+      float row[VEC];
+      load_some<VEC>(br + (int64_t)p * b_stride + c, row);
+      const float weight = b_weights[p];
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) {
+        if constexpr (sizeof(T) == 4) bw[e] += (double)weight * (double)row[e];
+        else bv[e] += weight * row[e];
+      }
+    }
+  } else {
+    if (br) load_some<VEC>(br + c, bv);
+    if constexpr (sizeof(T) == 4) {
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) bw[e] = (double)bv[e];
+    }
+  }
   if (bias) load_some<VEC>(bias + c, cv);
   if (shift) load_some<VEC>(shift + c, sv);
 #pragma unroll
   for (int e = 0; e < VEC; ++e) {
-    if constexpr (sizeof(T) == 4) value[e] = (float)((double)xv[e] + (double)scale * (((double)av[e] + (double)bv[e]) + (double)cv[e]) + (double)sv[e]);
+    if constexpr (sizeof(T) == 4) value[e] = (float)((double)xv[e] + (double)scale * (((double)av[e] + bw[e]) + (double)cv[e]) + (double)sv[e]);
     else value[e] = xv[e] + scale * ((av[e] + bv[e]) + cv[e]) + sv[e];
   }
 }
@@ -96,7 +119,7 @@ __device__ __forceinline__ void updated(const T* ar, const T* br, const float* b
 template <typename T, int VEC>
 __global__ __launch_bounds__(1024) void stream_update_norm_kernel(
     const T* __restrict__ a, int64_t a_stride, const T* __restrict__ b, int64_t b_stride,
-    const float* __restrict__ bias, const float* __restrict__ shift, float scale, float* __restrict__ stream,
+    const float* __restrict__ b_weights, int pieces, const float* __restrict__ bias, const float* __restrict__ shift, float scale, float* __restrict__ stream,
     const T* __restrict__ weight, T* __restrict__ out, const int* __restrict__ rows, int hidden, float eps) {
   __shared__ float scratch[16];
   __shared__ double scratch_wide[16];
@@ -105,7 +128,8 @@ __global__ __launch_bounds__(1024) void stream_update_norm_kernel(
   const int t = rows ? rows[r] : r;
   float* x = stream + (int64_t)t * hidden;
   const T* ar = a ? a + (int64_t)t * a_stride : nullptr;
-  const T* br = b ? b + (int64_t)t * b_stride : nullptr;
+  const T* br = b ? b + (int64_t)t * pieces * b_stride : nullptr;
+  const float* bwr = b_weights ? b_weights + (int64_t)t * pieces : nullptr;
   // a thread keeps the new values of its first columns (wider rows are made again below)
   constexpr int KEEP = 4;
   float kept[KEEP][VEC];
@@ -114,7 +138,7 @@ __global__ __launch_bounds__(1024) void stream_update_norm_kernel(
   int n = 0;
   for (int c = threadIdx.x * VEC; c < hidden; c += blockDim.x * VEC, ++n) {
     float value[VEC];
-    updated<T, VEC>(ar, br, bias, shift, scale, x, c, value);
+    updated<T, VEC>(ar, br, b_stride, bwr, pieces, bias, shift, scale, x, c, value);
 #pragma unroll
     for (int e = 0; e < VEC; ++e) {
       if constexpr (WIDE) squares_wide += (double)value[e] * (double)value[e];
@@ -145,7 +169,7 @@ __global__ __launch_bounds__(1024) void stream_update_norm_kernel(
     } else if (!rows) {
       load_some<VEC>(x + c, value);
     } else {  // made again: the stream was not written
-      updated<T, VEC>(ar, br, bias, shift, scale, x, c, value);
+      updated<T, VEC>(ar, br, b_stride, bwr, pieces, bias, shift, scale, x, c, value);
     }
     load_some<VEC>(weight + c, w);
 #pragma unroll
@@ -191,15 +215,18 @@ __global__ __launch_bounds__(256) void clamped_glu_kernel(const T* __restrict__ 
 
 }  // namespace
 
-// a, b: [rows of the stream, hidden] in the element type with row strides, or null; bias, shift:
+// a, b: [rows of the stream, hidden] in the element type with row strides, or null; with b_weights
+// (float32 [rows of the stream, pieces]) b is [rows of the stream * pieces, hidden] and row t gets the weighted sum
+// of its `pieces` rows (else pieces is 1 and b_weights null); bias, shift:
 // float32 [hidden] or null; weight (element type) with out [num_out_rows, hidden], or both null
 // (no norm); rows: int32 [num_out_rows] or null (every row of the stream, num_out_rows of them).
 extern "C" int mi_stream_update_norm(int dtype, const void* a, int64_t a_stride, const void* b, int64_t b_stride,
-                                     const float* bias, const float* shift, float scale, float* stream,
+                                     const float* b_weights, int pieces, const float* bias, const float* shift, float scale, float* stream,
                                      const void* weight, void* out, const int* rows, int num_out_rows, int hidden,
                                      float eps, hipStream_t stream_handle) {
   MI_REQUIRE(num_out_rows >= 0 && hidden > 0, "stream_update_norm: bad sizes rows=%d hidden=%d", num_out_rows, hidden);
   MI_REQUIRE(stream != nullptr, "stream_update_norm: no stream");
+  MI_REQUIRE(pieces >= 1 && (b_weights != nullptr ? b != nullptr : pieces == 1), "stream_update_norm: %d weighted rows a token", pieces);
   MI_REQUIRE((weight == nullptr) == (out == nullptr), "stream_update_norm: a norm weight and an output go together");
   MI_REQUIRE(weight != nullptr || rows == nullptr, "stream_update_norm: a row list only makes sense with the norm");
   MI_REQUIRE(weight == nullptr || eps > 0.f, "stream_update_norm: eps must be positive, got %g", (double)eps);
@@ -214,7 +241,7 @@ extern "C" int mi_stream_update_norm(int dtype, const void* a, int64_t a_stride,
                    ((uintptr_t)bias | (uintptr_t)shift | (uintptr_t)stream) % 16 == 0;
 #define MI_UPDATE_LAUNCH(T, VEC)                                                                                      \
   stream_update_norm_kernel<T, VEC><<<num_out_rows, threads, 0, stream_handle>>>(                                     \
-      (const T*)a, a_stride, (const T*)b, b_stride, bias, shift, scale, stream, (const T*)weight, (T*)out, rows, hidden, eps)
+      (const T*)a, a_stride, (const T*)b, b_stride, b_weights, pieces, bias, shift, scale, stream, (const T*)weight, (T*)out, rows, hidden, eps)
   if (dtype == MI_F32) { if (vec) MI_UPDATE_LAUNCH(float, 4); else MI_UPDATE_LAUNCH(float, 1); }
   else { if (vec) MI_UPDATE_LAUNCH(bf16_t, 4); else MI_UPDATE_LAUNCH(bf16_t, 1); }
 #undef MI_UPDATE_LAUNCH

@@ -7,7 +7,9 @@
 //                       a tie; logistic scores without a correction are ranked by z itself, of which
 //                       they are a rising function); leaves the chosen indices and their weights
 //                       s * route_scale (not renormalized), and, where a gate row is given,
-//                       logistic(gate . x) for a shared expert.
+//                       logistic(gate . x) for a shared expert.  With scores of the third kind the
+//                       correction is a bias of the logits, the largest biased logits are chosen and
+//                       weights are route_scale times the softmax over the chosen ones alone.
 //   route_logits, route_list   the same and the list of pairs by expert, for few bfloat16 tokens.
 //   expert_gate_up      few rows: for every (token, chosen expert) pair the expert's first product and
 //                       its activation, the weights read by expert index.
@@ -16,6 +18,7 @@
 //                       whose output is the token's input row itself.
 //   expert_combine      many rows: the same sum over rows of expert outputs that were made expert
 //                       by expert (sorted by expert; `where` maps a pair to its sorted row).
+//                       (A shared expert's rows without a shared_gate are added as they are.)
 //
 // Expert weights are stacked: gate|up [experts, 2 * ff, width] (an expert's gate rows, then its up
 // rows), or up [experts, ff, width] where experts have no gate; down [experts, width, ff].
@@ -69,15 +72,26 @@ __device__ __forceinline__ T expert_feature(A a, A b, A weight) {
   }
 }
 
+// How a token's scores are made of its logits.
+enum RouterScores { SCORES_SOFTMAX = 0, SCORES_LOGISTIC = 1, SCORES_CHOSEN_SOFTMAX = 2 };
+
 // A wave ranks a token's outputs, lane l those with e % 64 == l: the `top` largest choices and their weights.
 // `mine`: the token's logits in LDS, this wave's own (spent here: chosen ones are marked).
 template <typename A>
 __device__ __forceinline__ void rank_outputs(A* mine, const float* __restrict__ correction, int* __restrict__ chosen,
                                              float* __restrict__ weights, int outputs, int top, float route_scale,
-                                             int logistic, int lane) {
+                                             int scores, int lane) {
   const A taken = -(A)INFINITY;
   A most = taken, total_exp = 0;
-  if (!logistic) {
+  const bool logistic = scores == SCORES_LOGISTIC;
+  if (scores == SCORES_CHOSEN_SOFTMAX) {
+    // biased logits are what is ranked and what the weights are made of; the sum of exponentials is known
+    // only when all are chosen, so the weights are divided by it at the end
+    if (correction != nullptr) {
+      for (int e = lane; e < outputs; e += MI_WAVE) mine[e] += (A)correction[e];
+    }
+    correction = nullptr;
+  } else if (!logistic) {
     for (int e = lane; e < outputs; e += MI_WAVE) most = mine[e] > most ? mine[e] : most;
 #pragma unroll
     for (int off = MI_WAVE / 2; off > 0; off >>= 1) {
@@ -88,6 +102,7 @@ __device__ __forceinline__ void rank_outputs(A* mine, const float* __restrict__ 
     total_exp = lanes_total(total_exp);
   }
   const A inv = (A)1 / total_exp;  // (softmax)
+  A first_choice = taken;
   auto score_of = [&](A logit) { return logistic ? (A)1 / ((A)1 + exp_of(-logit)) : exp_of(logit - most) * inv; };
   // the choice is made on score + correction (without one on the logit, of which every score is a rising
   // function), the weight is the score alone
@@ -107,7 +122,15 @@ __device__ __forceinline__ void rank_outputs(A* mine, const float* __restrict__ 
       if (index < outputs && (best == outputs || other > best_choice || (other == best_choice && index < best))) best = index, best_choice = other;
     }
     if (best == outputs) best = 0;  // (more infinite logits than there are choices)
-    if (lane == 0) {
+    if (scores == SCORES_CHOSEN_SOFTMAX) {
+      if (k == 0) first_choice = best_choice;  // (the largest: no exponential below passes 1)
+      const A share = exp_of(best_choice - first_choice);
+      total_exp += share;
+      if (lane == 0) {
+        chosen[k] = best;
+        weights[k] = (float)share;
+      }
+    } else if (lane == 0) {
       chosen[k] = best;
       weights[k] = (float)(score_of(mine[best]) * (A)route_scale);
     }
@@ -115,6 +138,9 @@ __device__ __forceinline__ void rank_outputs(A* mine, const float* __restrict__ 
     __builtin_amdgcn_wave_barrier();
     if (lane == best % MI_WAVE) mine[best] = taken;
     __builtin_amdgcn_wave_barrier();
+  }
+  if (scores == SCORES_CHOSEN_SOFTMAX && lane == 0) {
+    for (int k = 0; k < top; ++k) weights[k] = (float)((A)weights[k] / total_exp * (A)route_scale);
   }
 }
 
@@ -124,7 +150,7 @@ template <typename T, int R>
 __global__ __launch_bounds__(1024) void route_top_k_kernel(
     const T* __restrict__ x, int64_t x_stride, const float* __restrict__ router, const float* __restrict__ correction,
     const float* __restrict__ gate_row, int* __restrict__ chosen, float* __restrict__ weights,
-    float* __restrict__ shared_gate, int num_tokens, int width, int outputs, int top, float route_scale, int logistic) {
+    float* __restrict__ shared_gate, int num_tokens, int width, int outputs, int top, float route_scale, int scores) {
   using A = typename SumOf<T>::type;
   extern __shared__ __align__(16) unsigned char lds_bytes[];
   A* z = reinterpret_cast<A*>(lds_bytes);                         // [R][outputs + 1]
@@ -195,7 +221,7 @@ __global__ __launch_bounds__(1024) void route_top_k_kernel(
     if (t >= num_tokens) break;
     A* mine = z + r * (outputs + 1);
     if (gate_row != nullptr && lane == 0) shared_gate[t] = (float)((A)1 / ((A)1 + exp_of(-mine[outputs])));
-    rank_outputs<A>(mine, correction, chosen + (int64_t)t * top, weights + (int64_t)t * top, outputs, top, route_scale, logistic, lane);
+    rank_outputs<A>(mine, correction, chosen + (int64_t)t * top, weights + (int64_t)t * top, outputs, top, route_scale, scores, lane);
   }
 }
 
@@ -272,7 +298,7 @@ __global__ __launch_bounds__(256) void expert_down_combine_kernel(
         sum += weight * (A)to_f32(from_f32<T>((float)y));
       }
     }
-    if (shared != nullptr) sum += (A)shared_gate[t] * (A)to_f32(shared[(int64_t)t * shared_stride + c]);
+    if (shared != nullptr) sum += (shared_gate != nullptr ? (A)shared_gate[t] : (A)1) * (A)to_f32(shared[(int64_t)t * shared_stride + c]);
     if (lane == 0) out[(int64_t)t * width + c] = from_f32<T>((float)sum);
   }
 }
@@ -302,7 +328,7 @@ __global__ __launch_bounds__(256) void expert_combine_kernel(
     float r[VEC];
     if (shared != nullptr) {
       mi_load_cols<T, VEC>(shared + (int64_t)t * shared_stride + c, r);
-      const A g = (A)shared_gate[t];
+      const A g = shared_gate != nullptr ? (A)shared_gate[t] : (A)1;
 #pragma unroll
       for (int j = 0; j < VEC; ++j) sum[j] += g * (A)r[j];
     }
@@ -423,7 +449,7 @@ __global__ __launch_bounds__(1024) void route_list_kernel(const float* __restric
                                                           int* __restrict__ chosen, float* __restrict__ weights,
                                                           float* __restrict__ shared_gate, int* __restrict__ listed,
                                                           int* __restrict__ first, int num_tokens, int outputs, int total,
-                                                          int experts, int top, float route_scale, int logistic) {
+                                                          int experts, int top, float route_scale, int scores) {
   extern __shared__ __align__(16) unsigned char lds_bytes[];
   float* z = reinterpret_cast<float*>(lds_bytes);                        // [waves][outputs]
   __shared__ int count[MI_SORT_MAX_EXPERTS + 1];
@@ -434,7 +460,7 @@ __global__ __launch_bounds__(1024) void route_list_kernel(const float* __restric
     for (int e = lane; e < outputs; e += MI_WAVE) mine[e] = logits[(int64_t)t * total + e];
     __builtin_amdgcn_wave_barrier();
     if (total > outputs && lane == 0) shared_gate[t] = 1.f / (1.f + expf(-logits[(int64_t)t * total + outputs]));
-    rank_outputs<float>(mine, correction, chosen + t * top, weights + t * top, outputs, top, route_scale, logistic, lane);
+    rank_outputs<float>(mine, correction, chosen + t * top, weights + t * top, outputs, top, route_scale, scores, lane);
   }
   __syncthreads();  // (what this block's waves have written to `chosen` is there for all of them)
   const int pairs = num_tokens * top;
@@ -698,10 +724,11 @@ __global__ __launch_bounds__(256) void weighted_squared_relu_kernel(const T* __r
 
 extern "C" int mi_route_top_k(int dtype, const void* x, int64_t x_stride, const float* router, const float* correction,
                               const float* gate_row, int* chosen, float* weights, float* shared_gate, int num_tokens,
-                              int width, int outputs, int top, float route_scale, int logistic, hipStream_t stream) {
+                              int width, int outputs, int top, float route_scale, int scores, hipStream_t stream) {
   MI_REQUIRE(num_tokens >= 0 && width > 0 && x_stride >= width, "route_top_k: bad sizes tokens=%d width=%d", num_tokens, width);
   MI_REQUIRE(outputs > 0 && outputs <= MI_ROUTER_MAX_OUTPUTS && top > 0 && top <= outputs,
              "route_top_k: %d router outputs (at most %d) of which %d are chosen", outputs, MI_ROUTER_MAX_OUTPUTS, top);
+  MI_REQUIRE(scores >= SCORES_SOFTMAX && scores <= SCORES_CHOSEN_SOFTMAX, "route_top_k: unknown scores %d", scores);
   MI_REQUIRE(gate_row == nullptr || shared_gate != nullptr, "route_top_k: a gate row needs a place for the gates");
   MI_REQUIRE(dtype == MI_F32 || dtype == MI_BF16, "route_top_k: unknown dtype %d", dtype);
   if (num_tokens == 0) return MI_OK;
@@ -715,7 +742,7 @@ extern "C" int mi_route_top_k(int dtype, const void* x, int64_t x_stride, const 
 #define MI_ROUTE(T, R)                                                                                               \
   route_top_k_kernel<T, R><<<blocks, threads, lds_for(R), stream>>>((const T*)x, x_stride, router, correction, gate_row, \
                                                                     chosen, weights, shared_gate, num_tokens, width,    \
-                                                                    outputs, top, route_scale, logistic)
+                                                                    outputs, top, route_scale, scores)
   if (dtype == MI_F32) {
     if (per_block == 4) MI_ROUTE(float, 4);
     else if (per_block == 2) MI_ROUTE(float, 2);
@@ -765,7 +792,7 @@ extern "C" int mi_expert_down_combine(int dtype, const void* act, const void* do
                                       int top, hipStream_t stream) {
   MI_REQUIRE(num_tokens >= 0 && width > 0 && ff > 0 && experts > 0 && top > 0 && x_stride >= width,
              "expert_down_combine: bad sizes tokens=%d width=%d ff=%d experts=%d top=%d", num_tokens, width, ff, experts, top);
-  MI_REQUIRE(shared == nullptr || (shared_gate != nullptr && shared_stride >= width), "expert_down_combine: a shared expert's rows come with their gates");
+  MI_REQUIRE(shared == nullptr || shared_stride >= width, "expert_down_combine: a shared expert's rows are shorter than a row");
   MI_REQUIRE(dtype == MI_F32 || dtype == MI_BF16, "expert_down_combine: unknown dtype %d", dtype);
   const size_t lds = (size_t)top * ff * (dtype == MI_F32 ? 4 : 2);
   MI_REQUIRE(lds <= 64 * 1024, "expert_down_combine: %d rows of %d do not fit the block's staging", top, ff);
@@ -792,7 +819,7 @@ extern "C" int mi_expert_combine(int dtype, const void* made, const int* where, 
                                  hipStream_t stream) {
   MI_REQUIRE(num_tokens >= 0 && width > 0 && experts > 0 && top > 0 && x_stride >= width,
              "expert_combine: bad sizes tokens=%d width=%d experts=%d top=%d", num_tokens, width, experts, top);
-  MI_REQUIRE(shared == nullptr || (shared_gate != nullptr && shared_stride >= width), "expert_combine: a shared expert's rows come with their gates");
+  MI_REQUIRE(shared == nullptr || shared_stride >= width, "expert_combine: a shared expert's rows are shorter than a row");
   MI_REQUIRE(dtype == MI_F32 || dtype == MI_BF16, "expert_combine: unknown dtype %d", dtype);
   if (num_tokens == 0) return MI_OK;
   const bool vec = width % 4 == 0 && x_stride % 4 == 0 && shared_stride % 4 == 0 && is_aligned16(made) && is_aligned16(x) &&
@@ -831,12 +858,13 @@ extern "C" int mi_route_few_takes(int num_tokens, int width, int outputs, int to
 // [num_tokens, outputs + (gate row ? 1 : 0)] floats.
 extern "C" int mi_route_few(const void* x, int64_t x_stride, const float* router, const float* correction, const float* gate_row,
                             float* logits, int* chosen, float* weights, float* shared_gate, int* listed, int* first,
-                            int num_tokens, int width, int outputs, int experts, int top, float route_scale, int logistic,
+                            int num_tokens, int width, int outputs, int experts, int top, float route_scale, int scores,
                             hipStream_t stream) {
   MI_REQUIRE(mi_route_few_takes(num_tokens, width, outputs, top) && x_stride >= width && x_stride % 4 == 0 && (uintptr_t)x % 8 == 0 &&
                  is_aligned16(router) && is_aligned16(gate_row),
              "route_few: %d tokens of %d columns, %d outputs", num_tokens, width, outputs);
   MI_REQUIRE(top > 0 && top <= outputs && experts > 0 && experts <= outputs, "route_few: %d of %d outputs, %d experts", top, outputs, experts);
+  MI_REQUIRE(scores >= SCORES_SOFTMAX && scores <= SCORES_CHOSEN_SOFTMAX, "route_few: unknown scores %d", scores);
   MI_REQUIRE(gate_row == nullptr || shared_gate != nullptr, "route_few: a gate row needs a place for the gates");
   const int total = outputs + (gate_row != nullptr ? 1 : 0);
   route_logits_kernel<<<dim3(total, ceil_div(num_tokens, 8)), 256, 0, stream>>>((const bf16_t*)x, x_stride, router, gate_row, logits,
@@ -844,7 +872,7 @@ extern "C" int mi_route_few(const void* x, int64_t x_stride, const float* router
   MI_CHECK_LAUNCH("route_logits");
   const int threads = min(1024, num_tokens * MI_WAVE);
   route_list_kernel<<<1, threads, (size_t)(threads / MI_WAVE) * outputs * 4, stream>>>(
-      logits, correction, chosen, weights, shared_gate, listed, first, num_tokens, outputs, total, experts, top, route_scale, logistic);
+      logits, correction, chosen, weights, shared_gate, listed, first, num_tokens, outputs, total, experts, top, route_scale, scores);
   MI_CHECK_LAUNCH("route_list");
   return MI_OK;
 }

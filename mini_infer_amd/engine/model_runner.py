@@ -74,6 +74,8 @@ class ModelRunner:
         self.vocab_size = model.vocab_size
         # the most positions a request may reach, if the model says (admission goes by it)
         self.max_model_len: int | None = getattr(model, "max_position_embeddings", None)
+        # positions the model has tensors for (a table of learned positions): a step past them is refused
+        self.num_positions: int | None = getattr(model, "num_positions", None)
         self.block_size = block_size
         self.num_blocks = num_blocks
         self.cache = CacheManager(
@@ -208,6 +210,12 @@ class ModelRunner:
                 if not 0 <= w < len(entry.tokens):
                     raise ValueError(
                         f"request {entry.request_id!r}: wanted place {w} is outside its {len(entry.tokens)} tokens"
+                    )
+            if self.num_positions is not None:
+                held = self.cache.length(entry.request_id) if self.cache.has_request(entry.request_id) else 0
+                if held + len(entry.tokens) > self.num_positions:
+                    raise ValueError(
+                        f"request {entry.request_id!r}: {held} + {len(entry.tokens)} tokens pass the model's {self.num_positions} positions"
                     )
         token_ids = np.concatenate([np.asarray(e.tokens, dtype=np.int64) for e in entries])
         if token_ids.min() < 0 or token_ids.max() >= self.vocab_size:

@@ -77,6 +77,11 @@ class DecoderModel:
         return self.spec.max_position_embeddings
 
     @property
+    def num_positions(self) -> int | None:
+        """The positions the model holds tensors for: no token can stand at or past this one (None: no such bound)."""
+        return getattr(self.embedding, "num_positions", None)
+
+    @property
     def graph_safe(self) -> bool:
         """Whether a decode step of this model can be recorded as a HIP graph."""
         parts = [self.embedding, self.final_norm, self.head, *self.blocks]

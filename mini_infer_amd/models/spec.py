@@ -99,7 +99,8 @@ class Architecture:
     contract, which is all the loader, the random-weights mode, the cache manager and the
     runner ask of a model:
 
-      dtype, device, vocab_size       attributes; `max_position_embeddings` (optional, may be None)
+      dtype, device, vocab_size       attributes; `max_position_embeddings`, `num_positions` (both
+                                      optional, may be None)
       graph_safe                      whether a step of single tokens may be recorded and replayed
       param_specs()                   {checkpoint name: ParamSpec} of every tensor it loads
       optional_names()                names a checkpoint may hold without the model needing them

@@ -62,12 +62,21 @@ ATTENTION_HEAD_DIM_STEP = 2
 ATTENTION_MAX_HEAD_DIM = 256
 
 
-def mfma_attention_supported(dtype: torch.dtype, head_dim: int, page_size: int) -> bool:
+MFMA_OWN_VALUE_HEAD_DIMS = (64, 96, 128, 192)  # key widths beside which value heads may have a width of their own
+MFMA_OWN_VALUE_MAX = 128  # up to this, in steps of 16, in pages of 16 slots
+
+
+def mfma_attention_supported(dtype: torch.dtype, head_dim: int, page_size: int, v_head_dim: int | None = None) -> bool:
     """Whether the matrix-core attention kernel takes this cache shape (else the plain kernel runs).
+    `v_head_dim`: the width of a value head where it is not the keys'.
 
     Caches it takes store their values transposed inside each page.
     """
-    return dtype == torch.bfloat16 and head_dim in MFMA_HEAD_DIMS and page_size % 16 == 0
+    if dtype != torch.bfloat16 or head_dim not in MFMA_HEAD_DIMS or page_size % 16 != 0:
+        return False
+    return v_head_dim in (None, head_dim) or (
+        head_dim in MFMA_OWN_VALUE_HEAD_DIMS and page_size == 16 and v_head_dim % 16 == 0 and 0 < v_head_dim <= MFMA_OWN_VALUE_MAX
+    )
 
 
 def _ptr(t: torch.Tensor | None) -> int | None:
@@ -90,19 +99,31 @@ def _stream() -> int:
 # ----------------------------------------------------------------------------
 
 
-def embed_gather(table: torch.Tensor, ids: torch.Tensor, scale: float = 1.0) -> torch.Tensor:
-    """`float32(table[ids]) * scale`: the start of the residual stream, [T, H] float32."""
-    _need_cuda(table, ids)
+def embed_gather(
+    table: torch.Tensor, ids: torch.Tensor, scale: float = 1.0, position_rows: torch.Tensor | None = None,
+    positions: torch.Tensor | None = None,
+) -> torch.Tensor:
+    """`float32(table[ids]) * scale`: the start of the residual stream, [T, H] float32; with `position_rows`
+    [N, H] (the table's dtype) plus `position_rows[positions]` (every position below N)."""
+    _need_cuda(table, ids, position_rows, positions)
     _need_contiguous("table", table)
     _need_contiguous("ids", ids)
     _need_int32("ids", ids)
     vocab, hidden = table.shape
+    if position_rows is not None:
+        _need_contiguous("position_rows", position_rows)
+        _need_contiguous("positions", positions)
+        _need_int32("positions", positions)
+        if (position_rows.dim() != 2 or position_rows.shape[1] != hidden or position_rows.dtype != table.dtype or positions is None
+                or positions.numel() != ids.numel()):
+            raise KernelShapeError(f"embed_gather: rows by position are {table.dtype} [N, {hidden}] and come with a position a token")
     out = torch.empty((ids.numel(), hidden), dtype=torch.float32, device=table.device)
     lib = library.load()
     library.check(
         lib.mi_embed_gather(
             _dtype_code(table), _ptr(table), _ptr(ids), _ptr(out), ids.numel(), hidden, vocab,
-            float(scale), _stream(),
+            float(scale), _ptr(position_rows), _ptr(positions) if position_rows is not None else None,
+            0 if position_rows is None else position_rows.shape[0], _stream(),
         )
     )
     return out
@@ -230,8 +251,8 @@ def add_rmsnorm(
     return out
 
 
-def rope_table(positions: torch.Tensor, inv_freq: torch.Tensor) -> tuple[torch.Tensor, torch.Tensor]:
-    """`cos, sin` of `position * inv_freq`, both [T, len(inv_freq)] float32."""
+def rope_table(positions: torch.Tensor, inv_freq: torch.Tensor, amplitude: float = 1.0) -> tuple[torch.Tensor, torch.Tensor]:
+    """`cos, sin` of `position * inv_freq`, times `amplitude`, both [T, len(inv_freq)] float32."""
     _need_cuda(positions, inv_freq)
     _need_contiguous("positions", positions)
     _need_contiguous("inv_freq", inv_freq)
@@ -243,7 +264,7 @@ def rope_table(positions: torch.Tensor, inv_freq: torch.Tensor) -> tuple[torch.T
     sin = torch.empty_like(cos)
     lib = library.load()
     library.check(
-        lib.mi_rope_table(_ptr(positions), _ptr(inv_freq), _ptr(cos), _ptr(sin), tokens, half, _stream())
+        lib.mi_rope_table(_ptr(positions), _ptr(inv_freq), _ptr(cos), _ptr(sin), tokens, half, float(amplitude), _stream())
     )
     return cos, sin
 
@@ -263,9 +284,11 @@ def rope_kv_write(
     interleaved: bool = False,
     v_transposed: bool = False,
     v_head_dim: int | None = None,
+    bias: torch.Tensor | None = None,
 ) -> None:
     """Rotate q in place inside `qkv`; rotate k and write k, v into their page slots.
     `v_head_dim`: the width of a value head where it is not the keys' (`head_dim`).
+    `bias` (float32, one number per column of q, k and v): added to the projection before anything else.
 
     `qkv` is [T, (q_heads + 2*kv_heads) * head_dim] (rows may be strided); pages are
     [num_pages, kv_heads, page_size, head_dim], value pages
@@ -292,6 +315,11 @@ def rope_kv_write(
         raise KernelShapeError(
             f"cos/sin must be float32 [{tokens}, {rotary_dim // 2}], got {tuple(cos.shape)} {cos.dtype}"
         )
+    if bias is not None:
+        _need_cuda(bias)
+        _need_contiguous("bias", bias)
+        if bias.dtype != torch.float32 or bias.numel() < (q_heads + kv_heads) * head_dim + kv_heads * v_dim:
+            raise KernelShapeError(f"rope_kv_write: the bias is float32, one number per column of q, k and v, got {bias.dtype} x {bias.numel()}")
     page_size = num_pages = 0
     if kv_heads > 0 and slot_mapping is not None:
         if k_pages is None or v_pages is None:
@@ -311,7 +339,7 @@ def rope_kv_write(
         lib.mi_rope_kv_write(
             _dtype_code(qkv), _ptr(qkv), qkv.stride(0), _ptr(cos), _ptr(sin), _ptr(slot_mapping),
             _ptr(k_pages), _ptr(v_pages), tokens, q_heads, kv_heads, head_dim, rotary_dim,
-            int(interleaved), page_size, num_pages, int(v_transposed), v_dim, _stream(),
+            int(interleaved), page_size, num_pages, int(v_transposed), v_dim, _ptr(bias), _stream(),
         )
     )
 
@@ -372,15 +400,16 @@ def gemm_skinny_bf16(a: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
     return c
 
 
-def linear_f32_out(x: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
-    """`x @ weight.T` as float32, whatever the operands' dtype: what an output head returns.
+def linear_f32_out(x: torch.Tensor, weight: torch.Tensor, scale: float = 1.0) -> torch.Tensor:
+    """`x @ weight.T` as float32, times `scale`, whatever the operands' dtype: what an output head returns.
 
     Few bfloat16 rows: the weight-streaming kernel writes float32 itself (no cast launch); its
     values are those of `linear(...).float()`, rounded to bfloat16 on the way, so that a row's
     logits do not depend on how many rows its step had.  More rows: the vendor library's
     product, cast.  float32 operands: `gemm_f32`."""
     if x.dtype == torch.float32:
-        return gemm_f32(x, weight)
+        logits = gemm_f32(x, weight)
+        return logits if scale == 1.0 else logits.mul_(scale)
     _need_cuda(x, weight)
     if (
         x.dtype == torch.bfloat16
@@ -397,11 +426,13 @@ def linear_f32_out(x: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
         out = torch.empty((m, n), dtype=torch.float32, device=x.device)
         library.check(
             library.load().mi_gemm_skinny_f32out_bf16(
-                _ptr(x), x.stride(0), _ptr(weight), weight.stride(0), _ptr(out), out.stride(0), m, n, k, _stream()
+                _ptr(x), x.stride(0), _ptr(weight), weight.stride(0), _ptr(out), out.stride(0), m, n, k, float(scale),
+                _stream(),
             )
         )
         return out
-    return torch.matmul(x, weight.t()).float()
+    logits = torch.matmul(x, weight.t()).float()
+    return logits if scale == 1.0 else logits.mul_(scale)
 
 
 def skinny_gemm_takes(m: int, k: int, lda: int, ldw: int, max_rows: int = SKINNY_MAX_ROWS) -> bool:
@@ -914,6 +945,8 @@ def paged_attention(
     chunk: int | None = None,
     sinks: torch.Tensor | None = None,
     softcap: float | None = None,
+    gate: torch.Tensor | None = None,
+    out: torch.Tensor | None = None,
 ) -> torch.Tensor | AttentionPieces:
     """Causal attention of every token over its request's pages; returns [T, q_heads*head_dim].
 
@@ -921,7 +954,12 @@ def paged_attention(
     [T, q_heads*v_head_dim]); with `v_pages=None` a value row is the first `v_head_dim` entries
     of its key row.  `sink_logit`: the softmax's denominator gets one more term
     exp(sink_logit), a sink that carries no value (both attention kernels know it; uncombined
-    `AttentionPieces` do not).  Values of a width of their own run the plain kernel.
+    `AttentionPieces` do not).  Values of a width of their own run on the matrix cores where
+    `mfma_attention_supported` says so (and their pages are transposed), else the plain kernel.
+
+    `gate` ([T, q_heads] in q's dtype, rows may be strided): head h's result for token t is multiplied by
+    `logistic(gate[t, h])` (both kernels; uncombined `AttentionPieces` are not made with it).  `out`
+    ([T, q_heads*value width] in q's dtype, rows may be strided): where the result is written.
 
     `sinks` (float32 [q_heads], optional): a sink logit per query head instead of one for all
     (both kernels).  `softcap`: every scaled score becomes `softcap * tanh(score / softcap)` before
@@ -958,14 +996,24 @@ def paged_attention(
         if sink_logit is not None:
             raise KernelShapeError("a sink logit for all heads or one per head, not both")
     has_sink = sink_logit is not None or sinks is not None
-    if v_pages is None or (v_head_dim is not None and v_head_dim != head_dim) or (
-        (has_sink or chunk is not None or softcap is not None) and not v_transposed
-    ):
+    v_dim = head_dim if v_head_dim is None else int(v_head_dim)
+    tokens = q.shape[0]
+    if gate is not None:
+        _need_cuda(gate)
+        if gate.dim() != 2 or tuple(gate.shape) != (tokens, q_heads) or gate.dtype != q.dtype or (q_heads > 1 and gate.stride(1) != 1):
+            raise KernelShapeError(f"the gate is {q.dtype} [{tokens}, {q_heads}] with unit inner stride, got {gate.dtype} {tuple(gate.shape)}")
+    if out is None:
+        out = torch.empty((tokens, q_heads * v_dim), dtype=q.dtype, device=q.device)
+    elif out.dim() != 2 or tuple(out.shape) != (tokens, q_heads * v_dim) or out.dtype != q.dtype or out.stride(1) != 1 or not out.is_cuda:
+        raise KernelShapeError(f"the result is {q.dtype} [{tokens}, {q_heads * v_dim}] with unit inner stride, got {out.dtype} {tuple(out.shape)}")
+    if v_pages is None or (not v_transposed and (
+        v_dim != head_dim or has_sink or chunk is not None or softcap is not None or gate is not None
+    )):
         return _paged_attention_general(
             q, k_pages, v_pages, block_table, token_request, positions, q_heads=q_heads, kv_heads=kv_heads,
-            head_dim=head_dim, v_head_dim=head_dim if v_head_dim is None else int(v_head_dim), scale=scale,
+            head_dim=head_dim, v_head_dim=v_dim, scale=scale,
             window=window, max_seq_len=max_seq_len, v_transposed=v_transposed, slopes=slopes, sink_logit=sink_logit,
-            chunk=chunk, sinks=sinks, softcap=softcap,
+            chunk=chunk, sinks=sinks, softcap=softcap, gate=gate, out=out,
         )
     _need_cuda(q, k_pages, v_pages, block_table, token_request, positions, cu_seqlens_q)
     for name, t in (("k_pages", k_pages), ("v_pages", v_pages), ("block_table", block_table),
@@ -983,8 +1031,7 @@ def paged_attention(
         raise KernelShapeError(
             f"pages must be [num_pages, {kv_heads}, page_size, {head_dim}], got {tuple(k_pages.shape)}"
         )
-    _check_v_pages(k_pages, v_pages, v_transposed)
-    tokens = q.shape[0]
+    _check_v_pages(k_pages, v_pages, v_transposed, v_dim)
     if token_request.numel() != tokens or positions.numel() != tokens:
         raise KernelShapeError("token_request and positions need one entry per token")
     if block_table.dim() != 2:
@@ -997,15 +1044,14 @@ def paged_attention(
     if host_cu_seqlens_q is not None and host_cu_seqlens_q[-1] != tokens:
         raise KernelShapeError(f"cu_seqlens_q ends at {host_cu_seqlens_q[-1]}, but there are {tokens} tokens")
     num_pages, page_size = k_pages.shape[0], k_pages.shape[2]
-    out = torch.empty((tokens, q_heads * head_dim), dtype=q.dtype, device=q.device)
     lib = library.load()
     group = q_heads // kv_heads
 
     use_mfma = v_transposed and not force_plain
-    if v_transposed and not mfma_attention_supported(q.dtype, head_dim, page_size):
+    if v_transposed and not mfma_attention_supported(q.dtype, head_dim, page_size, v_dim):
         raise KernelShapeError(
             f"transposed value pages need the matrix-core kernel, which does not take "
-            f"{q.dtype}, head_dim={head_dim}, page_size={page_size}"
+            f"{q.dtype}, head_dim={head_dim}, v_head_dim={v_dim}, page_size={page_size}"
         )
     if v_transposed and force_plain:
         raise KernelShapeError("the plain attention kernel reads value pages that are not transposed")
@@ -1019,9 +1065,15 @@ def paged_attention(
         if splits == 1:
             return None, None
         return (
-            torch.empty((rows * q_heads * splits, head_dim), dtype=torch.float32, device=q.device),
+            torch.empty((rows * q_heads * splits, v_dim), dtype=torch.float32, device=q.device),
             torch.empty((rows * q_heads * splits, 2), dtype=torch.float32, device=q.device),
         )
+
+    gate_args = (v_dim, _ptr(gate), 0 if gate is None else gate.stride(0))
+
+    def seen(tokens_per_tile: int) -> int:
+        """The most keys the tokens of one tile see (a chunked mask hides all but a chunk's)."""
+        return max_seq_len if chunk is None else min(max_seq_len, chunk + tokens_per_tile - 1)
 
     if use_mfma and host_cu_seqlens_q is None:
         # boundaries on the device only: one launch in the prefill shape, every wave finding its
@@ -1031,7 +1083,7 @@ def paged_attention(
         tokens_per_tile = lib.mi_attn_mfma_tokens_per_tile(q_heads, kv_heads, shape)
         num_tiles = tokens // tokens_per_tile + num_requests
         head_blocks = -(-group // min(group, 128))
-        splits = min(16, attention_splits(num_tiles * kv_heads * head_blocks, max_seq_len, target=512, min_keys=128))
+        splits = min(16, attention_splits(num_tiles * kv_heads * head_blocks, seen(tokens_per_tile), target=512, min_keys=128))
         part_acc, part_ml = partials(splits)
         library.check(
             lib.mi_attn_mfma(
@@ -1039,7 +1091,7 @@ def paged_attention(
                 _ptr(cu_seqlens_q), _ptr(positions), num_requests, tokens, num_tiles, _ptr(out), out.stride(0),
                 _ptr(part_acc), _ptr(part_ml), q_heads, kv_heads, head_dim, page_size, num_pages, float(scale),
                 int(window or 0), splits, shape, 0, 0, 1, int(has_sink), float(sink_logit or 0.0),
-                int(chunk or 0), _ptr(sinks), _ptr(slopes), float(softcap or 0.0), _stream(),
+                int(chunk or 0), _ptr(sinks), _ptr(slopes), float(softcap or 0.0), *gate_args, _stream(),
             )
         )
         return out
@@ -1071,8 +1123,9 @@ def paged_attention(
             target = 512 if shape == ATTN_SHAPE_PREFILL else 256
             # few requests with long contexts are cut finer (measured at batch 1: 128k keys
             # run 19 % faster in 32 ranges than in 16, 3k keys 4 % slower)
-            most = 16 if max_seq_len < 8192 else 32
-            splits = min(most, attention_splits(num_tiles * kv_heads * head_blocks, max_seq_len, target=target, min_keys=128))
+            keys = seen(tokens_per_tile)
+            most = 16 if keys < 8192 else 32
+            splits = min(most, attention_splits(num_tiles * kv_heads * head_blocks, keys, target=target, min_keys=128))
             part_acc, part_ml = partials(splits, first_token + run_tokens)
             library.check(
                 lib.mi_attn_mfma(
@@ -1083,7 +1136,7 @@ def paged_attention(
                     head_dim, page_size, num_pages, float(scale), int(window or 0), splits,
                     shape, int(one_tile_per_request), first_token,
                     0 if (leave_pieces and splits > 1) else 1, int(has_sink), float(sink_logit or 0.0),
-                    int(chunk or 0), _ptr(sinks), _ptr(slopes), float(softcap or 0.0), _stream(),
+                    int(chunk or 0), _ptr(sinks), _ptr(slopes), float(softcap or 0.0), *gate_args, _stream(),
                 )
             )
             if leave_pieces and splits > 1:
@@ -1101,7 +1154,7 @@ def paged_attention(
             run(0, leading_single)
             run(leading_single, num_requests)
         else:
-            pieces = run(0, num_requests, leave_pieces=not combine and not has_sink and chunk is None
+            pieces = run(0, num_requests, leave_pieces=not combine and not has_sink and chunk is None and gate is None and v_dim == head_dim
                          and leading_single == num_requests)
             if pieces is not None:
                 return pieces
@@ -1130,7 +1183,7 @@ def _paged_attention_general(
     token_request: torch.Tensor, positions: torch.Tensor, *, q_heads: int, kv_heads: int, head_dim: int,
     v_head_dim: int, scale: float, window: int | None, max_seq_len: int, v_transposed: bool,
     slopes: torch.Tensor | None, sink_logit: float | None, chunk: int | None = None,
-    sinks: torch.Tensor | None = None, softcap: float | None = None,
+    sinks: torch.Tensor | None = None, softcap: float | None = None, gate: torch.Tensor | None = None, out: torch.Tensor,
 ) -> torch.Tensor:
     """The plain attention kernel with everything it can be told: see `paged_attention`."""
     _need_cuda(q, k_pages, v_pages, block_table, token_request, positions, slopes, sinks)
@@ -1170,7 +1223,6 @@ def _paged_attention_general(
         raise KernelShapeError("token_request and positions need one entry per token, block_table is [requests, max_blocks]")
     if slopes is not None and (slopes.dtype != torch.float32 or slopes.numel() != q_heads):
         raise KernelShapeError(f"slopes must be float32 [{q_heads}], got {slopes.dtype} x {slopes.numel()}")
-    out = torch.empty((tokens, q_heads * v_head_dim), dtype=q.dtype, device=q.device)
     group = q_heads // kv_heads
     # (no row sees more keys than a chunk holds)
     splits = attention_splits(tokens * kv_heads * math.ceil(group / 4), min(max_seq_len, chunk) if chunk else max_seq_len)
@@ -1184,7 +1236,7 @@ def _paged_attention_general(
             _ptr(token_request), _ptr(positions), _ptr(out), out.stride(0), _ptr(part_acc), _ptr(part_ml), tokens,
             q_heads, kv_heads, head_dim, v_head_dim, v_row_stride, page_size, num_pages, float(scale), int(window or 0),
             splits, _ptr(slopes), int(sink_logit is not None or sinks is not None), float(sink_logit or 0.0), int(chunk or 0),
-            float(softcap or 0.0), _ptr(sinks), _stream(),
+            float(softcap or 0.0), _ptr(sinks), _ptr(gate), 0 if gate is None else gate.stride(0), _stream(),
         )
     )
     return out
@@ -1569,13 +1621,14 @@ class StreamUpdate:
 
         x += scale * (a + b + bias) + shift
 
-    `a`, `b`: a layer's sublayer outputs [T, H] in the compute dtype (either may be None);
+    `a`, `b`: a layer's sublayer outputs [T, H] in the compute dtype (either may be None; `b` may be
+    `WeightedRows`);
     `bias`, `shift`: float32 [H] or None.  A norm that knows it makes the update and its own
     statistics in one launch (`stream_update_norm`); anything else calls `finish()`, which
     returns the whole right-hand side as one float32 tensor to add."""
 
     a: torch.Tensor | None
-    b: torch.Tensor | None = None
+    b: "torch.Tensor | WeightedRows | None" = None
     bias: torch.Tensor | None = None
     shift: torch.Tensor | None = None
     scale: float = 1.0
@@ -1589,6 +1642,7 @@ class StreamUpdate:
         total = None
         for part in (self.a, self.b, self.bias):
             if part is not None:
+                part = part.finish() if isinstance(part, WeightedRows) else part
                 total = part.float() if total is None else total + part.float()
         if total is not None:
             total = total * self.scale
@@ -1607,7 +1661,14 @@ def stream_update_norm(
     new rows times `weight` (compute dtype) -> [T, H] or [len(rows), H]; `weight=None`: the
     update alone."""
     update = update if update is not None else StreamUpdate(None)
-    _need_cuda(update.a, update.b, update.bias, update.shift, residual, weight, rows)
+    b, b_weights, pieces = update.b, None, 1
+    if isinstance(b, WeightedRows):
+        b, b_weights, pieces = b.rows, b.weights, b.weights.shape[1]
+        _need_contiguous("b's weights", b_weights)
+        _need_f32("b's weights", b_weights)
+        if b_weights.shape[0] != residual.shape[0]:
+            raise KernelShapeError(f"stream update: weights of {b_weights.shape[0]} tokens for {residual.shape[0]} rows")
+    _need_cuda(update.a, b, b_weights, update.bias, update.shift, residual, weight, rows)
     for name, t in (("residual", residual), ("weight", weight), ("rows", rows), ("bias", update.bias), ("shift", update.shift)):
         _need_contiguous(name, t)
     _need_int32("rows", rows)
@@ -1616,8 +1677,8 @@ def stream_update_norm(
     _need_f32("shift", update.shift)
     tokens, hidden = residual.shape
     dtype = weight.dtype if weight is not None else (update.a.dtype if update.a is not None else torch.float32)
-    for name, t in (("a", update.a), ("b", update.b)):
-        if t is not None and (t.dim() != 2 or tuple(t.shape) != (tokens, hidden) or t.stride(1) != 1 or t.dtype != dtype):
+    for name, t, count in (("a", update.a, tokens), ("b", b, tokens * pieces)):
+        if t is not None and (t.dim() != 2 or tuple(t.shape) != (count, hidden) or t.stride(1) != 1 or t.dtype != dtype):
             raise KernelShapeError(f"stream update: {name} {tuple(t.shape)} {t.dtype} does not fit the stream {(tokens, hidden)} in {dtype}")
     for name, t in (("bias", update.bias), ("shift", update.shift), ("weight", weight)):
         if t is not None and t.numel() != hidden:
@@ -1629,17 +1690,19 @@ def stream_update_norm(
     code = F32 if dtype == torch.float32 else BF16
     library.check(
         library.load().mi_stream_update_norm(
-            code, _ptr(update.a), 0 if update.a is None else update.a.stride(0), _ptr(update.b),
-            0 if update.b is None else update.b.stride(0), _ptr(update.bias), _ptr(update.shift), float(update.scale),
+            code, _ptr(update.a), 0 if update.a is None else update.a.stride(0), _ptr(b),
+            0 if b is None else b.stride(0), _ptr(b_weights), pieces, _ptr(update.bias), _ptr(update.shift), float(update.scale),
             _ptr(residual), _ptr(weight), _ptr(out), _ptr(rows), n_out, hidden, float(eps), _stream(),
         )
     )
     return out
 
 
-def clamped_glu(gate_up: torch.Tensor, bias: torch.Tensor | None, limit: float, slope: float) -> torch.Tensor:
+def clamped_glu(
+    gate_up: torch.Tensor, bias: torch.Tensor | None, limit: float, slope: float, out: torch.Tensor | None = None,
+) -> torch.Tensor:
     """Rows [gate | up] (+ `bias`, float32 [2I]) -> `g * logistic(slope * g) * (u + 1)` with
-    g = min(gate, limit), u = clamp(up, -limit, limit); returns [T, I]."""
+    g = min(gate, limit), u = clamp(up, -limit, limit); returns [T, I] (`out`, whose rows may be strided, if given)."""
     _need_cuda(gate_up, bias)
     _need_contiguous("bias", bias)
     _need_f32("bias", bias)
@@ -1648,7 +1711,7 @@ def clamped_glu(gate_up: torch.Tensor, bias: torch.Tensor | None, limit: float, 
     tokens, inter = gate_up.shape[0], gate_up.shape[1] // 2
     if bias is not None and bias.numel() != 2 * inter:
         raise KernelShapeError(f"clamped_glu: the bias has {bias.numel()} entries for {2 * inter} columns")
-    out = torch.empty((tokens, inter), dtype=gate_up.dtype, device=gate_up.device)
+    out = _out_rows(out, tokens, inter, gate_up)
     library.check(
         library.load().mi_clamped_glu(
             _dtype_code(gate_up), _ptr(gate_up), gate_up.stride(0), _ptr(bias), _ptr(out), out.stride(0), tokens, inter,
@@ -1658,14 +1721,14 @@ def clamped_glu(gate_up: torch.Tensor, bias: torch.Tensor | None, limit: float, 
     return out
 
 
-def linear_clamped_glu(x: torch.Tensor, gate_up_weight: torch.Tensor, bias: torch.Tensor, limit: float, slope: float) -> torch.Tensor:
+def linear_clamped_glu(x: torch.Tensor, gate_up_weight: torch.Tensor, bias: torch.Tensor | None, limit: float, slope: float) -> torch.Tensor:
     """`clamped_glu(x @ [gate; up].T, bias, limit, slope)`.  bfloat16 with at most 32 rows runs as ONE
     kernel (the weight-streaming product with biases, clamps and activation in its last step);
     otherwise the product and `clamped_glu` run in turn.  Both round the two products to the element
     type first and then do the same float32 arithmetic, so the results agree bit for bit."""
     rows, width = gate_up_weight.shape
-    if rows % 2 or bias.numel() != rows:
-        raise KernelShapeError(f"linear_clamped_glu: stacked weight of {rows} rows, bias of {bias.numel()}")
+    if rows % 2 or (bias is not None and bias.numel() != rows):
+        raise KernelShapeError(f"linear_clamped_glu: stacked weight of {rows} rows, bias of {None if bias is None else bias.numel()}")
     if (
         x.dtype == torch.bfloat16
         and gate_up_weight.dtype == torch.bfloat16
@@ -1688,6 +1751,124 @@ def linear_clamped_glu(x: torch.Tensor, gate_up_weight: torch.Tensor, bias: torc
         )
         return out
     return clamped_glu(linear(x, gate_up_weight), bias, limit, slope)
+
+
+@dataclasses.dataclass(frozen=True)
+class LayerInputs:
+    """How the rows of a layer's stacked input projection lie, for a layer whose sublayers read one norm:
+    `[q | k | v | head gates | feed-forward gate | feed-forward up]`.  `kv_heads=0`: the layer reads another's keys
+    and values; `gate_rows=0`: no head gates (else at least `q_heads`, filled up with zero rows); `ff=0`: its
+    feed-forward is made elsewhere.  The feed-forward ends as `clamped_glu(limit, slope)` does, or, with
+    `limit=0`, as `silu(gate) * up`."""
+
+    q_heads: int
+    kv_heads: int
+    head_dim: int
+    v_head_dim: int
+    gate_rows: int = 0
+    ff: int = 0
+    limit: float = 0.0
+    slope: float = 1.0
+
+    @property
+    def qkv_rows(self) -> int:
+        return (self.q_heads + self.kv_heads) * self.head_dim + self.kv_heads * self.v_head_dim
+
+    @property
+    def rows(self) -> int:
+        return self.qkv_rows + self.gate_rows + 2 * self.ff
+
+
+def layer_in_rows_fit(layout: LayerInputs, rotary_dim: int, interleaved: bool) -> bool:
+    """Whether the one-kernel form takes a stacked projection of this layout (in steps of few bfloat16 rows)."""
+    return (
+        not interleaved
+        and rotary_dim % 8 == 0
+        and rotary_dim <= layout.head_dim
+        and layout.head_dim % 8 == 0
+        and layout.v_head_dim % 8 == 0
+        and layout.gate_rows % 8 == 0
+        and layout.ff % 4 == 0
+    )
+
+
+def layer_in_takes(x: "torch.Tensor | ScaledRows", weight: torch.Tensor, layout: LayerInputs, rotary_dim: int, interleaved: bool) -> bool:
+    """Whether `layer_in` runs these operands: at most 32 bfloat16 rows (16 as `ScaledRows`)."""
+    max_rows = SKINNY_WIDE_MAX_ROWS
+    if isinstance(x, ScaledRows):
+        if not _scaled_rows_fit(x):
+            return False
+        x, max_rows = x.values, SKINNY_MAX_ROWS
+    return (
+        x.dtype == torch.bfloat16
+        and weight.dtype == torch.bfloat16
+        and x.dim() == 2
+        and x.stride(1) == 1
+        and weight.stride(1) == 1
+        and skinny_gemm_takes(x.shape[0], x.shape[1], x.stride(0), weight.stride(0), max_rows)
+        and layer_in_rows_fit(layout, rotary_dim, interleaved)
+    )
+
+
+def layer_in(
+    x: "torch.Tensor | ScaledRows", weight: torch.Tensor, layout: LayerInputs, cos: torch.Tensor | None, sin: torch.Tensor | None,
+    rotary_dim: int, slot_mapping: torch.Tensor | None, k_pages: torch.Tensor | None, v_pages: torch.Tensor | None, *,
+    v_transposed: bool = False, bias: torch.Tensor | None = None, activated: torch.Tensor | None = None,
+) -> "tuple[torch.Tensor, torch.Tensor | None]":
+    """The stacked input projection of a layer whose sublayers read one norm, with everything that follows it row by
+    row, as ONE kernel for few rows: biases, the rotation of the first `rotary_dim` dims of queries and keys
+    (halves paired), the cache write, and the feed-forward's activation (into `activated` [M, ff], rows may be
+    strided).  Returns the rotated queries [M, q_heads*head_dim] and the head gates [M, q_heads] (not
+    activated; None without gate rows).  The values are those of `linear`, `rope_kv_write(bias=)` and
+    `clamped_glu` / `gated_mul("silu")` in turn (all round the product to bfloat16 first).  `x` may be `ScaledRows`."""
+    scaled = x if isinstance(x, ScaledRows) else None
+    if scaled is not None:
+        x = scaled.values
+        _need_cuda(scaled.sumsq)
+    if not layer_in_takes(scaled if scaled is not None else x, weight, layout, rotary_dim, False):
+        raise KernelShapeError(f"layer_in: x {tuple(x.shape)} {x.dtype} with {layout}, rotary_dim={rotary_dim} is not taken")
+    _need_cuda(x, weight, cos, sin, slot_mapping, k_pages, v_pages, bias, activated)
+    for name, t in (("cos", cos), ("sin", sin), ("slot_mapping", slot_mapping), ("k_pages", k_pages), ("v_pages", v_pages), ("bias", bias)):
+        _need_contiguous(name, t)
+    _need_int32("slot_mapping", slot_mapping)
+    _need_f32("bias", bias)
+    m, k = x.shape
+    if weight.dim() != 2 or weight.shape[0] < layout.rows or weight.shape[1] != k:
+        raise KernelShapeError(f"layer_in: weight {tuple(weight.shape)} does not hold {layout.rows} rows of {k}")
+    if bias is not None and bias.numel() != layout.qkv_rows:
+        raise KernelShapeError(f"layer_in: {layout.qkv_rows} biases of q, k and v, got {bias.numel()}")
+    for t in (cos, sin):
+        if rotary_dim > 0 and (t is None or tuple(t.shape) != (m, rotary_dim // 2) or t.dtype != torch.float32):
+            raise KernelShapeError(f"layer_in: cos/sin are float32 [{m}, {rotary_dim // 2}]")
+    page_size = num_pages = 0
+    if layout.kv_heads > 0:
+        if slot_mapping is None or k_pages is None or v_pages is None or slot_mapping.numel() != m:
+            raise KernelShapeError("layer_in: writing keys and values needs a slot a row, k_pages and v_pages")
+        if k_pages.dtype != torch.bfloat16 or v_pages.dtype != torch.bfloat16:
+            raise KernelShapeError("layer_in writes bfloat16 pages")
+        if k_pages.dim() != 4 or k_pages.shape[1] != layout.kv_heads or k_pages.shape[3] != layout.head_dim:
+            raise KernelShapeError(f"layer_in: k_pages {tuple(k_pages.shape)} do not hold {layout.kv_heads} heads of {layout.head_dim}")
+        _check_v_pages(k_pages, v_pages, v_transposed, layout.v_head_dim)
+        num_pages, page_size = k_pages.shape[0], k_pages.shape[2]
+    if layout.ff > 0:
+        if activated is None or tuple(activated.shape) != (m, layout.ff) or activated.dtype != torch.bfloat16 or activated.stride(1) != 1 \
+                or activated.stride(0) % 4 != 0 or activated.data_ptr() % 8 != 0:
+            raise KernelShapeError(f"layer_in: the activation goes to bfloat16 [{m}, {layout.ff}] rows on 8-byte boundaries")
+    q_out = torch.empty((m, layout.q_heads * layout.head_dim), dtype=torch.bfloat16, device=x.device)
+    gates = torch.empty((m, layout.q_heads), dtype=torch.bfloat16, device=x.device) if layout.gate_rows > 0 else None
+    writes = layout.kv_heads > 0
+    library.check(
+        library.load().mi_gemm_skinny_layer_in_bf16(
+            _ptr(x), x.stride(0), None if scaled is None else _ptr(scaled.sumsq), 0 if scaled is None else scaled.sumsq.shape[0],
+            0.0 if scaled is None else scaled.eps, _ptr(weight), weight.stride(0), _ptr(q_out), q_out.stride(0),
+            _ptr(cos) if rotary_dim > 0 else None, _ptr(sin) if rotary_dim > 0 else None, _ptr(slot_mapping) if writes else None,
+            _ptr(k_pages) if writes else None, _ptr(v_pages) if writes else None, _ptr(bias), _ptr(gates),
+            0 if gates is None else gates.stride(0), _ptr(activated) if layout.ff > 0 else None,
+            activated.stride(0) if layout.ff > 0 else 0, m, k, layout.q_heads, layout.kv_heads, layout.head_dim, layout.v_head_dim,
+            rotary_dim // 2, layout.gate_rows, layout.ff, layout.limit, layout.slope, page_size, num_pages, int(v_transposed), _stream(),
+        )
+    )
+    return q_out, gates
 
 
 def linear_geglu(x: torch.Tensor, gate_up_weight: torch.Tensor) -> torch.Tensor:
@@ -2268,7 +2449,17 @@ def head_norm_rope_kv_write(
 GATE_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1, "logistic": 2}
 
 
-def gated_mul(a: torch.Tensor, b: torch.Tensor, activation: str) -> torch.Tensor:
+def _out_rows(out: torch.Tensor | None, tokens: int, width: int, like: torch.Tensor) -> torch.Tensor:
+    """`out` if it is [tokens, width] rows (which may be strided) like `like`'s, or new ones."""
+    if out is None:
+        return torch.empty((tokens, width), dtype=like.dtype, device=like.device)
+    _need_cuda(out)
+    if out.dim() != 2 or tuple(out.shape) != (tokens, width) or out.dtype != like.dtype or out.stride(1) != 1:
+        raise KernelShapeError(f"results go to {like.dtype} [{tokens}, {width}] with unit inner stride, got {out.dtype} {tuple(out.shape)}")
+    return out
+
+
+def gated_mul(a: torch.Tensor, b: torch.Tensor, activation: str, out: torch.Tensor | None = None) -> torch.Tensor:
     """`act(a) * b` elementwise for [T, W] column ranges of rows (rows may be strided):
     `silu`, `gelu_tanh` (0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3)))) or `logistic`."""
     if activation not in GATE_ACTIVATIONS:
@@ -2277,7 +2468,7 @@ def gated_mul(a: torch.Tensor, b: torch.Tensor, activation: str) -> torch.Tensor
     if a.dim() != 2 or a.shape != b.shape or a.stride(1) != 1 or b.stride(1) != 1 or a.dtype != b.dtype:
         raise KernelShapeError(f"gated_mul: two [T, W] ranges of one dtype with unit inner stride, got {tuple(a.shape)} {tuple(b.shape)}")
     tokens, width = a.shape
-    out = torch.empty((tokens, width), dtype=a.dtype, device=a.device)
+    out = _out_rows(out, tokens, width, a)
     library.check(
         library.load().mi_gated_mul(
             _dtype_code(a), GATE_ACTIVATIONS[activation], _ptr(a), a.stride(0), _ptr(b), b.stride(0), _ptr(out), out.stride(0),
@@ -2456,7 +2647,7 @@ def qkv_norm_write(
 # ----------------------------------------------------------------------------
 
 ROUTER_MAX_OUTPUTS = 1024
-ROUTER_SCORES = ("softmax", "logistic")
+ROUTER_SCORES = ("softmax", "logistic", "chosen_softmax")
 # an expert's activation -> (mode of its first product's kernel, weight rows a feature of that product has)
 EXPERT_ACTIVATIONS = {"silu_gated": (1, 2), "squared_relu": (2, 1)}
 
@@ -2479,7 +2670,8 @@ def route_top_k(
     [outputs] or None; the lower index wins a tie) -> their indices int32 [T, top] and weights
     `score * route_scale` float32 [T, top] (not renormalized); with `gate_row` (float32 [W]) also
     `logistic(gate_row . x)` float32 [T].  `scores="logistic"`: every output's score is `logistic(z)` of its
-    own logit.
+    own logit.  `scores="chosen_softmax"`: `correction` is a bias of the logits, the largest biased logits are
+    chosen, and the weights are `route_scale` times the softmax over the chosen logits alone.
 
     With `experts` (how many of the outputs are real experts) a fourth result is the list of (row, choice) pairs
     by expert that `experts_by_expert` works from: for few bfloat16 rows it is made in the same launch
@@ -2518,12 +2710,12 @@ def route_top_k(
             library.check(lib.mi_route_few(
                 _ptr(x), x.stride(0), _ptr(router), _ptr(correction), _ptr(gate_row), _ptr(logits), _ptr(chosen), _ptr(weights),
                 _ptr(gates), _ptr(lists.listed), _ptr(lists.first), tokens, width, outputs, experts, int(top), float(route_scale),
-                int(scores == "logistic"), _stream()))
+                ROUTER_SCORES.index(scores), _stream()))
             return chosen, weights, gates, lists
     library.check(
         library.load().mi_route_top_k(
             _dtype_code(x), _ptr(x), x.stride(0), _ptr(router), _ptr(correction), _ptr(gate_row), _ptr(chosen), _ptr(weights),
-            _ptr(gates), tokens, width, outputs, int(top), float(route_scale), int(scores == "logistic"), _stream(),
+            _ptr(gates), tokens, width, outputs, int(top), float(route_scale), ROUTER_SCORES.index(scores), _stream(),
         )
     )
     if lists is not None:
@@ -2555,8 +2747,8 @@ def _check_experts(x, gate_up, down, chosen, weights, shared, shared_gate, activ
     if chosen.dim() != 2 or chosen.shape[0] != tokens or tuple(weights.shape) != tuple(chosen.shape):
         raise KernelShapeError("routed experts: chosen and weights are [T, top]")
     if shared is not None and (shared.dim() != 2 or shared.stride(1) != 1 or tuple(shared.shape) != (tokens, width) or shared.dtype != x.dtype
-                               or shared_gate is None or shared_gate.numel() != tokens):
-        raise KernelShapeError("routed experts: a shared expert's rows are [T, W] and come with one gate a row")
+                               or (shared_gate is not None and shared_gate.numel() != tokens)):
+        raise KernelShapeError("routed experts: a shared expert's rows are [T, W], with one gate a row or none")
     return tokens, width, experts, ff, chosen.shape[1]
 
 
@@ -2564,6 +2756,21 @@ def _expert_weights(activation: str, weights: torch.Tensor, weight_on: str):
     """(mode of the first product, weights it applies to what an expert reads, weights of the final sum)."""
     mode = EXPERT_ACTIVATIONS[activation][0]
     return (mode, weights, None) if weight_on == "input" else (mode, None, weights)
+
+
+@dataclasses.dataclass
+class WeightedRows:
+    """A weighted sum that has not been made yet: row t of the result is the sum over p of `weights[t, p]` (float32
+    [T, pieces]) times row `t * pieces + p` of `rows` [T * pieces, W].  A norm that knows it adds the rows up on
+    its way (`stream_update_norm`); anything else calls `finish()`."""
+
+    rows: torch.Tensor
+    weights: torch.Tensor
+
+    def finish(self) -> torch.Tensor:
+        tokens, pieces = self.weights.shape
+        wide = self.rows.view(tokens, pieces, self.rows.shape[1]).float() * self.weights[:, :, None]
+        return wide.sum(dim=1).to(self.rows.dtype)
 
 
 @dataclasses.dataclass
@@ -2647,7 +2854,7 @@ def experts_by_expert(
     x: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, chosen: torch.Tensor, weights: torch.Tensor,
     shared: torch.Tensor | None = None, shared_gate: torch.Tensor | None = None, tiles: str | None = None, *,
     activation: str = "silu_gated", weight_on: str = "output", combine: bool = True, lists: ExpertLists | None = None,
-) -> "torch.Tensor | SummedRows":
+) -> "torch.Tensor | SummedRows | WeightedRows":
     """The same sum as `experts_few_rows`, expert by expert without the host knowing anything: one small
     kernel lists the (row, expert) pairs by expert, then every chosen expert's block streams its
     weights once for up to eight of the expert's rows at a time (the rows wait in LDS), and one kernel adds
@@ -2656,12 +2863,13 @@ def experts_by_expert(
     gets): "rows" is that form; for prompts (bfloat16) "direct", blocks of 64 features that take 64 of an
     expert's rows a pass, and "lds", tiles of 128 rows x 128 features with both operands staged through LDS
     (rows in steps of 64 elements).  `combine=False`
-    (weights on the input, no shared or identity experts): the rows are left for a norm to add up (`SummedRows`).
+    (no shared or identity experts): the rows are left for a norm to add up (`SummedRows`; weights on the
+    output: `WeightedRows`).
     `lists`: the pairs by expert where `route_top_k` has made them already."""
     tokens, width, experts, ff, top = _check_experts(x, gate_up, down, chosen, weights, shared, shared_gate, activation, weight_on)
     mode, on_input, on_output = _expert_weights(activation, weights, weight_on)
-    if not combine and (weight_on != "input" or shared is not None):
-        raise KernelShapeError("experts_by_expert: rows are left apart only where the final sum is a plain one")
+    if not combine and shared is not None:
+        raise KernelShapeError("experts_by_expert: rows are left apart only where nothing joins their sum")
     if not experts_by_expert_take(x, gate_up, activation):
         raise KernelShapeError(f"experts_by_expert: rows of {width} and {ff} are not read 16 bytes at a time, or do not fit")
     pairs = tokens * top
@@ -2691,7 +2899,7 @@ def experts_by_expert(
         library.check(lib.mi_expert_rows(code, 0, _ptr(act), ff, 1, _ptr(down), _ptr(listed), _ptr(first), None, _ptr(made),
                                          width, experts, ff, width, many, _stream()))
     if not combine:
-        return SummedRows(made, top)
+        return SummedRows(made, top) if on_output is None else WeightedRows(made, weights)
     out = torch.empty((tokens, width), dtype=x.dtype, device=x.device)
     library.check(lib.mi_expert_combine(
         code, _ptr(made), None, _ptr(chosen), _ptr(on_output), _ptr(x), x.stride(0), _ptr(shared),

@@ -14,26 +14,26 @@ from pathlib import Path
 from mini_infer_amd.exceptions import ExtensionMissingError, KernelShapeError
 from mini_infer_amd.ops import build as _build
 
-ABI_VERSION = 36
+ABI_VERSION = 37
 
 _lib: ctypes.CDLL | None = None
 _lib_path: Path | None = None
 
 _P = c_void_p
 _SIGNATURES: dict[str, list] = {
-    "mi_embed_gather": [c_int, _P, _P, _P, c_int, c_int, c_int, c_float, _P],
+    "mi_embed_gather": [c_int, _P, _P, _P, c_int, c_int, c_int, c_float, _P, _P, c_int, _P],
     "mi_take_device_tokens": [_P, _P, _P, c_int, c_int, c_int, _P],
     "mi_begin_step": [_P, _P, _P, c_int, c_int, c_int, _P, _P, _P, c_int, c_int, _P],
     "mi_add_rmsnorm": [c_int, _P, _P, _P, _P, _P, c_int, c_int, c_float, _P, c_int, c_int64, _P],
-    "mi_rope_table": [_P, _P, _P, _P, c_int, c_int, _P],
+    "mi_rope_table": [_P, _P, _P, _P, c_int, c_int, c_float, _P],
     "mi_rope_kv_write": [
         c_int, _P, c_int64, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
-        c_int, c_int, c_int, _P,
+        c_int, c_int, c_int, _P, _P,
     ],
     "mi_silu_mul": [c_int, _P, _P, c_int, c_int, _P],
     "mi_gemm_f32": [_P, c_int64, _P, c_int64, _P, c_int64, c_int, c_int, c_int, _P],
     "mi_gemm_skinny_bf16": [_P, c_int64, _P, c_int64, _P, c_int64, c_int, c_int, c_int, _P],
-    "mi_gemm_skinny_f32out_bf16": [_P, c_int64, _P, c_int64, _P, c_int64, c_int, c_int, c_int, _P],
+    "mi_gemm_skinny_f32out_bf16": [_P, c_int64, _P, c_int64, _P, c_int64, c_int, c_int, c_int, c_float, _P],
     "mi_gemm_mid_partial_bf16": [_P, c_int64, _P, c_int64, _P, c_int, c_int, c_int, _P],
     "mi_gemm_mid_bf16_ranges": [c_int, c_int],
     "mi_gemm_mid_bf16_supported": [c_int, c_int, c_int, c_int64, c_int64],
@@ -50,6 +50,10 @@ _SIGNATURES: dict[str, list] = {
         _P, c_int64, _P, c_int, c_float, _P, c_int64, _P, c_int64, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_int,
         c_int, c_int, c_int, c_int, _P,
     ],
+    "mi_gemm_skinny_layer_in_bf16": [
+        _P, c_int64, _P, c_int, c_float, _P, c_int64, _P, c_int64, _P, _P, _P, _P, _P, _P, _P, c_int64, _P, c_int64, c_int, c_int,
+        c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_int, c_int, c_int, _P,
+    ],
     "mi_gemm_skinny_bf16_supported": [c_int, c_int, c_int, c_int64, c_int64],
     "mi_gemm_skinny_wide_bf16_supported": [c_int, c_int, c_int, c_int64, c_int64],
     "mi_attn_generic": [
@@ -58,7 +62,8 @@ _SIGNATURES: dict[str, list] = {
     ],
     "mi_attn_mfma": [
         _P, c_int64, _P, _P, _P, c_int, _P, _P, c_int, c_int, c_int, _P, c_int64, _P, _P, c_int,
-        c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, _P, _P, c_float, _P,
+        c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, _P, _P, c_float, c_int, _P,
+        c_int64, _P,
     ],
     "mi_gemm_skinny_addnorm_pieces": [c_int],
     "mi_gemm_skinny_addnorm_bf16": [
@@ -67,6 +72,7 @@ _SIGNATURES: dict[str, list] = {
     "mi_gemm_skinny_swiglu_scaled_bf16": [_P, c_int64, _P, c_int, c_float, _P, c_int64, _P, c_int64, c_int, c_int, c_int, _P],
     "mi_attn_mfma_tokens_per_tile": [c_int, c_int, c_int],
     "mi_attn_mfma_supported": [c_int, c_int],
+    "mi_attn_mfma_values_supported": [c_int, c_int, c_int],
     "mi_sample": [c_int, _P, c_int64, c_int, c_int, _P, _P, _P, _P, _P, _P, _P, _P],
     "mi_sample_slots": [c_int, _P, c_int64, c_int, c_int, _P, _P, c_int, _P, _P],
     "mi_embed_sinusoid": [c_int, _P, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_float, _P],
@@ -81,9 +87,9 @@ _SIGNATURES: dict[str, list] = {
     "mi_gated_table_rows": [c_int, _P, c_int64, _P, c_int64, _P, _P, c_int, c_int, c_int, c_int, _P],
     "mi_attn_general": [
         c_int, _P, c_int64, _P, _P, _P, c_int, _P, _P, _P, c_int64, _P, _P, c_int, c_int, c_int, c_int, c_int,
-        c_int64, c_int, c_int, c_float, c_int, c_int, _P, c_int, c_float, c_int, c_float, _P, _P,
+        c_int64, c_int, c_int, c_float, c_int, c_int, _P, c_int, c_float, c_int, c_float, _P, _P, c_int64, _P,
     ],
-    "mi_stream_update_norm": [c_int, _P, c_int64, _P, c_int64, _P, _P, c_float, _P, _P, _P, _P, c_int, c_int, c_float, _P],
+    "mi_stream_update_norm": [c_int, _P, c_int64, _P, c_int64, _P, c_int, _P, _P, c_float, _P, _P, _P, _P, c_int, c_int, c_float, _P],
     "mi_clamped_glu": [c_int, _P, c_int64, _P, _P, c_int64, c_int, c_int, c_float, c_float, _P],
     "mi_short_conv": [
         c_int, _P, c_int64, _P, _P, c_int64, _P, _P, _P, _P, c_int64, c_int, c_int, c_int, c_int, c_int, _P, c_int, _P,

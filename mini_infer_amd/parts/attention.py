@@ -8,7 +8,8 @@ q and k fused with the write of k and v into cache pages
 projection.  A window, if given, limits each query to the last `window` keys; a chunk to
 the keys of its own stretch of `chunk` positions.  Queries and keys may be normed head by
 head before the rotation, and the attended rows may be gated by a projection of the
-layer's input before the output projection.
+layer's input before the output projection.  The projections of q, k and v may have biases, and a
+layer may have none of keys and values at all (it then attends to another layer's).
 """
 
 from __future__ import annotations
@@ -56,6 +57,9 @@ class GQAttention(Mixer):
         chunk: int | None = None,
         head_norm: dict | None = None,
         gate: dict | None = None,
+        bias_suffix: str | None = None,
+        own_keys: bool = True,
+        cache_chunk: int | None = None,
     ) -> None:
         """`v_head_dim`: value heads of another width than the query and key heads (`head_dim`).
         `sink_logit`: the softmax's denominator gets one more term exp(sink_logit), a sink that
@@ -67,7 +71,13 @@ class GQAttention(Mixer):
         entries that the heads share, before the rotation.
         `gate` = {"name": n, "activation": "logistic"}: one more projection of the layer's input, as wide as
         the concatenated value heads; the attended rows are multiplied by its activation, element
-        by element, before the output projection."""
+        by element, before the output projection.  With `"per_head": True` the projection has one number per
+        query head instead, by whose logistic the head's whole result is multiplied.
+        `bias_suffix`: q, k and v have biases, float32 tensors of the projections' names with this added.
+        `own_keys=False`: the layer has no tensors of keys and values; a call of it reads another call's cache
+        (rotated keys and values as they lie there), whose head counts, widths and rotation are its own.
+        `cache_chunk`: every reader of the cache sees only keys of its own stretch of this many positions, so
+        earlier stretches are given back."""
         super().__init__(dtype, device)
         if num_heads % num_kv_heads != 0:
             raise ValueError(f"num_heads={num_heads} is not a multiple of num_kv_heads={num_kv_heads}")
@@ -80,9 +90,18 @@ class GQAttention(Mixer):
         self.head_norm_names = None if head_norm is None else tuple(head_norm.get("names", ("q_norm", "k_norm")))
         self.gate_name = None if gate is None else str(gate["name"])
         self.gate_activation = None if gate is None else str(gate.get("activation", "logistic"))
+        self.head_gate = gate is not None and bool(gate.get("per_head", False))
+        if self.head_gate and self.gate_activation != "logistic":
+            raise NotImplementedError(f"attention: a gate of one number per head is a logistic one, got {self.gate_activation!r}")
+        self.bias_suffix, self.own_keys, self.cache_chunk = bias_suffix, bool(own_keys), cache_chunk
+        self.bias: torch.Tensor | None = None  # float32 [q | k | v] ([q] without own keys)
         # the few-row kernels that fold projection, rotation and cache write (and the output
-        # projection's hand-over) know neither head norms nor gates
-        self._plain_heads = head_norm is None and gate is None
+        # projection's hand-over) know neither head norms nor gates nor biases
+        self._plain_heads = head_norm is None and gate is None and bias_suffix is None and self.own_keys
+        if not self._plain_heads and head_norm is not None and (bias_suffix is not None or not self.own_keys):
+            raise NotImplementedError("attention: head norms beside biases, or without keys of its own; not built")
+        if not self.own_keys and gate is not None and not self.head_gate:
+            raise NotImplementedError("attention: a gate as wide as the attended rows without keys of its own; not built")
         self.q_norm_weight: torch.Tensor | None = None
         self.k_norm_weight: torch.Tensor | None = None
         if head_dim <= 0 or head_dim % ops.ATTENTION_HEAD_DIM_STEP != 0 or head_dim > ops.ATTENTION_MAX_HEAD_DIM:
@@ -114,24 +133,36 @@ class GQAttention(Mixer):
         self.out = Linear(num_heads * self.v_head_dim, hidden_size, names[3], dtype, device, suffix=suffix)
 
     def _input_projection(self, hidden_size: int, q_width: int, kv_width: int, names, suffix: str) -> Linear:
-        """The stacked product that feeds the attention: q | k | v here."""
+        """The stacked product that feeds the attention: q | k | v here (q alone without keys of its own)."""
         v_width = self.num_kv_heads * self.v_head_dim
-        widths, parts = [q_width, kv_width, v_width], list(names[:3])
+        self._bias_names = [names[0] + suffix]
+        widths, parts = [q_width], [names[0]]
+        if self.own_keys:
+            self._bias_names += [names[1] + suffix, names[2] + suffix]
+            widths, parts = widths + [kv_width, v_width], parts + list(names[1:3])
+        self.qkv_width = sum(widths)
         if self.gate_name is not None:  # q | k | v | gate
-            widths.append(self.num_heads * self.v_head_dim)
+            widths.append(self.num_heads if self.head_gate else self.num_heads * self.v_head_dim)
             parts.append(self.gate_name)
-        return Linear(hidden_size, widths, parts, self.dtype, self.device, suffix=suffix)
+        self._bias_widths = widths[: len(self._bias_names)]
+        # (a gate of one number per head: filled up with zero rows, so that rows of the product stay aligned)
+        return Linear(hidden_size, widths, parts, self.dtype, self.device, suffix=suffix, row_step=8 if self.head_gate else 1)
 
     def param_specs(self, prefix: str) -> dict[str, ParamSpec]:
         specs = {**self.qkv.param_specs(prefix), **self.out.param_specs(prefix)}
         if self.head_norm_names is not None:
             for name in self.head_norm_names:
                 specs[prefix + name] = ParamSpec((self.head_dim,), init="norm_weight", dtype="float32")
+        if self.bias_suffix is not None:
+            for name, width in zip(self._bias_names, self._bias_widths):
+                specs[prefix + name + self.bias_suffix] = ParamSpec((width,), dtype="float32")
         return specs
 
     def load_params(self, prefix: str, get: TensorGetter) -> None:
         self.qkv.load_params(prefix, get)
         self.out.load_params(prefix, get)
+        if self.bias_suffix is not None:
+            self.bias = torch.cat([get(prefix + name + self.bias_suffix).float() for name in self._bias_names]).contiguous()
         if self.head_norm_names is not None:
             self.q_norm_weight = get(prefix + self.head_norm_names[0]).float().contiguous()
             self.k_norm_weight = get(prefix + self.head_norm_names[1]).float().contiguous()
@@ -152,14 +183,80 @@ class GQAttention(Mixer):
     def cache_needs(self, page_size: int) -> CacheNeeds:
         # values lie transposed inside a page where the matrix-core kernel will read them
         # (that kernel knows no score bias: such layers keep the plain layout and kernel)
-        transposed = (
-            self.slopes is None and self._same_widths
-            and ops.mfma_attention_supported(self.dtype, self.head_dim, page_size)
-        )
         v_head_dim = None if self.v_head_dim == self.head_dim else self.v_head_dim
-        return CacheNeeds(
-            pages=PagedKVNeeds(self.num_kv_heads, self.head_dim, self.window, v_head_dim=v_head_dim, v_transposed=transposed)
+        transposed = (
+            self.slopes is None and (self._same_widths or self._rows_stay_aligned)
+            and ops.mfma_attention_supported(self.dtype, self.head_dim, page_size, v_head_dim)
         )
+        return CacheNeeds(
+            pages=PagedKVNeeds(self.num_kv_heads, self.head_dim, self.window, v_head_dim=v_head_dim, v_transposed=transposed,
+                               chunk=self.cache_chunk)
+        )
+
+    @property
+    def _rows_stay_aligned(self) -> bool:
+        """Whether queries lie in rows of the stacked product on the boundaries the matrix-core kernel reads from."""
+        return self.qkv.padded_features % 8 == 0
+
+    # -- a layer whose sublayers' products are made together (`parts.joint`) ------------------
+
+    @property
+    def can_join(self) -> bool:  # type: ignore[override]
+        return self.head_norm_eps is None and (self.gate_name is None or self.head_gate)
+
+    @property
+    def joint_input(self) -> Linear:
+        return self.qkv
+
+    @property
+    def joint_output(self) -> Linear:
+        return self.out
+
+    def joint_layout(self, ff: int, limit: float, slope: float) -> ops.LayerInputs:
+        """How the stacked input rows lie when a feed-forward's follow the attention's."""
+        return ops.LayerInputs(
+            self.num_heads, self.num_kv_heads if self.own_keys else 0, self.head_dim, self.v_head_dim,
+            self.qkv.padded_features - self.qkv_width if self.head_gate else 0, ff, limit, slope)
+
+    def rotation(self) -> tuple[int, bool] | None:
+        """`(rotary_dim, interleaved)` known before a step ((0, False) without positions), or None."""
+        return (0, False) if self.position is None else self.position.rotary_layout()
+
+    def _tables(self, ctx: StepContext, like: torch.Tensor):
+        """cos, sin, rotated dims and pairing of a step."""
+        rotary = self.position.rotary(ctx) if self.position is not None else None
+        if rotary is not None:
+            return rotary.cos, rotary.sin, rotary.rotary_dim, rotary.interleaved
+        empty = torch.empty((ctx.num_tokens, 0), dtype=torch.float32, device=like.device)
+        return empty, empty, 0, False
+
+    def forward_projected(self, columns: torch.Tensor, ctx: StepContext, cache: LayerCache, writes_cache: bool, out: torch.Tensor | None = None):
+        """What stands between the two products: `columns` are rows of the stacked input product (rotated in
+        place; rows may be strided); the attended (and gated) rows go to `out` if it is given."""
+        if writes_cache != self.own_keys:
+            raise ValueError("attention without keys of its own reads another call's, and only that")
+        cos, sin, rotary_dim, interleaved = self._tables(ctx, columns)
+        ops.rope_kv_write(
+            columns, cos, sin, ctx.slot_mapping[cache.group] if writes_cache else None, cache.k_pages, cache.v_pages,
+            q_heads=self.num_heads, kv_heads=self.num_kv_heads if writes_cache else 0, head_dim=self.head_dim,
+            rotary_dim=rotary_dim, interleaved=interleaved, v_transposed=cache.v_transposed, v_head_dim=self.v_head_dim,
+            bias=self.bias,
+        )
+        gate = columns[:, self.qkv_width:self.qkv_width + self.num_heads] if self.head_gate else None
+        return self._attend(columns, ctx, cache, gate, out)
+
+    def forward_layer_in(self, x, weight: torch.Tensor, layout: ops.LayerInputs, ctx: StepContext, cache: LayerCache, writes_cache: bool,
+                         activated: torch.Tensor | None, out: torch.Tensor):
+        """The same for few rows, the stacked product of the whole layer included: `ops.layer_in`, then the attention."""
+        if writes_cache != self.own_keys:
+            raise ValueError("attention without keys of its own reads another call's, and only that")
+        rows = x.values if isinstance(x, ops.ScaledRows) else x
+        cos, sin, rotary_dim, _ = self._tables(ctx, rows)
+        queries, gates = ops.layer_in(
+            x, weight, layout, cos, sin, rotary_dim, ctx.slot_mapping[cache.group] if writes_cache else None, cache.k_pages,
+            cache.v_pages, v_transposed=cache.v_transposed, bias=self.bias, activated=activated,
+        )
+        return self._attend(queries, ctx, cache, gates, out)
 
     def forward(
         self, x: torch.Tensor, ctx: StepContext, cache: LayerCache, writes_cache: bool = True
@@ -167,6 +264,9 @@ class GQAttention(Mixer):
         assert cache.group is not None and cache.k_pages is not None and cache.v_pages is not None
         q_width = self.num_heads * self.head_dim
         assert self.qkv.weight is not None
+        if self.bias_suffix is not None or self.head_gate or not self.own_keys:
+            x = x.finish() if isinstance(x, ops.ScaledRows) else x
+            return self._project(self.forward_projected(self.qkv.forward(x), ctx, cache, writes_cache))
         rotary = self.position.rotary(ctx) if self.position is not None else None
         if isinstance(x, ops.ScaledRows) and not (
             rotary is not None
@@ -237,13 +337,15 @@ class GQAttention(Mixer):
             return ops.linear_from_attention(attended, self.out.weight)
         return self.out.forward(attended, partial_ok=self.emit_partial_sums)
 
-    def _attend(self, queries: torch.Tensor, ctx: StepContext, cache: LayerCache):
-        """Attention of the rotated queries (the first columns of `queries`) over the cache pages.
+    def _attend(self, queries: torch.Tensor, ctx: StepContext, cache: LayerCache, gate: torch.Tensor | None = None,
+                out: torch.Tensor | None = None):
+        """Attention of the rotated queries (the first columns of `queries`) over the cache pages, times the
+        logistic of `gate` ([T, heads]) if there is one, into `out` if it is given.
         At the smallest batches the key ranges may come back uncombined, for the output
         projection to combine on its way (one launch less a layer)."""
         few = (
             queries.dtype == torch.bfloat16 and self._same_widths and self.sink_logit is None
-            and self._plain_heads and self.chunk is None
+            and self._plain_heads and self.chunk is None and out is None
             and ops.attention_pieces_pay(ctx.num_tokens, self.num_heads, self.head_dim)
         )
         return ops.paged_attention(
@@ -251,7 +353,7 @@ class GQAttention(Mixer):
             ctx.positions, ctx.cu_seqlens_q, ctx.host_cu_seqlens_q, q_heads=self.num_heads,
             kv_heads=self.num_kv_heads, head_dim=self.head_dim, scale=self.scale, window=self.window,
             max_seq_len=ctx.max_seq_len, v_transposed=cache.v_transposed, combine=not few, slopes=self.slopes,
-            v_head_dim=self.v_head_dim, sink_logit=self.sink_logit, chunk=self.chunk,
+            v_head_dim=self.v_head_dim, sink_logit=self.sink_logit, chunk=self.chunk, gate=gate, out=out,
         )
 
 
@@ -277,6 +379,8 @@ class KeysAsValuesAttention(GQAttention):
         self.norm_names = tuple(norm_names)
         self.q_norm: torch.Tensor | None = None
         self.k_norm: torch.Tensor | None = None
+
+    can_join = False
 
     def _input_projection(self, hidden_size, q_width, kv_width, names, suffix):
         return Linear(hidden_size, [q_width, kv_width], [names[0], names[1]], self.dtype, self.device, suffix=suffix)
@@ -333,6 +437,7 @@ class WholeNormAttention(GQAttention):
 
     What is cached is the normed key and the (mixed) value, so decoding reads them as they are."""
 
+    can_join = False
     can_defer_output = False
     takes_scaled_rows = False
 
@@ -470,7 +575,8 @@ def build_gqa_attention(desc: dict, dtype: torch.dtype, device, shared: dict | N
             position = POSITION_ENCODINGS.lookup(pos_desc["kind"])(pos_desc, dtype, device, shared)
             if shared is not None:
                 shared[key] = position
-    extra = {k: desc[k] for k in ("suffix", "v_head_dim", "sink_logit", "chunk", "head_norm", "gate") if k in desc}
+    extra = {k: desc[k] for k in ("suffix", "v_head_dim", "sink_logit", "chunk", "head_norm", "gate", "bias_suffix", "own_keys",
+                                 "cache_chunk") if k in desc}
     if "names" in desc:
         extra["names"] = tuple(desc["names"])
     return GQAttention(

@@ -71,7 +71,8 @@ class PagedKVNeeds:
     stream at all, the mixer keeps a single stream and gets no value pages).
 
     `window=None` keeps every token; with a window, pages that no future query can see
-    are given back.  `v_transposed` is the layout of a value page, chosen by the mixer
+    are given back; so are, with a chunk, pages of earlier stretches of `chunk` positions (counted from
+    position 0) than the next token's.  `v_transposed` is the layout of a value page, chosen by the mixer
     for the kernel that will read it: `[slot][dim]` (False) or `[dim][slot]` (True).
     Layer calls whose needs are equal share one page group.
     """
@@ -81,6 +82,7 @@ class PagedKVNeeds:
     window: int | None = None
     v_head_dim: int | None = None
     v_transposed: bool = False
+    chunk: int | None = None
 
     @property
     def value_dim(self) -> int:
@@ -290,8 +292,13 @@ class Mixer(Part):
     `ops.PendingProduct` (its last product, not made yet) instead of a tensor.
     `takes_scaled_rows`: `x` may be an `ops.ScaledRows` (a norm's output but for the rows'
     factors); the block then lets the norm before the mixer emit them, and the norm asks
-    `wants_scaled_rows(rows)` before it does so in a step of `rows` rows."""
+    `wants_scaled_rows(rows)` before it does so in a step of `rows` rows.
 
+    `can_join`: the mixer's first and last step are products, of its input and of its inner rows, and a
+    block whose sublayers read one norm may make them together with its feed-forward's
+    (`parts.joint.JointProducts` says what such a mixer offers)."""
+
+    can_join = False
     emit_partial_sums = False
     can_defer_output = False
     emit_pending_output = False
@@ -322,7 +329,17 @@ class FeedForward(Part):
     `takes_scaled_rows`: `x` may be an `ops.ScaledRows` (a norm's output but for the rows'
     factors).  `can_defer_output`, `emit_pending_output`: as for `Mixer`; here it is the
     model that sets the latter (`Block.enable_pending_output`), since the norm that follows
-    belongs to whatever comes next in the model's order."""
+    belongs to whatever comes next in the model's order.
+
+    `joint_partner()`: the gated feed-forward (the part itself, or a part inside it that runs for every
+    token and whose result is added as it is) whose products a block whose sublayers read one norm may make
+    together with its mixer's, or None.  A block that does so sets `partner_joined`: `forward` then leaves the partner out
+    (and is not called at all where the part is its own partner)."""
+
+    partner_joined = False
+
+    def joint_partner(self) -> "FeedForward | None":
+        return None
 
     emit_partial_sums = False
     takes_scaled_rows = False

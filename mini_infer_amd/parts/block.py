@@ -135,13 +135,35 @@ class ParallelBlock(Block):
 
     The add is left to whatever norm comes next, as `ops.StreamUpdate` (with the bias of the
     feed-forward's last product, where it has one, riding along): a norm that knows such an
-    update makes it in the launch that also begins the next layer."""
+    update makes it in the launch that also begins the next layer.
+
+    `joint`: the sublayers' first products are made as one, and so are their last
+    (`parts.joint.JointProducts`); of a routed feed-forward it is the shared expert that joins, and the rest is
+    added beside it.  Where nothing is added beside, the last product may be left unmade for the norm that
+    follows (`ops.PendingProduct`), or in pieces (`ops.PartialSums`), as in `PreNormBlock`."""
 
     def __init__(self, norm: Norm, mixer: Mixer, feed_forward: FeedForward | None, scale: float,
-                 names: dict[str, str], dtype: torch.dtype, device) -> None:
+                 names: dict[str, str], dtype: torch.dtype, device, *, joint: bool = False) -> None:
         super().__init__(dtype, device)
         self.norm, self.mixer, self.feed_forward = norm, mixer, feed_forward
         self.scale, self.names = float(scale), names
+        self.joint = None
+        self.beside = feed_forward  # what of the feed-forward is not made with the joint products
+        self.emit_pending_output = self.emit_partial_sums = False
+        if joint:
+            from mini_infer_amd.parts.joint import JointProducts
+
+            partner = feed_forward.joint_partner() if feed_forward is not None else None
+            if partner is not None:
+                feed_forward.partner_joined = True
+                if partner is feed_forward:
+                    self.beside = None
+            self.joint = JointProducts(mixer, partner, dtype)
+            if self.beside is None and norm.takes_pending_products:
+                norm.emit_scaled_rows = True
+                norm.scaled_rows_consumer = self.joint
+            if self.beside is not None and hasattr(self.beside, "leave_rows_apart"):
+                self.beside.leave_rows_apart = True
 
     def _children(self):
         parts = [(self.names["norm"], self.norm), (self.names["mixer"], self.mixer)]
@@ -157,6 +179,16 @@ class ParallelBlock(Block):
     def takes_pending_products(self) -> bool:  # type: ignore[override]
         return self.norm.takes_pending_products
 
+    def enable_pending_output(self) -> None:
+        self.emit_pending_output = self.joint is not None
+
+    @property
+    def takes_partial_sums(self) -> bool:  # type: ignore[override]
+        return self.joint is not None and self.norm.takes_partial_sums
+
+    def enable_partial_sums(self) -> None:
+        self.emit_partial_sums = self.joint is not None
+
     def param_specs(self, prefix: str) -> dict[str, ParamSpec]:
         specs: dict[str, ParamSpec] = {}
         for sub, part in self._children():
@@ -166,11 +198,29 @@ class ParallelBlock(Block):
     def load_params(self, prefix: str, get: TensorGetter) -> None:
         for sub, part in self._children():
             part.load_params(prefix + sub, get)
+        if self.joint is not None:
+            self.joint.join()
+
+    def _forward_joint(self, h, ctx: StepContext, cache: LayerCache, writes_cache: bool):
+        from mini_infer_amd import ops
+
+        weight = self.joint.output_weight
+        if self.beside is None and self.scale == 1.0:
+            inner = self.joint.inner_rows(h, ctx, cache, writes_cache)
+            if (self.emit_pending_output and self.dtype == torch.bfloat16
+                    and ops.pending_product_pays(inner.shape[0], *weight.shape, self.emit_partial_sums)):
+                return ops.PendingProduct(inner, weight)
+            return ops.linear(inner, weight, partial_ok=self.emit_partial_sums)
+        h = h.finish() if hasattr(h, "finish") else h
+        added = ops.linear(self.joint.inner_rows(h, ctx, cache, writes_cache), weight)
+        return ops.StreamUpdate(added, None if self.beside is None else self.beside.forward(h, ctx), None, None, self.scale)
 
     def forward(self, delta, residual: torch.Tensor, ctx: StepContext, cache: LayerCache, writes_cache: bool = True):
         from mini_infer_amd import ops
 
         h = self.norm.forward(delta, residual)
+        if self.joint is not None:
+            return self._forward_joint(h, ctx, cache, writes_cache)
         if hasattr(h, "finish"):
             h = h.finish()
         mixed = self.mixer.forward(h, ctx, cache, writes_cache)
@@ -186,14 +236,15 @@ class ParallelBlock(Block):
 @register_block("parallel")
 def build_parallel_block(desc: dict, dtype: torch.dtype, device, shared: dict | None = None) -> ParallelBlock:
     """`desc`: `norm`, `mixer`, optional `feed_forward` (descriptions with a `kind`), `scale` (the
-    number the sublayers' sum is multiplied with before it is added) and `names`."""
+    number the sublayers' sum is multiplied with before it is added), `joint` (whether the sublayers'
+    products are made together) and `names`."""
     shared = {} if shared is None else shared
     ffn = desc.get("feed_forward")
     return ParallelBlock(
         NORMS.lookup(desc["norm"]["kind"])(desc["norm"], dtype, device, shared),
         MIXERS.lookup(desc["mixer"]["kind"])(desc["mixer"], dtype, device, shared),
         FEED_FORWARDS.lookup(ffn["kind"])(ffn, dtype, device, shared) if ffn is not None else None,
-        float(desc.get("scale", 1.0)), dict(desc["names"]), dtype, device,
+        float(desc.get("scale", 1.0)), dict(desc["names"]), dtype, device, joint=bool(desc.get("joint", False)),
     )
 
 

@@ -52,6 +52,30 @@ class ScaledEmbedding(TokenEmbedding):
         return ops.embed_gather(self.weight, ctx.token_ids, self.scale)
 
 
+class LearnedPositionEmbedding(ScaledEmbedding):
+    """`table[token] * scale` plus a learned row of the token's position (which is not scaled).  A request
+    cannot grow past the rows there are (`num_positions`)."""
+
+    def __init__(self, vocab_size: int, hidden_size: int, name: str, scale: float, position_name: str, num_positions: int,
+                 dtype: torch.dtype, device) -> None:
+        super().__init__(vocab_size, hidden_size, name, scale, dtype, device)
+        if num_positions <= 0:
+            raise ValueError(f"learned positions: a positive number of rows, got {num_positions}")
+        self.position_name, self.num_positions = position_name, int(num_positions)
+        self.position_rows: torch.Tensor | None = None
+
+    def param_specs(self, prefix: str) -> dict[str, ParamSpec]:
+        return {**super().param_specs(prefix), prefix + self.position_name: ParamSpec((self.num_positions, self.hidden_size))}
+
+    def load_params(self, prefix: str, get: TensorGetter) -> None:
+        super().load_params(prefix, get)
+        self.position_rows = get(prefix + self.position_name).contiguous()
+
+    def forward(self, ctx: StepContext, cache: LayerCache | None = None) -> torch.Tensor:
+        assert self.weight is not None and self.position_rows is not None, "embedding used before its tables were loaded"
+        return ops.embed_gather(self.weight, ctx.token_ids, self.scale, self.position_rows, ctx.positions)
+
+
 SINUSOID_BASE = 10000.0
 STREAM_CAST = "stream_cast"  # key in `StepContext.shared`: (the stream, its latest copy in the compute dtype)
 
@@ -107,8 +131,11 @@ class OutputHead(Head):
         device,
         *,
         tied_to: TokenEmbedding | None = None,
+        scale: float = 1.0,
     ) -> None:
+        """`scale`: the logits are multiplied by this."""
         super().__init__(dtype, device)
+        self.scale = float(scale)
         self.hidden_size = hidden_size
         self.vocab_size = vocab_size
         self.name = name
@@ -136,7 +163,7 @@ class OutputHead(Head):
 
     def forward(self, h: torch.Tensor, ctx: StepContext | None = None) -> torch.Tensor:
         """Logits [rows, vocab] in float32."""
-        return ops.linear_f32_out(h, self.weight)
+        return ops.linear_f32_out(h, self.weight, self.scale)
 
 
 @register_embedding("token_embedding")
@@ -147,6 +174,14 @@ def build_token_embedding(desc: dict, dtype: torch.dtype, device, shared: dict |
 @register_embedding("scaled_embedding")
 def build_scaled_embedding(desc: dict, dtype: torch.dtype, device, shared: dict | None = None) -> ScaledEmbedding:
     return ScaledEmbedding(int(desc["vocab_size"]), int(desc["hidden_size"]), str(desc["name"]), float(desc["scale"]), dtype, device)
+
+
+@register_embedding("learned_position_embedding")
+def build_learned_position_embedding(desc: dict, dtype: torch.dtype, device, shared: dict | None = None) -> LearnedPositionEmbedding:
+    return LearnedPositionEmbedding(
+        int(desc["vocab_size"]), int(desc["hidden_size"]), str(desc["name"]), float(desc.get("scale", 1.0)),
+        str(desc["position_name"]), int(desc["num_positions"]), dtype, device,
+    )
 
 
 @register_embedding("scaled_sinusoid_embedding")
@@ -167,7 +202,8 @@ def build_linear_head(desc: dict, dtype: torch.dtype, device, shared: dict | Non
         if tied_to is None or not hasattr(tied_to, "weight"):
             raise ValueError("a tied output head needs the model's embedding part to hold a `weight` table")
     return OutputHead(
-        int(desc["hidden_size"]), int(desc["vocab_size"]), str(desc["name"]), dtype, device, tied_to=tied_to
+        int(desc["hidden_size"]), int(desc["vocab_size"]), str(desc["name"]), dtype, device, tied_to=tied_to,
+        scale=float(desc.get("scale", 1.0)),
     )
 
 

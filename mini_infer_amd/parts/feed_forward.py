@@ -52,6 +52,19 @@ class SwiGLU(FeedForward):
         return (self.activation == "silu" and self.dtype == torch.bfloat16
                 and ops.scaled_rows_product_takes(rows, self.gate_up.weight, self.hidden_size))
 
+    def joint_partner(self) -> "FeedForward | None":
+        return self if self.activation == "silu" else None
+
+    @property
+    def joint_limits(self) -> tuple[float, float]:
+        """`limit` and `slope` of the activation as `ops.LayerInputs` counts them (0: plain silu)."""
+        return 0.0, 1.0
+
+    def forward_projected(self, columns: torch.Tensor, out: torch.Tensor) -> None:
+        """The activation of rows [gate | up] into `out` (rows of either may be strided)."""
+        n = self.intermediate_size
+        ops.gated_mul(columns[:, :n], columns[:, n:2 * n], self.activation, out=out)
+
     def forward(self, x: "torch.Tensor | ops.ScaledRows", ctx: StepContext) -> torch.Tensor:
         assert self.gate_up.weight is not None, "SwiGLU used before its weights were loaded"
         assert self.down.weight is not None
@@ -198,7 +211,7 @@ GATE_SLOPE = 1.702  # of the logistic that gates: g * logistic(1.702 g) approxim
 
 
 class ClampedGatedFeedForward(FeedForward):
-    """Gated, with biases on all three products and both branches clamped before they meet:
+    """Gated, with biases on all three products (`biases=False`: none) and both branches clamped before they meet:
 
         g = min(W_gate x + b_gate, limit)          u = clamp(W_up x + b_up, -limit, limit)
         y = W_down (g * logistic(slope * g) * (u + 1)) + b_down
@@ -212,13 +225,13 @@ class ClampedGatedFeedForward(FeedForward):
 
     def __init__(self, hidden_size: int, intermediate_size: int, limit: float, dtype: torch.dtype, device, *,
                  slope: float = GATE_SLOPE, names: tuple[str, str, str] = ("gate", "up", "down"), suffix: str = "",
-                 bias_suffix: str = ".b") -> None:
+                 bias_suffix: str = ".b", biases: bool = True) -> None:
         super().__init__(dtype, device)
         if limit <= 0:
             raise ValueError(f"clamped gated feed-forward: the limit must be positive, got {limit}")
         self.hidden_size, self.intermediate_size = hidden_size, intermediate_size
         self.limit, self.slope = float(limit), float(slope)
-        self.names, self.suffix, self.bias_suffix = tuple(names), suffix, bias_suffix
+        self.names, self.suffix, self.bias_suffix, self.biases = tuple(names), suffix, bias_suffix, bool(biases)
         self.gate_up = Linear(hidden_size, [intermediate_size, intermediate_size], [names[0], names[1]], dtype, device, suffix=suffix)
         self.down = Linear(intermediate_size, hidden_size, names[2], dtype, device, suffix=suffix)
         self.gate_up_bias: torch.Tensor | None = None
@@ -228,8 +241,11 @@ class ClampedGatedFeedForward(FeedForward):
         return prefix + self.names[which] + self.suffix + self.bias_suffix
 
     def param_specs(self, prefix: str) -> dict[str, ParamSpec]:
+        products = {**self.gate_up.param_specs(prefix), **self.down.param_specs(prefix)}
+        if not self.biases:
+            return products
         return {
-            **self.gate_up.param_specs(prefix), **self.down.param_specs(prefix),
+            **products,
             self._bias_name(prefix, 0): ParamSpec((self.intermediate_size,), dtype="float32"),
             self._bias_name(prefix, 1): ParamSpec((self.intermediate_size,), dtype="float32"),
             self._bias_name(prefix, 2): ParamSpec((self.hidden_size,), dtype="float32"),
@@ -238,11 +254,24 @@ class ClampedGatedFeedForward(FeedForward):
     def load_params(self, prefix: str, get: TensorGetter) -> None:
         self.gate_up.load_params(prefix, get)
         self.down.load_params(prefix, get)
+        if not self.biases:
+            return
         self.gate_up_bias = torch.cat([get(self._bias_name(prefix, 0)).float(), get(self._bias_name(prefix, 1)).float()]).contiguous()
         self.output_bias = get(self._bias_name(prefix, 2)).float().contiguous()
 
+    def joint_partner(self) -> "FeedForward | None":
+        return None if self.biases else self
+
+    @property
+    def joint_limits(self) -> tuple[float, float]:
+        return self.limit, self.slope
+
+    def forward_projected(self, columns: torch.Tensor, out: torch.Tensor) -> None:
+        """As `SwiGLU.forward_projected`."""
+        ops.clamped_glu(columns[:, :2 * self.intermediate_size], self.gate_up_bias, self.limit, self.slope, out=out)
+
     def forward(self, x, ctx: StepContext) -> torch.Tensor:
-        assert self.gate_up_bias is not None, "feed-forward used before its weights were loaded"
+        assert self.gate_up_bias is not None or not self.biases, "feed-forward used before its weights were loaded"
         if isinstance(x, ops.ScaledRows):
             x = x.finish()
         assert self.gate_up.weight is not None
@@ -253,7 +282,7 @@ class ClampedGatedFeedForward(FeedForward):
 
 @register_feed_forward("clamped_glu")
 def build_clamped_gated_feed_forward(desc: dict, dtype: torch.dtype, device, shared: dict | None = None) -> ClampedGatedFeedForward:
-    extra = {k: desc[k] for k in ("slope", "suffix", "bias_suffix") if k in desc}
+    extra = {k: desc[k] for k in ("slope", "suffix", "bias_suffix", "biases") if k in desc}
     if "names" in desc:
         extra["names"] = tuple(desc["names"])
     return ClampedGatedFeedForward(int(desc["hidden_size"]), int(desc["intermediate_size"]), float(desc["limit"]), dtype, device, **extra)
@@ -267,12 +296,14 @@ class RoutedExperts(FeedForward):
         y = sum over the `top` outputs e with the largest choice of  (s_e * route_scale) * expert_e(x)
 
     The weights are the scores themselves (without the correction, not renormalized).  `scores="logistic"`:
-    every output's score is the logistic function of its own logit.  `activation="squared_relu"`: experts
+    every output's score is the logistic function of its own logit.  `scores="chosen_softmax"`: the correction is a
+    bias of the logits, the largest biased logits are chosen, and the weights are the softmax over the chosen
+    ones alone (times `route_scale`).  `activation="squared_relu"`: experts
     have no gate, `W_down relu(W_up x)^2`.  `weight_on="input"`: the weight multiplies what an expert
     READS, `y = sum expert_e(s_e * x)`; it is applied to the first product's sums, `W (s x) = s (W x)`.  The last
     `identity` router outputs stand for experts without tensors whose output is their input.  A
     shared expert of the same form may run for every token beside them, gated by one number a
-    token, `logistic(w_sg . x)`.
+    token, `logistic(w_sg . x)`, or (`shared_gated=False`) added as it is.
 
     Few rows (and every step that is recorded to be replayed) run expert by expert without the host
     knowing anything: the (token, expert) pairs are listed by expert on the device, and every chosen
@@ -291,7 +322,7 @@ class RoutedExperts(FeedForward):
     def __init__(self, hidden_size: int, intermediate_size: int, experts: int, top: int, dtype: torch.dtype, device, *,
                  identity: int = 0, route_scale: float = 1.0, correction: bool = True, shared_size: int | None = None,
                  names: dict[str, str] | None = None, scores: str = "softmax", activation: str = "silu_gated",
-                 weight_on: str = "output") -> None:
+                 weight_on: str = "output", shared_gated: bool = True) -> None:
         super().__init__(dtype, device)
         if scores not in ops.kernels.ROUTER_SCORES or activation not in ops.kernels.EXPERT_ACTIVATIONS:
             raise NotImplementedError(f"routed experts: scores {scores!r} (built: {ops.kernels.ROUTER_SCORES}), activation {activation!r} "
@@ -309,6 +340,7 @@ class RoutedExperts(FeedForward):
         self.hidden_size, self.intermediate_size = hidden_size, intermediate_size
         self.experts, self.identity, self.top, self.route_scale = experts, identity, top, float(route_scale)
         self.has_correction, self.shared_size = bool(correction), shared_size
+        self.shared_gated = bool(shared_gated)
         self.names = {"router": "router", "correction": "correction", "expert": "e{}.", "gate": "gate", "up": "up",
                       "down": "down", "shared": "shared.", "shared_gate": "shared.sg", **(names or {})}
         self.shared = None if shared_size is None else SwiGLU(
@@ -340,6 +372,7 @@ class RoutedExperts(FeedForward):
             specs[self._expert_name(prefix, e, "down")] = ParamSpec((hidden, ff))
         if self.shared is not None:
             specs.update(self.shared.param_specs(prefix))
+        if self.shared is not None and self.shared_gated:
             specs[prefix + self.names["shared_gate"]] = ParamSpec((1, hidden), dtype="float32")
         return specs
 
@@ -359,6 +392,7 @@ class RoutedExperts(FeedForward):
             self.down[e] = get(self._expert_name(prefix, e, "down"))
         if self.shared is not None:
             self.shared.load_params(prefix, get)
+        if self.shared is not None and self.shared_gated:
             self.shared_gate_row = get(prefix + self.names["shared_gate"]).float().reshape(-1).contiguous()
 
     def _grouped(self, x: torch.Tensor, ctx: StepContext) -> bool:
@@ -372,6 +406,10 @@ class RoutedExperts(FeedForward):
         expert_bytes = (3 if self.gated else 2) * self.intermediate_size * self.hidden_size * element
         return x.shape[0] * self.top * expert_bytes > self.experts * self.GROUPED_BYTES_PER_EXPERT
 
+    def joint_partner(self) -> "FeedForward | None":
+        """The shared expert, where its result is added as it is."""
+        return self.shared if self.shared is not None and not self.shared_gated else None
+
     def forward(self, x, ctx: StepContext) -> torch.Tensor:
         assert self.router is not None and self.gate_up is not None and self.down is not None, \
             "feed-forward used before its weights were loaded"
@@ -384,7 +422,7 @@ class RoutedExperts(FeedForward):
             x, self.router, self.correction, self.shared_gate_row, top=self.top, route_scale=self.route_scale, scores=self.scores,
             experts=self.experts if by_expert else None)
         shared = None
-        if self.shared is not None:
+        if self.shared is not None and not self.partner_joined:
             shared = self.shared.forward(x, ctx)
             shared = shared.finish() if hasattr(shared, "finish") else shared
         how = {"activation": self.activation, "weight_on": self.weight_on}
@@ -393,7 +431,7 @@ class RoutedExperts(FeedForward):
         elif by_expert:
             run = ops.experts_by_expert
             how["lists"] = lists[0]
-            how["combine"] = not (self.leave_rows_apart and self.weight_on == "input" and shared is None)
+            how["combine"] = not (self.leave_rows_apart and shared is None and (self.weight_on == "input" or not self.identity))
         else:
             run = ops.experts_few_rows
         return run(x, self.gate_up, self.down, chosen, weights, shared, gates, **how)
@@ -401,7 +439,8 @@ class RoutedExperts(FeedForward):
 
 @register_feed_forward("routed_experts")
 def build_routed_experts(desc: dict, dtype: torch.dtype, device, shared: dict | None = None) -> RoutedExperts:
-    extra = {k: desc[k] for k in ("identity", "route_scale", "correction", "shared_size", "names", "scores", "activation", "weight_on")
+    extra = {k: desc[k] for k in ("identity", "route_scale", "correction", "shared_size", "names", "scores", "activation", "weight_on",
+                                 "shared_gated")
              if k in desc}
     return RoutedExperts(int(desc["hidden_size"]), int(desc["intermediate_size"]), int(desc["experts"]), int(desc["top"]),
                          dtype, device, **extra)

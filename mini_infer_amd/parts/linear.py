@@ -27,7 +27,10 @@ class Linear(Part):
         device,
         *,
         suffix: str = ".weight",
+        row_step: int = 1,
     ) -> None:
+        """`row_step`: the stacked matrix is filled up with zero rows to a multiple of this (the columns of the
+        product past `out_features` are then zero; a row of the product begins on a boundary of as many elements)."""
         super().__init__(dtype, device)
         self.suffix = suffix  # what follows a block's name in the checkpoint ("" where the name is the tensor's)
         self.in_features = in_features
@@ -36,6 +39,7 @@ class Linear(Part):
         if len(self.out_splits) != len(self.names):
             raise ValueError("one name per stacked output block")
         self.out_features = sum(self.out_splits)
+        self.padded_features = -(-self.out_features // row_step) * row_step
         self.weight: torch.Tensor | None = None
 
     def param_specs(self, prefix: str) -> dict[str, ParamSpec]:
@@ -46,6 +50,8 @@ class Linear(Part):
 
     def load_params(self, prefix: str, get: TensorGetter) -> None:
         blocks = [get(prefix + name + self.suffix) for name in self.names]
+        if self.padded_features > self.out_features:
+            blocks.append(blocks[0].new_zeros((self.padded_features - self.out_features, self.in_features)))
         self.weight = (blocks[0] if len(blocks) == 1 else torch.cat(blocks, dim=0)).contiguous()
 
     def forward(self, x: torch.Tensor, partial_ok: bool = False):

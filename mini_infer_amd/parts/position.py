@@ -52,11 +52,33 @@ def llama3_inv_freq(
     return torch.where(medium, smoothed, scaled)
 
 
+def yarn_inv_freq(inv_freq: torch.Tensor, theta: float, factor: float, original: float, fast: float, slow: float) -> torch.Tensor:
+    """Frequencies rescaled by how often a pair turns within `original` positions: pairs that turn `fast` times or
+    more keep theirs, pairs that turn `slow` times or less have it divided by `factor`, and in between the two are
+    blended along the pair's number (whole numbers mark the ends of the blend)."""
+    pairs = inv_freq.numel()
+    dims = 2 * pairs
+
+    def pair_turning(times: float) -> float:
+        return dims * math.log(original / (2 * math.pi * times)) / (2 * math.log(theta))
+
+    first = max(math.floor(pair_turning(fast)), 0)
+    last = min(math.ceil(pair_turning(slow)), dims - 1)
+    blend = ((torch.arange(pairs, dtype=torch.float64) - first) / max(last - first, 0.001)).clamp(0.0, 1.0).to(inv_freq.dtype)
+    return inv_freq / factor * blend + inv_freq * (1 - blend)
+
+
+def yarn_amplitude(factor: float) -> float:
+    """What cosines and sines are multiplied by beside `yarn_inv_freq`."""
+    return 0.1 * math.log(factor) + 1.0
+
+
 class RotaryPosition(PositionEncoding):
     """Rotation of the first `rotary_dim` dims of each head.
 
     `interleaved=False` pairs dim j with j + rotary_dim/2 (the Llama way,
-    rope.py:411-416); `interleaved=True` pairs 2j with 2j+1.
+    rope.py:411-416); `interleaved=True` pairs 2j with 2j+1.  `yarn` = {"factor", "original", "fast", "slow"}:
+    frequencies rescaled by `yarn_inv_freq`, cosines and sines by `yarn_amplitude`.
     """
 
     def __init__(
@@ -70,6 +92,7 @@ class RotaryPosition(PositionEncoding):
         interleaved: bool = False,
         llama3: dict | None = None,
         exact_frequencies: bool = False,
+        yarn: dict | None = None,
     ) -> None:
         super().__init__(dtype, device)
         self.head_dim = head_dim
@@ -89,6 +112,12 @@ class RotaryPosition(PositionEncoding):
                 float(llama3["high_freq_factor"]),
                 int(llama3["original_max_position_embeddings"]),
             )
+        self.amplitude = 1.0
+        if yarn is not None:
+            if llama3 is not None:
+                raise ValueError("rotary frequencies are rescaled one way, not two")
+            table = yarn_inv_freq(table, float(theta), float(yarn["factor"]), float(yarn["original"]), float(yarn["fast"]), float(yarn["slow"]))
+            self.amplitude = yarn_amplitude(float(yarn["factor"]))
         self.inv_freq_host = table.to(torch.float32)
         self._inv_freq_device: torch.Tensor | None = None
 
@@ -102,7 +131,7 @@ class RotaryPosition(PositionEncoding):
         """cos, sin [T, rotary_dim/2] float32 for this step's positions (made once a step)."""
         key = ("rotary_tables", id(self))
         if key not in ctx.shared:
-            ctx.shared[key] = ops.rope_table(ctx.positions, self.inv_freq)
+            ctx.shared[key] = ops.rope_table(ctx.positions, self.inv_freq, self.amplitude)
         return ctx.shared[key]
 
     def rotary_layout(self) -> tuple[int, bool]:
@@ -124,6 +153,7 @@ def build_rotary(desc: dict, dtype: torch.dtype, device, shared: dict | None = N
         interleaved=bool(desc.get("interleaved", False)),
         llama3=desc.get("llama3"),
         exact_frequencies=bool(desc.get("exact_frequencies", False)),
+        yarn=desc.get("yarn"),
     )
 
 
