@@ -524,11 +524,36 @@ def figosun_config(sizes: dict, layers: int) -> dict:
             "embedding": {"scale": float(h) ** 0.5}, "layers": [layer for _ in range(layers)]}
 
 
+BEMULORN_CHUNK = 8192
+BEMULORN_EXPERTS = 16
+BEMULORN_TOP = 2
+
+
+def bemulorn_config(sizes: dict, layers: int) -> dict:
+    """A Bemulorn model with the widths of a Llama configuration, four layers at a time: one with a dense
+    clamped feed-forward of Llama's width, one with 16 experts a quarter as wide, of which a token takes 2,
+    beside a shared expert of the same width, and the two again without keys and values of their own, reading those of
+    the second.  The attention has Llama's heads, key/value heads and head size, value heads three quarters as
+    wide, half of every head rotated (frequencies rescaled by 8 from 8,192 positions), in chunks of 8,192."""
+    h, heads, kv, d = sizes["hidden_size"], sizes["num_attention_heads"], sizes["num_key_value_heads"], sizes["head_dim"]
+    ff = sizes["intermediate_size"]
+    mixer = {"heads": heads, "kv_heads": kv, "dim": d, "vdim": 3 * d // 4, "scale": d ** -0.5, "mask": {"size": BEMULORN_CHUNK},
+             "rot": {"base": 500000.0, "dims": d // 2, "scaling": {"factor": 8.0, "original": 8192, "fast": 32.0, "slow": 1.0}}}
+    dense = {"kind": "dense", "ff": ff, "limit": 7.0}
+    moe = {"kind": "moe", "expert": {"ff": ff // 4}, "shared": {"ff": ff // 4}, "router": {"experts": BEMULORN_EXPERTS, "top": BEMULORN_TOP}}
+    entries = []
+    for i in range(layers):
+        reads = {"kv_from": i - i % 4 + 1} if i % 4 >= 2 else {}
+        entries.append({"type": "attention", "mixer": {**mixer, **reads}, "mlp": moe if i % 2 else dense})
+    return {"architecture": "Bemulorn", "vocab": sizes["vocab_size"], "width": h, "norm": {"eps": 1e-6}, "max_positions": 8192,
+            "embedding": {"scale": float(h) ** 0.5}, "logit_scale": 0.5, "layers": entries}
+
+
 def model_costs(model, raw: dict, tokens: int, context: float) -> dict:
     """What a step must move and compute, from the model's own list of tensors: bytes of every matrix
     a decode step streams (tables that are only gathered from are left out), multiply-adds of its
     products per token, and per layer kind what attention reads and computes at `context` keys."""
-    gathered = {"embed", "side.embed", "model.embed_tokens.weight"}
+    gathered = {"embed", "pos", "side.embed", "model.embed_tokens.weight"}
     specs = model.param_specs()
     matrix = sum(int(s.shape[0]) * int(s.shape[1]) for n, s in specs.items() if len(s.shape) == 2 and n not in gathered)
     if "lm_head.weight" not in specs and "head" not in specs and "model.embed_tokens.weight" in specs:  # a tied head streams the embedding's table
@@ -551,6 +576,20 @@ def model_costs(model, raw: dict, tokens: int, context: float) -> dict:
         # (the latent's key and value maps are applied per head to queries and outputs: counted with the matrices)
         return {"matrix_values": matrix, "kv_values_per_request": kv_values, "state_bytes_per_request": state_bytes,
                 "prefill_flops": 2.0 * tokens * (matrix - head) + 2.0 * head + attention_flops}
+    if raw.get("architecture") == "Bemulorn":
+        # attention inside chunks, also where a layer reads another's keys and values; experts as for Kunudra
+        mixers = [l["mixer"] for l in raw["layers"]]
+        routed = [l["mlp"] for l in raw["layers"] if l["mlp"] is not None and l["mlp"]["kind"] == "moe"]
+        expert_values = sum(3 * m["expert"]["ff"] * raw["width"] for m in routed)
+        matrix -= BEMULORN_EXPERTS * expert_values
+        chunk_of = lambda m: m["mask"]["size"]  # noqa: E731
+        kv_values = sum(m["kv_heads"] * (m["dim"] + m["vdim"]) * (context % chunk_of(m) + 1) for m in mixers)
+        pairs = lambda c: sum(i % c + 1 for i in range(tokens))  # noqa: E731
+        attention_flops = sum(2.0 * pairs(chunk_of(m)) * m["heads"] * (m["dim"] + m["vdim"]) for m in mixers)
+        expert_flops = 2.0 * tokens * BEMULORN_TOP * expert_values
+        return {"matrix_values": matrix, "kv_values_per_request": kv_values, "expert_values": expert_values,
+                "experts": BEMULORN_EXPERTS, "top": BEMULORN_TOP,
+                "prefill_flops": 2.0 * tokens * (matrix - head) + 2.0 * head + attention_flops + expert_flops}
     if raw.get("architecture") == "Kunudra":
         # windowed attention: keys and values of every key/value head inside the window; latent attention:
         # one row [latent | rotated part] per token inside the window; experts: a decode step streams only
@@ -697,6 +736,9 @@ def measure_design(design: str, sizes_name: str, dtype: str, layers: int | None,
         sides = [(design, kunudra_config(sizes, layers)), ("zekonex", zekonex_config(sizes, layers)), ("llama", theirs)]
     elif design == "figosun":  # beside the other design with latent attention and routed experts, and beside Llama
         sides = [(design, figosun_config(sizes, layers)), ("kunudra", kunudra_config(sizes, layers)), ("llama", theirs)]
+    elif design == "bemulorn":  # beside the other designs with parallel layers and with routed experts, and beside Llama
+        sides = [(design, bemulorn_config(sizes, layers)), ("zekonex", zekonex_config(sizes, layers)),
+                 ("kunudra", kunudra_config(sizes, layers)), ("llama", theirs)]
     else:
         raise ValueError(f"no design {design!r} to compare")
     line = {"design": design, "sizes": f"{model_name} layer sizes", "layers": layers, "dtype": dtype, "window": DESIGN_WINDOW,
@@ -744,10 +786,10 @@ def main() -> int:
                         help="with --serving / --reference-workload: launch steps that have portions of prompts in them kernel "
                         "by kernel, however few their tokens (recorded steps of single tokens stay)")
     parser.add_argument(
-        "--design", default=None, choices=("nadosun", "zekonex", "kemurax", "kunudra", "figosun"),
+        "--design", default=None, choices=("nadosun", "zekonex", "kemurax", "kunudra", "figosun", "bemulorn"),
         help="instead of the default run: prefill (one 2,048-token prompt) and decode (batch 1, --batch and 64; --steps "
         "steps, default 64 here) of that design beside Llama at the layer sizes of --sizes and equal depth "
-        "(--layers, default 12; zekonex also beside nadosun, kemurax and kunudra beside zekonex, figosun beside kunudra); prints one JSON line and exits",
+        "(--layers, default 12; zekonex also beside nadosun, kemurax and kunudra beside zekonex, figosun beside kunudra, bemulorn beside zekonex and kunudra); prints one JSON line and exits",
     )
     parser.add_argument("--design-alone", action="store_true", help="with --design: leave the Llama side out (for profiles)")
     parser.add_argument("--attention-batch", type=int, default=0)

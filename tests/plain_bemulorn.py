@@ -24,6 +24,10 @@ def keep(a):
     return a
 
 
+def f32_round(a):
+    return np.asarray(a, dtype=np.float32).astype(np.float64)
+
+
 def bf16_round(a: np.ndarray) -> np.ndarray:
     import torch
 
@@ -66,17 +70,26 @@ def frequencies(rot: dict) -> tuple[list[float], float]:
     return blended, 0.1 * math.log(scaling["factor"]) + 1.0
 
 
-def rotate_halves(v: np.ndarray, position: int, rot: dict) -> np.ndarray:
-    """Turn the first `dims` entries of `v`, entry i with entry i + dims/2; the rest pass."""
-    turns, amplitude = frequencies(rot)
-    out = np.array(v, dtype=np.float64)
+def rotate_halves(rows: np.ndarray, position: int, rot: dict, turns=None) -> np.ndarray:
+    """Turn the first `dims` entries of every row of `rows` [n, d], entry i with entry i + dims/2; the rest
+    pass.  `turns`: what `frequencies(rot)` gives, if the caller has it."""
+    speeds, amplitude = frequencies(rot) if turns is None else turns
+    out = np.array(rows, dtype=np.float64)
     half = rot["dims"] // 2
-    for i, f in enumerate(turns):
+    for i, f in enumerate(speeds):
         angle = float(ANGLE_TYPE(position) * ANGLE_TYPE(f))
         c, s = math.cos(angle) * amplitude, math.sin(angle) * amplitude
-        out[i] = v[i] * c - v[i + half] * s
-        out[i + half] = v[i + half] * c + v[i] * s
+        out[:, i] = rows[:, i] * c - rows[:, i + half] * s
+        out[:, i + half] = rows[:, i + half] * c + rows[:, i] * s
     return out
+
+
+def rotate_all(heads: np.ndarray, rot: dict | None, store=keep) -> np.ndarray:
+    """Heads [T, n, d] of positions 0 .. T - 1, each turned by its position (no rotation: as they are)."""
+    if rot is None:
+        return heads
+    turns = frequencies(rot)
+    return store(np.stack([rotate_halves(heads[t], t, rot, turns) for t in range(heads.shape[0])]))
 
 
 def embed(tokens, weights: dict, scale: float) -> np.ndarray:
@@ -101,23 +114,20 @@ def keys_and_values(h: np.ndarray, w: dict, m: dict, store=keep) -> tuple[np.nda
     T, G = h.shape[0], m["kv_heads"]
     k = store(h @ w["k"].T + w["k.b"]).reshape(T, G, m["dim"])
     v = store(h @ w["v"].T + w["v.b"]).reshape(T, G, m["vdim"])
-    if m.get("rot") is not None:
-        k = store(np.stack([[rotate_halves(k[t, g], t, m["rot"]) for g in range(G)] for t in range(T)]))
-    return k, v
+    return rotate_all(k, m.get("rot"), store), v
 
 
 def attention(h: np.ndarray, w: dict, m: dict, keys: np.ndarray, values: np.ndarray, store=keep) -> np.ndarray:
     """Queries of h over the keys and values given (the layer's own or an earlier layer's)."""
     T, H, G, d, dv = h.shape[0], m["heads"], m["kv_heads"], m["dim"], m["vdim"]
-    q = store(h @ w["q"].T + w["q.b"]).reshape(T, H, d)
+    q = rotate_all(store(h @ w["q"].T + w["q.b"]).reshape(T, H, d), m.get("rot"), store)
     gate = logistic(store(h @ w["g"].T))  # [T, H]
     out = np.zeros((T, H, dv))
     for a in range(H):
         g = a // (H // G)
         for i in range(T):
-            turned = store(rotate_halves(q[i, a], i, m["rot"])) if m.get("rot") is not None else q[i, a]
             js = visible(i, m.get("mask"))
-            p = softmax_plus_one(keys[js.start:js.stop, g] @ turned * m["scale"])
+            p = softmax_plus_one(keys[js.start:js.stop, g] @ q[i, a] * m["scale"])
             out[i, a] = p @ values[js.start:js.stop, g] * gate[i, a]
     return store(store(out.reshape(T, H * dv)) @ w["o"].T)
 
