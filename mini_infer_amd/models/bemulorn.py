@@ -114,7 +114,7 @@ class BemulornConfig:
         entries = raw.get("layers")
         if not isinstance(entries, list) or not entries:
             raise ConfigError("config.json needs a non-empty list under 'layers'")
-        layers = tuple(_parse_layer(f"layers[{i}]", entry) for i, entry in enumerate(entries))
+        layers = tuple(_parse_layer(f"layers[{i}]", _with_sources_sizes(entry, entries)) for i, entry in enumerate(entries))
         for i, layer in enumerate(layers):
             _check_source(i, layer, layers)
         return cls(
@@ -127,6 +127,18 @@ class BemulornConfig:
             norm_eps=_positive("norm.eps", _section(raw, "norm").get("eps")),
             layers=layers,
         )
+
+
+def _with_sources_sizes(entry: Any, entries: list) -> Any:
+    """A layer that reads another's keys and values may leave out what has to equal that layer's."""
+    mixer = entry.get("mixer") if isinstance(entry, dict) else None
+    source = mixer.get("kv_from") if isinstance(mixer, dict) else None
+    if not isinstance(source, int) or isinstance(source, bool) or not 0 <= source < len(entries) or not isinstance(entries[source], dict):
+        return entry
+    theirs = entries[source].get("mixer")
+    if not isinstance(theirs, dict):
+        return entry
+    return {**entry, "mixer": {**{key: theirs[key] for key in ("kv_heads", "dim", "vdim", "rot") if key in theirs}, **mixer}}
 
 
 def _check_source(i: int, layer: BemulornLayer, layers: tuple[BemulornLayer, ...]) -> None:

@@ -400,8 +400,10 @@ def gemm_skinny_bf16(a: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
     return c
 
 
-def linear_f32_out(x: torch.Tensor, weight: torch.Tensor, scale: float = 1.0) -> torch.Tensor:
+def linear_f32_out(x: torch.Tensor, weight: torch.Tensor, scale: float = 1.0, scale_row: torch.Tensor | None = None) -> torch.Tensor:
     """`x @ weight.T` as float32, times `scale`, whatever the operands' dtype: what an output head returns.
+    `scale_row`: the scale once more as a float32 tensor of one entry on the device (with it the widening and
+    the scaling of the library's product are one launch).
 
     Few bfloat16 rows: the weight-streaming kernel writes float32 itself (no cast launch); its
     values are those of `linear(...).float()`, rounded to bfloat16 on the way, so that a row's
@@ -431,8 +433,10 @@ def linear_f32_out(x: torch.Tensor, weight: torch.Tensor, scale: float = 1.0) ->
             )
         )
         return out
-    logits = torch.matmul(x, weight.t()).float()
-    return logits if scale == 1.0 else logits.mul_(scale)
+    product = torch.matmul(x, weight.t())
+    if scale == 1.0:
+        return product.float()
+    return torch.mul(product, scale_row) if scale_row is not None else product.float().mul_(scale)
 
 
 def skinny_gemm_takes(m: int, k: int, lda: int, ldw: int, max_rows: int = SKINNY_MAX_ROWS) -> bool:

@@ -207,6 +207,8 @@ class ParallelBlock(Block):
         weight = self.joint.output_weight
         if self.beside is None and self.scale == 1.0:
             inner = self.joint.inner_rows(h, ctx, cache, writes_cache)
+            if self.joint.apart_out(inner.shape[0]):
+                return ops.StreamUpdate(*self.joint.outputs(inner))
             if (self.emit_pending_output and self.dtype == torch.bfloat16
                     and ops.pending_product_pays(inner.shape[0], *weight.shape, self.emit_partial_sums)):
                 return ops.PendingProduct(inner, weight)

@@ -136,6 +136,7 @@ class OutputHead(Head):
         """`scale`: the logits are multiplied by this."""
         super().__init__(dtype, device)
         self.scale = float(scale)
+        self._scale_row: torch.Tensor | None = None  # the scale on the device
         self.hidden_size = hidden_size
         self.vocab_size = vocab_size
         self.name = name
@@ -154,6 +155,8 @@ class OutputHead(Head):
     def load_params(self, prefix: str, get: TensorGetter) -> None:
         if self.tied_to is None:
             self._weight = get(prefix + self.name).contiguous()
+        if self.scale != 1.0:
+            self._scale_row = torch.full((1,), self.scale, dtype=torch.float32, device=self.device)
 
     @property
     def weight(self) -> torch.Tensor:
@@ -163,7 +166,7 @@ class OutputHead(Head):
 
     def forward(self, h: torch.Tensor, ctx: StepContext | None = None) -> torch.Tensor:
         """Logits [rows, vocab] in float32."""
-        return ops.linear_f32_out(h, self.weight, self.scale)
+        return ops.linear_f32_out(h, self.weight, self.scale, self._scale_row)
 
 
 @register_embedding("token_embedding")

@@ -12,7 +12,9 @@ both results are sums, the two last ones are one product with the matrices side 
 (the sum of the sublayers is then rounded once, not three times).  A layer is two products of
 twice the size with the mixer's own work between them: at few rows the weights of a whole layer stream
 through two launches, and the first of them ends with everything that follows it row by row
-(`ops.layer_in`); a prompt's products are larger ones.
+(`ops.layer_in`).  For many rows the vendor library makes both products and the pieces of a very large one are
+faster apart, so a prompt takes the parts' own views of the stacked matrices where they are (`apart_in`,
+`apart_out`).
 
 What a mixer that joins offers (`Mixer.can_join`): `joint_input` and `joint_output` (its first and
 last `Linear`), `joint_layout(ff, limit, slope)` (how the stacked rows lie), `rotation()`,
@@ -30,6 +32,18 @@ from mini_infer_amd import ops
 from mini_infer_amd.parts.base import FeedForward, LayerCache, Mixer, StepContext
 
 ROW_STEP = 8  # rows of stacked products and of joined inner rows begin on boundaries of as many elements
+
+
+# Where bfloat16 products are made apart (bfloat16 only; the 32-bit engine's own product has no such choice).
+# The first product, by rows x stacked features, microseconds together / apart at 8B and 1B widths:
+#     512 x 34592    147 / 128      1024 x 13088    96 / 108      256 x 34592     83 / 94
+#     2048 x 34592   466 / 430      2048 x 11296   255 / 155      2048 x 6176     59 / 61
+#     4096 x 34592   936 / 794      2048 x 19360   182 / 130      1024 x 19360    81 / 75
+APART_IN_OUTPUTS = 1 << 24
+# The last product, by rows and by K (3072 + 14336, 1536 + 8192, 3072 + 3584 into 4096 or 2048 features), 256 /
+# 512 / 2048 rows: 113 / 70, 176 / 100, 377 / 239; 28 / 43, 33 / 47, 78 / 87; 25 / 40, 41 / 45, 91 / 98.  (Up to
+# 128 rows a long K goes to the engine's own product in pieces.)
+APART_OUT_ROWS, APART_OUT_K = 128, 12288
 
 
 def _aligned(count: int) -> int:
@@ -93,8 +107,23 @@ class JointProducts:
             self.mixer.forward_layer_in(h, self.input_weight, self.layout, ctx, cache, writes_cache, activated, mixed)
         else:
             h = h.finish() if isinstance(h, ops.ScaledRows) else h
-            columns = ops.linear(h, self.input_weight)
-            self.mixer.forward_projected(columns[:, : self.mixer_columns], ctx, cache, writes_cache, mixed)
+            if self.partner is not None and self.dtype == torch.bfloat16 and rows.shape[0] * self.input_weight.shape[0] >= APART_IN_OUTPUTS:
+                own, gated = ops.linear(h, self.mixer.joint_input.weight), ops.linear(h, self.partner.gate_up.weight)
+            else:
+                columns = ops.linear(h, self.input_weight)
+                own, gated = columns[:, : self.mixer_columns], columns[:, self.mixer_columns: self.mixer_columns + 2 * self.ff]
+            self.mixer.forward_projected(own, ctx, cache, writes_cache, mixed)
             if self.partner is not None:
-                self.partner.forward_projected(columns[:, self.mixer_columns: self.mixer_columns + 2 * self.ff], activated)
+                self.partner.forward_projected(gated, activated)
         return joined[:, : self.inner + self.ff]
+
+    def apart_out(self, rows: int) -> bool:
+        """Whether the last product of so many rows is made in its two parts."""
+        return (self.partner is not None and self.dtype == torch.bfloat16 and rows > APART_OUT_ROWS
+                and self.inner + self.ff >= APART_OUT_K)
+
+    def outputs(self, joined: torch.Tensor) -> tuple[torch.Tensor, torch.Tensor]:
+        """The two parts of the last product of `inner_rows`."""
+        assert self.partner is not None
+        return (ops.linear(joined[:, : self.inner], self.mixer.joint_output.weight),
+                ops.linear(joined[:, self.inner:], self.partner.down.weight))

@@ -80,6 +80,14 @@ def test_configurations_the_design_does_not_have_are_refused(change, message):
         architecture_for(cfg).parse_config(cfg)
 
 
+def test_a_reader_may_leave_out_what_equals_its_source():
+    cfg = json.loads(json.dumps(tb.CONFIGS["A"][0]))
+    for key in ("kv_heads", "dim", "vdim", "rot"):
+        del cfg["layers"][1]["mixer"][key]
+    parse = architecture_for(cfg).parse_config
+    assert parse(cfg) == parse(tb.CONFIGS["A"][0])
+
+
 def test_the_number_of_positions_may_be_the_tables_alone():
     cfg = {k: v for k, v in tb.CONFIGS["D"][0].items() if k != "max_positions"}
     arch = architecture_for(cfg)

@@ -113,6 +113,9 @@ def test_logits_times_a_number(dtype, rows):
     scaled = ops.linear_f32_out(dev(h, TORCH[dtype]), dev(w, TORCH[dtype]), 1.75).cpu().numpy()
     plain = ops.linear_f32_out(dev(h, TORCH[dtype]), dev(w, TORCH[dtype])).cpu().numpy()
     np.testing.assert_array_equal(scaled, plain * np.float32(1.75))
+    one_launch = ops.linear_f32_out(dev(h, TORCH[dtype]), dev(w, TORCH[dtype]), 1.75, dev(np.array([1.75], dtype=np.float32)))
+    assert one_launch.dtype == torch.float32
+    np.testing.assert_array_equal(one_launch.cpu().numpy(), scaled)
     np.testing.assert_allclose(plain, rounded(h, dtype) @ rounded(w, dtype).T, rtol=0, atol=tolerance(dtype, 30))
 
 
@@ -538,6 +541,36 @@ def test_products_made_together_and_apart_agree(folders, dtype, name):
                        runner_for(folder, dtype, block, pages=8, seats=1, graphs=graphs)):
             got = np.concatenate([runner.step([StepEntry("a", part, list(range(len(part))))]).cpu().numpy() for part in portions])
             assert_close(got, want, dtype, f"{name} graphs={graphs}", bf16_max_factor=2.5)
+
+
+@pytest.mark.parametrize("name", ["A", "C", "E"])
+def test_a_prompts_products_made_in_their_two_parts_agree_too(folders, name, monkeypatch):
+    """What very large products of many rows do, with limits so low that the tiny ones do it: the parts' own views of
+    the stacked matrices, in whole prompts, portions and decoded tokens."""
+    from mini_infer_amd.engine import StepEntry
+    from mini_infer_amd.parts import joint
+
+    name, cfg, block, weights, folder = folders[name, "bfloat16"]
+    tokens = tb.random_tokens(cfg, 60, seed=17)
+    want = oracle(name, cfg, weights, tokens)
+    made = {"out": 0}
+    original = joint.JointProducts.outputs
+
+    def counted(self, joined):
+        made["out"] += 1
+        return original(self, joined)
+
+    monkeypatch.setattr(joint.JointProducts, "outputs", counted)
+    for rows, outputs in ((2, 1), (0, 1), (2, 1 << 40)):
+        monkeypatch.setattr(joint, "APART_IN_OUTPUTS", outputs)
+        monkeypatch.setattr(joint, "APART_OUT_ROWS", rows)
+        monkeypatch.setattr(joint, "APART_OUT_K", 0)
+        before = made["out"]
+        runner = runner_for(folder, "bfloat16", block, pages=8, seats=1, graphs=False)
+        portions = [tokens[:40], tokens[40:42]] + [[t] for t in tokens[42:]]
+        got = np.concatenate([runner.step([StepEntry("a", part, list(range(len(part))))]).cpu().numpy() for part in portions])
+        assert_close(got, want, "bfloat16", f"{name} {rows} {outputs}", bf16_max_factor=2.5)
+        assert made["out"] > before
 
 
 def test_a_step_past_the_table_of_positions_is_refused_and_changes_nothing(tmp_path):
